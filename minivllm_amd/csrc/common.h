@@ -113,6 +113,12 @@ __device__ __forceinline__ void store4_stream(void* p, uint32_t v) {
 
 __device__ __forceinline__ float fast_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
 
+// A softmax denominator l, counted in units of 2^m, with one further term exp(sink): a learned number per query head
+// that has neither key nor value.  A row that saw no key (m = -inf) keeps its zero.
+__device__ __forceinline__ float add_sink(float l, float m, float sink) {
+  return m == -INFINITY ? l : l + fast_exp2(sink * kLog2e - m);
+}
+
 // x / d for many x and one d: r = 1 / d is computed once (correctly rounded), then each quotient costs a
 // multiply and two FMAs instead of a full division sequence: q = x r, q + (x - q d) r.  With a correctly rounded
 // reciprocal the corrected quotient is the correctly rounded x / d for normal operands (Markstein), up to rare

@@ -66,6 +66,7 @@ struct DecodeArgs {
   int num_parts;          // partitions per sequence in the grid / workspace
   float scale_log2;       // scale * log2(e)
   int head_chunks;        // MFMA kernels: slices of up to 16 query heads per kv head (1 unless a kv head has more than 16)
+  const float* sink;      // [num_heads] or null: one more exp(sink) in a head's denominator (added where it is inverted)
 };
 
 // The query heads one wave of the MFMA kernels works for.  A wave holds up to 16 query heads as the 16 columns of its
@@ -288,6 +289,7 @@ __device__ __forceinline__ void finish_head(HEAD& hd, const DecodeArgs& a, int b
   hd.l += __shfl_xor(hd.l, 32, 64);
   if (direct) {
     T* out = reinterpret_cast<T*>(a.out);
+    if (a.sink != nullptr && (lane & 15) < group) hd.l = add_sink(hd.l, hd.m, a.sink[head0 + (lane & 15)]);
     const float linv = hd.l > 0.f ? 1.f / hd.l : 0.f;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
@@ -1370,6 +1372,7 @@ __global__ __launch_bounds__(64) void decode_generic_kernel(const DecodeArgs a) 
 
   if (direct) {
     T* out = reinterpret_cast<T*>(a.out) + ((int64_t)b * a.num_heads + h) * D;
+    if (a.sink != nullptr) l = add_sink(l, m, a.sink[h]);
     const float linv = l > 0.f ? 1.f / l : 0.f;
 #pragma unroll
     for (int r = 0; r < kGenericMaxR; ++r) {
@@ -1432,6 +1435,7 @@ __global__ __launch_bounds__(256) void decode_reduce_kernel(const DecodeArgs a) 
     mx = mn;
   }
   T* out = reinterpret_cast<T*>(a.out) + ((int64_t)b * a.num_heads + h) * D;
+  if (a.sink != nullptr) lsum = add_sink(lsum, mx, a.sink[h]);
   const float linv = lsum > 0.f ? 1.f / lsum : 0.f;
 #pragma unroll
   for (int r = 0; r < kGenericMaxR; ++r) {
@@ -1484,6 +1488,7 @@ __global__ __launch_bounds__(256) void decode_reduce_vec_kernel(const DecodeArgs
       }
     }
   }
+  if (a.sink != nullptr) lsum = add_sink(lsum, mx, a.sink[h]);
   const float linv = lsum > 0.f ? 1.f / lsum : 0.f;
   T o4[4];
 #pragma unroll
@@ -1653,7 +1658,7 @@ static int decode_entry(void* out, const void* q, const void* k_cache, const voi
                         const float* k_scale, const float* v_scale, bool int8,
                         const int32_t* block_tables, int max_num_blocks, const void* context_lens,
                         int ctx_is_i64, int batch, int num_heads, int num_kv_heads, int head_dim,
-                        int block_size, int64_t num_blocks, float scale, int dtype, void* workspace,
+                        int block_size, int64_t num_blocks, float scale, const float* sink, int dtype, void* workspace,
                         size_t workspace_bytes, void* stream) {
   const int bad = decode_check(out, q, k_cache, v_cache, k_scale, v_scale, int8, block_tables, max_num_blocks,
                                context_lens, batch, num_heads, num_kv_heads, head_dim, block_size, num_blocks, dtype);
@@ -1675,6 +1680,7 @@ static int decode_entry(void* out, const void* q, const void* k_cache, const voi
   a.part_tokens = plan.part_tokens;
   a.num_parts = plan.num_parts;
   a.scale_log2 = scale * kLog2e;
+  a.sink = sink;
   a.ws_acc = nullptr; a.ws_ml = nullptr;
   if (a.num_parts > 1) {
     const size_t need = workspace_bytes_for(batch, num_heads, head_dim, max_num_blocks, block_size);
@@ -1758,7 +1764,17 @@ extern "C" int mvllm_paged_decode(void* out, const void* q, const void* k_cache,
                                   size_t workspace_bytes, void* stream) {
   return decode_entry(out, q, k_cache, v_cache, nullptr, nullptr, false, block_tables, max_num_blocks,
                       context_lens, ctx_is_i64, batch, num_heads, num_kv_heads, head_dim, block_size,
-                      num_blocks, scale, dtype, workspace, workspace_bytes, stream);
+                      num_blocks, scale, nullptr, dtype, workspace, workspace_bytes, stream);
+}
+
+extern "C" int mvllm_paged_decode_sink(void* out, const void* q, const void* k_cache, const void* v_cache,
+                                       const int32_t* block_tables, int max_num_blocks, const void* context_lens,
+                                       int ctx_is_i64, int batch, int num_heads, int num_kv_heads, int head_dim,
+                                       int block_size, int64_t num_blocks, float scale, const float* sink, int dtype,
+                                       void* workspace, size_t workspace_bytes, void* stream) {
+  return decode_entry(out, q, k_cache, v_cache, nullptr, nullptr, false, block_tables, max_num_blocks,
+                      context_lens, ctx_is_i64, batch, num_heads, num_kv_heads, head_dim, block_size,
+                      num_blocks, scale, sink, dtype, workspace, workspace_bytes, stream);
 }
 
 // ---------------------------------------------------------------------------
@@ -1814,7 +1830,7 @@ extern "C" int mvllm_paged_decode_noalloc(void* out, const void* q, const void* 
   // all run), so nothing in the array has to start at zero.
   return decode_entry(out, q, k_cache, v_cache, nullptr, nullptr, false, block_tables, max_num_blocks,
                       context_lens, ctx_is_i64, batch, num_heads, num_kv_heads, head_dim, block_size,
-                      num_blocks, scale, dtype, ws, kStaticScratchBytes, stream);
+                      num_blocks, scale, nullptr, dtype, ws, kStaticScratchBytes, stream);
 }
 
 extern "C" int mvllm_paged_decode_int8(void* out, const void* q, const int8_t* k_cache, const int8_t* v_cache,
@@ -1825,5 +1841,5 @@ extern "C" int mvllm_paged_decode_int8(void* out, const void* q, const int8_t* k
                                        size_t workspace_bytes, void* stream) {
   return decode_entry(out, q, k_cache, v_cache, k_scale, v_scale, true, block_tables, max_num_blocks,
                       context_lens, ctx_is_i64, batch, num_heads, num_kv_heads, head_dim, block_size,
-                      num_blocks, scale, dtype, workspace, workspace_bytes, stream);
+                      num_blocks, scale, nullptr, dtype, workspace, workspace_bytes, stream);
 }

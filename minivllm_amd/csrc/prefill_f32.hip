@@ -232,7 +232,7 @@ __global__ __launch_bounds__(64 * kPfWaves, 2) void prefill_f32_kernel(const Pre
   // ---- output: lane (row l32, hi) holds dims 32 t + 8 (r / 4) + 4 hi + r % 4 ----
   const float row_sum = sum_with_lane_xor32(l);   // (every lane takes part in the exchange)
   if (active && qrow < seq_len) {
-    const float inv = 1.f / row_sum;
+    const float inv = 1.f / (a.sink != nullptr ? add_sink(row_sum, m, a.sink[h]) : row_sum);
     float* dst = reinterpret_cast<float*>(a.out) + ((int64_t)(seq_start + qrow) * a.num_heads + h) * D;
 #pragma unroll
     for (int t = 0; t < kTD; ++t)

@@ -42,6 +42,7 @@ struct PrefillArgs {
   const int32_t* q_pos = nullptr;
   float* lse = nullptr;
   int64_t q_period = 0;
+  const float* sink = nullptr;   // optional, [num_heads]: one more exp(sink) in a row's denominator (not with lse: the merge adds it)
   int band_shift = 0;   // MFMA path: log2 of the row tiles per band of the item order (locate_banded)
 };
 
@@ -712,7 +713,8 @@ __global__ __launch_bounds__(64 * kPfWaves, D == 256 ? 1 : 2) void prefill_mfma_
   if (!active) return;
   char* ot = &lds.k[0][0] + wave * (kWaveRows * kRowB);   // 4 waves x 32 rows = both K buffers
   {
-    const float lt = l + __shfl_xor(l, 32, 64);
+    float lt = l + __shfl_xor(l, 32, 64);
+    if (a.sink != nullptr) lt = add_sink(lt, -neg_m[0], a.sink[h]);
     const float inv = 1.f / lt;
     if (PAGED && a.lse != nullptr && hi == 0 && qrow < seq_len)
       a.lse[(int64_t)(seq_start + qrow) * a.num_heads + h] = __log2f(lt) - neg_m[0];

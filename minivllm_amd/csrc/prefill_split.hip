@@ -99,6 +99,7 @@ struct MergeArgs {
   const float* lse;        // [splits * total_q, Hq]
   const int32_t* cu_seqlens_q;
   const int32_t* ws_cu_k;
+  const float* sink;       // [Hq] or null: one more exp(sink) in every row's denominator
   int num_seqs;
   int splits;
   int total_q;
@@ -153,6 +154,7 @@ __global__ __launch_bounds__(256) void split_merge_kernel(const MergeArgs a) {
       acc[2 * e + 1] = w != 0.f ? fmaf(w, hi_to_float<T>(words[e]), acc[2 * e + 1]) : acc[2 * e + 1];
     }
   }
+  if (a.sink != nullptr) den = add_sink(den, top, a.sink[h]);
   const float inv = den > 0.f ? 1.f / den : 0.f;
   uint4 o;
   o.x = pack2<T>(acc[0] * inv, acc[1] * inv);
@@ -262,7 +264,7 @@ static int run_split(void* out, const void* q, const void* k_cache, const void* 
                      const float* v_scale, bool int8, const int32_t* block_tables, int max_num_blocks,
                      const int32_t* cu_seqlens_q, const int32_t* cu_seqlens_k, int num_seqs, int64_t total_q_tokens,
                      int max_kv_len, int num_heads, int num_kv_heads, int head_dim, int block_size, int64_t num_blocks,
-                     float scale, int dtype, int splits, void* workspace, size_t workspace_bytes, void* stream) {
+                     float scale, const float* sink, int dtype, int splits, void* workspace, size_t workspace_bytes, void* stream) {
   if (dtype_size(dtype) == 0) return MVLLM_ERR_BAD_DTYPE;
   if (num_seqs < 0 || total_q_tokens < 0 || max_kv_len < 0 || num_heads <= 0 || num_kv_heads <= 0 || head_dim <= 0 ||
       block_size <= 0 || num_blocks < 0 || max_num_blocks < 0 || num_heads % num_kv_heads != 0 || !(scale > 0.f))
@@ -308,6 +310,7 @@ static int run_split(void* out, const void* q, const void* k_cache, const void* 
 
   MergeArgs m;
   m.out = out; m.part = part; m.lse = lse; m.cu_seqlens_q = cu_seqlens_q; m.ws_cu_k = sp.ws_cu_k;
+  m.sink = sink;
   m.num_seqs = num_seqs; m.splits = splits; m.total_q = (int)total_q_tokens; m.num_heads = num_heads; m.head_dim = head_dim;
   const int heads_per_wg = 256 / (head_dim / 8);
   const dim3 grid((unsigned)total_q_tokens, (unsigned)((num_heads + heads_per_wg - 1) / heads_per_wg));
@@ -323,7 +326,18 @@ extern "C" int mvllm_prefill_paged_split(void* out, const void* q, const void* k
                                          float scale, int dtype, int splits, void* workspace, size_t workspace_bytes,
                                          void* stream) {
   return run_split(out, q, k_cache, v_cache, nullptr, nullptr, false, block_tables, max_num_blocks, cu_seqlens_q, cu_seqlens_k,
-                   num_seqs, total_q_tokens, max_kv_len, num_heads, num_kv_heads, head_dim, block_size, num_blocks, scale, dtype,
+                   num_seqs, total_q_tokens, max_kv_len, num_heads, num_kv_heads, head_dim, block_size, num_blocks, scale, nullptr, dtype,
+                   splits, workspace, workspace_bytes, stream);
+}
+
+extern "C" int mvllm_prefill_paged_split_sink(void* out, const void* q, const void* k_cache, const void* v_cache,
+                                              const int32_t* block_tables, int max_num_blocks, const int32_t* cu_seqlens_q,
+                                              const int32_t* cu_seqlens_k, int num_seqs, int64_t total_q_tokens, int max_kv_len,
+                                              int num_heads, int num_kv_heads, int head_dim, int block_size, int64_t num_blocks,
+                                              float scale, const float* sink, int dtype, int splits, void* workspace,
+                                              size_t workspace_bytes, void* stream) {
+  return run_split(out, q, k_cache, v_cache, nullptr, nullptr, false, block_tables, max_num_blocks, cu_seqlens_q, cu_seqlens_k,
+                   num_seqs, total_q_tokens, max_kv_len, num_heads, num_kv_heads, head_dim, block_size, num_blocks, scale, sink, dtype,
                    splits, workspace, workspace_bytes, stream);
 }
 
@@ -334,6 +348,6 @@ extern "C" int mvllm_prefill_paged_int8_split(void* out, const void* q, const in
                                               int num_kv_heads, int head_dim, int block_size, int64_t num_blocks, float scale,
                                               int dtype, int splits, void* workspace, size_t workspace_bytes, void* stream) {
   return run_split(out, q, k_cache, v_cache, k_scale, v_scale, true, block_tables, max_num_blocks, cu_seqlens_q, cu_seqlens_k,
-                   num_seqs, total_q_tokens, max_kv_len, num_heads, num_kv_heads, head_dim, block_size, num_blocks, scale, dtype,
+                   num_seqs, total_q_tokens, max_kv_len, num_heads, num_kv_heads, head_dim, block_size, num_blocks, scale, nullptr, dtype,
                    splits, workspace, workspace_bytes, stream);
 }

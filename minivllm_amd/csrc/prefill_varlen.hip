@@ -81,6 +81,7 @@ __global__ __launch_bounds__(256) void prefill_generic_kernel(const PrefillArgs 
       m = m_new;
     }
     T* op = out + (int64_t)(seq_start + r) * qrow + (int64_t)h * D;
+    if (a.sink != nullptr) l = add_sink(l, m, a.sink[h]);
     const float linv = l > 0.f ? 1.f / l : 0.f;
 #pragma unroll
     for (int i = 0; i < kGenMaxR; ++i) {
@@ -179,10 +180,9 @@ extern "C" int mvllm_prefill_plan(int num_heads, int num_kv_heads, int head_dim,
   return MVLLM_OK;
 }
 
-extern "C" int mvllm_prefill_varlen(void* out, const void* q, const void* k, const void* v,
-                                    const int32_t* cu_seqlens, int num_seqs, int64_t total_tokens,
-                                    int num_heads, int num_kv_heads, int head_dim, float scale, int dtype,
-                                    void* stream) {
+static int prefill_varlen_entry(void* out, const void* q, const void* k, const void* v, const int32_t* cu_seqlens,
+                                int num_seqs, int64_t total_tokens, int num_heads, int num_kv_heads, int head_dim,
+                                float scale, const float* sink, int dtype, void* stream) {
   if (dtype_size(dtype) == 0) return MVLLM_ERR_BAD_DTYPE;
   if (num_seqs < 0 || total_tokens < 0 || num_heads <= 0 || num_kv_heads <= 0 || head_dim <= 0)
     return MVLLM_ERR_BAD_SHAPE;
@@ -197,12 +197,12 @@ extern "C" int mvllm_prefill_varlen(void* out, const void* q, const void* k, con
   a.num_kv_heads = num_kv_heads; a.head_dim = head_dim; a.scale_log2 = scale * kLog2e;
   a.tiles_x = 0; a.heads_y = 0; a.band_bits = 0;
   a.cu_seqlens_k = nullptr; a.block_tables = nullptr; a.max_num_blocks = 0; a.block_size = 0; a.num_blocks = 0;
-  a.k_scale = nullptr; a.v_scale = nullptr;
+  a.k_scale = nullptr; a.v_scale = nullptr; a.sink = sink;
   const bool aligned = aligned16(q) && aligned16(k) && aligned16(v) && aligned16(out);
   const int kind = aligned ? prefill_kernel_for(num_heads, num_kv_heads, head_dim, 0, dtype, false, false) : 0;
   const bool mfma_ok = kind == 2;
   if (mfma_ok && dtype == MVLLM_F32) return launch_prefill_f32(a, false, (hipStream_t)stream);
-  if (mfma_ok && scale > 0.f && prefill_pp_takes(num_seqs, num_heads, num_kv_heads, head_dim, dtype, 0)) {
+  if (mfma_ok && !sink && scale > 0.f && prefill_pp_takes(num_seqs, num_heads, num_kv_heads, head_dim, dtype, 0)) {
     PrefillPpArgs p;
     p.out = out; p.q = q; p.k = k; p.v = v; p.cu_seqlens = cu_seqlens; p.total_tokens = total_tokens;
     p.num_seqs = num_seqs; p.num_heads = num_heads; p.num_kv_heads = num_kv_heads; p.scale_log2 = scale * kLog2e;
@@ -212,6 +212,7 @@ extern "C" int mvllm_prefill_varlen(void* out, const void* q, const void* k, con
     return launch_prefill_pp(p, dtype, (hipStream_t)stream);
   }
   // fp32, and 16-bit head dims 32, 80, 96, 112 and 256: 16-row tiles on the decode kernel's tile arithmetic (paged_decode.hip)
+  if (kind == 1 && sink) return MVLLM_ERR_UNSUPPORTED;
   if (kind == 1) {
     PrefillRowsArgs r;
     r.out = out; r.q = q; r.k = k; r.v = v; r.cu_seqlens = cu_seqlens; r.total_tokens = total_tokens;
@@ -223,11 +224,27 @@ extern "C" int mvllm_prefill_varlen(void* out, const void* q, const void* k, con
   return prefill_dispatch<false>(a, dtype, mfma_ok, (hipStream_t)stream);
 }
 
-extern "C" int mvllm_prefill_paged(void* out, const void* q, const void* k_cache, const void* v_cache,
-                                   const int32_t* block_tables, int max_num_blocks, const int32_t* cu_seqlens_q,
-                                   const int32_t* cu_seqlens_k, int num_seqs, int64_t total_q_tokens,
-                                   int num_heads, int num_kv_heads, int head_dim, int block_size,
-                                   int64_t num_blocks, float scale, int dtype, void* stream) {
+extern "C" int mvllm_prefill_varlen(void* out, const void* q, const void* k, const void* v,
+                                    const int32_t* cu_seqlens, int num_seqs, int64_t total_tokens,
+                                    int num_heads, int num_kv_heads, int head_dim, float scale, int dtype,
+                                    void* stream) {
+  return prefill_varlen_entry(out, q, k, v, cu_seqlens, num_seqs, total_tokens, num_heads, num_kv_heads, head_dim, scale,
+                              nullptr, dtype, stream);
+}
+
+extern "C" int mvllm_prefill_varlen_sink(void* out, const void* q, const void* k, const void* v,
+                                         const int32_t* cu_seqlens, int num_seqs, int64_t total_tokens,
+                                         int num_heads, int num_kv_heads, int head_dim, float scale,
+                                         const float* sink, int dtype, void* stream) {
+  return prefill_varlen_entry(out, q, k, v, cu_seqlens, num_seqs, total_tokens, num_heads, num_kv_heads, head_dim, scale,
+                              sink, dtype, stream);
+}
+
+static int prefill_paged_entry(void* out, const void* q, const void* k_cache, const void* v_cache,
+                               const int32_t* block_tables, int max_num_blocks, const int32_t* cu_seqlens_q,
+                               const int32_t* cu_seqlens_k, int num_seqs, int64_t total_q_tokens,
+                               int num_heads, int num_kv_heads, int head_dim, int block_size,
+                               int64_t num_blocks, float scale, const float* sink, int dtype, void* stream) {
   if (dtype_size(dtype) == 0) return MVLLM_ERR_BAD_DTYPE;
   if (num_seqs < 0 || total_q_tokens < 0 || num_heads <= 0 || num_kv_heads <= 0 || head_dim <= 0 ||
       block_size <= 0 || num_blocks < 0 || max_num_blocks < 0)
@@ -245,11 +262,12 @@ extern "C" int mvllm_prefill_paged(void* out, const void* q, const void* k_cache
   a.tiles_x = 0; a.heads_y = 0; a.band_bits = 0;
   a.cu_seqlens_k = cu_seqlens_k; a.block_tables = block_tables; a.max_num_blocks = max_num_blocks;
   a.block_size = block_size; a.num_blocks = num_blocks; a.k_scale = nullptr; a.v_scale = nullptr;
+  a.sink = sink;
   const bool aligned = aligned16(q) && aligned16(k_cache) && aligned16(v_cache) && aligned16(out);
   const int kind = aligned ? prefill_kernel_for(num_heads, num_kv_heads, head_dim, block_size, dtype, true, false) : 0;
   const bool mfma_ok = kind == 2;
   if (mfma_ok && dtype == MVLLM_F32) return launch_prefill_f32(a, true, (hipStream_t)stream);
-  if (mfma_ok && scale > 0.f && prefill_pp_takes(num_seqs, num_heads, num_kv_heads, head_dim, dtype, block_size)) {
+  if (mfma_ok && !sink && scale > 0.f && prefill_pp_takes(num_seqs, num_heads, num_kv_heads, head_dim, dtype, block_size)) {
     PrefillPpArgs p;
     p.out = out; p.q = q; p.k = k_cache; p.v = v_cache; p.cu_seqlens = cu_seqlens_q; p.total_tokens = total_q_tokens;
     p.num_seqs = num_seqs; p.num_heads = num_heads; p.num_kv_heads = num_kv_heads; p.scale_log2 = scale * kLog2e;
@@ -259,6 +277,7 @@ extern "C" int mvllm_prefill_paged(void* out, const void* q, const void* k_cache
     p.timeline = nullptr; p.timeline_entries = 0; p.timeline_block = 0;
     return launch_prefill_pp(p, dtype, (hipStream_t)stream);
   }
+  if (kind == 1 && sink) return MVLLM_ERR_UNSUPPORTED;
   if (kind == 1) {
     PrefillRowsArgs r;
     r.out = out; r.q = q; r.k = k_cache; r.v = v_cache; r.cu_seqlens = cu_seqlens_q; r.total_tokens = total_q_tokens;
@@ -268,6 +287,24 @@ extern "C" int mvllm_prefill_paged(void* out, const void* q, const void* k_cache
     return launch_prefill_rows16(r, head_dim, dtype, (hipStream_t)stream);
   }
   return prefill_dispatch<true>(a, dtype, mfma_ok, (hipStream_t)stream);
+}
+
+extern "C" int mvllm_prefill_paged(void* out, const void* q, const void* k_cache, const void* v_cache,
+                                   const int32_t* block_tables, int max_num_blocks, const int32_t* cu_seqlens_q,
+                                   const int32_t* cu_seqlens_k, int num_seqs, int64_t total_q_tokens,
+                                   int num_heads, int num_kv_heads, int head_dim, int block_size,
+                                   int64_t num_blocks, float scale, int dtype, void* stream) {
+  return prefill_paged_entry(out, q, k_cache, v_cache, block_tables, max_num_blocks, cu_seqlens_q, cu_seqlens_k, num_seqs,
+                             total_q_tokens, num_heads, num_kv_heads, head_dim, block_size, num_blocks, scale, nullptr, dtype, stream);
+}
+
+extern "C" int mvllm_prefill_paged_sink(void* out, const void* q, const void* k_cache, const void* v_cache,
+                                   const int32_t* block_tables, int max_num_blocks, const int32_t* cu_seqlens_q,
+                                   const int32_t* cu_seqlens_k, int num_seqs, int64_t total_q_tokens,
+                                   int num_heads, int num_kv_heads, int head_dim, int block_size,
+                                   int64_t num_blocks, float scale, const float* sink, int dtype, void* stream) {
+  return prefill_paged_entry(out, q, k_cache, v_cache, block_tables, max_num_blocks, cu_seqlens_q, cu_seqlens_k, num_seqs,
+                             total_q_tokens, num_heads, num_kv_heads, head_dim, block_size, num_blocks, scale, sink, dtype, stream);
 }
 
 extern "C" int mvllm_prefill_paged_int8(void* out, const void* q, const int8_t* k_cache, const int8_t* v_cache,

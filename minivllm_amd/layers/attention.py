@@ -91,6 +91,21 @@ def _check_cache(name, cache, num_kv_heads, head_dim):
         raise ValueError(f"{name} must be contiguous")
 
 
+def _output(like, out):
+    if out is None:
+        return torch.empty_like(like)
+    if out.shape != like.shape or out.dtype != like.dtype or out.device != like.device or not out.is_contiguous():
+        raise ValueError("out must be a contiguous tensor like q")
+    return out
+
+
+def _sink_ptr(sink, num_heads):
+    _C.require_cuda(sink)
+    if sink.dtype != torch.float32 or tuple(sink.shape) != (num_heads,) or not sink.is_contiguous():
+        raise ValueError(f"sink must be contiguous float32 ({num_heads},)")
+    return sink.data_ptr()
+
+
 def _slots(slot_mapping):
     if slot_mapping.dtype != torch.int64:
         slot_mapping = slot_mapping.to(torch.int64)
@@ -159,11 +174,14 @@ def store_kvcache_int8(key: torch.Tensor, value: torch.Tensor, k_cache: torch.Te
 
 
 def flash_attention_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, cu_seqlens: torch.Tensor,
-                            scale: float, num_heads: int, num_kv_heads: int, head_dim: int) -> torch.Tensor:
+                            scale: float, num_heads: int, num_kv_heads: int, head_dim: int, *,
+                            sink: torch.Tensor | None = None, out: torch.Tensor | None = None) -> torch.Tensor:
     """Causal attention over a packed ragged batch.  Reference: attention.py:212-280.
 
     q: (total_tokens, num_heads, head_dim); k, v: (total_tokens, num_kv_heads,
     head_dim); cu_seqlens: int32 (num_seqs + 1,).  Returns a tensor like q.
+    ``sink`` (float32 (num_heads,), not in the reference): one more exp(sink) per head in the softmax denominators;
+    ``out``: contiguous tensor like q to write to.
     No device->host synchronisation happens here.
     """
     _C.require_cuda(q, k, v, cu_seqlens)
@@ -181,10 +199,16 @@ def flash_attention_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, c
     if cu_seqlens.dtype != torch.int32:
         cu_seqlens = cu_seqlens.to(torch.int32)
     cu_seqlens = cu_seqlens.contiguous()
-    output = torch.empty_like(q)
+    output = _output(q, out)
     num_seqs = cu_seqlens.shape[0] - 1
     _warn_if_generic("prefill", num_heads, num_kv_heads, head_dim, 0, q.dtype, False)
     lib = _C.load()
+    if sink is not None:
+        st = lib.mvllm_prefill_varlen_sink(_ptr(output), _ptr(q), _ptr(k), _ptr(v), _ptr(cu_seqlens), num_seqs, total,
+                                           num_heads, num_kv_heads, head_dim, float(scale), _sink_ptr(sink, num_heads),
+                                           _C.dtype_code(q.dtype), _C.current_stream_ptr(q.device))
+        _C.check(st, "flash_attention_prefill (sink)")
+        return output
     st = lib.mvllm_prefill_varlen(_ptr(output), _ptr(q), _ptr(k), _ptr(v), _ptr(cu_seqlens), num_seqs, total,
                                   num_heads, num_kv_heads, head_dim, float(scale), _C.dtype_code(q.dtype),
                                   _C.current_stream_ptr(q.device))
@@ -196,7 +220,8 @@ def flash_attention_prefill_paged(q: torch.Tensor, k_cache: torch.Tensor, v_cach
                                   block_tables: torch.Tensor, cu_seqlens_q: torch.Tensor,
                                   cu_seqlens_k: torch.Tensor, scale: float, num_heads: int, num_kv_heads: int,
                                   head_dim: int, block_size: int, max_seqlen_k: int | None = None,
-                                  key_splits: int | None = None) -> torch.Tensor:
+                                  key_splits: int | None = None, *, sink: torch.Tensor | None = None,
+                                  out: torch.Tensor | None = None) -> torch.Tensor:
     """Causal prefill of the tokens that follow each sequence's cached prefix, with every key read from the
     paged cache.  Consumes the metadata ``ModelRunner.prepare_prefill`` builds for prefix-cache hits
     (model_runner.py:192-226), which the reference's ``Attention.forward`` ignores (attention.py:518-523).
@@ -211,6 +236,8 @@ def flash_attention_prefill_paged(q: torch.Tensor, k_cache: torch.Tensor, v_cach
     With ``max_seqlen_k`` given, a batch of few new tokens behind long prefixes (too few query tiles to occupy the
     chip) has every sequence's keys cut into ranges that are walked side by side and merged; ``key_splits`` forces the
     number of ranges (0 or 1: never split; None: the library's ``mvllm_prefill_paged_split_plan`` decides).
+    ``sink`` and ``out`` as in ``flash_attention_prefill`` (with a sink, block sizes that are not a multiple of 16 stay on
+    the generic kernel).
     """
     _C.require_cuda(q, k_cache, v_cache, block_tables, cu_seqlens_q, cu_seqlens_k)
     if q.dim() != 3 or tuple(q.shape[1:]) != (num_heads, head_dim):
@@ -232,9 +259,10 @@ def flash_attention_prefill_paged(q: torch.Tensor, k_cache: torch.Tensor, v_cach
     block_tables = block_tables.to(torch.int32).contiguous()
     cu_seqlens_q = cu_seqlens_q.to(torch.int32).contiguous()
     cu_seqlens_k = cu_seqlens_k.to(torch.int32).contiguous()
-    output = torch.empty_like(q)
+    output = _output(q, out)
+    sink_ptr = 0 if sink is None else _sink_ptr(sink, num_heads)
     lib = _C.load()
-    if max_seqlen_k is not None and int(max_seqlen_k) > 0 and block_size % 16 != 0:
+    if max_seqlen_k is not None and int(max_seqlen_k) > 0 and block_size % 16 != 0 and sink is None:
         need = lib.mvllm_prefill_paged_staged_workspace_bytes(num_seqs, int(max_seqlen_k), num_heads, num_kv_heads, head_dim,
                                                               _C.dtype_code(q.dtype), 0)
         if 0 < need <= STAGED_PREFILL_MAX_BYTES:
@@ -260,18 +288,18 @@ def flash_attention_prefill_paged(q: torch.Tensor, k_cache: torch.Tensor, v_cach
                 raise ValueError(f"key_splits={key_splits}: the split form is not built for this shape")
         if 0 < need <= STAGED_PREFILL_MAX_BYTES:
             workspace = torch.empty(need, dtype=torch.uint8, device=q.device)
-            st = lib.mvllm_prefill_paged_split(_ptr(output), _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
-                                               block_tables.shape[1], _ptr(cu_seqlens_q), _ptr(cu_seqlens_k), num_seqs,
-                                               q.shape[0], int(max_seqlen_k), num_heads, num_kv_heads, head_dim, block_size,
-                                               k_cache.shape[0], float(scale), code, splits, _ptr(workspace), need,
-                                               _C.current_stream_ptr(q.device))
+            st = lib.mvllm_prefill_paged_split_sink(
+                _ptr(output), _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_tables), block_tables.shape[1],
+                _ptr(cu_seqlens_q), _ptr(cu_seqlens_k), num_seqs, q.shape[0], int(max_seqlen_k), num_heads, num_kv_heads,
+                head_dim, block_size, k_cache.shape[0], float(scale), sink_ptr, code, splits, _ptr(workspace), need,
+                _C.current_stream_ptr(q.device))
             _C.check(st, "flash_attention_prefill_paged (split over keys)")
             return output
     _warn_if_generic("prefill", num_heads, num_kv_heads, head_dim, block_size, q.dtype, False)
-    st = lib.mvllm_prefill_paged(_ptr(output), _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
-                                 block_tables.shape[1], _ptr(cu_seqlens_q), _ptr(cu_seqlens_k), num_seqs,
-                                 q.shape[0], num_heads, num_kv_heads, head_dim, block_size, k_cache.shape[0],
-                                 float(scale), _C.dtype_code(q.dtype), _C.current_stream_ptr(q.device))
+    st = lib.mvllm_prefill_paged_sink(_ptr(output), _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
+                                      block_tables.shape[1], _ptr(cu_seqlens_q), _ptr(cu_seqlens_k), num_seqs,
+                                      q.shape[0], num_heads, num_kv_heads, head_dim, block_size, k_cache.shape[0],
+                                      float(scale), sink_ptr, _C.dtype_code(q.dtype), _C.current_stream_ptr(q.device))
     _C.check(st, "flash_attention_prefill_paged")
     return output
 
@@ -410,14 +438,16 @@ def prefill_plan(num_heads: int, num_kv_heads: int, head_dim: int, block_size: i
 def paged_attention_decode(query: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                            block_tables: torch.Tensor, context_lens: torch.Tensor, scale: float,
                            num_heads: int, num_kv_heads: int, head_dim: int, block_size: int, *,
-                           workspace: torch.Tensor | None = None) -> torch.Tensor:
+                           workspace: torch.Tensor | None = None, sink: torch.Tensor | None = None,
+                           out: torch.Tensor | None = None) -> torch.Tensor:
     """One query token per sequence over its paged KV.  Reference: attention.py:418-473.
 
     query: (batch, num_heads, head_dim); caches (num_blocks, block_size, Hkv, D);
     block_tables int32 (batch, max_num_blocks), -1 padded; context_lens int32 or
     int64 (batch,).  Returns a tensor like query; rows with context_len 0 are zeros.
     ``workspace`` (optional, not in the reference): a uint8 device tensor the caller owns for the split-K
-    partials; without it, or when it is too small, a per-device buffer of this module is used.
+    partials; without it, or when it is too small, a per-device buffer of this module is used.  ``sink`` and ``out`` as in
+    ``flash_attention_prefill``.
     """
     _C.require_cuda(query, k_cache, v_cache, block_tables, context_lens)
     if k_cache.dtype != query.dtype or v_cache.dtype != query.dtype:
@@ -425,13 +455,21 @@ def paged_attention_decode(query: torch.Tensor, k_cache: torch.Tensor, v_cache: 
     query, block_tables, context_lens = _decode_common(query, k_cache, v_cache, block_tables, context_lens,
                                                        num_heads, num_kv_heads, head_dim, block_size)
     batch, max_blocks = block_tables.shape
-    output = torch.empty_like(query)
+    output = _output(query, out)
     if batch == 0:
         return output
     _warn_if_generic("decode", num_heads, num_kv_heads, head_dim, block_size, query.dtype, False)
     lib = _C.load()
     nbytes = lib.mvllm_paged_decode_workspace_bytes(batch, num_heads, head_dim, max_blocks, block_size)
     ws = _decode_workspace(query.device, nbytes, workspace)
+    if sink is not None:
+        st = lib.mvllm_paged_decode_sink(_ptr(output), _ptr(query), _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
+                                         max_blocks, _ptr(context_lens), int(context_lens.dtype == torch.int64), batch,
+                                         num_heads, num_kv_heads, head_dim, block_size, k_cache.shape[0], float(scale),
+                                         _sink_ptr(sink, num_heads), _C.dtype_code(query.dtype), _ptr(ws),
+                                         0 if ws is None else ws.numel(), _C.current_stream_ptr(query.device))
+        _C.check(st, "paged_attention_decode (sink)")
+        return output
     st = lib.mvllm_paged_decode(_ptr(output), _ptr(query), _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
                                 max_blocks, _ptr(context_lens), int(context_lens.dtype == torch.int64), batch,
                                 num_heads, num_kv_heads, head_dim, block_size, k_cache.shape[0], float(scale),
