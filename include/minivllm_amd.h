@@ -457,6 +457,111 @@ int mvllm_norm_linear_small_m(void* out, void* residual_out, const void* x, cons
  */
 int mvllm_linear_small_m_plan(int M, int N, int K, int norm, int glu, int dtype, int* waves);
 
+/*
+ * Attention with a sink: the four calls below are mvllm_paged_decode, mvllm_prefill_varlen, mvllm_prefill_paged and
+ * mvllm_prefill_paged_split with one more term in every softmax denominator, exp(sink[h]): a learned number per query
+ * head that has neither key nor value and is not scaled (no counterpart in the reference).  sink fp32 [Hq] on the device.
+ * The prefill forms run on the one-group, fp32 and generic kernels; a paged cache whose blocks hold 2^31 bytes or more
+ * is MVLLM_ERR_UNSUPPORTED.
+ */
+int mvllm_paged_decode_sink(void* out, const void* q, const void* k_cache, const void* v_cache,
+                            const int32_t* block_tables, int max_num_blocks, const void* context_lens, int ctx_is_i64,
+                            int batch, int num_heads, int num_kv_heads, int head_dim, int block_size,
+                            int64_t num_blocks, float scale, const float* sink, int dtype, void* workspace,
+                            size_t workspace_bytes, void* stream);
+int mvllm_prefill_varlen_sink(void* out, const void* q, const void* k, const void* v, const int32_t* cu_seqlens,
+                              int num_seqs, int64_t total_tokens, int num_heads, int num_kv_heads, int head_dim,
+                              float scale, const float* sink, int dtype, void* stream);
+int mvllm_prefill_paged_sink(void* out, const void* q, const void* k_cache, const void* v_cache,
+                             const int32_t* block_tables, int max_num_blocks, const int32_t* cu_seqlens_q,
+                             const int32_t* cu_seqlens_k, int num_seqs, int64_t total_q_tokens, int num_heads,
+                             int num_kv_heads, int head_dim, int block_size, int64_t num_blocks, float scale,
+                             const float* sink, int dtype, void* stream);
+int mvllm_prefill_paged_split_sink(void* out, const void* q, const void* k_cache, const void* v_cache,
+                                   const int32_t* block_tables, int max_num_blocks, const int32_t* cu_seqlens_q,
+                                   const int32_t* cu_seqlens_k, int num_seqs, int64_t total_q_tokens, int max_kv_len,
+                                   int num_heads, int num_kv_heads, int head_dim, int block_size, int64_t num_blocks,
+                                   float scale, const float* sink, int dtype, int splits, void* workspace,
+                                   size_t workspace_bytes, void* stream);
+
+/*
+ * Between two sublayers that have a norm on either side and a short causal convolution in front (no counterpart in the
+ * reference; the residual stream is fp32):
+ *     x' = x + rms(y) * post;   h = rms(x') * pre;   out_t = h_t + sum_j conv[j] * h_(t - taps + 1 + j)
+ *   out      [rows, width] dtype;  x_out fp32 [rows, width] = x' or NULL (must not be x)
+ *   x        fp32 [rows, width], or NULL with embed [vocab, width] dtype and tokens int64 [rows] (x = embed[token])
+ *   y        [rows, width] dtype or NULL (x' = x);  post, pre: fp32 gains, one number (stride 0) or [width] (stride 1)
+ *   conv     fp32 [taps, width] or NULL (out = h), taps 1 .. 8;  state fp32 [num_banks, taps - 1, width]: the last
+ *            taps - 1 rows of h, read before an entry's first row (zeros before position 0) and written after its last
+ *   cu_seqlens int32 [entries + 1] rows of the entries (all rows covered), row_entry int32 [rows], bank_in / bank_out
+ *            int32 [entries] (they must differ for entries of more than one row), positions int64 [rows]
+ * bf16 and fp32, width up to 16384 (4096 where it is not a multiple of 4).
+ */
+int mvllm_norm_conv(void* out, float* x_out, const float* x, const void* embed, const int64_t* tokens, int64_t vocab,
+                    const void* y, const float* post, int post_stride, const float* pre, int pre_stride, float eps,
+                    const float* conv, int taps, float* state, int64_t num_banks, const int32_t* cu_seqlens,
+                    const int32_t* row_entry, const int32_t* bank_in, const int32_t* bank_out, const int64_t* positions,
+                    int64_t rows, int width, int dtype, void* stream);
+
+/*
+ * Per-head norms, rotary embedding in either pair layout, rotated values and the cache store for heads whose key and
+ * value sizes may differ (models/qwen3.py:104-110 is the reference's case of it).
+ *   proj [rows, proj_row_stride]: q [Hq, dim] | k [Hkv, dim] | v [Hkv, vdim] | anything
+ *   q_out [*, Hq, head_dim], k_out / v_out [*, Hkv, head_dim] or NULL: row dst_row[t] (NULL: t); dims past dim / vdim
+ *   are zeros.  k_cache / v_cache [num_slots, Hkv, head_dim] rows slots[t] (< 0 or NULL: none).
+ *   gain_q / gain_k fp32 [dim] or NULL (no norm); q_scale multiplies q last.
+ *   rot_table fp32 [max_position, rot_dims / 2, 2], v_table fp32 [max_position, vdim / 2, 2] or NULL: (cos, sin) per
+ *   pair; interleaved: pair i is dims 2i, 2i + 1, else i, i + n / 2.
+ * bf16 and fp32, head_dim up to 512.
+ */
+int mvllm_head_rope_store(void* q_out, void* k_out, void* v_out, const void* proj, int64_t proj_row_stride,
+                          const float* gain_q, const float* gain_k, float eps, float q_scale, const float* rot_table,
+                          int rot_dims, const float* v_table, int interleaved, int64_t max_position,
+                          const int64_t* positions, const int32_t* dst_row, const int64_t* slots, void* k_cache,
+                          void* v_cache, int64_t num_slots, int64_t rows, int num_heads, int num_kv_heads, int dim,
+                          int vdim, int head_dim, int dtype, void* stream);
+
+/*
+ * Behind attention over rotated values: out[t, h, :vdim] = rotate(o[dst_row[t], h], -position) * sigmoid(gate[t, h]).
+ * o [*, Hq, head_dim]; gate [rows, gate_row_stride] dtype, Hq values per row, or NULL; v_table as above or NULL.
+ */
+int mvllm_head_unrotate_gate(void* out, const void* o, const void* gate, int64_t gate_row_stride, const float* v_table,
+                             int interleaved, int64_t max_position, const int64_t* positions, const int32_t* dst_row,
+                             int64_t rows, int num_heads, int vdim, int head_dim, int dtype, void* stream);
+
+/*
+ * Decode metadata of a cache that holds one attention chunk per sequence (chunk 0: the whole sequence): for a row with
+ * context length c > 0, chunk_lens = (c - 1) mod chunk + 1 and slots = the slot of that last token; 0 and -1 otherwise.
+ * All int64 [batch] but block_tables int32 [batch, max_num_blocks].
+ */
+int mvllm_chunk_decode_step(int64_t* chunk_lens, int64_t* slots, const int64_t* context_lens,
+                            const int32_t* block_tables, int max_num_blocks, int chunk, int block_size, int batch,
+                            void* stream);
+
+/*
+ * out[rows, N] (fp32) = act(x W^T + bias): columns below `split` get cap * tanh(z / cap) (cap 0: z), the others
+ * logsigmoid of that.  x [rows, K], w [N, K] dtype; bias fp32 [N] or NULL.  For the gates of a recurrence, N small.
+ */
+int mvllm_gate_linear(float* out, const void* x, int64_t x_row_stride, const void* w, const float* bias, int64_t rows,
+                      int N, int K, int split, float cap, int dtype, void* stream);
+
+/*
+ * mLSTM matrix-memory recurrence (csrc/mlstm.hip has the equations): every row of every entry in turn.
+ *   num fp32 [rows, H, vdim], den fp32 [rows, H] (the floor added), m_next fp32 [entries, H]
+ *   proj [rows, proj_row_stride]: q [H, dim] | k [H, dim] | v [H, vdim] | anything;  gates fp32 [rows, 2 H]
+ *   state of slot slots[e]: s_state fp32 [*, H, dim, vdim], n_state [*, H, dim], m_state [*, H]; s and n are updated,
+ *   m by mvllm_mlstm_output; an entry that starts at position 0 starts from zeros.  slots < 0: the entry is skipped.
+ * mvllm_mlstm_output: out [rows, H * vdim] = rms(num / den) * weight * sigmoid(gate), m_state[slot] = m_next.
+ */
+int mvllm_mlstm_recurrent(float* num, float* den, float* m_next, const void* proj, int64_t proj_row_stride,
+                          const float* gates, float* s_state, float* n_state, const float* m_state,
+                          const int32_t* cu_seqlens, const int32_t* slots, const int64_t* positions, int entries,
+                          int num_heads, int dim, int vdim, float q_scale, float floor, int dtype, void* stream);
+int mvllm_mlstm_output(void* out, const float* num, const float* den, const float* weight, const void* gate,
+                       int64_t gate_row_stride, float eps, const float* m_next, float* m_state,
+                       const int32_t* cu_seqlens, const int32_t* row_entry, const int32_t* slots, int64_t rows,
+                       int num_heads, int vdim, int dtype, void* stream);
+
 #ifdef __cplusplus
 }
 #endif

@@ -12,6 +12,7 @@ import torch
 
 _LIB_PATH = os.path.join(os.path.dirname(os.path.abspath(__file__)), "libminivllm_amd.so")
 _lib = None
+_partial = None      # path of a library that holds some of the entry points only (use_library)
 
 DTYPE_CODES = {torch.float32: 0, torch.bfloat16: 1, torch.float16: 2}
 
@@ -71,6 +72,29 @@ SIGNATURES = {
     "mvllm_qk_norm_rope_store": (c_int, [c_void_p] * 6 + [c_int64] * 3 + [c_void_p, c_float, c_void_p, c_int64,
                                                            c_void_p, c_void_p] + [c_void_p] * 4 +
                                  [c_int, c_int64, c_int64, c_int, c_int, c_int, c_int, c_void_p]),
+    "mvllm_paged_decode_sink": (c_int, [c_void_p] * 5 + [c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                                                          c_int64, c_float, c_void_p, c_int, c_void_p, c_size_t, c_void_p]),
+    "mvllm_prefill_varlen_sink": (c_int, [c_void_p] * 5 + [c_int, c_int64, c_int, c_int, c_int, c_float, c_void_p, c_int,
+                                                            c_void_p]),
+    "mvllm_prefill_paged_sink": (c_int, [c_void_p] * 5 + [c_int, c_void_p, c_void_p, c_int, c_int64, c_int, c_int, c_int,
+                                                           c_int, c_int64, c_float, c_void_p, c_int, c_void_p]),
+    "mvllm_prefill_paged_split_sink": (c_int, [c_void_p] * 5 + [c_int, c_void_p, c_void_p, c_int, c_int64, c_int, c_int, c_int,
+                                                 c_int, c_int, c_int64, c_float, c_void_p, c_int, c_int, c_void_p, c_size_t,
+                                                 c_void_p]),
+    "mvllm_norm_conv": (c_int, [c_void_p] * 5 + [c_int64, c_void_p, c_void_p, c_int, c_void_p, c_int, c_float, c_void_p,
+                                                  c_int, c_void_p, c_int64] + [c_void_p] * 5 + [c_int64, c_int, c_int, c_void_p]),
+    "mvllm_head_rope_store": (c_int, [c_void_p] * 4 + [c_int64, c_void_p, c_void_p, c_float, c_float, c_void_p, c_int,
+                                                        c_void_p, c_int, c_int64] + [c_void_p] * 5 + [c_int64, c_int64] +
+                              [c_int] * 6 + [c_void_p]),
+    "mvllm_head_unrotate_gate": (c_int, [c_void_p] * 3 + [c_int64, c_void_p, c_int, c_int64, c_void_p, c_void_p, c_int64] +
+                                 [c_int] * 4 + [c_void_p]),
+    "mvllm_chunk_decode_step": (c_int, [c_void_p] * 4 + [c_int] * 4 + [c_void_p]),
+    "mvllm_gate_linear": (c_int, [c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_int, c_int, c_float,
+                                  c_int, c_void_p]),
+    "mvllm_mlstm_recurrent": (c_int, [c_void_p] * 4 + [c_int64] + [c_void_p] * 7 + [c_int] * 4 + [c_float, c_float, c_int,
+                                                                                              c_void_p]),
+    "mvllm_mlstm_output": (c_int, [c_void_p] * 5 + [c_int64, c_float] + [c_void_p] * 5 + [c_int64, c_int, c_int, c_int,
+                                                                                      c_void_p]),
 }
 
 
@@ -82,17 +106,30 @@ def lib_path() -> str:
     return _LIB_PATH
 
 
+def use_library(path: str) -> None:
+    """Load ``path`` instead of the full library (before the first call into it); entry points it lacks stay unbound."""
+    global _partial
+    if path == _LIB_PATH or path == _partial:
+        return
+    if _lib is not None:
+        raise MinivllmAmdError("another library is already loaded")
+    _partial = path
+
+
 def load():
     """Load the shared library once; raise if it has not been built."""
     global _lib
     if _lib is not None:
         return _lib
-    if not os.path.exists(_LIB_PATH):
+    path = _partial or _LIB_PATH
+    if not os.path.exists(path):
         raise MinivllmAmdError(
-            f"{_LIB_PATH} not found: build it with `python -m minivllm_amd._build` "
+            f"{path} not found: build it with `python -m minivllm_amd._build` "
             "(there is no fallback path)")
-    lib = ctypes.CDLL(_LIB_PATH)
+    lib = ctypes.CDLL(path)
     for name, (restype, argtypes) in SIGNATURES.items():
+        if _partial and not hasattr(lib, name):
+            continue
         fn = getattr(lib, name)      # AttributeError if the symbol is missing
         fn.restype = restype
         fn.argtypes = argtypes

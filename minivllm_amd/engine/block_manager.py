@@ -67,6 +67,20 @@ class BlockManager:
         self.used_block_ids.remove(block_id)
         self.free_block_ids.append(block_id)
 
+    def take_block(self) -> int:
+        """A free block for a caller that keeps its own tables (nothing is hashed or shared)."""
+        return self._allocate_block(self.free_block_ids[0]).block_id
+
+    def give_back(self, block_id: int) -> None:
+        block = self.blocks[block_id]
+        block.ref_count -= 1
+        if block.ref_count == 0:
+            self._deallocate_block(block_id)
+
+    def holds(self, tokens: int) -> bool:
+        """Whether a sequence of that many tokens fits an empty pool."""
+        return -(-tokens // self.block_size) <= len(self.blocks)
+
     def can_allocate(self, seq: Sequence) -> bool:
         return len(self.free_block_ids) >= seq.num_blocks
 

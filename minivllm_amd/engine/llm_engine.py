@@ -5,28 +5,34 @@ from __future__ import annotations
 
 import time
 
-from minivllm_amd.engine.model_runner import ModelRunner
 from minivllm_amd.engine.scheduler import Scheduler
 from minivllm_amd.engine.sequence import Sequence
+from minivllm_amd.models.registry import make_runner, read_model_config
 from minivllm_amd.sampling_parameters import SamplingParams
 
 
 class LLMEngine:
     def __init__(self, config: dict, model_runner=None):
         self.block_size = config.get("block_size", 256)
+        self.model_runner = model_runner if model_runner is not None else make_runner(config)
         self.scheduler = Scheduler(
             max_num_sequences=config.get("max_num_sequences", 16),
             max_num_batched_tokens=config.get("max_num_batched_tokens", 1024),
             max_cached_blocks=config.get("max_cached_blocks", 1024),
             block_size=self.block_size,
-            eos=config.get("eos", 50256))
-        self.model_runner = model_runner if model_runner is not None else ModelRunner(config)
+            eos=config.get("eos", 50256),
+            cache_manager=getattr(self.model_runner, "cache_manager", None))
         # longest sequence (prompt + new tokens) the rotary table and the graph's block-table buffer are sized for
         self.max_model_length = min(config.get("max_model_length", config.get("max_position", 4096)),
                                     config.get("max_position", 4096))
         self.async_decode = config.get("async_decode", True)
         self.pending = None          # (ids on their way, placeholders to fill, sequences that step finished)
         self.stats = {"prefill_tokens": 0, "decode_tokens": 0, "prefill_s": 0.0, "decode_s": 0.0, "steps": 0}
+
+    @classmethod
+    def from_pretrained(cls, model_dir: str, **engine_config) -> "LLMEngine":
+        """An engine for a checkpoint folder (config.json, model.safetensors); keywords are engine keys."""
+        return cls({**read_model_config(model_dir), "model_dir": model_dir, **engine_config})
 
     def add_prompt(self, prompt_token_ids: list[int], sampling_params: SamplingParams) -> None:
         """Queue a prompt.  A request that could outgrow ``max_model_length`` / ``max_position`` is refused here:
@@ -42,12 +48,11 @@ class LLMEngine:
         # llm_engine.py:62-75): a sequence is re-admitted as a whole after a preemption, so its full length must fit
         # the token budget of a step, and its blocks the pool
         slots = longest - 1                                     # the last sampled token is never fed back
-        if slots > self.scheduler.max_num_batched_tokens:
+        if slots > self.scheduler.max_num_batched_tokens and not self.scheduler.ragged:
             raise ValueError(f"prompt + max_tokens - 1 = {slots} tokens exceed max_num_batched_tokens "
                              f"{self.scheduler.max_num_batched_tokens}")
-        pool = len(self.scheduler.block_manager.blocks)
-        if -(-slots // self.block_size) > pool:
-            raise ValueError(f"{slots} tokens need {-(-slots // self.block_size)} blocks of {self.block_size}, the pool has {pool}")
+        if not self.scheduler.block_manager.holds(slots):
+            raise ValueError(f"{slots} tokens need more blocks of {self.block_size} than the pool has")
         self.scheduler.add_sequence(Sequence(prompt_token_ids, sampling_params, self.block_size))
 
     def step(self):
@@ -89,7 +94,10 @@ class LLMEngine:
         token_ids = runner.run(seqs, is_prefill)
         self.scheduler.postprocess(seqs, token_ids)
         finished += [(seq.seq_id, seq.completion_token_ids) for seq in seqs if seq.is_finished]
-        processed = sum(len(seq) - 1 for seq in seqs) if is_prefill else len(seqs)
+        if self.scheduler.ragged:
+            processed = sum(seq.num_scheduled_tokens for seq in seqs)
+        else:
+            processed = sum(len(seq) - 1 for seq in seqs) if is_prefill else len(seqs)
         return finished, processed, is_prefill
 
     def flush(self):

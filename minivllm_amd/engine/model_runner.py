@@ -72,19 +72,7 @@ class ModelRunner:
         self.num_blocks = config.get("max_cached_blocks", 1024)
         self.dtype = _DTYPES[config.get("dtype", "bf16")]
         self.kv_cache_dtype = config.get("kv_cache_dtype", "auto")
-        head_dim = config.get("head_dim") or config["hidden_size"] // config["num_heads"]
-        self.model = Qwen3ForCausalLM(
-            vocab_size=config["vocab_size"], hidden_size=config["hidden_size"], num_heads=config["num_heads"],
-            head_dim=head_dim, scale=config.get("scale", 1.0), num_kv_heads=config.get("num_kv_heads"),
-            rms_norm_epsilon=config.get("rms_norm_epsilon", 1e-6), qkv_bias=config.get("qkv_bias", False),
-            base=config.get("base", 1_000_000), max_position=config.get("max_position", 4096),
-            intermediate_size=config["intermediate_size"], ffn_bias=config.get("ffn_bias", True),
-            num_layers=config["num_layers"], tie_word_embeddings=config.get("tie_word_embeddings", True),
-            block_size=self.block_size, kv_cache_dtype=self.kv_cache_dtype,
-            fused_qk=config.get("fused_qk", True), fused_elementwise=config.get("fused_elementwise", True),
-            small_rows=config.get("linear_small_rows", 64), norm_rows=config.get("linear_norm_rows", 32))
-        self.model.reset_parameters(seed=config.get("seed", 0))
-        self.model.to(device=self.device, dtype=self.dtype).eval()
+        self.model = self.build_model()
         self.sampler = Sampler()
         self.fused_sampler = config.get("fused_sampler", True)
         self.fused_lm_head = self.fused_sampler and config.get("fused_lm_head", True)
@@ -99,6 +87,22 @@ class ModelRunner:
         self.graphs = {}
         if not config.get("enforce_eager", True):
             self.capture_decode_graphs()
+
+    def build_model(self):
+        config = self.config
+        head_dim = config.get("head_dim") or config["hidden_size"] // config["num_heads"]
+        model = Qwen3ForCausalLM(
+            vocab_size=config["vocab_size"], hidden_size=config["hidden_size"], num_heads=config["num_heads"],
+            head_dim=head_dim, scale=config.get("scale", 1.0), num_kv_heads=config.get("num_kv_heads"),
+            rms_norm_epsilon=config.get("rms_norm_epsilon", 1e-6), qkv_bias=config.get("qkv_bias", False),
+            base=config.get("base", 1_000_000), max_position=config.get("max_position", 4096),
+            intermediate_size=config["intermediate_size"], ffn_bias=config.get("ffn_bias", True),
+            num_layers=config["num_layers"], tie_word_embeddings=config.get("tie_word_embeddings", True),
+            block_size=self.block_size, kv_cache_dtype=self.kv_cache_dtype,
+            fused_qk=config.get("fused_qk", True), fused_elementwise=config.get("fused_elementwise", True),
+            small_rows=config.get("linear_small_rows", 64), norm_rows=config.get("linear_norm_rows", 32))
+        model.reset_parameters(seed=config.get("seed", 0))
+        return model.to(device=self.device, dtype=self.dtype).eval()
 
     def allocate_kv_cache(self):
         """One pool ``[2, L, num_blocks, block_size, Hkv, D]``; each ``Attention`` gets its layer's views
@@ -216,10 +220,10 @@ class ModelRunner:
         self._own_decode_workspace(buckets, max_blocks)
         pool = None
         for bs in reversed(buckets):
-            set_context(False, slot_mapping=v["slot_mapping"][:bs], context_lens=v["context_lens"][:bs],
-                        block_tables=v["block_tables"][:bs])
+            prepare = self._captured_context(bs)
 
             def forward():
+                prepare()
                 hidden = self.model(v["input_ids"][:bs], v["positions"][:bs])
                 if not self.fused_sampler:                 # the module-chain sampler draws from a host-side generator
                     v["outputs"][:bs] = hidden
@@ -250,6 +254,13 @@ class ModelRunner:
         self._dev_step = None                            # value of the device counter, unknown after the warm-ups
         torch.cuda.synchronize()
         self._pinned.zero_()                             # the warm-ups left their sequence numbers: steps count from 1
+
+    def _captured_context(self, bs):
+        """Set the context a captured step of ``bs`` rows runs under; returns what the step launches before the model."""
+        v = self.graph_vars
+        set_context(False, slot_mapping=v["slot_mapping"][:bs], context_lens=v["context_lens"][:bs],
+                    block_tables=v["block_tables"][:bs])
+        return lambda: None
 
     def _own_decode_workspace(self, buckets, max_blocks):
         """One split-K scratch buffer for every decode call of this runner, allocated before any graph is

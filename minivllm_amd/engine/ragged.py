@@ -1,0 +1,177 @@
+"""Metadata of a ragged step: entries of any length (portions of prompts beside single decoded tokens) in one packed batch.
+
+Rows are packed entry by entry, entries of one token first.  Attention sees a row's entry cut at chunk borders: the piece
+that goes on in a chunk whose earlier tokens are cached reads the cache (``prefixed``), pieces that start a chunk read the
+packed keys and values of the step (``fresh``), single tokens take the decode kernel.  Pieces are sorted in that order
+(``dst_row``), so that each kernel runs over consecutive rows.  Only the tokens of an entry's last chunk stay cached; where
+the entry also reads the chunk before, whose blocks they go to, they are stored after attention (``late_slots``)."""
+from __future__ import annotations
+
+from dataclasses import dataclass, field
+from typing import Optional
+
+import numpy as np
+import torch
+
+
+@dataclass
+class WindowStep:
+    """One attention window's view of the step."""
+    num_decode: int = 0
+    num_prefixed: int = 0                             # rows of pieces with a cached prefix
+    num_fresh: int = 0
+    dst_row: Optional[torch.Tensor] = None            # int32 [T], None: rows stay in order
+    slots: Optional[torch.Tensor] = None              # int64 [T], stored before attention (-1: not)
+    late_slots: Optional[torch.Tensor] = None         # int64 [T] in dst_row order, stored after attention, or None
+    chunk_lens: Optional[torch.Tensor] = None         # int64 [num_decode]
+    decode_tables: Optional[torch.Tensor] = None      # int32 [num_decode, width]
+    prefixed_cu_q: Optional[torch.Tensor] = None      # int32 [pieces + 1]
+    prefixed_cu_k: Optional[torch.Tensor] = None
+    prefixed_tables: Optional[torch.Tensor] = None
+    prefixed_max_k: int = 0
+    fresh_cu: Optional[torch.Tensor] = None
+
+
+@dataclass
+class RaggedStep:
+    num_tokens: int
+    num_entries: int
+    num_single: int                                   # entries of one token, packed first
+    input_ids: torch.Tensor                           # int64 [T]
+    positions: torch.Tensor                           # int64 [T]
+    cu_seqlens: torch.Tensor                          # int32 [entries + 1]
+    row_entry: torch.Tensor                           # int32 [T]
+    bank_in: torch.Tensor                             # int32 [entries]: banks of the short-convolution state
+    bank_out: torch.Tensor
+    state_slots: torch.Tensor                         # int32 [entries]
+    windows: list = field(default_factory=list)       # WindowStep per window
+    long_rows: int = 0                                # rows of entries with more than one token
+    order: list = field(default_factory=list)         # entry e of the packing is sequence order[e] of the caller
+    starts: list = field(default_factory=list)        # first packed row of the caller's sequence i
+
+
+def _pad_tables(tables):
+    width = max((len(t) for t in tables), default=1) or 1
+    out = np.full((len(tables), width), -1, dtype=np.int32)
+    for i, t in enumerate(tables):
+        out[i, :len(t)] = t
+    return out
+
+
+def _window_arrays(items, window, index, block_size, cu):
+    """Host arrays of one window; items: (tokens before, new tokens, sequence) in packing order."""
+    total = int(cu[-1])
+    slots = np.full(total, -1, dtype=np.int64)
+    late = np.full(total, -1, dtype=np.int64)
+    any_late = False
+    chunk_lens, decode_tables = [], []
+    pre_rows, pre_q, pre_k, pre_tables = [], [0], [0], []
+    fresh_rows, fresh_q = [], [0]
+    single = 0
+    for e, (p0, n, seq) in enumerate(items):
+        table = np.asarray(seq.group_tables[index], dtype=np.int64)
+        at = int(cu[e])
+        local = np.arange(p0, p0 + n)
+        size = window or p0 + n
+        place = local % size
+        where = table[place // block_size] * block_size + place % block_size
+        if n == 1:
+            chunk_lens.append(int(place[0]) + 1)
+            decode_tables.append(seq.group_tables[index])
+            slots[at] = where[0]
+            single += 1
+            continue
+        head = 0
+        if p0 % size:
+            head = min(size - p0 % size, n)
+            pre_rows.append(np.arange(at, at + head))
+            pre_q.append(pre_q[-1] + head)
+            pre_k.append(pre_k[-1] + p0 % size + head)
+            pre_tables.append(seq.group_tables[index])
+            slots[at:at + head] = where[:head]
+        if head < n:
+            fresh_rows.append(np.arange(at + head, at + n))
+            cuts = list(range(head + size, n, size)) + [n]
+            base = fresh_q[-1] - head
+            fresh_q.extend(base + c for c in cuts)
+            last = cuts[-2] if len(cuts) > 1 else head
+            if head:
+                late[at + last:at + n] = where[last:]
+                any_late = True
+            else:
+                slots[at + last:at + n] = where[last:]
+    order = np.concatenate([np.arange(single), *pre_rows, *fresh_rows]).astype(np.int64)     # packed row of each sorted row
+    sorted_as_packed = bool((order == np.arange(total)).all())
+    dst = np.empty(total, dtype=np.int32)
+    dst[order] = np.arange(total, dtype=np.int32)
+    out = dict(slots=slots)
+    if not sorted_as_packed:
+        out["dst_row"] = dst
+    if any_late:
+        out["late_slots"] = late[order]
+    if single:
+        out["chunk_lens"] = np.asarray(chunk_lens, dtype=np.int64)
+        out["decode_tables"] = _pad_tables(decode_tables)
+    if pre_rows:
+        out["prefixed_cu_q"] = np.asarray(pre_q, dtype=np.int32)
+        out["prefixed_cu_k"] = np.asarray(pre_k, dtype=np.int32)
+        out["prefixed_tables"] = _pad_tables(pre_tables)
+    if fresh_rows:
+        out["fresh_cu"] = np.asarray(fresh_q, dtype=np.int32)
+    counts = dict(num_decode=single, num_prefixed=pre_q[-1], num_fresh=fresh_q[-1],
+                  prefixed_max_k=int(np.diff(pre_k).max()) if pre_rows else 0)
+    return out, counts
+
+
+def ragged_arrays(seqs, windows, block_size):
+    """Host side of a step over ``seqs``: each runs its tokens [num_computed_tokens, + num_scheduled_tokens).  Returns
+    (arrays, window arrays, window counts, facts), everything in numpy; the sequences' convolution banks flip for entries
+    of more than one token."""
+    order = sorted(range(len(seqs)), key=lambda i: seqs[i].num_scheduled_tokens > 1)        # stable
+    items = [(seqs[i].num_computed_tokens, seqs[i].num_scheduled_tokens, seqs[i]) for i in order]
+    lens = np.asarray([n for _, n, _ in items], dtype=np.int64)
+    cu = np.concatenate([[0], np.cumsum(lens)]).astype(np.int32)
+    ids = np.concatenate([np.asarray(s.token_ids[p:p + n], dtype=np.int64) for p, n, s in items])
+    positions = np.concatenate([np.arange(p, p + n, dtype=np.int64) for p, n, _ in items])
+    bank_in, bank_out = [], []
+    for _, n, s in items:
+        bank_in.append(2 * s.state_slot + s.state_bank)
+        if n > 1:
+            s.state_bank ^= 1
+        bank_out.append(2 * s.state_slot + s.state_bank)
+    arrays = dict(input_ids=ids, positions=positions, cu_seqlens=cu,
+                  row_entry=np.repeat(np.arange(len(items), dtype=np.int32), lens),
+                  bank_in=np.asarray(bank_in, dtype=np.int32), bank_out=np.asarray(bank_out, dtype=np.int32),
+                  state_slots=np.asarray([s.state_slot for _, _, s in items], dtype=np.int32))
+    per_window = [_window_arrays(items, w, g, block_size, cu) for g, w in enumerate(windows)]
+    starts = [0] * len(seqs)
+    for e, i in enumerate(order):
+        starts[i] = int(cu[e])
+    singles = int((lens == 1).sum())
+    facts = dict(num_tokens=int(cu[-1]), num_entries=len(items), num_single=singles, long_rows=int(cu[-1]) - singles,
+                 order=order, starts=starts)
+    return arrays, [a for a, _ in per_window], [c for _, c in per_window], facts
+
+
+def ragged_step(seqs, windows, block_size, device) -> RaggedStep:
+    """The step's device tensors: one copy per integer type, every tensor a 16-byte aligned slice of it."""
+    arrays, window_arrays, counts, facts = ragged_arrays(seqs, windows, block_size)
+    named = [((None, k), a) for k, a in arrays.items()]
+    for g, wa in enumerate(window_arrays):
+        named += [((g, k), a) for k, a in wa.items()]
+    placed = {}
+    for np_dtype, torch_dtype in ((np.int32, torch.int32), (np.int64, torch.int64)):
+        mine = [(key, a) for key, a in named if a.dtype == np_dtype]
+        offsets, total = [], 0
+        for _, a in mine:
+            offsets.append(total)
+            total += -(-a.size // 4) * 4
+        host = torch.empty(max(total, 1), dtype=torch_dtype, pin_memory=device.type == "cuda")
+        view = host.numpy()
+        for (_, a), at in zip(mine, offsets):
+            view[at:at + a.size] = a.reshape(-1)
+        dev = host.to(device, non_blocking=True)
+        for (key, a), at in zip(mine, offsets):
+            placed[key] = dev[at:at + a.size].view(a.shape)
+    ws = [WindowStep(**counts[g], **{k: placed[(g, k)] for k in wa}) for g, wa in enumerate(window_arrays)]
+    return RaggedStep(windows=ws, **{k: placed[(None, k)] for k in arrays}, **facts)

@@ -1,4 +1,5 @@
-"""Prefill-first continuous batching (src/myvllm/engine/scheduler.py:6-82).
+"""Prefill-first continuous batching (src/myvllm/engine/scheduler.py:6-82), or, for models with a cache manager of their
+own (``cache_manager``), steps that mix portions of prompts with decoded tokens.
 
 Intended semantics where the reference is broken: limits are checked before a
 sequence is popped from ``running`` (the reference pops then breaks, losing
@@ -16,8 +17,10 @@ from minivllm_amd.engine.sequence import Sequence, SequenceStatus
 
 class Scheduler:
     def __init__(self, max_num_sequences: int, max_num_batched_tokens: int, max_cached_blocks: int,
-                 block_size: int, eos: int):
-        self.block_manager = BlockManager(max_cached_blocks, block_size)
+                 block_size: int, eos: int, cache_manager=None):
+        # a cache manager of the model's own means ragged steps: portions of prompts beside decoded tokens
+        self.ragged = cache_manager is not None
+        self.block_manager = cache_manager if self.ragged else BlockManager(max_cached_blocks, block_size)
         self.max_num_batched_tokens = max_num_batched_tokens
         self.max_num_sequences = max_num_sequences
         self.waiting: deque[Sequence] = deque()
@@ -30,11 +33,51 @@ class Scheduler:
     def add_sequence(self, sequence: Sequence):
         self.waiting.append(sequence)
 
+    def _schedule_ragged(self) -> list[Sequence]:
+        """A step that brings prompt tokens: one token of every decoding sequence, then portions of the prompts under
+        way, then of waiting ones, as far as the token budget, the batch slots and the cache reach."""
+        scheduled: list[Sequence] = []
+        budget = self.max_num_batched_tokens
+        for seq in sorted(self.running, key=lambda s: len(s) - s.num_computed_tokens > 1):     # stable: decoding ones first
+            if seq not in self.running or budget == 0 or len(scheduled) == self.max_num_sequences:
+                continue                                       # preempted by an earlier one of this step, or no room
+            while not self.block_manager.can_append(seq):
+                # scheduled sequences keep their blocks: their step is decided
+                victim = next((s for s in reversed(self.running) if s is not seq and s not in scheduled), seq)
+                self.running.remove(victim)
+                self.preempt(victim)
+                if victim is seq:
+                    break
+            else:
+                self.block_manager.append(seq)
+                seq.num_scheduled_tokens = min(len(seq) - seq.num_computed_tokens, budget)
+                budget -= seq.num_scheduled_tokens
+                scheduled.append(seq)
+        while self.waiting and budget > 0 and len(self.running) < self.max_num_sequences:
+            seq = self.waiting[0]
+            if not self.block_manager.can_allocate(seq):
+                break
+            self.waiting.popleft()
+            self.block_manager.allocate(seq)
+            seq.status = SequenceStatus.RUNNING
+            seq.num_scheduled_tokens = min(len(seq), budget)
+            budget -= seq.num_scheduled_tokens
+            self.running.append(seq)
+            scheduled.append(seq)
+        return scheduled
+
     def schedule(self) -> tuple[list[Sequence], bool]:
         scheduled: list[Sequence] = []
         num_tokens = 0
+        if self.ragged:
+            under_way = any(len(seq) - seq.num_computed_tokens > 1 for seq in self.running)
+            admit = (self.waiting and len(self.running) < self.max_num_sequences
+                     and self.block_manager.can_allocate(self.waiting[0]))
+            if under_way or admit:
+                return self._schedule_ragged(), True
+            # every running sequence decodes: an ordinary decode step
         # prefill: admit waiting sequences while blocks, token budget and batch slots last
-        while self.waiting and len(scheduled) < self.max_num_sequences:
+        while not self.ragged and self.waiting and len(scheduled) < self.max_num_sequences:
             seq = self.waiting[0]
             if len(seq) + num_tokens > self.max_num_batched_tokens or not self.block_manager.can_allocate(seq):
                 break
@@ -58,6 +101,7 @@ class Scheduler:
                     break
             else:
                 self.block_manager.append(seq)
+                seq.num_scheduled_tokens = 1
                 scheduled.append(seq)
                 num_tokens += 1
         if scheduled:
@@ -83,6 +127,7 @@ class Scheduler:
                 slots.append(None)
                 continue
             seq.append_token(self.PLACEHOLDER)
+            seq.num_computed_tokens += 1
             slots.append((seq, seq.num_tokens - 1))
             if seq.num_completion_tokens >= seq.max_tokens:
                 seq.status = SequenceStatus.FINISHED
@@ -117,7 +162,11 @@ class Scheduler:
         return ended
 
     def postprocess(self, seqs: list[Sequence], token_ids: list[int]) -> None:
+        """``token_ids[i]`` is None where sequence i still has prompt tokens to come (ragged steps)."""
         for seq, token_id in zip(seqs, token_ids):
+            seq.num_computed_tokens += seq.num_scheduled_tokens
+            if token_id is None:
+                continue
             seq.append_token(int(token_id))
             if (not seq.ignore_eos and token_id == self.eos) or seq.num_completion_tokens >= seq.max_tokens:
                 seq.status = SequenceStatus.FINISHED

@@ -37,6 +37,12 @@ class Sequence:
         self.num_prompt_tokens = len(self.token_ids)
         self.num_cached_tokens = 0
         self.block_table: list[int] = []
+        # models that run ragged steps (engine/ragged.py): what is in the cache, what the next step brings, where it lies
+        self.num_computed_tokens = 0
+        self.num_scheduled_tokens = 0
+        self.group_tables: list[list[int]] = []
+        self.state_slot = -1
+        self.state_bank = 0
         self.temperature = sampling_params.temperature
         self.max_tokens = sampling_params.max_tokens
         self.ignore_eos = sampling_params.ignore_eos

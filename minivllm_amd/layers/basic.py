@@ -4,6 +4,8 @@ operations and, with ``fused=True``, as single HIP launches (minivllm_amd.layers
 exponential-race sampler (layers/sampler.py:14-19)."""
 from __future__ import annotations
 
+import math
+
 import torch
 import torch.nn as nn
 import torch.nn.functional as F
@@ -84,6 +86,21 @@ class RotaryEmbedding(nn.Module):
         cos, sin = self.cos_sin_cache[positions].chunk(2, dim=-1)      # (T, D/2) each, fp32
         cos, sin = cos.unsqueeze(1), sin.unsqueeze(1)
         return self._rotate(query, cos, sin), self._rotate(key, cos, sin)
+
+
+def rotary_pair_table(base: float, dims: int, max_position: int, scaling: dict | None = None) -> torch.Tensor:
+    """float32 (max_position, dims / 2, 2): cos and sin of position * base^(-2 i / dims), angles in double precision.
+
+    ``scaling`` (``factor``, ``low``, ``high``, ``original``) stretches the slow pairs: wavelengths beyond original / low
+    by ``factor``, those below original / high not at all, a blend linear in original / wavelength between them."""
+    freq = float(base) ** (-torch.arange(0, dims, 2, dtype=torch.float64) / dims)
+    if scaling is not None:
+        turns = scaling["original"] * freq / (2 * math.pi)                 # of a pair over the original context
+        keep = ((turns - scaling["low"]) / (scaling["high"] - scaling["low"])).clamp(0.0, 1.0) if (
+            scaling["high"] != scaling["low"]) else (turns > scaling["high"]).double()
+        freq = (1.0 - keep) * freq / scaling["factor"] + keep * freq
+    angle = torch.outer(torch.arange(max_position, dtype=torch.float64), freq)
+    return torch.stack([angle.cos(), angle.sin()], dim=-1).float().contiguous()
 
 
 class SiluAndMul(nn.Module):

@@ -17,7 +17,8 @@ import torch
 from minivllm_amd import _C
 
 __all__ = ["qk_norm_rope_store", "sample_tokens", "sample_tokens_into", "decode_advance", "add_rms_norm", "silu_and_mul", "linear_small_m", "linear_small_m_takes", "norm_linear_small_m", "norm_linear_small_m_takes",
-           "lm_head_sample", "lm_head_sample_takes", "lm_head_sample_workspace_bytes"]
+           "lm_head_sample", "lm_head_sample_takes", "lm_head_sample_workspace_bytes", "norm_conv", "head_rope_store",
+           "head_unrotate_gate", "chunk_decode_step"]
 
 
 def _ptr(t):
@@ -378,3 +379,141 @@ def lm_head_sample(hidden: torch.Tensor, weight: torch.Tensor, temperatures: tor
                                         _C.current_stream_ptr(hidden.device))
     _C.check(st, "lm_head_sample")
     return out
+
+
+def _check(t, dtype, shape, name):
+    if t.dtype != dtype or tuple(t.shape) != tuple(shape) or not t.is_contiguous():
+        raise ValueError(f"{name} must be contiguous {dtype} {tuple(shape)}, got {t.dtype} {tuple(t.shape)}")
+
+
+def norm_conv(step, pre: torch.Tensor, eps: float, dtype: torch.dtype, x: torch.Tensor | None = None,
+              tokens: torch.Tensor | None = None, embed: torch.Tensor | None = None, y: torch.Tensor | None = None,
+              post: torch.Tensor | None = None, conv: torch.Tensor | None = None, state: torch.Tensor | None = None,
+              want_x: bool = True):
+    """The launch between two sublayers: ``x' = x + rms(y) * post``, ``h = rms(x') * pre``, ``h + conv(h)`` over time.
+
+    x float32 (T, W), or ``embed`` (vocab, W) with ``tokens`` int64 (T,); y (T, W) in ``dtype`` or None; post / pre
+    float32 gains, one number () or per channel (W,); conv float32 (taps, W) or None with ``state`` float32
+    (banks, taps - 1, W); ``step``: the ragged step (entries, banks, positions).  Returns (out in ``dtype``, x')."""
+    _C.require_cuda(pre, x, tokens, embed, y, post, conv, state)
+    src = x if x is not None else embed
+    rows, width = (x.shape[0] if x is not None else tokens.numel()), src.shape[1]
+    if x is not None:
+        _check(x, torch.float32, (rows, width), "x")
+    else:
+        _check(embed, dtype, embed.shape, "embed")
+        _check(tokens, torch.int64, (rows,), "tokens")
+    if y is not None:
+        _check(y, dtype, (rows, width), "y")
+    for name, g in (("pre", pre), ("post", post)):
+        if g is not None and (g.dtype != torch.float32 or g.numel() not in (1, width) or not g.is_contiguous()):
+            raise ValueError(f"{name} must be float32, one number or ({width},)")
+    taps = banks = 0
+    if conv is not None:
+        taps = conv.shape[0]
+        _check(conv, torch.float32, (taps, width), "conv")
+        if taps > 1:
+            banks = state.shape[0]
+            _check(state, torch.float32, (banks, taps - 1, width), "state")
+        banks = max(banks, 1)
+        if step.num_tokens != rows:
+            raise ValueError("the step's rows and x's differ")
+    out = torch.empty((rows, width), dtype=dtype, device=src.device)
+    x_out = torch.empty((rows, width), dtype=torch.float32, device=src.device) if want_x and (y is not None or x is None) else None
+    st = _C.load().mvllm_norm_conv(
+        _ptr(out), _ptr(x_out), _ptr(x), _ptr(embed if x is None else None), _ptr(tokens if x is None else None),
+        0 if embed is None else embed.shape[0], _ptr(y), _ptr(post if y is not None else None),
+        int(post is not None and post.numel() > 1), _ptr(pre), int(pre.numel() > 1), float(eps), _ptr(conv), taps,
+        _ptr(state if taps > 1 else None), banks, _ptr(step.cu_seqlens if taps else None),
+        _ptr(step.row_entry if taps else None), _ptr(step.bank_in if taps else None), _ptr(step.bank_out if taps else None),
+        _ptr(step.positions if taps else None), rows, width, _C.dtype_code(dtype), _C.current_stream_ptr(src.device))
+    _C.check(st, "norm_conv")
+    return out, (x_out if x_out is not None else x)
+
+
+def head_rope_store(proj: torch.Tensor, positions: torch.Tensor, num_heads: int, num_kv_heads: int, dim: int, vdim: int,
+                    head_dim: int, gain_q: torch.Tensor | None = None, gain_k: torch.Tensor | None = None,
+                    eps: float = 1e-6, q_scale: float = 1.0, rot_table: torch.Tensor | None = None,
+                    v_table: torch.Tensor | None = None, interleaved: bool = True, dst_row: torch.Tensor | None = None,
+                    slots: torch.Tensor | None = None, k_cache: torch.Tensor | None = None,
+                    v_cache: torch.Tensor | None = None, need_kv: bool = True):
+    """Per-head norms, rotary embedding, rotated values and the cache store of packed projection rows [q | k | v | ...].
+
+    ``rot_table`` float32 (max_position, rot_dims / 2, 2) and ``v_table`` (max_position, vdim / 2, 2) hold (cos, sin) per
+    pair; ``interleaved`` pairs dims 2i and 2i + 1, otherwise the halves.  Heads leave ``head_dim`` wide, zeros past
+    ``dim`` / ``vdim``; row t goes to row ``dst_row[t]`` of the packed results.  Returns (q, k, v), k and v None unless
+    ``need_kv``."""
+    _C.require_cuda(proj, positions, gain_q, gain_k, rot_table, v_table, dst_row, slots, k_cache, v_cache)
+    rows = proj.shape[0]
+    if proj.dim() != 2 or (proj.shape[1] > 1 and proj.stride(1) != 1) or proj.shape[1] < num_heads * dim + num_kv_heads * (dim + vdim):
+        raise ValueError("proj must be (T, >= q + k + v columns) with dense rows")
+    _check(positions, torch.int64, (rows,), "positions")
+    for name, g in (("gain_q", gain_q), ("gain_k", gain_k)):
+        if g is not None:
+            _check(g, torch.float32, (dim,), name)
+    tables = [t for t in (rot_table, v_table) if t is not None]
+    max_position = min((t.shape[0] for t in tables), default=1 << 62)
+    rot = 0 if rot_table is None else 2 * rot_table.shape[1]
+    for name, t, n in (("rot_table", rot_table, rot // 2), ("v_table", v_table, vdim // 2)):
+        if t is not None:
+            _check(t, torch.float32, (t.shape[0], n, 2), name)
+    if dst_row is not None:
+        _check(dst_row, torch.int32, (rows,), "dst_row")
+    num_slots = 0
+    if slots is not None:
+        _check(slots, torch.int64, (rows,), "slots")
+        for name, c in (("k_cache", k_cache), ("v_cache", v_cache)):
+            _check(c, proj.dtype, (*c.shape[:2], num_kv_heads, head_dim), name)
+        num_slots = min(k_cache.shape[0] * k_cache.shape[1], v_cache.shape[0] * v_cache.shape[1])
+    q = torch.empty((rows, num_heads, head_dim), dtype=proj.dtype, device=proj.device)
+    k = torch.empty((rows, num_kv_heads, head_dim), dtype=proj.dtype, device=proj.device) if need_kv else None
+    v = torch.empty_like(k) if need_kv else None
+    st = _C.load().mvllm_head_rope_store(
+        _ptr(q), _ptr(k), _ptr(v), _ptr(proj), proj.stride(0) if rows > 1 else proj.shape[1], _ptr(gain_q), _ptr(gain_k),
+        float(eps), float(q_scale), _ptr(rot_table), rot, _ptr(v_table), int(interleaved), max_position, _ptr(positions),
+        _ptr(dst_row), _ptr(slots), _ptr(k_cache if slots is not None else None), _ptr(v_cache if slots is not None else None),
+        num_slots, rows, num_heads, num_kv_heads, dim, vdim, head_dim, _C.dtype_code(proj.dtype),
+        _C.current_stream_ptr(proj.device))
+    _C.check(st, "head_rope_store")
+    return q, k, v
+
+
+def head_unrotate_gate(o: torch.Tensor, positions: torch.Tensor, vdim: int, gate: torch.Tensor | None = None,
+                       v_table: torch.Tensor | None = None, interleaved: bool = True,
+                       dst_row: torch.Tensor | None = None) -> torch.Tensor:
+    """``o`` (T, heads, head_dim) from attention over rotated values -> (T, heads * vdim): every head turned back by its
+    position (``v_table`` None: not) and multiplied by ``sigmoid(gate)``, gate (T, heads) with dense rows or None; row t is
+    read from row ``dst_row[t]``."""
+    _C.require_cuda(o, positions, gate, v_table, dst_row)
+    rows, heads, head_dim = o.shape
+    _check(o, o.dtype, (rows, heads, head_dim), "o")
+    _check(positions, torch.int64, (rows,), "positions")
+    if gate is not None and (gate.dtype != o.dtype or tuple(gate.shape) != (rows, heads) or (heads > 1 and gate.stride(1) != 1)):
+        raise ValueError("gate must be (T, heads) in o's dtype with dense rows")
+    if v_table is not None:
+        _check(v_table, torch.float32, (v_table.shape[0], vdim // 2, 2), "v_table")
+    if dst_row is not None:
+        _check(dst_row, torch.int32, (rows,), "dst_row")
+    out = torch.empty((rows, heads * vdim), dtype=o.dtype, device=o.device)
+    st = _C.load().mvllm_head_unrotate_gate(
+        _ptr(out), _ptr(o), _ptr(gate), heads if gate is None or rows == 1 else gate.stride(0), _ptr(v_table), int(interleaved),
+        1 << 62 if v_table is None else v_table.shape[0], _ptr(positions), _ptr(dst_row), rows, heads, vdim, head_dim,
+        _C.dtype_code(o.dtype), _C.current_stream_ptr(o.device))
+    _C.check(st, "head_unrotate_gate")
+    return out
+
+
+def chunk_decode_step(context_lens: torch.Tensor, block_tables: torch.Tensor, chunk: int, block_size: int,
+                      chunk_lens: torch.Tensor, slots: torch.Tensor) -> None:
+    """Per row of a decode batch over a cache that holds one attention chunk per sequence (``chunk`` 0: all of it): the
+    context length inside the chunk and the cache slot of the row's token, written to ``chunk_lens`` and ``slots`` (int64,
+    in place); 0 and -1 for rows whose context length is 0."""
+    _C.require_cuda(context_lens, block_tables, chunk_lens, slots)
+    batch = context_lens.numel()
+    for name, t in (("context_lens", context_lens), ("chunk_lens", chunk_lens), ("slots", slots)):
+        _check(t, torch.int64, (batch,), name)
+    _check(block_tables, torch.int32, (batch, block_tables.shape[1]), "block_tables")
+    st = _C.load().mvllm_chunk_decode_step(_ptr(chunk_lens), _ptr(slots), _ptr(context_lens), _ptr(block_tables),
+                                           block_tables.shape[1], int(chunk), block_size, batch,
+                                           _C.current_stream_ptr(context_lens.device))
+    _C.check(st, "chunk_decode_step")

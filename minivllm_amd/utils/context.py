@@ -22,6 +22,7 @@ class Context:
     slot_mapping: Optional[torch.Tensor] = None     # int64 [T], -1 = do not store
     context_lens: Optional[torch.Tensor] = None     # int64 (engine) or int32 [B]
     block_tables: Optional[torch.Tensor] = None     # int32 [B, MB], -1 padded
+    ragged: Optional[object] = None                 # engine.ragged.RaggedStep, for models that run ragged steps
 
 
 _context = Context()
@@ -37,7 +38,7 @@ def reset_context() -> None:
 
 
 def set_context(is_prefill, cu_seqlens_q=None, cu_seqlens_k=None, max_seqlen_q=0, max_seqlen_k=0,
-                slot_mapping=None, context_lens=None, block_tables=None) -> None:
+                slot_mapping=None, context_lens=None, block_tables=None, ragged=None) -> None:
     global _context
     _context = Context(is_prefill, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, max_seqlen_k,
-                       slot_mapping, context_lens, block_tables)
+                       slot_mapping, context_lens, block_tables, ragged)

@@ -31,6 +31,9 @@ def test_header_declares_expected_entry_points():
               "mvllm_prefill_paged", "mvllm_prefill_paged_int8", "mvllm_prefill_paged_int8_staged", "mvllm_prefill_paged_staged", "mvllm_prefill_paged_staged_workspace_bytes", "mvllm_prefill_paged_split", "mvllm_prefill_paged_int8_split", "mvllm_prefill_paged_split_plan", "mvllm_prefill_paged_split_workspace_bytes", "mvllm_qk_norm_rope_store", "mvllm_sample_tokens", "mvllm_sample_tokens_dev_offset", "mvllm_decode_advance", "mvllm_sample_tokens_workspace_bytes",
               "mvllm_add_rms_norm", "mvllm_linear_small_m", "mvllm_norm_linear_small_m", "mvllm_linear_small_m_plan",
               "mvllm_lm_head_sample", "mvllm_lm_head_sample_workspace_bytes",
+              "mvllm_paged_decode_sink", "mvllm_prefill_varlen_sink", "mvllm_prefill_paged_sink",
+              "mvllm_prefill_paged_split_sink", "mvllm_norm_conv", "mvllm_head_rope_store", "mvllm_head_unrotate_gate",
+              "mvllm_chunk_decode_step", "mvllm_gate_linear", "mvllm_mlstm_recurrent", "mvllm_mlstm_output",
               "mvllm_silu_and_mul", "mvllm_version", "mvllm_status_string"]:
         assert n in names
 
