@@ -552,11 +552,22 @@ int mvllm_gate_linear(float* out, const void* x, int64_t x_row_stride, const voi
  *   state of slot slots[e]: s_state fp32 [*, H, dim, vdim], n_state [*, H, dim], m_state [*, H]; s and n are updated,
  *   m by mvllm_mlstm_output; an entry that starts at position 0 starts from zeros.  slots < 0: the entry is skipped.
  * mvllm_mlstm_output: out [rows, H * vdim] = rms(num / den) * weight * sigmoid(gate), m_state[slot] = m_next.
+ * mvllm_mlstm_chunked: the recurrence's results for entries of many rows in blocks of 64 rows on the matrix unit (bf16,
+ *   dim <= 256, dim and vdim multiples of 8; others: MVLLM_ERR_UNSUPPORTED).  segments int32 [num_segments, 4]: entry,
+ *   first row, rows, flags (1 first, 2 last, 4 the only one of its entry), the segments of an entry in order and next to
+ *   each other, all but the last a multiple of 64 rows.  split != 0 (some entry has several): workspace of
+ *   mvllm_mlstm_chunked_workspace_bytes.
  */
 int mvllm_mlstm_recurrent(float* num, float* den, float* m_next, const void* proj, int64_t proj_row_stride,
                           const float* gates, float* s_state, float* n_state, const float* m_state,
                           const int32_t* cu_seqlens, const int32_t* slots, const int64_t* positions, int entries,
                           int num_heads, int dim, int vdim, float q_scale, float floor, int dtype, void* stream);
+size_t mvllm_mlstm_chunked_workspace_bytes(int num_segments, int num_heads, int dim, int vdim);
+int mvllm_mlstm_chunked(float* num, float* den, float* m_next, const void* proj, int64_t proj_row_stride,
+                        const float* gates, float* s_state, float* n_state, const float* m_state,
+                        const int32_t* cu_seqlens, const int32_t* slots, const int64_t* positions,
+                        const int32_t* segments, int num_segments, int split, int num_heads, int dim, int vdim,
+                        float q_scale, float floor, int dtype, void* workspace, size_t workspace_bytes, void* stream);
 int mvllm_mlstm_output(void* out, const float* num, const float* den, const float* weight, const void* gate,
                        int64_t gate_row_stride, float eps, const float* m_next, float* m_state,
                        const int32_t* cu_seqlens, const int32_t* row_entry, const int32_t* slots, int64_t rows,

@@ -93,6 +93,9 @@ SIGNATURES = {
                                   c_int, c_void_p]),
     "mvllm_mlstm_recurrent": (c_int, [c_void_p] * 4 + [c_int64] + [c_void_p] * 7 + [c_int] * 4 + [c_float, c_float, c_int,
                                                                                               c_void_p]),
+    "mvllm_mlstm_chunked_workspace_bytes": (c_size_t, [c_int] * 4),
+    "mvllm_mlstm_chunked": (c_int, [c_void_p] * 4 + [c_int64] + [c_void_p] * 8 + [c_int] * 5 + [c_float, c_float, c_int,
+                                                                                            c_void_p, c_size_t, c_void_p]),
     "mvllm_mlstm_output": (c_int, [c_void_p] * 5 + [c_int64, c_float] + [c_void_p] * 5 + [c_int64, c_int, c_int, c_int,
                                                                                       c_void_p]),
 }

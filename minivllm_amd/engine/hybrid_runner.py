@@ -43,8 +43,8 @@ class HybridModelRunner(ModelRunner):
     @torch.inference_mode()
     def forward_step(self, seqs, layer_outputs=None):
         """Run every sequence's scheduled tokens; returns (hidden rows, the step)."""
-        step = ragged_step(seqs, self.model.windows, self.block_size, self.device)
-        set_context(step.long_rows > 0, ragged=step)
+        step = ragged_step(seqs, self.model.windows, self.block_size, self.device, self.model.memory_units)
+        set_context(step.multi_rows > 0, ragged=step)
         try:
             hidden = self.model(step.input_ids, step.positions, layer_outputs)
         finally:
@@ -115,7 +115,7 @@ class HybridModelRunner(ModelRunner):
         lens, slots = [t[:bs] for t in v["chunk_lens"]], [t[:bs] for t in v["chunk_slots"]]
         tables = [t[:bs] for t in v["tables"]]
         windows = [WindowStep(num_decode=bs, slots=s, chunk_lens=n, decode_tables=t) for s, n, t in zip(slots, lens, tables)]
-        step = RaggedStep(num_tokens=bs, num_entries=bs, num_single=bs, input_ids=v["input_ids"][:bs],
+        step = RaggedStep(num_tokens=bs, num_entries=bs, num_single=bs, num_short=bs, input_ids=v["input_ids"][:bs],
                           positions=v["positions"][:bs], cu_seqlens=v["cu_seqlens"][:bs + 1], row_entry=v["row_entry"][:bs],
                           bank_in=v["banks"][:bs], bank_out=v["banks"][:bs], state_slots=v["state_slots"][:bs], windows=windows)
         set_context(False, ragged=step)

@@ -1,10 +1,12 @@
 """Metadata of a ragged step: entries of any length (portions of prompts beside single decoded tokens) in one packed batch.
 
-Rows are packed entry by entry, entries of one token first.  Attention sees a row's entry cut at chunk borders: the piece
+Rows are packed entry by entry: entries of one token first, then short ones, then long ones.  Attention sees a row's entry cut at chunk borders: the piece
 that goes on in a chunk whose earlier tokens are cached reads the cache (``prefixed``), pieces that start a chunk read the
 packed keys and values of the step (``fresh``), single tokens take the decode kernel.  Pieces are sorted in that order
 (``dst_row``), so that each kernel runs over consecutive rows.  Only the tokens of an entry's last chunk stay cached; where
-the entry also reads the chunk before, whose blocks they go to, they are stored after attention (``late_slots``)."""
+the entry also reads the chunk before, whose blocks they go to, they are stored after attention (``late_slots``).
+A recurrence takes single and short entries row by row and long ones in blocks of rows, cut into ``segments`` that run side
+by side where there are too few of them to fill the GPU."""
 from __future__ import annotations
 
 from dataclasses import dataclass, field
@@ -45,9 +47,37 @@ class RaggedStep:
     bank_out: torch.Tensor
     state_slots: torch.Tensor                         # int32 [entries]
     windows: list = field(default_factory=list)       # WindowStep per window
-    long_rows: int = 0                                # rows of entries with more than one token
+    multi_rows: int = 0                               # rows of entries with more than one token
+    num_short: int = 0                                # entries below LONG_ROWS (the first ones)
+    segments: Optional[torch.Tensor] = None           # int32 [n, 4] of long entries: entry, first row, rows, flags
+    split: bool = False                               # some long entry has more than one segment
     order: list = field(default_factory=list)         # entry e of the packing is sequence order[e] of the caller
     starts: list = field(default_factory=list)        # first packed row of the caller's sequence i
+
+
+LONG_ROWS = 32                 # an entry of at least this many rows is long
+BLOCK_ROWS = 64                # rows per block of a recurrence's block form: segments are whole blocks
+FILL_WORKGROUPS = 512          # segments are made shorter until there are this many workgroups ...
+MIN_SEGMENT_ROWS = 256         # ... but not shorter than this
+
+
+def _segments(lens, cu, units):
+    """[entry, first row, rows, flags (1 first, 2 last, 4 only)] of every long entry."""
+    long_entries = [e for e, n in enumerate(lens) if n >= LONG_ROWS]
+    total = int(sum(lens[e] for e in long_entries))
+    length = total
+    if long_entries and units and len(long_entries) * units < FILL_WORKGROUPS // 2:
+        length = max(-(-total * units // (FILL_WORKGROUPS * BLOCK_ROWS)) * BLOCK_ROWS, MIN_SEGMENT_ROWS)
+    out = []
+    for e in long_entries:
+        n, at = int(lens[e]), int(cu[e])
+        pieces = max(-(-n // length), 1)
+        size = -(-n // (pieces * BLOCK_ROWS)) * BLOCK_ROWS
+        cuts = list(range(0, n, size)) + [n]
+        for i, (lo, hi) in enumerate(zip(cuts, cuts[1:])):
+            first, last = i == 0, hi == n
+            out.append([e, at + lo, hi - lo, int(first) | 2 * int(last) | 4 * int(first and last)])
+    return out
 
 
 def _pad_tables(tables):
@@ -123,11 +153,12 @@ def _window_arrays(items, window, index, block_size, cu):
     return out, counts
 
 
-def ragged_arrays(seqs, windows, block_size):
+def ragged_arrays(seqs, windows, block_size, memory_units=0):
     """Host side of a step over ``seqs``: each runs its tokens [num_computed_tokens, + num_scheduled_tokens).  Returns
     (arrays, window arrays, window counts, facts), everything in numpy; the sequences' convolution banks flip for entries
     of more than one token."""
-    order = sorted(range(len(seqs)), key=lambda i: seqs[i].num_scheduled_tokens > 1)        # stable
+    kind = [(n > 1) + (n >= LONG_ROWS) for n in (s.num_scheduled_tokens for s in seqs)]
+    order = sorted(range(len(seqs)), key=lambda i: kind[i])                                  # stable
     items = [(seqs[i].num_computed_tokens, seqs[i].num_scheduled_tokens, seqs[i]) for i in order]
     lens = np.asarray([n for _, n, _ in items], dtype=np.int64)
     cu = np.concatenate([[0], np.cumsum(lens)]).astype(np.int32)
@@ -148,14 +179,17 @@ def ragged_arrays(seqs, windows, block_size):
     for e, i in enumerate(order):
         starts[i] = int(cu[e])
     singles = int((lens == 1).sum())
-    facts = dict(num_tokens=int(cu[-1]), num_entries=len(items), num_single=singles, long_rows=int(cu[-1]) - singles,
-                 order=order, starts=starts)
+    segments = _segments(lens, cu, memory_units) if memory_units else []
+    if segments:
+        arrays["segments"] = np.asarray(segments, dtype=np.int32)
+    facts = dict(num_tokens=int(cu[-1]), num_entries=len(items), num_single=singles, multi_rows=int(cu[-1]) - singles,
+                 num_short=int((lens < LONG_ROWS).sum()), split=any(not s[3] & 4 for s in segments), order=order, starts=starts)
     return arrays, [a for a, _ in per_window], [c for _, c in per_window], facts
 
 
-def ragged_step(seqs, windows, block_size, device) -> RaggedStep:
+def ragged_step(seqs, windows, block_size, device, memory_units=0) -> RaggedStep:
     """The step's device tensors: one copy per integer type, every tensor a 16-byte aligned slice of it."""
-    arrays, window_arrays, counts, facts = ragged_arrays(seqs, windows, block_size)
+    arrays, window_arrays, counts, facts = ragged_arrays(seqs, windows, block_size, memory_units)
     named = [((None, k), a) for k, a in arrays.items()]
     for g, wa in enumerate(window_arrays):
         named += [((g, k), a) for k, a in wa.items()]

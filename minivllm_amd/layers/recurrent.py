@@ -48,6 +48,12 @@ def gate_linear(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None
     return out
 
 
+def chunked_takes(proj: torch.Tensor, dim: int, vdim: int) -> bool:
+    """Whether the block form is built for this layer (otherwise every row goes through the recurrence in turn)."""
+    return (proj.dtype == torch.bfloat16 and dim % 8 == 0 and vdim % 8 == 0 and dim <= 256 and proj.data_ptr() % 16 == 0
+            and proj.shape[1] % 8 == 0 and (proj.shape[0] == 1 or proj.stride(0) % 8 == 0))
+
+
 def mlstm(step, proj: torch.Tensor, gates: torch.Tensor, gate_col: int, weight: torch.Tensor, state: MlstmState,
           eps: float) -> torch.Tensor:
     """The mLSTM mixer between its projections: (T, H * vdim) = rms(recurrence) * weight * sigmoid(gate).
@@ -74,10 +80,19 @@ def mlstm(step, proj: torch.Tensor, gates: torch.Tensor, gate_col: int, weight: 
     out = torch.empty((rows, heads * vdim), dtype=proj.dtype, device=dev)
     lib = _C.load()
     scale = dim ** -0.5
-    _C.check(lib.mvllm_mlstm_recurrent(
-        _ptr(num), _ptr(den), _ptr(m_next), _ptr(proj), stride, _ptr(gates), _ptr(state.s), _ptr(state.n), _ptr(state.m),
-        _ptr(step.cu_seqlens), _ptr(step.state_slots), _ptr(step.positions), step.num_entries, heads, dim, vdim, scale,
-        DEN_FLOOR, code, stream), "mlstm_recurrent")
+    common = (_ptr(num), _ptr(den), _ptr(m_next), _ptr(proj), stride, _ptr(gates), _ptr(state.s), _ptr(state.n), _ptr(state.m),
+              _ptr(step.cu_seqlens), _ptr(step.state_slots), _ptr(step.positions))
+    blocks = step.segments is not None and chunked_takes(proj, dim, vdim)
+    row_by_row = step.num_short if blocks else step.num_entries
+    if row_by_row:
+        _C.check(lib.mvllm_mlstm_recurrent(*common, row_by_row, heads, dim, vdim, scale, DEN_FLOOR, code, stream),
+                 "mlstm_recurrent")
+    if blocks:
+        count = step.segments.shape[0]
+        nbytes = lib.mvllm_mlstm_chunked_workspace_bytes(count, heads, dim, vdim) if step.split else 0
+        ws = torch.empty(nbytes, dtype=torch.uint8, device=dev) if nbytes else None
+        _C.check(lib.mvllm_mlstm_chunked(*common, _ptr(step.segments), count, int(step.split), heads, dim, vdim, scale,
+                                         DEN_FLOOR, code, _ptr(ws), nbytes, stream), "mlstm_chunked")
     _C.check(lib.mvllm_mlstm_output(
         _ptr(out), _ptr(num), _ptr(den), _ptr(weight), proj.data_ptr() + gate_col * proj.element_size(), stride, float(eps),
         _ptr(m_next), _ptr(state.m), _ptr(step.cu_seqlens), _ptr(step.row_entry), _ptr(step.state_slots), rows, heads, vdim,

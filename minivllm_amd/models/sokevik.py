@@ -47,7 +47,7 @@ def kernel_sources(config: dict) -> list[str]:
     """The csrc files a model of this configuration runs on."""
     sources = ["capi.hip", "activation.hip", "linear_small.hip", "norm_conv.hip"]
     if any(e["type"] == "mlstm" for e in config["layers"]):
-        sources += ["gate_linear.hip", "mlstm.hip"]
+        sources += ["gate_linear.hip", "mlstm.hip", "mlstm_chunk.hip"]
     attention = [e["mixer"] for e in config["layers"] if e["type"] == "attention"]
     if attention:
         sources += ["head_rope.hip", "store_kvcache.hip", "paged_decode.hip", "prefill_varlen.hip", "prefill_split.hip",
@@ -152,6 +152,9 @@ class SokevikForCausalLM(nn.Module):
         self.windows = sorted({_window(e["mixer"]) for e in layers if e["type"] == "attention"})
         self.layer_stack = nn.ModuleList([
             SokevikLayer(shared[j], layers[i], self.windows, block_size, dtype, self.eps) for i, j in enumerate(self.owners)])
+        # workgroups per segment of the block form of the matrix memory (0: no such layer): how far portions are cut
+        self.memory_units = min((e["mixer"]["heads"] * -(-e["mixer"]["vdim"] // 128) for e in layers if e["type"] == "mlstm"),
+                                default=0)
         max_position, tables = config.get("max_position", 4096), {}
 
         def table(base, dims, scaling):
@@ -186,7 +189,7 @@ class SokevikForCausalLM(nn.Module):
         width = c["width"]
 
         def normal(*shape, std=1.0, mean=0.0):
-            return (torch.randn(*shape, generator=g, device=self.device) * std + mean).to(torch.bfloat16)
+            return (torch.randn(shape, generator=g, device=self.device) * std + mean).to(torch.bfloat16)
 
         t = {"embed": normal(c["vocab"], width), "head": normal(c["vocab"], width, std=width ** -0.5),
              "final.norm": normal(mean=1.0, std=0.0)}

@@ -169,7 +169,7 @@ def random_weights(config, seed=0, dtype=torch.bfloat16):
     width, taps = config["width"], config["canon"]["taps"]
 
     def normal(*shape, std=1.0, mean=0.0):
-        return (torch.randn(*shape, generator=g) * std + mean).to(dtype)
+        return (torch.randn(shape, generator=g) * std + mean).to(dtype)
 
     w = {"embed": normal(config["vocab"], width), "head": normal(config["vocab"], width, std=width ** -0.5),
          "final.norm": normal(std=0.1, mean=1.0)}

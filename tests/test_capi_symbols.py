@@ -34,6 +34,7 @@ def test_header_declares_expected_entry_points():
               "mvllm_paged_decode_sink", "mvllm_prefill_varlen_sink", "mvllm_prefill_paged_sink",
               "mvllm_prefill_paged_split_sink", "mvllm_norm_conv", "mvllm_head_rope_store", "mvllm_head_unrotate_gate",
               "mvllm_chunk_decode_step", "mvllm_gate_linear", "mvllm_mlstm_recurrent", "mvllm_mlstm_output",
+              "mvllm_mlstm_chunked", "mvllm_mlstm_chunked_workspace_bytes",
               "mvllm_silu_and_mul", "mvllm_version", "mvllm_status_string"]:
         assert n in names
 
