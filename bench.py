@@ -38,7 +38,7 @@ def parse_args():
     ap.add_argument("--warmup", type=int, default=5)
     ap.add_argument("--seed", type=int, default=0)
     ap.add_argument("--block-size", type=int, default=16, help="block size of the headline decode workload")
-    ap.add_argument("--only", default="", help="comma list out of decode256,prefill,prefill_long,store,int8,reference_shapes,decode_small,demo_shape,head_dims,fused_qk,sampler,mfma_probe,prefill_timeline,loads_probe,engine,engine16,engine64,cpu to restrict the extras (the headline decode always runs)")
+    ap.add_argument("--only", default="", help="comma list out of decode256,prefill,prefill_long,store,int8,reference_shapes,decode_small,demo_shape,head_dims,fused_qk,sampler,mfma_probe,prefill_timeline,loads_probe,engine,engine16,engine64,cpu to restrict the extras (the headline decode always runs); only when named: sokevik, the Sokevik design beside the Qwen3-style decoder, models and kernels (sokevik_kernels: kernels alone)")
     ap.add_argument("--no-cpu", action="store_true", help="skip the cpu_baseline leg")
     ap.add_argument("--calib-copy", action="store_true",
                     help="also launch three 1 GiB device copies (reads 1 GiB, writes 1 GiB each) so a rocprofv3 "
@@ -910,6 +910,195 @@ def bench_engine(args, max_num_sequences, graph):
     }
 
 
+def graph_call_ms(args, fn, calls=20):
+    """Time of one call among ``calls`` of them inside a hipGraph (a small call is latency, which back-to-back launches
+    from the host would hide behind the host's own)."""
+    import torch
+    for _ in range(3):
+        fn()
+    torch.cuda.synchronize()
+    g = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(g):
+        for _ in range(calls):
+            fn()
+    return time_steps(g.replay, args.steps, 2, EXTRA_WARM_MS)[1] / calls
+
+
+# widths, heads and feed-forwards of decoders of about 1.7 and 8 billion parameters, a few layers of them
+SOKEVIK_SIZES = {"w2048": dict(width=2048, heads=16, kv=8, ff=6144, layers=8), "w4096": dict(width=4096, heads=32, kv=8, ff=12288, layers=4)}
+SOKEVIK_CHUNK, SOKEVIK_DIM, SOKEVIK_VDIM = 1024, 128, 256      # attention chunk; key and value size of a memory head
+
+
+def sokevik_models(size, block_size=16):
+    """Sokevik (attention and matrix-memory layers in turn, a feed-forward behind each) and the Qwen3-style decoder of the
+    same width, heads, feed-forward and number of layers, as engine configurations."""
+    z, vocab = SOKEVIK_SIZES[size], 32000
+    mlp = {"kind": "dense", "ff": z["ff"]}
+    attn = {"type": "attention", "mlp": mlp, "mixer": {
+        "heads": z["heads"], "kv_heads": z["kv"], "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": SOKEVIK_CHUNK},
+        "rot": {"base": 500000.0, "dims": 128, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}}
+    memory = {"type": "mlstm", "mlp": mlp, "mixer": {"heads": z["width"] // SOKEVIK_VDIM, "dim": SOKEVIK_DIM, "vdim": SOKEVIK_VDIM, "gate_cap": 15.0}}
+    sokevik = {"architecture": "Sokevik", "width": z["width"], "vocab": vocab, "canon": {"taps": 4}, "norm": {"eps": 1e-6},
+               "layers": [(attn, memory)[i % 2] for i in range(z["layers"])]}
+    qwen3 = dict(vocab_size=vocab, hidden_size=z["width"], num_layers=z["layers"], num_heads=z["heads"], num_kv_heads=z["kv"], head_dim=128,
+                 intermediate_size=z["ff"], base=1_000_000, rms_norm_epsilon=1e-6, qkv_bias=False, ffn_bias=False, scale=128 ** -0.5,
+                 tie_word_embeddings=False)
+    return sokevik, qwen3
+
+
+def engine_throughput(args, config, prompts, prompt_len, new_tokens):
+    """Prompt and output tokens per second of ``LLMEngine.generate`` (sampling, scheduling and metadata included)."""
+    import torch
+    from minivllm_amd.engine.llm_engine import LLMEngine
+    from minivllm_amd.sampling_parameters import SamplingParams
+    longest = prompt_len + new_tokens
+    engine = LLMEngine({**config, "block_size": 16, "max_num_batched_tokens": max(prompts * prompt_len, longest), "max_num_sequences": prompts,
+                        "max_cached_blocks": prompts * -(-longest // 16), "max_position": longest, "max_model_length": longest,
+                        "enforce_eager": False, "dtype": "bf16", "eos": -1, "seed": args.seed})
+    g = torch.Generator().manual_seed(args.seed)
+    for timed in (False, False, True):                     # the same load twice before it counts, with other tokens each time
+        ids = [torch.randint(0, 32000, (prompt_len,), generator=g).tolist() for _ in range(prompts)]
+        for key in engine.stats:
+            engine.stats[key] = 0
+        torch.cuda.synchronize()
+        engine.generate(ids, SamplingParams(temperature=0.6, max_tokens=new_tokens, ignore_eos=True))
+    st = engine.stats
+    return {"prefill_tok_per_s": prompts * prompt_len / st["prefill_s"], "decode_tok_per_s": prompts * (new_tokens - 1) / st["decode_s"]}
+
+
+def bench_sokevik(args, with_models=True):
+    """The Sokevik design beside the Qwen3-style decoder at equal width, heads, feed-forward and layers (random weights):
+    whole-engine prefill and decode throughput, and every kernel of the design beside the like kernel of the other model,
+    each against its own roofline (the larger of its bytes over the HBM peak and its flops over the matrix peak)."""
+    import torch
+    out = {"models": {}, "kernels": {}}
+    for size in SOKEVIK_SIZES if with_models else ():
+        for prompts, prompt_len, new in ((4, 2048, 128), (32, 512, 128), (1, 16384, 64)):
+            leg = {}
+            for name, config in zip(("sokevik", "qwen3"), sokevik_models(size)):
+                leg[name] = engine_throughput(args, config, prompts, prompt_len, new)
+                torch.cuda.empty_cache()
+            out["models"][f"{size}_{prompts}x{prompt_len}+{new}"] = leg
+    for rows, calls in ((8192, 4), (64, 20)):
+        with torch.inference_mode():
+            out["kernels"][f"{rows}_rows"] = bench_sokevik_kernels(args, rows, calls)
+        torch.cuda.empty_cache()
+    return out
+
+
+def bench_sokevik_kernels(args, rows, calls):
+    """Kernels at width 4096: 8192 prompt rows (8 prompts of 1024, one attention chunk each), or 64 decoded rows with 1024
+    tokens in the chunk (the matrix memory and attention over 256 sequences there: their states must not fit a cache)."""
+    import torch
+    import torch.nn.functional as F
+    from minivllm_amd.engine.hybrid_cache import HybridCacheManager
+    from minivllm_amd.engine.ragged import ragged_step
+    from minivllm_amd.engine.sequence import Sequence
+    from minivllm_amd.layers.attention import flash_attention_prefill, paged_attention_decode
+    from minivllm_amd.layers.basic import RotaryEmbedding, rotary_pair_table
+    from minivllm_amd.layers.fused import (add_rms_norm, head_rope_store, head_unrotate_gate, linear_small_m, norm_conv,
+                                           qk_norm_rope_store, silu_and_mul)
+    from minivllm_amd.layers.recurrent import MlstmState, gate_linear, mlstm
+
+    dev = torch.device("cuda:0")
+    gen = torch.Generator(device=dev).manual_seed(args.seed)
+    rnd = lambda *shape, dtype=torch.bfloat16: torch.randn(*shape, generator=gen, device=dev).to(dtype)
+    prefill = rows > 64
+    width, hq, hkv, d, chunk, bs = 4096, 32, 8, 128, SOKEVIK_CHUNK, 16
+    heads, dim, vdim = width // SOKEVIK_VDIM, SOKEVIK_DIM, SOKEVIK_VDIM
+
+    def step_of(lengths, before, slots=None):
+        m = HybridCacheManager([chunk], len(lengths) * chunk // bs, bs, slots or len(lengths))
+        seqs = []
+        for n, p0 in zip(lengths, before):
+            seq = Sequence([0] * (p0 + n), block_size=bs)
+            m.allocate(seq)
+            seq.num_computed_tokens, seq.num_scheduled_tokens = p0, n
+            seqs.append(seq)
+        return ragged_step(seqs, [chunk], bs, dev, heads * -(-vdim // 128))
+
+    lengths = [chunk] * (rows // chunk) if prefill else [1] * rows
+    step = step_of(lengths, [0] * len(lengths) if prefill else [chunk - 1] * rows)
+    entries = len(lengths)
+    res = {}
+
+    def leg(name, kernel, nbytes, like, like_kernel, like_bytes, flops=0.0, like_flops=0.0):
+        def one(fn, b, f):
+            ms = graph_call_ms(args, fn, calls)
+            floor = max(b / (HBM_PEAK_GBS * 1e9), f / (MFMA_BF16_PEAK_TFLOPS * 1e12)) * 1e3
+            return {"us": ms * 1e3, "roofline_us": floor * 1e3, "frac": floor / ms}
+        mine, other = one(kernel, nbytes, flops), one(like, like_bytes, like_flops)
+        res[name] = {**mine, "like": {"name": like_kernel, **other}, "times_further": other["frac"] / mine["frac"]}
+
+    # norm, residual, norm and short convolution | residual norm
+    x, y, z = rnd(rows, width, dtype=torch.float32), rnd(rows, width), rnd(rows, width)
+    state = torch.zeros(2 * entries + 1, 3, width, device=dev)
+    one_gain, gains, taps = torch.ones((), device=dev), torch.ones(width, device=dev), rnd(4, width, dtype=torch.float32)
+    leg("norm_conv", lambda: norm_conv(step, one_gain, 1e-6, torch.bfloat16, x=x, y=y, post=one_gain, conv=taps, state=state),
+        rows * width * 12 + (1 if prefill else 2) * entries * 3 * width * 4 + 4 * width * 4,
+        lambda: add_rms_norm(y, gains, 1e-6, z), "add_rms_norm", rows * width * 8)
+    # norms, rotations (values too) and cache store | q / k norm, rotation and cache store
+    cols = hq * d + 2 * hkv * d
+    proj, positions = rnd(rows, cols + hq), step.positions
+    gain, table = torch.ones(d, device=dev), rotary_pair_table(500000.0, d, 2048, None).to(dev)
+    kc = torch.zeros(entries * chunk // bs, bs, hkv, d, dtype=torch.bfloat16, device=dev)
+    vc, w = torch.zeros_like(kc), step.windows[0]
+    packed = 2 * hkv if prefill else 0                     # keys and values packed for prefill as well
+    moved = rows * (2 * cols + (hq + packed + 2 * hkv) * d * 2 + 16)
+    q = proj[:, :hq * d].unflatten(-1, (hq, d))
+    k, v = (proj[:, i * hkv * d + hq * d:(i + 1) * hkv * d + hq * d].unflatten(-1, (hkv, d)) for i in range(2))
+    rotary = RotaryEmbedding(1_000_000, d, 2048).to(dev)
+    leg("head_rope_store", lambda: head_rope_store(proj, positions, hq, hkv, d, d, d, gain, gain, 1e-6, 1.0, table, table, True, w.dst_row,
+                                                   w.slots, kc, vc, need_kv=prefill),
+        moved, lambda: qk_norm_rope_store(q, k, v, positions, rotary.cos_sin_cache, gain, 1e-6, w.slots, kc, vc, need_kv=prefill),
+        "qk_norm_rope_store", moved)
+    # values turned back and gated | silu and product (elementwise)
+    wide = hq * d * 4 // 6 // 8 * 8                        # as many bytes
+    o, gate, act = rnd(rows, hq, d), proj[:, cols:cols + hq], rnd(rows, 2 * wide)
+    leg("head_unrotate_gate", lambda: head_unrotate_gate(o, positions, d, gate, table), rows * (hq * d * 4 + hq * 2),
+        lambda: silu_and_mul(act), "silu_and_mul", rows * wide * 6)
+    del x, y, z, state, act, o
+    # attention with a sink | without
+    sink, scale = torch.ones(hq, device=dev), d ** -0.5
+    if prefill:
+        q, k, v = rnd(rows, hq, d), rnd(rows, hkv, d), rnd(rows, hkv, d)
+        att = (0, rows * (2 * hq + 2 * hkv) * d * 2, 4.0 * hq * d * entries * chunk * (chunk + 1) / 2)
+        leg("attention", lambda: flash_attention_prefill(q, k, v, w.fresh_cu, scale, hq, hkv, d, sink=sink), att[1],
+            lambda: flash_attention_prefill(q, k, v, w.fresh_cu, scale, hq, hkv, d), "packed prefill", att[1], att[2], att[2])
+        plain = lambda: flash_attention_prefill(q, k, v, w.fresh_cu, scale, hq, hkv, d)
+    else:
+        batch = 256
+        step = step_of([1] * batch, [chunk - 1] * batch)
+        w, entries, rows = step.windows[0], batch, batch
+        kc, vc, q = rnd(batch * chunk // bs, bs, hkv, d), rnd(batch * chunk // bs, bs, hkv, d), rnd(batch, hq, d)
+        att = (0, batch * (chunk * 2 * hkv * d * 2 + 2 * hq * d * 2 + 4 * chunk // bs), 0.0)
+        run = lambda **kw: paged_attention_decode(q, kc, vc, w.decode_tables, w.chunk_lens, scale, hq, hkv, d, bs, **kw)
+        leg("attention", lambda: run(sink=sink), att[1], run, "paged decode", att[1])
+        plain = run
+    # the matrix memory (recurrence, norm and output gate) | attention of the same rows
+    n = heads * (2 * dim + vdim)
+    proj = rnd(rows, n + heads * vdim)
+    gates = torch.cat([rnd(rows, heads, dtype=torch.float32), F.logsigmoid(rnd(rows, heads, dtype=torch.float32) + 4)], 1).contiguous()
+    memory = MlstmState.allocate(entries, heads, dim, vdim, dev)
+    weight = torch.ones(heads * vdim, device=dev)
+    nbytes = rows * (2 * (n + heads * vdim) + 2 * heads * vdim + 8 * heads) + (1 if prefill else 2) * entries * heads * dim * (vdim + 1) * 4
+    # per row and head: the state's update and its product with q; in blocks also the weighted scores and values of half a block
+    flops = rows * heads * (4.0 * dim * vdim + (64.0 * (dim + vdim) if prefill else 0.0))
+    leg("mlstm", lambda: mlstm(step, proj, gates, n, weight, memory, 1e-6), nbytes, plain, "attention of the same rows", att[1],
+        flops if prefill else 0.0, att[2])
+    # gate projections | a plain projection of as many columns
+    h, gw, bias = rnd(rows, width), rnd(2 * heads, width), torch.zeros(2 * heads, device=dev)
+    gate_bytes = rows * width * 2 + 2 * heads * width * 2
+    if prefill:
+        like, like_name, gb, hh = (lambda: F.linear(h, gw)), "library product", gate_bytes + rows * heads * 4, h
+    else:
+        hh = h[:64].contiguous()
+        gate_bytes = 64 * width * 2 + 2 * heads * width * 2
+        like, like_name, gb = (lambda: linear_small_m(hh, gw)), "linear_small_m", gate_bytes + 64 * heads * 4
+    leg("gate_linear", lambda: gate_linear(hh, gw, bias, heads, 15.0), gate_bytes + hh.shape[0] * heads * 8, like, like_name, gb)
+    return res
+
+
 def summary_of(line):
     """The figures of every quantity the metric names, in a few hundred characters, for the end of the JSON line."""
     ex = line["extra"]
@@ -1013,6 +1202,10 @@ def main():
             extra["engine_16seq_graph"] = bench_engine(args, 16, True)
         if "engine64" in only:
             extra["engine_64seq_graph"] = bench_engine(args, 64, True)
+    if "sokevik" in only:
+        extra["sokevik"] = bench_sokevik(args)
+    elif "sokevik_kernels" in only:                    # without the models, as a kernel trace wants
+        extra["sokevik"] = bench_sokevik(args, with_models=False)
 
     if "loads_only" in head:
         extra["decode_loads_only"] = head["loads_only"]

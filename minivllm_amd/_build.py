@@ -88,8 +88,14 @@ def build_library(verbose: bool = True, jobs: int = 8) -> str:
 
 
 def part_path(sources) -> str:
-    tag = hashlib.sha1(" ".join(sorted(sources)).encode()).hexdigest()[:10]
-    return os.path.join(PKG_DIR, f"libminivllm_part_{tag}.so")
+    """Named after the sources' names and contents and the headers: a changed checkout builds another one."""
+    digest = hashlib.sha1(" ".join(HIPCC_FLAGS).encode())
+    headers = [f for f in os.listdir(CSRC) if f.endswith(".h")]
+    for name in sorted([*sources, "absent_kernels.hip", *headers]):
+        digest.update(name.encode())
+        with open(os.path.join(CSRC, name), "rb") as f:
+            digest.update(f.read())
+    return os.path.join(PKG_DIR, f"libminivllm_part_{digest.hexdigest()[:10]}.so")
 
 
 def build_part(sources, verbose: bool = False, jobs: int = 8) -> str:

@@ -2,6 +2,8 @@
 #pragma once
 #include <hip/hip_runtime.h>
 #include <stdint.h>
+#include <type_traits>
+
 #include "../../include/minivllm_amd.h"
 
 namespace mvllm {
@@ -85,6 +87,23 @@ __device__ __forceinline__ float wave_max(float x) {
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) x = fmaxf(x, __shfl_xor(x, o, 64));
   return x;
+}
+
+// Sum over the 16 lanes of a row, in every lane, without the LDS pipe (lane permutations inside the vector unit), and the
+// sum of four such rows' sums.
+__device__ __forceinline__ float row16_sum(float x) {
+  auto moved = [](float v, auto CTRL) __attribute__((always_inline)) {
+    return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), decltype(CTRL)::value, 0xf, 0xf, false));
+  };
+  x += moved(x, std::integral_constant<int, 0xB1>{});      // lane ^ 1
+  x += moved(x, std::integral_constant<int, 0x4E>{});      // lane ^ 2
+  x += moved(x, std::integral_constant<int, 0x141>{});     // mirrored half rows: the other four of eight
+  x += moved(x, std::integral_constant<int, 0x140>{});     // mirrored rows: the other eight
+  return x;
+}
+__device__ __forceinline__ float four_rows_sum(float x) {
+  auto row = [x](int lane) __attribute__((always_inline)) { return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(x), lane)); };
+  return (row(0) + row(16)) + (row(32) + row(48));
 }
 
 // 16-byte global load with the non-temporal hint: for data that is read once and should stream through the

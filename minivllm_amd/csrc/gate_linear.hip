@@ -1,7 +1,7 @@
 // Gate projections of a recurrent layer: out[T, N] = act(x[T, K] W[N, K]^T + bias), N small, fp32 accumulation and fp32
 // output (a recurrence's gates enter exponentials, where a 16-bit result would be a few per cent off).  Columns below
 // `split` get a soft cap, cap * tanh(z / cap), the others logsigmoid of the same.
-//   bf16: one workgroup = 16 rows x 16 columns; its four waves take 32-wide steps of K in turn on
+//   bf16: one workgroup = 16 rows x 16 or 32 columns; its four waves take 32-wide steps of K in turn on
 //         v_mfma_f32_16x16x32_bf16 and meet in LDS.
 //   fp32: the same tile with one fp32 dot product per thread over K chunks staged in LDS.
 #include "common.h"
@@ -35,30 +35,58 @@ __device__ __forceinline__ uint4 load_k8(const bf16_t* row, int k, int K, bool l
   return *reinterpret_cast<const uint4*>(v);
 }
 
+// NT column tiles per workgroup (one pass over x for all of them); kFull: K is a multiple of 32 and rows are 16-byte
+// aligned, so that loads need no guards (rows and columns past the end load the last one and are not stored).
+template <int NT, bool kFull>
 __global__ __launch_bounds__(256) void gate_linear_bf16_kernel(const GateArgs a, bool vec) {
-  __shared__ float4 part[3][64];
+  __shared__ float4 part[3][NT][64];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int row = blockIdx.x * 16 + (lane & 15), col = blockIdx.y * 16 + (lane & 15);
-  const bf16_t* x = reinterpret_cast<const bf16_t*>(a.x) + (int64_t)row * a.x_stride;
-  const bf16_t* w = reinterpret_cast<const bf16_t*>(a.w) + (int64_t)col * a.K;
+  const int row = blockIdx.x * 16 + (lane & 15), col0 = blockIdx.y * 16 * NT + (lane & 15);
   const int k0 = 8 * (lane >> 4);
-  v4f acc = {0.f, 0.f, 0.f, 0.f};
+  const bf16_t* x = reinterpret_cast<const bf16_t*>(a.x) + (int64_t)(kFull ? min(row, a.rows - 1) : row) * a.x_stride;
+  const bf16_t* w[NT];
+#pragma unroll
+  for (int n = 0; n < NT; ++n) {
+    const int col = col0 + 16 * n;
+    w[n] = reinterpret_cast<const bf16_t*>(a.w) + (int64_t)(kFull ? min(col, a.N - 1) : col) * a.K;
+  }
+  v4f acc[NT];
+#pragma unroll
+  for (int n = 0; n < NT; ++n) acc[n] = v4f{0.f, 0.f, 0.f, 0.f};
+  if constexpr (kFull) {
+#pragma unroll 8
+    for (int k = 32 * wave + k0; k < a.K; k += 128) {
+      const uint4 xv = *reinterpret_cast<const uint4*>(x + k);
+#pragma unroll
+      for (int n = 0; n < NT; ++n) acc[n] = mfma16x16x32<bf16_t>(*reinterpret_cast<const uint4*>(w[n] + k), xv, acc[n]);
+    }
+  } else {
 #pragma unroll 4
-  for (int k = 32 * wave; k < a.K; k += 128)
-    acc = mfma16x16x32<bf16_t>(load_k8(w, k + k0, a.K, col < a.N, vec), load_k8(x, k + k0, a.K, row < a.rows, vec), acc);
+    for (int k = 32 * wave; k < a.K; k += 128) {
+      const uint4 xv = load_k8(x, k + k0, a.K, row < a.rows, vec);
+#pragma unroll
+      for (int n = 0; n < NT; ++n) acc[n] = mfma16x16x32<bf16_t>(load_k8(w[n], k + k0, a.K, col0 + 16 * n < a.N, vec), xv, acc[n]);
+    }
+  }
   // lane holds row l % 16, columns 4 (l / 16) + r
-  if (wave > 0) part[wave - 1][lane] = make_float4(acc[0], acc[1], acc[2], acc[3]);
+  if (wave > 0) {
+#pragma unroll
+    for (int n = 0; n < NT; ++n) part[wave - 1][n][lane] = make_float4(acc[n][0], acc[n][1], acc[n][2], acc[n][3]);
+  }
   __syncthreads();
   if (wave > 0 || row >= a.rows) return;
 #pragma unroll
-  for (int i = 0; i < 3; ++i) {
-    const float4 p = part[i][lane];
-    acc[0] += p.x; acc[1] += p.y; acc[2] += p.z; acc[3] += p.w;
-  }
+  for (int n = 0; n < NT; ++n) {
 #pragma unroll
-  for (int r = 0; r < 4; ++r) {
-    const int n = blockIdx.y * 16 + 4 * (lane >> 4) + r;
-    if (n < a.N) a.out[(int64_t)row * a.N + n] = gate_activation(a, acc[r], n);
+    for (int i = 0; i < 3; ++i) {
+      const float4 p = part[i][n][lane];
+      acc[n][0] += p.x; acc[n][1] += p.y; acc[n][2] += p.z; acc[n][3] += p.w;
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int c = (blockIdx.y * NT + n) * 16 + 4 * (lane >> 4) + r;
+      if (c < a.N) a.out[(int64_t)row * a.N + c] = gate_activation(a, acc[n][r], c);
+    }
   }
 }
 
@@ -99,9 +127,13 @@ extern "C" int mvllm_gate_linear(float* out, const void* x, int64_t x_row_stride
   GateArgs a;
   a.out = out; a.x = x; a.w = w; a.bias = bias; a.x_stride = x_row_stride; a.rows = (int)rows; a.N = N; a.K = K;
   a.split = split; a.cap = cap;
-  const dim3 grid((unsigned)((rows + 15) / 16), (unsigned)((N + 15) / 16));
+  const unsigned tiles = (unsigned)((rows + 15) / 16);
+  const dim3 grid(tiles, (unsigned)((N + 15) / 16)), grid2(tiles, (unsigned)((N + 31) / 32));
   hipStream_t s = (hipStream_t)stream;
+  const bool vec = K % 8 == 0 && x_row_stride % 8 == 0 && aligned16(x) && aligned16(w), full = vec && K % 32 == 0;
   if (dtype == MVLLM_F32) gate_linear_f32_kernel<<<grid, dim3(256), 0, s>>>(a);
-  else gate_linear_bf16_kernel<<<grid, dim3(256), 0, s>>>(a, K % 8 == 0 && x_row_stride % 8 == 0 && aligned16(x) && aligned16(w));
+  else if (!full) gate_linear_bf16_kernel<1, false><<<grid, dim3(256), 0, s>>>(a, vec);
+  else if (N <= 16) gate_linear_bf16_kernel<1, true><<<grid, dim3(256), 0, s>>>(a, vec);
+  else gate_linear_bf16_kernel<2, true><<<grid2, dim3(256), 0, s>>>(a, vec);
   return launch_status();
 }

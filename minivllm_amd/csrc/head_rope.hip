@@ -11,7 +11,8 @@
 //   dst = dst_row[t] (null: t) reorders the rows for attention, which runs over groups of rows.
 // mvllm_head_unrotate_gate: attention output rows [*, H, D] ->
 //     out[t, h * vdim + d] = rotate(o[dst_row[t], h], -pos)[d] * sigmoid(gate[t, h])
-// Sixteen lanes own one head vector, eight consecutive dims per lane and step; everything is computed in fp32 from the
+// Sixteen lanes own one head vector, eight consecutive dims per lane and step (in long batches four heads of a row, which
+// share the row's angles); everything is computed in fp32 from the
 // loaded values and rounded once.
 #include "common.h"
 
@@ -53,30 +54,40 @@ template <typename T> __device__ __forceinline__ void store8(T* p, int n, const 
     if (i < n) p[i] = r[i];
 }
 
-// Rotation of one lane's eight dims d0 .. d0 + 7.  cs: this position's (cos, sin) pairs, rot / 2 of them; `partner` holds
-// the eight dims of the other half (half-split layout only, where dim m pairs with m + rot / 2).
-__device__ __forceinline__ void rotate8(float* x, const float* partner, int d0, int rot, bool interleaved,
-                                        const float2* cs, float sign) {
-  if (interleaved) {
+// (cos, sin) of the four pairs among dims d0 .. d0 + 7 of a row of angles, rot / 2 of them; pairs past the end stay as
+// they are.
+__device__ __forceinline__ void load_angles(float2* angle, const float2* cs, int d0, int rot) {
+  if (d0 + 8 <= rot && (reinterpret_cast<uintptr_t>(cs) & 15u) == 0) {
+    const float4 a = reinterpret_cast<const float4*>(cs)[d0 / 4], b = reinterpret_cast<const float4*>(cs)[d0 / 4 + 1];
+    angle[0] = make_float2(a.x, a.y); angle[1] = make_float2(a.z, a.w);
+    angle[2] = make_float2(b.x, b.y); angle[3] = make_float2(b.z, b.w);
+    return;
+  }
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      if (d0 + 2 * i < rot) {
-        const float2 c = cs[d0 / 2 + i];
-        const float s = c.y * sign, u = x[2 * i], v = x[2 * i + 1];
-        x[2 * i] = u * c.x - v * s;
-        x[2 * i + 1] = v * c.x + u * s;
-      }
-    }
-  } else {
-    const int half = rot / 2;
+  for (int i = 0; i < 4; ++i) angle[i] = d0 + 2 * i < rot ? cs[d0 / 2 + i] : make_float2(1.f, 0.f);
+}
+
+// Rotation of one lane's eight dims, pairs (2i, 2i + 1).
+__device__ __forceinline__ void turn_pairs(float* x, const float2* angle, float sign) {
 #pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      const int d = d0 + i;
-      if (d < rot) {
-        const bool low = d < half;
-        const float2 c = cs[low ? d : d - half];
-        x[i] = low ? x[i] * c.x - partner[i] * (c.y * sign) : x[i] * c.x + partner[i] * (c.y * sign);
-      }
+  for (int i = 0; i < 4; ++i) {
+    const float2 c = angle[i];
+    const float s = c.y * sign, u = x[2 * i], v = x[2 * i + 1];
+    x[2 * i] = u * c.x - v * s;
+    x[2 * i + 1] = v * c.x + u * s;
+  }
+}
+
+// The same for pairs (m, m + rot / 2): `partner` holds the eight dims of the other half.
+__device__ __forceinline__ void turn_halves(float* x, const float* partner, int d0, int rot, const float2* cs, float sign) {
+  const int half = rot / 2;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const int d = d0 + i;
+    if (d < rot) {
+      const bool low = d < half;
+      const float2 c = cs[low ? d : d - half];
+      x[i] = low ? x[i] * c.x - partner[i] * (c.y * sign) : x[i] * c.x + partner[i] * (c.y * sign);
     }
   }
 }
@@ -118,68 +129,88 @@ struct HeadRopeArgs {
   float eps, q_scale;
 };
 
-template <typename T>
-__global__ __launch_bounds__(256) void head_rope_store_kernel(const HeadRopeArgs a) {
-  const int per_row = a.heads + 2 * a.kv_heads;
-  const int64_t item = (int64_t)blockIdx.x * (256 / kLanes) + threadIdx.x / kLanes;
+// Sixteen lanes take kUnits heads of one row that turn by the same table (q and k heads, or v heads), so that the row's
+// angles are read once for all of them; kSteps steps of 128 dims.
+template <typename T, int kSteps, int kUnits>
+__global__ __launch_bounds__(256) void head_rope_store_kernel(const HeadRopeArgs a, unsigned parts_qk, unsigned parts) {
+  const unsigned item = blockIdx.x * (256 / kLanes) + threadIdx.x / kLanes;
   const int li = threadIdx.x % kLanes;
-  const bool live = item < a.rows * per_row;
-  const int64_t t = live ? item / per_row : 0;
-  const int u = live ? (int)(item - t * per_row) : 0;
-  const bool is_q = u < a.heads, is_v = u >= a.heads + a.kv_heads;
-  const int head = is_q ? u : is_v ? u - a.heads - a.kv_heads : u - a.heads;
+  const bool live = item < (unsigned)a.rows * parts;
+  const int64_t t = live ? item / parts : 0;
+  const unsigned part = live ? item - (unsigned)t * parts : 0;
+  const bool is_v = part >= parts_qk;
+  const int u0 = (int)(is_v ? part - parts_qk : part) * kUnits;        // first head: q and k heads counted through, or v heads
+  const int count = live ? min(kUnits, (is_v ? a.kv_heads : a.heads + a.kv_heads) - u0) : 0;
   const int n = is_v ? a.vdim : a.dim;
-  const T* src = reinterpret_cast<const T*>(a.proj) + t * a.proj_stride +
-                 (is_q ? (int64_t)head * a.dim
-                       : is_v ? (int64_t)(a.heads + a.kv_heads) * a.dim + (int64_t)head * a.vdim
-                              : (int64_t)(a.heads + head) * a.dim);
-  const float* gain = is_q ? a.gain_q : is_v ? nullptr : a.gain_k;
-  float x[kMaxSteps][8];
-  float ss = 0.f;
+  const T* src = reinterpret_cast<const T*>(a.proj) + t * a.proj_stride + (is_v ? (int64_t)(a.heads + a.kv_heads) * a.dim : 0) + (int64_t)u0 * n;
+  float x[kUnits][kSteps][8];
 #pragma unroll
-  for (int s = 0; s < kMaxSteps; ++s) {
-    const int d0 = 8 * (li + kLanes * s);
+  for (int j = 0; j < kUnits; ++j)
 #pragma unroll
-    for (int i = 0; i < 8; ++i) x[s][i] = 0.f;
-    if (live && d0 < n) load8(src + d0, min(8, n - d0), x[s]);
+    for (int s = 0; s < kSteps; ++s) {
+      const int d0 = 8 * (li + kLanes * s);
 #pragma unroll
-    for (int i = 0; i < 8; ++i) ss = fmaf(x[s][i], x[s][i], ss);
-  }
-#pragma unroll
-  for (int o = 1; o < kLanes; o <<= 1) ss += __shfl_xor(ss, o, 64);
-  if (!live) return;
-  const float scale = gain ? 1.0f / sqrtf(ss / (float)n + a.eps) : 1.0f;
+      for (int i = 0; i < 8; ++i) x[j][s][i] = 0.f;
+      if (j < count && d0 < n) load8(src + j * n + d0, min(8, n - d0), x[j][s]);
+    }
   int64_t pos = a.positions[t];
   pos = pos < 0 ? 0 : pos >= a.max_position ? a.max_position - 1 : pos;
   const int rot = is_v ? (a.v_table ? a.vdim : 0) : (a.rot_table ? a.rot : 0);
   const float2* cs = rot == 0 ? nullptr : (is_v ? a.v_table : a.rot_table) + pos * (rot / 2);
   const int64_t dst = a.dst_row ? a.dst_row[t] : t;
-  const int64_t slot = !is_q && a.slots ? a.slots[t] : -1;
-  T* packed = reinterpret_cast<T*>(is_q ? a.q_out : is_v ? a.v_out : a.k_out);
-  const int groups = is_q ? a.heads : a.kv_heads;
-  if (packed) packed += (dst * groups + head) * a.D;
-  T* cached = nullptr;
-  if (slot >= 0 && slot < a.num_slots) cached = reinterpret_cast<T*>(is_v ? a.v_cache : a.k_cache) + (slot * a.kv_heads + head) * a.D;
+  const int64_t own_slot = a.slots ? a.slots[t] : -1;
+  float2 angle[kSteps][4];                                             // of the lane's pairs (interleaved layout)
 #pragma unroll
-  for (int s = 0; s < kMaxSteps; ++s) {
-    const int d0 = 8 * (li + kLanes * s);
-    if (d0 >= a.D) continue;
-    if (gain) {
+  for (int s = 0; s < kSteps; ++s) load_angles(angle[s], cs, 8 * (li + kLanes * s), a.interleaved ? rot : 0);
 #pragma unroll
-      for (int i = 0; i < 8; ++i) x[s][i] = d0 + i < n ? x[s][i] * scale * gain[d0 + i] : 0.f;
-    }
-    if (d0 < rot) {
-      float partner[8];
-      if (!a.interleaved) load_partner(src, gain, scale, d0, rot, partner);
-      rotate8(x[s], partner, d0, rot, a.interleaved != 0, cs, 1.f);
-    }
-    if (is_q) {
+  for (int j = 0; j < kUnits; ++j) {
+    const int u = u0 + j;
+    const bool is_q = !is_v && u < a.heads;
+    const float* gain = is_v ? nullptr : is_q ? a.gain_q : a.gain_k;
+    float scale = 1.f;
+    if (gain) {                                                        // the same for the sixteen lanes
+      float ss = 0.f;
 #pragma unroll
-      for (int i = 0; i < 8; ++i) x[s][i] *= a.q_scale;
+      for (int s = 0; s < kSteps; ++s)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) ss = fmaf(x[j][s][i], x[j][s][i], ss);
+      scale = 1.0f / sqrtf(row16_sum(ss) / (float)n + a.eps);
     }
-    const int m = min(8, a.D - d0);
-    if (packed) store8(packed + d0, m, x[s]);
-    if (cached) store8(cached + d0, m, x[s]);
+    if (j >= count) continue;
+    const int head = is_q || is_v ? u : u - a.heads, groups = is_q ? a.heads : a.kv_heads;
+    T* packed = reinterpret_cast<T*>(is_q ? a.q_out : is_v ? a.v_out : a.k_out);
+    if (packed) packed += (dst * groups + head) * a.D;
+    const int64_t slot = is_q ? -1 : own_slot;
+    T* cached = nullptr;
+    if (slot >= 0 && slot < a.num_slots) cached = reinterpret_cast<T*>(is_v ? a.v_cache : a.k_cache) + (slot * a.kv_heads + head) * a.D;
+#pragma unroll
+    for (int s = 0; s < kSteps; ++s) {
+      const int d0 = 8 * (li + kLanes * s);
+      if (d0 >= a.D) continue;
+      float* v = x[j][s];
+      if (gain) {
+        float g[8];
+        load8(gain + d0, max(min(8, n - d0), 0), g);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[i] = v[i] * scale * g[i];
+      }
+      if (d0 < rot) {
+        if (a.interleaved) {
+          turn_pairs(v, angle[s], 1.f);
+        } else {
+          float partner[8];
+          load_partner(src + j * n, gain, scale, d0, rot, partner);
+          turn_halves(v, partner, d0, rot, cs, 1.f);
+        }
+      }
+      if (is_q) {
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[i] *= a.q_scale;
+      }
+      const int m = min(8, a.D - d0);
+      if (packed) store8(packed + d0, m, v);
+      if (cached) store8(cached + d0, m, v);
+    }
   }
 }
 
@@ -197,37 +228,53 @@ struct UnrotateGateArgs {
   int interleaved;
 };
 
-template <typename T>
-__global__ __launch_bounds__(256) void head_unrotate_gate_kernel(const UnrotateGateArgs a) {
-  const int64_t item = (int64_t)blockIdx.x * (256 / kLanes) + threadIdx.x / kLanes;
+template <typename T, int kSteps, int kUnits>
+__global__ __launch_bounds__(256) void head_unrotate_gate_kernel(const UnrotateGateArgs a, unsigned parts) {
+  const unsigned item = blockIdx.x * (256 / kLanes) + threadIdx.x / kLanes;
   const int li = threadIdx.x % kLanes;
-  if (item >= a.rows * a.heads) return;
-  const int64_t t = item / a.heads;
-  const int h = (int)(item - t * a.heads);
+  if (item >= (unsigned)a.rows * parts) return;
+  const int64_t t = item / parts;
+  const int h0 = (int)(item - (unsigned)t * parts) * kUnits, count = min(kUnits, a.heads - h0);
   const int64_t src_row = a.dst_row ? a.dst_row[t] : t;
-  const T* src = reinterpret_cast<const T*>(a.o) + (src_row * a.heads + h) * a.D;
-  T* dst = reinterpret_cast<T*>(a.out) + (t * a.heads + h) * a.vdim;
-  float g = 1.f;
-  if (a.gate) g = 1.0f / (1.0f + __expf(-to_float(reinterpret_cast<const T*>(a.gate)[t * a.gate_stride + h])));
+  const T* src = reinterpret_cast<const T*>(a.o) + (src_row * a.heads + h0) * a.D;
+  T* dst = reinterpret_cast<T*>(a.out) + (t * a.heads + h0) * a.vdim;
+  float x[kUnits][kSteps][8], g[kUnits];
+#pragma unroll
+  for (int j = 0; j < kUnits; ++j) {
+#pragma unroll
+    for (int s = 0; s < kSteps; ++s) {
+      const int d0 = 8 * (li + kLanes * s);
+      if (j < count && d0 < a.vdim) load8(src + j * a.D + d0, min(8, a.vdim - d0), x[j][s]);
+    }
+    g[j] = 1.f;
+    if (a.gate && j < count) g[j] = 1.0f / (1.0f + __expf(-to_float(reinterpret_cast<const T*>(a.gate)[t * a.gate_stride + h0 + j])));
+  }
   int64_t pos = a.positions[t];
   pos = pos < 0 ? 0 : pos >= a.max_position ? a.max_position - 1 : pos;
   const int rot = a.v_table ? a.vdim : 0;
   const float2* cs = rot ? a.v_table + pos * (rot / 2) : nullptr;
 #pragma unroll
-  for (int s = 0; s < kMaxSteps; ++s) {
+  for (int s = 0; s < kSteps; ++s) {
     const int d0 = 8 * (li + kLanes * s);
     if (d0 >= a.vdim) continue;
-    const int n = min(8, a.vdim - d0);
-    float x[8];
-    load8(src + d0, n, x);
-    if (d0 < rot) {
-      float partner[8];
-      if (!a.interleaved) load_partner(src, nullptr, 1.f, d0, rot, partner);
-      rotate8(x, partner, d0, rot, a.interleaved != 0, cs, -1.f);
-    }
+    float2 angle[4];
+    load_angles(angle, cs, d0, a.interleaved ? rot : 0);
 #pragma unroll
-    for (int i = 0; i < 8; ++i) x[i] *= g;
-    store8(dst + d0, n, x);
+    for (int j = 0; j < kUnits; ++j) {
+      if (j >= count) break;
+      if (d0 < rot) {
+        if (a.interleaved) {
+          turn_pairs(x[j][s], angle, -1.f);
+        } else {
+          float partner[8];
+          load_partner(src + j * a.D, nullptr, 1.f, d0, rot, partner);
+          turn_halves(x[j][s], partner, d0, rot, cs, -1.f);
+        }
+      }
+#pragma unroll
+      for (int i = 0; i < 8; ++i) x[j][s][i] *= g[j];
+      store8(dst + j * a.vdim + d0, min(8, a.vdim - d0), x[j][s]);
+    }
   }
 }
 
@@ -255,7 +302,18 @@ __global__ __launch_bounds__(256) void chunk_decode_step_kernel(int64_t* chunk_l
 
 using namespace mvllm;
 
+constexpr int kRowUnits = 4;       // heads per sixteen lanes where there are rows enough to fill the chip anyway
+constexpr int kManyRows = 512;
+
 static unsigned head_blocks(int64_t items) { return (unsigned)((items + 256 / kLanes - 1) / (256 / kLanes)); }
+
+// f(steps, units): compile-time counts of 128-dim steps and of heads per sixteen lanes
+template <typename F> static void with_steps(int head_dim, int64_t rows, F f) {
+  using std::integral_constant;
+  if (head_dim > 8 * kLanes) f(integral_constant<int, kMaxSteps>{}, integral_constant<int, 1>{});
+  else if (rows < kManyRows) f(integral_constant<int, 1>{}, integral_constant<int, 1>{});
+  else f(integral_constant<int, 1>{}, integral_constant<int, kRowUnits>{});
+}
 
 extern "C" int mvllm_head_rope_store(void* q_out, void* k_out, void* v_out, const void* proj, int64_t proj_row_stride,
                                      const float* gain_q, const float* gain_k, float eps, float q_scale,
@@ -270,7 +328,8 @@ extern "C" int mvllm_head_rope_store(void* q_out, void* k_out, void* v_out, cons
       (v_table && vdim % 2 != 0) || max_position <= 0 || num_slots < 0 ||
       proj_row_stride < (int64_t)num_heads * dim + (int64_t)num_kv_heads * (dim + vdim))
     return MVLLM_ERR_BAD_SHAPE;
-  if (dtype == MVLLM_F16 || head_dim > 8 * kLanes * kMaxSteps) return MVLLM_ERR_UNSUPPORTED;
+  if (dtype == MVLLM_F16 || head_dim > 8 * kLanes * kMaxSteps || rows > ((int64_t)1 << 31) / (num_heads + 2 * (int64_t)num_kv_heads))
+    return MVLLM_ERR_UNSUPPORTED;
   if (rows == 0) return MVLLM_OK;
   if (!q_out || !proj || !positions || (slots && (!k_cache || !v_cache)) || (rot_dims && !rot_table)) return MVLLM_ERR_NULL_POINTER;
   HeadRopeArgs a;
@@ -281,9 +340,13 @@ extern "C" int mvllm_head_rope_store(void* q_out, void* k_out, void* v_out, cons
   a.proj_stride = proj_row_stride; a.max_position = max_position; a.num_slots = num_slots; a.rows = rows;
   a.heads = num_heads; a.kv_heads = num_kv_heads; a.dim = dim; a.vdim = vdim; a.D = head_dim; a.rot = rot_dims;
   a.interleaved = interleaved; a.eps = eps; a.q_scale = q_scale;
-  const unsigned grid = head_blocks(rows * (num_heads + 2 * (int64_t)num_kv_heads));
-  if (dtype == MVLLM_F32) head_rope_store_kernel<float><<<dim3(grid), dim3(256), 0, (hipStream_t)stream>>>(a);
-  else head_rope_store_kernel<bf16_t><<<dim3(grid), dim3(256), 0, (hipStream_t)stream>>>(a);
+  with_steps(head_dim, rows, [&](auto STEPS, auto UNITS) {
+    constexpr int kSteps = decltype(STEPS)::value, kUnits = decltype(UNITS)::value;
+    const unsigned parts_qk = (unsigned)(num_heads + num_kv_heads + kUnits - 1) / kUnits, parts = parts_qk + (unsigned)(num_kv_heads + kUnits - 1) / kUnits;
+    const dim3 grid(head_blocks(rows * parts));
+    if (dtype == MVLLM_F32) head_rope_store_kernel<float, kSteps, kUnits><<<grid, dim3(256), 0, (hipStream_t)stream>>>(a, parts_qk, parts);
+    else head_rope_store_kernel<bf16_t, kSteps, kUnits><<<grid, dim3(256), 0, (hipStream_t)stream>>>(a, parts_qk, parts);
+  });
   return launch_status();
 }
 
@@ -295,16 +358,20 @@ extern "C" int mvllm_head_unrotate_gate(void* out, const void* o, const void* ga
   if (rows < 0 || num_heads <= 0 || vdim <= 0 || head_dim < vdim || (v_table && vdim % 2 != 0) || max_position <= 0 ||
       (gate && gate_row_stride < num_heads))
     return MVLLM_ERR_BAD_SHAPE;
-  if (dtype == MVLLM_F16 || head_dim > 8 * kLanes * kMaxSteps) return MVLLM_ERR_UNSUPPORTED;
+  if (dtype == MVLLM_F16 || head_dim > 8 * kLanes * kMaxSteps || rows > ((int64_t)1 << 31) / num_heads) return MVLLM_ERR_UNSUPPORTED;
   if (rows == 0) return MVLLM_OK;
   if (!out || !o || !positions) return MVLLM_ERR_NULL_POINTER;
   UnrotateGateArgs a;
   a.out = out; a.o = o; a.gate = gate; a.v_table = reinterpret_cast<const float2*>(v_table); a.positions = positions;
   a.dst_row = dst_row; a.gate_stride = gate_row_stride; a.max_position = max_position; a.rows = rows;
   a.heads = num_heads; a.vdim = vdim; a.D = head_dim; a.interleaved = interleaved;
-  const unsigned grid = head_blocks(rows * num_heads);
-  if (dtype == MVLLM_F32) head_unrotate_gate_kernel<float><<<dim3(grid), dim3(256), 0, (hipStream_t)stream>>>(a);
-  else head_unrotate_gate_kernel<bf16_t><<<dim3(grid), dim3(256), 0, (hipStream_t)stream>>>(a);
+  with_steps(head_dim, rows, [&](auto STEPS, auto UNITS) {
+    constexpr int kSteps = decltype(STEPS)::value, kUnits = decltype(UNITS)::value;
+    const unsigned parts = (unsigned)(num_heads + kUnits - 1) / kUnits;
+    const dim3 grid(head_blocks(rows * parts));
+    if (dtype == MVLLM_F32) head_unrotate_gate_kernel<float, kSteps, kUnits><<<grid, dim3(256), 0, (hipStream_t)stream>>>(a, parts);
+    else head_unrotate_gate_kernel<bf16_t, kSteps, kUnits><<<grid, dim3(256), 0, (hipStream_t)stream>>>(a, parts);
+  });
   return launch_status();
 }
 

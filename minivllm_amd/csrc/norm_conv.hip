@@ -71,25 +71,27 @@ template <typename T> struct Chunk<T, 1> {
   static __device__ __forceinline__ void store(T* p, const float* v) { *p = from_float<T>(v[0]); }
 };
 
-// Sums of N values per thread over the workgroup, the same in every thread.
+// Sums of N values per thread over the workgroup, the same in every thread: rows of 16 lanes in registers, the rows of all
+// waves (at most 64) through LDS.  Consecutive calls take the two halves of `lds` in turn (`flip`): whoever writes a half
+// again has passed the barrier of the call in between, which everybody reaches after reading it.
 template <int N>
-__device__ __forceinline__ void block_sums(float* v, float* lds, int waves) {
+__device__ __forceinline__ void block_sums(float* v, float* lds, int waves, int& flip) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
 #pragma unroll
-  for (int i = 0; i < N; ++i) v[i] = wave_sum(v[i]);
-  if (waves == 1) return;
-  if (lane == 0) {
+  for (int i = 0; i < N; ++i) v[i] = row16_sum(v[i]);
+  if (waves > 1) {
+    lds += flip * (kMaxThreads / 16) * N;
+    flip ^= 1;
+    if ((lane & 15) == 0) {
 #pragma unroll
-    for (int i = 0; i < N; ++i) lds[wave * N + i] = v[i];
-  }
-  __syncthreads();
+      for (int i = 0; i < N; ++i) lds[(wave * 4 + (lane >> 4)) * N + i] = v[i];
+    }
+    __syncthreads();
 #pragma unroll
-  for (int i = 0; i < N; ++i) {
-    float s = 0.f;
-    for (int w = 0; w < waves; ++w) s += lds[w * N + i];
-    v[i] = s;
+    for (int i = 0; i < N; ++i) v[i] = row16_sum(lane < 4 * waves ? lds[lane * N + i] : 0.f);
   }
-  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < N; ++i) v[i] = four_rows_sum(v[i]);
 }
 
 // NC chunks of VEC channels per thread.
@@ -99,7 +101,8 @@ __global__ __launch_bounds__(kMaxThreads) void norm_conv_kernel(const NormConvAr
   constexpr int kHist = TAPS > 1 ? TAPS - 1 : 1;
   constexpr int kBatch = NC == 1 ? kRowsTogether : 1;
   constexpr bool kKeepConv = NC == 1;       // taps and gains in registers; wide rows read them again for every row
-  __shared__ float lds[(kMaxThreads / 64) * kRowsTogether];
+  __shared__ __attribute__((aligned(16))) float lds[2 * (kMaxThreads / 16) * kRowsTogether];
+  int flip = 0;
   const int waves = blockDim.x >> 6;
   const int W = a.width;
   const int first = blockIdx.x * a.rows_per_wg;
@@ -169,7 +172,7 @@ __global__ __launch_bounds__(kMaxThreads) void norm_conv_kernel(const NormConvAr
 #pragma unroll
         for (int c = 0; c < C; ++c) sums[r] = fmaf(yv[r][c], yv[r][c], sums[r]);
       }
-      block_sums<kBatch>(sums, lds, waves);
+      block_sums<kBatch>(sums, lds, waves, flip);
 #pragma unroll
       for (int r = 0; r < kBatch; ++r) {
         const float d = sqrtf(sums[r] * inv_w + a.eps);
@@ -184,7 +187,7 @@ __global__ __launch_bounds__(kMaxThreads) void norm_conv_kernel(const NormConvAr
 #pragma unroll
       for (int c = 0; c < C; ++c) sums[r] = fmaf(x[r][c], x[r][c], sums[r]);
     }
-    block_sums<kBatch>(sums, lds, waves);
+    block_sums<kBatch>(sums, lds, waves, flip);
 #pragma unroll
     for (int r = 0; r < kBatch; ++r) {
       if (r >= n) break;
