@@ -1,7 +1,7 @@
 // Gate projections of a recurrent layer: out[T, N] = act(x[T, K] W[N, K]^T + bias), N small, fp32 accumulation and fp32
 // output (a recurrence's gates enter exponentials, where a 16-bit result would be a few per cent off).  Columns below
 // `split` get a soft cap, cap * tanh(z / cap), the others logsigmoid of the same.
-//   bf16: one workgroup = 16 rows x 16 or 32 columns; its four waves take 32-wide steps of K in turn on
+//   bf16: one workgroup = 16 rows x 16 or 32 columns; its waves take 64-wide steps of K in turn on
 //         v_mfma_f32_16x16x32_bf16 and meet in LDS.
 //   fp32: the same tile with one fp32 dot product per thread over K chunks staged in LDS.
 #include "common.h"
@@ -35,11 +35,13 @@ __device__ __forceinline__ uint4 load_k8(const bf16_t* row, int k, int K, bool l
   return *reinterpret_cast<const uint4*>(v);
 }
 
-// NT column tiles per workgroup (one pass over x for all of them); kFull: K is a multiple of 32 and rows are 16-byte
+constexpr int kFewRows = 512;        // up to here K is split over sixteen waves: the call is one memory round trip
+
+// kWaves waves share K; NT column tiles per workgroup (one pass over x for all of them); kFull: K is a multiple of 64 and rows are 16-byte
 // aligned, so that loads need no guards (rows and columns past the end load the last one and are not stored).
-template <int NT, bool kFull>
-__global__ __launch_bounds__(256) void gate_linear_bf16_kernel(const GateArgs a, bool vec) {
-  __shared__ float4 part[3][NT][64];
+template <int kWaves, int NT, bool kFull>
+__global__ __launch_bounds__(64 * kWaves) void gate_linear_bf16_kernel(const GateArgs a, bool vec) {
+  __shared__ float4 part[kWaves][NT][64];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int row = blockIdx.x * 16 + (lane & 15), col0 = blockIdx.y * 16 * NT + (lane & 15);
   const int k0 = 8 * (lane >> 4);
@@ -54,40 +56,34 @@ __global__ __launch_bounds__(256) void gate_linear_bf16_kernel(const GateArgs a,
 #pragma unroll
   for (int n = 0; n < NT; ++n) acc[n] = v4f{0.f, 0.f, 0.f, 0.f};
   if constexpr (kFull) {
-#pragma unroll 8
-    for (int k = 32 * wave + k0; k < a.K; k += 128) {
-      const uint4 xv = *reinterpret_cast<const uint4*>(x + k);
+#pragma unroll 4
+    for (int k = 64 * wave + 2 * k0; k < a.K; k += 64 * kWaves) {      // a lane's 32 bytes: whole lines per row and wave
 #pragma unroll
-      for (int n = 0; n < NT; ++n) acc[n] = mfma16x16x32<bf16_t>(*reinterpret_cast<const uint4*>(w[n] + k), xv, acc[n]);
+      for (int half = 0; half < 16; half += 8) {
+        const uint4 xv = *reinterpret_cast<const uint4*>(x + k + half);
+#pragma unroll
+        for (int n = 0; n < NT; ++n) acc[n] = mfma16x16x32<bf16_t>(*reinterpret_cast<const uint4*>(w[n] + k + half), xv, acc[n]);
+      }
     }
   } else {
 #pragma unroll 4
-    for (int k = 32 * wave; k < a.K; k += 128) {
+    for (int k = 32 * wave; k < a.K; k += 32 * kWaves) {
       const uint4 xv = load_k8(x, k + k0, a.K, row < a.rows, vec);
 #pragma unroll
       for (int n = 0; n < NT; ++n) acc[n] = mfma16x16x32<bf16_t>(load_k8(w[n], k + k0, a.K, col0 + 16 * n < a.N, vec), xv, acc[n]);
     }
   }
-  // lane holds row l % 16, columns 4 (l / 16) + r
-  if (wave > 0) {
+  // lane holds row l % 16, columns 4 (l / 16) + r of every tile; the activations are spread over the workgroup
 #pragma unroll
-    for (int n = 0; n < NT; ++n) part[wave - 1][n][lane] = make_float4(acc[n][0], acc[n][1], acc[n][2], acc[n][3]);
-  }
+  for (int n = 0; n < NT; ++n) part[wave][n][lane] = make_float4(acc[n][0], acc[n][1], acc[n][2], acc[n][3]);
   __syncthreads();
-  if (wave > 0 || row >= a.rows) return;
+  static_assert(256 * NT <= 64 * kWaves, "one output per thread");
+  const int t = threadIdx.x, n = t >> 8, c = (t >> 4) & 15, out_row = blockIdx.x * 16 + (t & 15), out_col = (blockIdx.y * NT + n) * 16 + c;
+  if (n >= NT || out_row >= a.rows || out_col >= a.N) return;
+  float z = 0.f;
 #pragma unroll
-  for (int n = 0; n < NT; ++n) {
-#pragma unroll
-    for (int i = 0; i < 3; ++i) {
-      const float4 p = part[i][n][lane];
-      acc[n][0] += p.x; acc[n][1] += p.y; acc[n][2] += p.z; acc[n][3] += p.w;
-    }
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int c = (blockIdx.y * NT + n) * 16 + 4 * (lane >> 4) + r;
-      if (c < a.N) a.out[(int64_t)row * a.N + c] = gate_activation(a, acc[n][r], c);
-    }
-  }
+  for (int i = 0; i < kWaves; ++i) z += reinterpret_cast<const float*>(&part[i][n][16 * (c >> 2) + (t & 15)])[c & 3];
+  a.out[(int64_t)out_row * a.N + out_col] = gate_activation(a, z, out_col);
 }
 
 __global__ __launch_bounds__(256) void gate_linear_f32_kernel(const GateArgs a) {
@@ -130,10 +126,11 @@ extern "C" int mvllm_gate_linear(float* out, const void* x, int64_t x_row_stride
   const unsigned tiles = (unsigned)((rows + 15) / 16);
   const dim3 grid(tiles, (unsigned)((N + 15) / 16)), grid2(tiles, (unsigned)((N + 31) / 32));
   hipStream_t s = (hipStream_t)stream;
-  const bool vec = K % 8 == 0 && x_row_stride % 8 == 0 && aligned16(x) && aligned16(w), full = vec && K % 32 == 0;
+  const bool vec = K % 8 == 0 && x_row_stride % 8 == 0 && aligned16(x) && aligned16(w), full = vec && K % 64 == 0;
   if (dtype == MVLLM_F32) gate_linear_f32_kernel<<<grid, dim3(256), 0, s>>>(a);
-  else if (!full) gate_linear_bf16_kernel<1, false><<<grid, dim3(256), 0, s>>>(a, vec);
-  else if (N <= 16) gate_linear_bf16_kernel<1, true><<<grid, dim3(256), 0, s>>>(a, vec);
-  else gate_linear_bf16_kernel<2, true><<<grid2, dim3(256), 0, s>>>(a, vec);
+  else if (!full) gate_linear_bf16_kernel<4, 1, false><<<grid, dim3(256), 0, s>>>(a, vec);
+  else if (rows <= kFewRows) gate_linear_bf16_kernel<16, 1, true><<<grid, dim3(1024), 0, s>>>(a, vec);
+  else if (N <= 16) gate_linear_bf16_kernel<8, 1, true><<<grid, dim3(512), 0, s>>>(a, vec);
+  else gate_linear_bf16_kernel<8, 2, true><<<grid2, dim3(512), 0, s>>>(a, vec);
   return launch_status();
 }

@@ -46,7 +46,7 @@ template <typename T> __device__ __forceinline__ void store8(T* p, int n, const 
   for (int i = 0; i < 8; ++i) r[i] = from_float<T>(v[i]);
   if (n == 8 && (reinterpret_cast<uintptr_t>(p) & 15u) == 0) {
 #pragma unroll
-    for (int i = 0; i < (int)(sizeof(r) / 16); ++i) reinterpret_cast<uint4*>(p)[i] = reinterpret_cast<const uint4*>(r)[i];
+    for (int i = 0; i < (int)(sizeof(r) / 16); ++i) store16_stream(reinterpret_cast<uint4*>(p) + i, reinterpret_cast<const uint4*>(r)[i]);
     return;
   }
 #pragma unroll

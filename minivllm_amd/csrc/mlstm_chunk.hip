@@ -362,7 +362,7 @@ __global__ __launch_bounds__(64 * kWaves, DIMP == 256 ? 1 : 2) void mlstm_chunk_
       for (int rt = 0; rt < 2; ++rt)
 #pragma unroll
         for (int r = 0; r < 16; ++r)
-          __builtin_amdgcn_raw_buffer_store_b32(__float_as_uint(o[rt][r]), rsrc, voff + (uint32_t)(32 * rt + 8 * (r >> 2) + (r & 3)) * pitch, 0, 0);
+          __builtin_amdgcn_raw_buffer_store_b32(__float_as_uint(o[rt][r]), rsrc, voff + (uint32_t)(32 * rt + 8 * (r >> 2) + (r & 3)) * pitch, 0, 2 /* nt */);
     }
     __syncthreads();                                // everybody is done with this block's LDS
   }

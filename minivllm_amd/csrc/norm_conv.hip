@@ -52,7 +52,9 @@ template <> struct Chunk<float, 4> {
     const float4 f = *reinterpret_cast<const float4*>(p);
     v[0] = f.x; v[1] = f.y; v[2] = f.z; v[3] = f.w;
   }
-  static __device__ __forceinline__ void store(float* p, const float* v) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
+  static __device__ __forceinline__ void store(float* p, const float* v) {
+    store16_stream(p, make_uint4(__float_as_uint(v[0]), __float_as_uint(v[1]), __float_as_uint(v[2]), __float_as_uint(v[3])));
+  }
 };
 template <> struct Chunk<bf16_t, 4> {
   static __device__ __forceinline__ void load(const bf16_t* p, float* v) {
@@ -63,7 +65,7 @@ template <> struct Chunk<bf16_t, 4> {
   static __device__ __forceinline__ void store(bf16_t* p, const float* v) {
     bf16_t r[4];
     for (int i = 0; i < 4; ++i) r[i] = from_float<bf16_t>(v[i]);
-    *reinterpret_cast<uint2*>(p) = *reinterpret_cast<const uint2*>(r);
+    store8_stream(p, *reinterpret_cast<const uint2*>(r));
   }
 };
 template <typename T> struct Chunk<T, 1> {
