@@ -1086,6 +1086,10 @@ def bench_sokevik_kernels(args, rows, calls):
     flops = rows * heads * (4.0 * dim * vdim + (64.0 * (dim + vdim) if prefill else 0.0))
     leg("mlstm", lambda: mlstm(step, proj, gates, n, weight, memory, 1e-6), nbytes, plain, "attention of the same rows", att[1],
         flops if prefill else 0.0, att[2])
+    if prefill:                                            # the rows as one prompt, in segments side by side
+        whole = step_of([rows], [0])
+        leg("mlstm_one_prompt", lambda: mlstm(whole, proj, gates, n, weight, memory, 1e-6),
+            nbytes - (entries - 1) * heads * dim * (vdim + 1) * 4, plain, "attention of the same rows", att[1], flops, att[2])
     # gate projections | a plain projection of as many columns
     h, gw, bias = rnd(rows, width), rnd(2 * heads, width), torch.zeros(2 * heads, device=dev)
     gate_bytes = rows * width * 2 + 2 * heads * width * 2

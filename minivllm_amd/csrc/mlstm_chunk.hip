@@ -44,6 +44,10 @@ struct MlstmChunkArgs {
   float q_scale, floor;
 };
 
+__device__ __forceinline__ uint4 load16(__amdgpu_buffer_rsrc_t rows, uint32_t offset) {
+  return __builtin_bit_cast(uint4, __builtin_amdgcn_raw_buffer_load_b128(rows, offset, 0, 0));
+}
+
 // x = hi + lo with both bf16, eight values at a time as operand fragments
 struct Split8 { uint4 hi, lo; };
 __device__ __forceinline__ Split8 split8(const float* x) {
@@ -101,15 +105,19 @@ __global__ __launch_bounds__(64 * kWaves, DIMP == 256 ? 1 : 2) void mlstm_chunk_
     s_in = a.ws_s + ((int64_t)seg * H + h) * dim * vdim;
     n_in = a.ws_n + ((int64_t)seg * H + h) * dim;
   }
-  static_for<kTD>([&](auto TD) {
-    constexpr int td = decltype(TD)::value;
+  // bounds-checked: rows past dim and columns past vdim (and everything without a state) arrive as zeros
+  const uint32_t s_bytes = (uint32_t)(dim * vdim) * 4u;
+  const uint32_t s_first = has_col ? (uint32_t)(4 * hi * vdim + col) * 4u : 0x80000000u;
+  {
+    const auto state = __builtin_amdgcn_make_buffer_rsrc(const_cast<float*>(s_in), 0, s_in != nullptr ? s_bytes : 0u, 0x00020000);
+    static_for<kTD>([&](auto TD) {
+      constexpr int td = decltype(TD)::value;
 #pragma unroll
-    for (int r = 0; r < 16; ++r) {
-      const int d = 32 * td + 8 * (r >> 2) + 4 * hi + (r & 3);
-      s[td][r] = s_in != nullptr && d < dim && has_col ? s_in[d * vdim + col] : 0.f;
-    }
-    __builtin_amdgcn_sched_barrier(0);
-  });
+      for (int r = 0; r < 16; ++r)
+        s[td][r] = __uint_as_float(__builtin_amdgcn_raw_buffer_load_b32(state, s_first + (uint32_t)((32 * td + 8 * (r >> 2) + (r & 3)) * vdim) * 4u, 0, 0));
+      __builtin_amdgcn_sched_barrier(0);
+    });
+  }
   if (n_owner)
     for (int d = tid; d < DIMP; d += kThreads) n_lds[d] = n_in != nullptr && d < dim ? n_in[d] : 0.f;
 
@@ -121,22 +129,28 @@ __global__ __launch_bounds__(64 * kWaves, DIMP == 256 ? 1 : 2) void mlstm_chunk_
   const bf16_t* vg = a.proj + (int64_t)2 * H * dim + (int64_t)h * vdim + tile * VT;
   constexpr int kQStep = kThreads / (DIMP / 8), kVStep = kThreads / (VT / 8);      // rows between a thread's loads
   const int q_r = tid / (DIMP / 8), q_d = (tid % (DIMP / 8)) * 8, v_r = tid / (VT / 8), v_d = (tid % (VT / 8)) * 8;
+  // bounds-checked: rows past the segment's end and columns past dim / vdim arrive as zeros
+  const uint32_t pitch_in = (uint32_t)a.proj_stride * 2u;
+  const uint32_t q_first = q_d < dim ? (uint32_t)q_r * pitch_in + (uint32_t)q_d * 2u : 0x80000000u;
+  const uint32_t v_first = tile * VT + v_d < vdim ? (uint32_t)v_r * pitch_in + (uint32_t)v_d * 2u : 0x80000000u;
   auto fetch = [&](int at) __attribute__((always_inline)) {
     const int64_t base = (int64_t)(row0 + at) * a.proj_stride;
-    int q_off = q_r * (int)a.proj_stride + q_d, v_off = v_r * (int)a.proj_stride + v_d;
+    const uint32_t reach = (uint32_t)(min(kBlock, rows - at) - 1) * pitch_in;
+    auto rows_of = [&](const bf16_t* p, int cols) {
+      return __builtin_amdgcn_make_buffer_rsrc(const_cast<bf16_t*>(p + base), 0, reach + (uint32_t)cols * 2u, 0x00020000);
+    };
+    uint32_t q_off = q_first, v_off = v_first;
     asm volatile("" : "+v"(q_off), "+v"(v_off));    // (offsets of all loads kept across the loop would not fit the registers)
+    const auto k_rows = rows_of(kg, dim), v_rows = rows_of(vg, vdim - tile * VT);
+    if constexpr (!kStateOnly) {
+      const auto q_rows = rows_of(qg, dim);
 #pragma unroll
-    for (int i = 0; i < kQLoads; ++i) {
-      const bool live = at + q_r + i * kQStep < rows && q_d < dim;
-      const int off = q_off + i * kQStep * (int)a.proj_stride;
-      if constexpr (!kStateOnly) qr[i] = live ? *reinterpret_cast<const uint4*>(qg + base + off) : make_uint4(0u, 0u, 0u, 0u);
-      kr[i] = live ? *reinterpret_cast<const uint4*>(kg + base + off) : make_uint4(0u, 0u, 0u, 0u);
+      for (int i = 0; i < kQLoads; ++i) qr[i] = load16(q_rows, q_off + (uint32_t)(i * kQStep) * pitch_in);
     }
 #pragma unroll
-    for (int i = 0; i < kVLoads; ++i) {
-      const bool live = at + v_r + i * kVStep < rows && tile * VT + v_d < vdim;
-      vr[i] = live ? *reinterpret_cast<const uint4*>(vg + base + v_off + i * kVStep * (int)a.proj_stride) : make_uint4(0u, 0u, 0u, 0u);
-    }
+    for (int i = 0; i < kQLoads; ++i) kr[i] = load16(k_rows, q_off + (uint32_t)(i * kQStep) * pitch_in);
+#pragma unroll
+    for (int i = 0; i < kVLoads; ++i) vr[i] = load16(v_rows, v_off + (uint32_t)(i * kVStep) * pitch_in);
     const bool live = at + lane < rows;
     const float* g = a.gates + (int64_t)(row0 + at + (live ? lane : 0)) * 2 * H;
     gate_i = live ? g[h] : -INFINITY;
@@ -200,6 +214,8 @@ __global__ __launch_bounds__(64 * kWaves, DIMP == 256 ? 1 : 2) void mlstm_chunk_
         }
         // key column sx of the lane, rows 32 rt + 4 hi + 8 (r / 4) + r % 4; past the diagonal the weight is exp(-inf)
         const int sx = 32 * ct + l32, t0 = 32 * rt + 4 * hi;
+        int past = l32 - 4 * hi;                    // on the diagonal: rows `up` below it are past the key
+        asm volatile("" : "+v"(past));              // (sixteen lane masks kept across the loop would not fit the registers)
         const float as = sc_a[sx];
         uint16_t* hp = &ph[t0 * kPRow + sx];
         uint16_t* lp = &pl[t0 * kPRow + sx];
@@ -208,7 +224,7 @@ __global__ __launch_bounds__(64 * kWaves, DIMP == 256 ? 1 : 2) void mlstm_chunk_
         for (int r = 0; r < 16; ++r) {
           constexpr float kNever = -INFINITY;
           const int up = 8 * (r >> 2) + (r & 3);
-          const float arg = rt == ct && sx > t0 + up ? kNever : as - Mp[up];
+          const float arg = rt == ct && past > up ? kNever : as - Mp[up];
           const float x = p[r] * (a.q_scale * __expf(arg));
           const bf16_t top = from_float<bf16_t>(x);
           hp[up * kPRow] = top.bits;
@@ -352,7 +368,8 @@ __global__ __launch_bounds__(64 * kWaves, DIMP == 256 ? 1 : 2) void mlstm_chunk_
     }
     if constexpr (!kStateOnly) {
       // bounds-checked stores: rows past the segment and columns past vdim are dropped
-      const uint32_t pitch = (uint32_t)(H * vdim) * 4u;
+      uint32_t pitch = (uint32_t)(H * vdim) * 4u;
+      asm volatile("" : "+s"(pitch));
       const int n_rows = min(kBlock, rows - at);
       const auto rsrc = __builtin_amdgcn_make_buffer_rsrc(a.num + ((int64_t)(row0 + at) * H + h) * vdim, 0,
                                                           (uint32_t)(n_rows - 1) * pitch + (uint32_t)vdim * 4u, 0x00020000);
@@ -370,13 +387,14 @@ __global__ __launch_bounds__(64 * kWaves, DIMP == 256 ? 1 : 2) void mlstm_chunk_
   // ---- the state behind the segment: contribution -> workspace (kStateOnly), the last one -> the slot ----
   if (!kStateOnly && !(flags & 2)) return;
   float* s_out = kStateOnly ? a.ws_s + ((int64_t)seg * H + h) * dim * vdim : a.s_state + ((int64_t)slot * H + h) * dim * vdim;
+  const auto state = __builtin_amdgcn_make_buffer_rsrc(s_out, 0, s_bytes, 0x00020000);
+  uint32_t s_pitch = (uint32_t)vdim * 4u;
+  asm volatile("" : "+s"(s_pitch));
   static_for<kTD>([&](auto TD) {
     constexpr int td = decltype(TD)::value;
 #pragma unroll
-    for (int r = 0; r < 16; ++r) {
-      const int d = 32 * td + 8 * (r >> 2) + 4 * hi + (r & 3);
-      if (d < dim && has_col) s_out[d * vdim + col] = s[td][r];
-    }
+    for (int r = 0; r < 16; ++r)
+      __builtin_amdgcn_raw_buffer_store_b32(__float_as_uint(s[td][r]), state, s_first + (uint32_t)(32 * td + 8 * (r >> 2) + (r & 3)) * s_pitch, 0, 0);
     __builtin_amdgcn_sched_barrier(0);
   });
   if (n_owner) {
@@ -394,7 +412,10 @@ __global__ __launch_bounds__(64 * kWaves, DIMP == 256 ? 1 : 2) void mlstm_chunk_
 }
 
 // Contributions of an entry's segments -> the state in front of each of them, in place.  Workgroup = (first segment of an
-// entry, head, slice of the elements of S and n).
+// entry, head, slice of the elements of S and n).  A thread owns four consecutive elements; the contributions of kAhead
+// segments are loaded together, before the states that replace them are stored.
+constexpr int kCombineElements = 1024, kAhead = 8;
+
 __global__ __launch_bounds__(256) void mlstm_combine_kernel(const MlstmChunkArgs a) {
   const int seg0 = blockIdx.x, h = blockIdx.y;
   const int flags0 = a.segments[4 * seg0 + 3];
@@ -403,21 +424,40 @@ __global__ __launch_bounds__(256) void mlstm_combine_kernel(const MlstmChunkArgs
   if (slot < 0) return;
   const int H = a.heads;
   const bool fresh = a.positions[a.segments[4 * seg0 + 1]] == 0;
-  const int64_t per_s = (int64_t)a.dim * a.vdim, total = per_s + a.dim;
-  const int64_t at = (int64_t)blockIdx.z * 256 + threadIdx.x;
-  const bool live = at < total, in_s = at < per_s;
-  float x = 0.f, m = fresh ? 0.f : a.m_state[(int64_t)slot * H + h];
-  if (live && !fresh) x = in_s ? a.s_state[((int64_t)slot * H + h) * per_s + at] : a.n_state[((int64_t)slot * H + h) * a.dim + at - per_s];
-  for (int seg = seg0; seg < a.num_segments; ++seg) {
-    const bool last = (a.segments[4 * seg + 3] & 2) != 0;
-    float* p = in_s ? a.ws_s + ((int64_t)seg * H + h) * per_s + at : a.ws_n + ((int64_t)seg * H + h) * a.dim + at - per_s;
-    const float own = live && !last ? *p : 0.f;
-    if (live) *p = x;
-    if (last) break;
-    const float f = a.ws_f[(int64_t)seg * H + h], mo = a.ws_m[(int64_t)seg * H + h];
-    const float m_new = fmaxf(f + m, mo);
-    x = __expf(f + m - m_new) * x + __expf(mo - m_new) * own;
-    m = m_new;
+  const int64_t per_s = (int64_t)a.dim * a.vdim;
+  const int64_t at = (int64_t)blockIdx.z * kCombineElements + 4 * threadIdx.x;
+  if (at >= per_s + a.dim) return;                  // dim and dim * vdim are multiples of four
+  const bool in_s = at < per_s;
+  const int64_t pitch = in_s ? (int64_t)H * per_s : (int64_t)H * a.dim;         // between segments
+  float* ws = in_s ? a.ws_s + h * per_s + at : a.ws_n + (int64_t)h * a.dim + at - per_s;
+  float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
+  float m = fresh ? 0.f : a.m_state[(int64_t)slot * H + h];
+  if (!fresh)
+    x = *reinterpret_cast<const float4*>(in_s ? a.s_state + ((int64_t)slot * H + h) * per_s + at
+                                              : a.n_state + ((int64_t)slot * H + h) * a.dim + at - per_s);
+  for (int base = seg0;; base += kAhead) {
+    float4 own[kAhead];
+    float f[kAhead], mo[kAhead];
+    bool last[kAhead];
+#pragma unroll
+    for (int j = 0; j < kAhead; ++j) {              // past the entry's last segment: read, not used
+      const int seg = min(base + j, a.num_segments - 1);
+      own[j] = *reinterpret_cast<const float4*>(ws + seg * pitch);
+      f[j] = a.ws_f[(int64_t)seg * H + h];
+      mo[j] = a.ws_m[(int64_t)seg * H + h];
+      last[j] = base + j >= a.num_segments - 1 || (a.segments[4 * seg + 3] & 2) != 0;
+    }
+#pragma unroll
+    for (int j = 0; j < kAhead; ++j) {
+      *reinterpret_cast<float4*>(ws + (base + j) * pitch) = x;
+      if (last[j]) return;
+      const float m_new = fmaxf(f[j] + m, mo[j]), keep = __expf(f[j] + m - m_new), add = __expf(mo[j] - m_new);
+      x.x = keep * x.x + add * own[j].x;
+      x.y = keep * x.y + add * own[j].y;
+      x.z = keep * x.z + add * own[j].z;
+      x.w = keep * x.w + add * own[j].w;
+      m = m_new;
+    }
   }
 }
 // The maxima in front of the segments: after the kernel above, which still needs the contributions' own.
@@ -446,7 +486,7 @@ static int launch_chunked(const MlstmChunkArgs& a, bool split, hipStream_t s) {
     int status = launch_status();
     if (status != 0) return status;
     const int64_t elements = (int64_t)a.dim * a.vdim + a.dim;
-    mlstm_combine_kernel<<<dim3((unsigned)a.num_segments, (unsigned)a.heads, (unsigned)((elements + 255) / 256)), dim3(256), 0, s>>>(a);
+    mlstm_combine_kernel<<<dim3((unsigned)a.num_segments, (unsigned)a.heads, (unsigned)((elements + kCombineElements - 1) / kCombineElements)), dim3(256), 0, s>>>(a);
     mlstm_combine_max_kernel<<<dim3((unsigned)a.num_segments, (unsigned)((a.heads + 63) / 64)), dim3(64), 0, s>>>(a);
     status = launch_status();
     if (status != 0) return status;
@@ -486,6 +526,7 @@ extern "C" int mvllm_mlstm_chunked(float* num, float* den, float* m_next, const 
   if (!aligned16(proj)) return MVLLM_ERR_MISALIGNED;
   if (split && (!workspace || workspace_bytes < mvllm_mlstm_chunked_workspace_bytes(num_segments, num_heads, dim, vdim)))
     return MVLLM_ERR_WORKSPACE;
+  if (split && (!aligned16(workspace) || !aligned16(s_state) || !aligned16(n_state))) return MVLLM_ERR_MISALIGNED;
   MlstmChunkArgs a;
   a.num = num; a.den = den; a.m_next = m_next; a.proj = reinterpret_cast<const bf16_t*>(proj); a.gates = gates;
   a.s_state = s_state; a.n_state = n_state; a.m_state = m_state; a.cu = cu_seqlens; a.slot = slots; a.positions = positions;
