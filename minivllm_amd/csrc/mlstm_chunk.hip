@@ -412,12 +412,13 @@ __global__ __launch_bounds__(64 * kWaves, DIMP == 256 ? 1 : 2) void mlstm_chunk_
 }
 
 // Contributions of an entry's segments -> the state in front of each of them, in place.  Workgroup = (first segment of an
-// entry, head, slice of the elements of S and n).  A thread owns four consecutive elements; the contributions of kAhead
-// segments are loaded together, before the states that replace them are stored.
+// entry, slice of the elements of S and n; head).  Slices run fastest: with segments there, the one workgroup in
+// num_segments that has work would always fall to the same XCD.  A thread owns four consecutive elements; the
+// contributions of kAhead segments are loaded together, before the states that replace them are stored.
 constexpr int kCombineElements = 1024, kAhead = 8;
 
-__global__ __launch_bounds__(256) void mlstm_combine_kernel(const MlstmChunkArgs a) {
-  const int seg0 = blockIdx.x, h = blockIdx.y;
+__global__ __launch_bounds__(256) void mlstm_combine_kernel(const MlstmChunkArgs a, int slices) {
+  const int seg0 = blockIdx.x / slices, slice = blockIdx.x % slices, h = blockIdx.y;
   const int flags0 = a.segments[4 * seg0 + 3];
   if (!(flags0 & 1) || (flags0 & 4)) return;
   const int slot = a.slot[a.segments[4 * seg0]];
@@ -425,7 +426,7 @@ __global__ __launch_bounds__(256) void mlstm_combine_kernel(const MlstmChunkArgs
   const int H = a.heads;
   const bool fresh = a.positions[a.segments[4 * seg0 + 1]] == 0;
   const int64_t per_s = (int64_t)a.dim * a.vdim;
-  const int64_t at = (int64_t)blockIdx.z * kCombineElements + 4 * threadIdx.x;
+  const int64_t at = (int64_t)slice * kCombineElements + 4 * threadIdx.x;
   if (at >= per_s + a.dim) return;                  // dim and dim * vdim are multiples of four
   const bool in_s = at < per_s;
   const int64_t pitch = in_s ? (int64_t)H * per_s : (int64_t)H * a.dim;         // between segments
@@ -485,8 +486,9 @@ static int launch_chunked(const MlstmChunkArgs& a, bool split, hipStream_t s) {
     mlstm_chunk_kernel<DIMP, kWaves, true><<<grid, block, 0, s>>>(a);
     int status = launch_status();
     if (status != 0) return status;
-    const int64_t elements = (int64_t)a.dim * a.vdim + a.dim;
-    mlstm_combine_kernel<<<dim3((unsigned)a.num_segments, (unsigned)a.heads, (unsigned)((elements + kCombineElements - 1) / kCombineElements)), dim3(256), 0, s>>>(a);
+    const int slices = (a.dim * a.vdim + a.dim + kCombineElements - 1) / kCombineElements;
+    if ((int64_t)slices * a.num_segments >= 1 << 24) return MVLLM_ERR_BAD_SHAPE;
+    mlstm_combine_kernel<<<dim3((unsigned)(slices * a.num_segments), (unsigned)a.heads), dim3(256), 0, s>>>(a, slices);
     mlstm_combine_max_kernel<<<dim3((unsigned)a.num_segments, (unsigned)((a.heads + 63) / 64)), dim3(64), 0, s>>>(a);
     status = launch_status();
     if (status != 0) return status;
