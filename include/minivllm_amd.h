@@ -573,6 +573,92 @@ int mvllm_mlstm_output(void* out, const float* num, const float* den, const floa
                        const int32_t* cu_seqlens, const int32_t* row_entry, const int32_t* slots, int64_t rows,
                        int num_heads, int vdim, int dtype, void* stream);
 
+/*
+ * Between two sublayers of a decoder whose residual is `streams` fp32 streams (hyper-connections; csrc/stream_norm.hip):
+ *     y' = scale * y;   x'_t = sum_s mix[s, t] x_s + out[t] y';   h = rms(sum_t in[t] x'_t) * gain
+ *   out [rows, out_row_stride] dtype = h, zeros past width;  x_out fp32 [rows, streams, width] = x' or NULL (may be x)
+ *   x fp32 [rows, streams, width];  scale fp32 [width] or NULL;  hc_out [streams], hc_mix [streams, streams] (from x to),
+ *   hc_in [streams] or NULL (the plain sum), gain [width]: fp32
+ *   y: [rows, y_row_stride] dtype, or with parts: y = sum_k weights[t, k] parts[part_row[t, k]] + sigmoid(gate[t]) * y,
+ *   parts [*, part_row_stride] dtype, part_row int32 [rows, top] (NULL: row t * top + k), weights fp32 [rows, top],
+ *   gate fp32, one per row gate_row_stride apart (NULL: 1), y NULL: no such row.
+ * mvllm_stream_embed_norm starts the streams: x_s = embed[token] * embed_scale + bigram[b], b = (previous * mul_prev +
+ *   token * mul_cur) mod buckets, b = buckets for a sequence's first token; embed [vocab, width], bigram [buckets + 1, width]
+ *   or NULL.  The token before an entry's first row is prev_tokens[bank_in[entry]] (int64); its last row writes
+ *   prev_tokens[bank_out[entry]].  Banks must differ for entries of more than one row.
+ * bf16 and fp32, up to 8 streams, width up to 16384 (4096 where it is not a multiple of 4).
+ */
+int mvllm_stream_embed_norm(void* out, int64_t out_row_stride, float* x_out, const void* embed, int64_t vocab,
+                            float embed_scale, const void* bigram, int64_t buckets, int64_t mul_prev, int64_t mul_cur,
+                            int64_t* prev_tokens, const int64_t* tokens, const int64_t* positions,
+                            const int32_t* cu_seqlens, const int32_t* row_entry, const int32_t* bank_in,
+                            const int32_t* bank_out, const float* hc_in, const float* gain, float eps, int64_t rows,
+                            int streams, int width, int dtype, void* stream);
+int mvllm_stream_norm(void* out, int64_t out_row_stride, float* x_out, const float* x, const void* y, int64_t y_row_stride,
+                      const void* parts, int64_t part_row_stride, const int32_t* part_row, const float* weights, int top,
+                      const float* gate, int64_t gate_row_stride, const float* scale, const float* hc_out,
+                      const float* hc_mix, const float* hc_in, const float* gain, float eps, int64_t rows, int streams,
+                      int width, int dtype, void* stream);
+
+/*
+ * Matrix memory with a constant decay per head: S = decay S + k v^T, num = S^T q (csrc/decay_memory.hip).
+ *   proj [rows, proj_row_stride]: q [H, dim] | k [H, dim] | v [H, vdim] | anything; silu != 0: each through z sigmoid(z)
+ *   num fp32 [rows, H, vdim];  decay fp32 [H] (the chunked form: its natural logarithm);  s_state fp32 [*, H, dim, vdim]
+ *   everything else as for mvllm_mlstm_recurrent / mvllm_mlstm_chunked.
+ * mvllm_gated_row_norm: out [rows, out_row_stride] = rms(x) * weight * sigmoid(gate), zeros past width; x fp32 [rows, width].
+ */
+int mvllm_decay_memory_recurrent(float* num, const void* proj, int64_t proj_row_stride, const float* decay, float* s_state,
+                                 const int32_t* cu_seqlens, const int32_t* slots, const int64_t* positions, int entries,
+                                 int num_heads, int dim, int vdim, int silu, int dtype, void* stream);
+size_t mvllm_decay_memory_chunked_workspace_bytes(int num_segments, int num_heads, int dim, int vdim);
+int mvllm_decay_memory_chunked(float* num, const void* proj, int64_t proj_row_stride, const float* log_decay,
+                               float* s_state, const int32_t* cu_seqlens, const int32_t* slots, const int64_t* positions,
+                               const int32_t* segments, int num_segments, int split, int num_heads, int dim, int vdim,
+                               int silu, int dtype, void* workspace, size_t workspace_bytes, void* stream);
+int mvllm_gated_row_norm(void* out, int64_t out_row_stride, const float* x, const float* weight, const void* gate,
+                         int64_t gate_row_stride, float eps, int64_t rows, int width, int dtype, void* stream);
+
+/*
+ * Attention over latents (csrc/latent.hip): a cache of one row per token, `padded` (a multiple of 32) elements wide with
+ * zeros past the rank.
+ * mvllm_latent_norm_store: c = rms(in[:rank]) * weight -> out [rows, padded] (or NULL) and cache row slots[t] (< 0: none).
+ * mvllm_head_linear: out[t, h, :N] = W_h x[t, h, :K], w [H, N, K]; row and head strides in elements.  bf16: K % 8 == 0,
+ *   N % 16 == 0.
+ * mvllm_latent_decode: softmax(scale q . c) c over the first lens[t] (int64) rows of entry row_entry[t]'s table: q and out
+ *   [rows, H, padded], cache [num_blocks, block_size, padded], block_tables int32 [entries, table_width]; 0 keys: zeros.
+ *   workspace: mvllm_latent_decode_workspace_bytes (max_keys = table_width * block_size), 16-byte aligned.
+ */
+int mvllm_latent_norm_store(void* out, const void* in, int64_t in_row_stride, const float* weight, float eps, void* cache,
+                            int64_t num_slots, const int64_t* slots, int64_t rows, int rank, int padded, int dtype,
+                            void* stream);
+int mvllm_head_linear(void* out, int64_t out_row_stride, int64_t out_head_stride, const void* x, int64_t x_row_stride,
+                      int64_t x_head_stride, const void* w, int64_t rows, int num_heads, int N, int K, int dtype,
+                      void* stream);
+size_t mvllm_latent_decode_workspace_bytes(int rows, int num_heads, int padded, int64_t max_keys, int dtype);
+int mvllm_latent_decode(void* out, const void* q, const void* cache, const int32_t* block_tables, int table_width,
+                        const int32_t* row_entry, const int64_t* lens, int rows, int num_heads, int padded, int block_size,
+                        int64_t num_blocks, float scale, int dtype, void* workspace, size_t workspace_bytes, void* stream);
+
+/*
+ * Mixture of experts (csrc/moe.hip).
+ * mvllm_moe_route: ids int32 [rows, top], weights fp32 [rows, top] from fp32 logits: s = sigmoid(z), choice = s + correction
+ *   (fp32 [experts] or NULL); with groups > 1 only experts of the `keep` groups of neighbours with the largest sums of their
+ *   two largest choices are open; weights = s / (sum + 1e-20).
+ * mvllm_moe_plan: (token, choice) pairs sorted by expert, into `plan` (mvllm_moe_plan_bytes; its first `pairs` int32 are the
+ *   sorted place of every pair).
+ * mvllm_moe_linear: w [experts, N, K]; glu: gate and up rows in turns of 32, result silu(gate) * up.  With a plan: row p of
+ *   out is sorted place p, reading x row pair / per_token (per_token > 0) or row p.  Without (bf16, at most 4096 pairs, for
+ *   the few rows of a decode step): row p of out is pair p, reading x row p / per_token or row p.  K % 64 == 0,
+ *   N % 16 == 0 (glu: 64), bf16 and fp32.
+ */
+int mvllm_moe_route(int32_t* ids, float* weights, const float* logits, int64_t logit_row_stride, const float* correction,
+                    int64_t rows, int experts, int top, int groups, int keep, void* stream);
+size_t mvllm_moe_plan_bytes(int64_t pairs, int experts);
+int mvllm_moe_plan(void* plan, size_t plan_bytes, const int32_t* ids, int64_t pairs, int experts, void* stream);
+int mvllm_moe_linear(void* out, int64_t out_row_stride, const void* x, int64_t x_row_stride, const void* w,
+                     const int32_t* ids, void* plan, int64_t pairs, int experts, int N, int K, int per_token, int glu,
+                     int dtype, void* stream);
+
 #ifdef __cplusplus
 }
 #endif

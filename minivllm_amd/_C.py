@@ -96,6 +96,26 @@ SIGNATURES = {
     "mvllm_mlstm_chunked_workspace_bytes": (c_size_t, [c_int] * 4),
     "mvllm_mlstm_chunked": (c_int, [c_void_p] * 4 + [c_int64] + [c_void_p] * 8 + [c_int] * 5 + [c_float, c_float, c_int,
                                                                                             c_void_p, c_size_t, c_void_p]),
+    "mvllm_stream_embed_norm": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_float, c_void_p] + [c_int64] * 3 +
+                                [c_void_p] * 9 + [c_float, c_int64, c_int, c_int, c_int, c_void_p]),
+    "mvllm_stream_norm": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p,
+                                  c_int, c_void_p, c_int64] + [c_void_p] * 5 + [c_float, c_int64, c_int, c_int, c_int, c_void_p]),
+    "mvllm_decay_memory_recurrent": (c_int, [c_void_p, c_void_p, c_int64] + [c_void_p] * 5 + [c_int] * 6 + [c_void_p]),
+    "mvllm_decay_memory_chunked_workspace_bytes": (c_size_t, [c_int] * 4),
+    "mvllm_decay_memory_chunked": (c_int, [c_void_p, c_void_p, c_int64] + [c_void_p] * 6 + [c_int] * 7 + [c_void_p, c_size_t,
+                                                                                                         c_void_p]),
+    "mvllm_gated_row_norm": (c_int, [c_void_p, c_int64] + [c_void_p] * 3 + [c_int64, c_float, c_int64, c_int, c_int, c_void_p]),
+    "mvllm_latent_norm_store": (c_int, [c_void_p, c_void_p, c_int64, c_void_p, c_float, c_void_p, c_int64, c_void_p, c_int64,
+                                        c_int, c_int, c_int, c_void_p]),
+    "mvllm_head_linear": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_int64, c_int64, c_void_p, c_int64] + [c_int] * 4 +
+                          [c_void_p]),
+    "mvllm_latent_decode_workspace_bytes": (c_size_t, [c_int, c_int, c_int, c_int64, c_int]),
+    "mvllm_latent_decode": (c_int, [c_void_p] * 4 + [c_int, c_void_p, c_void_p] + [c_int] * 4 + [c_int64, c_float, c_int, c_void_p,
+                                                                                         c_size_t, c_void_p]),
+    "mvllm_moe_route": (c_int, [c_void_p] * 3 + [c_int64, c_void_p, c_int64] + [c_int] * 4 + [c_void_p]),
+    "mvllm_moe_plan_bytes": (c_size_t, [c_int64, c_int]),
+    "mvllm_moe_plan": (c_int, [c_void_p, c_size_t, c_void_p, c_int64, c_int, c_void_p]),
+    "mvllm_moe_linear": (c_int, [c_void_p, c_int64, c_void_p, c_int64] + [c_void_p] * 3 + [c_int64] + [c_int] * 6 + [c_void_p]),
     "mvllm_mlstm_output": (c_int, [c_void_p] * 5 + [c_int64, c_float] + [c_void_p] * 5 + [c_int64, c_int, c_int, c_int,
                                                                                       c_void_p]),
 }

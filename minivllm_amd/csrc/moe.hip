@@ -1,0 +1,515 @@
+// Mixture of experts: the router's choice, the rows sorted by expert, and the experts' products.
+//   moe_route   scores s = sigmoid(z), choice scores s + correction; groups of neighbouring experts by the sum of their two
+//               largest choice scores, the best `keep` groups stay open; the `top` largest choice scores of those are chosen,
+//               weights s / (sum of the chosen s + 1e-20)
+//   moe_plan    (token, choice) pairs sorted by expert, and tiles of 128 sorted rows per expert
+//   moe_linear  out[row] = x[row] W_e^T, optionally silu(gate) * up behind it: W_e [2 F, K] with gate and up rows in turns of
+//               32, so that both halves of an output are in one lane
+// Products, by the number of rows: few (a decode step: no plan; a workgroup gathers its expert's rows itself, its waves share
+// K, weights stream once), many (bf16: 128 x 128 tiles on the matrix unit over sorted rows), any (fp32, over sorted rows).
+#include "prefill_tiles.h"
+
+#pragma clang fp contract(off)
+
+namespace mvllm {
+
+// ---- routing ----
+struct RouteArgs {
+  int32_t* ids;            // [T, top]
+  float* weights;          // [T, top]
+  const float* z;          // [T, z_stride] logits
+  const float* correction; // [E] or null
+  int64_t z_stride;
+  int rows, experts, top, groups, keep;
+};
+
+// One token per wave; lane l has experts l, l + 64, ...
+template <int NE>
+__global__ __launch_bounds__(256) void moe_route_kernel(const RouteArgs a) {
+  __shared__ float choice_of[4][64 * NE], group_of[4][64];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int row = blockIdx.x * 4 + wave;
+  const bool live = row < a.rows;
+  const int E = a.experts;
+  float s[NE], choice[NE];
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const int e = lane + 64 * i;
+    s[i] = 0.f;
+    choice[i] = -INFINITY;
+    if (live && e < E) {
+      s[i] = 1.0f / (1.0f + expf(-a.z[(int64_t)row * a.z_stride + e]));
+      choice[i] = s[i] + (a.correction ? a.correction[e] : 0.f);
+    }
+    choice_of[wave][e] = choice[i];
+  }
+  if (a.groups > 1) {
+    const int size = E / a.groups;
+    __syncthreads();
+    if (lane < a.groups) {
+      float first = -INFINITY, second = -INFINITY;
+      for (int j = 0; j < size; ++j) {
+        const float x = choice_of[wave][lane * size + j];
+        second = fmaxf(second, fminf(first, x));
+        first = fmaxf(first, x);
+      }
+      group_of[wave][lane] = size > 1 ? first + second : first;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      const int e = lane + 64 * i;
+      if (e >= E) continue;
+      const int g = e / size;
+      const float mine = group_of[wave][g];
+      int before = 0;
+      for (int j = 0; j < a.groups; ++j) {
+        const float x = group_of[wave][j];
+        before += x > mine || (x == mine && j < g);
+      }
+      if (before >= a.keep) choice[i] = -INFINITY;
+    }
+  }
+  float my_s = 0.f, sum = 0.f;
+  int my_id = 0;
+  for (int k = 0; k < a.top; ++k) {
+    float best = -INFINITY, best_s = 0.f;
+    int id = 1 << 30;
+#pragma unroll
+    for (int i = 0; i < NE; ++i)
+      if (choice[i] > best) { best = choice[i]; best_s = s[i]; id = lane + 64 * i; }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float x = __shfl_xor(best, o, 64), xs = __shfl_xor(best_s, o, 64);
+      const int xi = __shfl_xor(id, o, 64);
+      if (x > best || (x == best && xi < id)) { best = x; best_s = xs; id = xi; }
+    }
+    if (id >= E) id = 0;                            // (nothing left to choose)
+#pragma unroll
+    for (int i = 0; i < NE; ++i)
+      if (lane + 64 * i == id) choice[i] = -INFINITY;
+    sum += best_s;
+    if (lane == k) { my_s = best_s; my_id = id; }
+  }
+  if (live && lane < a.top) {
+    a.ids[(int64_t)row * a.top + lane] = my_id;
+    a.weights[(int64_t)row * a.top + lane] = my_s / (sum + 1e-20f);
+  }
+}
+
+// ---- pairs sorted by expert ----
+constexpr int kTileRows = 128, kPlanPairs = 2048, kMaxExperts = 1024;
+
+struct PlanArgs {
+  const int32_t* ids;      // [pairs]
+  int32_t* hist;           // [blocks, E]
+  int32_t* sorted_pair;    // [pairs]: pair at a sorted place
+  int32_t* place;          // [pairs]: sorted place of a pair
+  int32_t* row_start;      // [E + 1]
+  int32_t* tile_expert;    // [max tiles]
+  int32_t* tile_row;       // [max tiles]: first sorted row
+  int32_t* num_tiles;      // [1]
+  int pairs, experts, blocks;
+};
+
+__global__ __launch_bounds__(256) void moe_count_kernel(const PlanArgs a) {
+  __shared__ int32_t count[kMaxExperts];
+  for (int e = threadIdx.x; e < a.experts; e += 256) count[e] = 0;
+  __syncthreads();
+  const int end = min((int)(blockIdx.x + 1) * kPlanPairs, a.pairs);
+  for (int p = blockIdx.x * kPlanPairs + threadIdx.x; p < end; p += 256) atomicAdd(&count[a.ids[p]], 1);
+  __syncthreads();
+  for (int e = threadIdx.x; e < a.experts; e += 256) a.hist[(int64_t)blockIdx.x * a.experts + e] = count[e];
+}
+
+__global__ __launch_bounds__(1024) void moe_place_kernel(const PlanArgs a) {
+  __shared__ int32_t total[kMaxExperts + 1], tiles[kMaxExperts + 1], cursor[kMaxExperts];
+  const int e = threadIdx.x;
+  int n = 0, mine = 0;
+  if (e < a.experts)
+    for (int b = 0; b < a.blocks; ++b) {
+      if (b == (int)blockIdx.x) mine = n;
+      n += a.hist[(int64_t)b * a.experts + e];
+    }
+  // inclusive sums over the experts
+  total[e + 1] = n;
+  tiles[e + 1] = (n + kTileRows - 1) / kTileRows;
+  if (e == 0) total[0] = tiles[0] = 0;
+  __syncthreads();
+  for (int o = 1; o < 1024; o <<= 1) {
+    const int x = e + 1 > o ? total[e + 1 - o] : 0, y = e + 1 > o ? tiles[e + 1 - o] : 0;
+    __syncthreads();
+    total[e + 1] += x;
+    tiles[e + 1] += y;
+    __syncthreads();
+  }
+  if (e < a.experts) cursor[e] = total[e] + mine;
+  __syncthreads();
+  const int end = min((int)(blockIdx.x + 1) * kPlanPairs, a.pairs);
+  for (int p = blockIdx.x * kPlanPairs + threadIdx.x; p < end; p += 1024) {
+    const int at = atomicAdd(&cursor[a.ids[p]], 1);
+    a.sorted_pair[at] = p;
+    a.place[p] = at;
+  }
+  if (blockIdx.x == 0 && e < a.experts) {
+    a.row_start[e] = total[e];
+    if (e == a.experts - 1) {
+      a.row_start[e + 1] = total[e + 1];
+      a.num_tiles[0] = tiles[e + 1];
+    }
+    for (int t = tiles[e]; t < tiles[e + 1]; ++t) {
+      a.tile_expert[t] = e;
+      a.tile_row[t] = total[e] + (t - tiles[e]) * kTileRows;
+    }
+  }
+}
+
+// ---- products ----
+struct ExpertLinearArgs {
+  void* out;                   // [pairs, out_stride]
+  const void* x;               // [*, x_stride]
+  const void* w;               // [E, N, K]
+  const int32_t* ids;          // [pairs] (few)
+  const int32_t* sorted_pair;  // (many, any) plan, see above
+  const int32_t* row_start;
+  const int32_t* tile_expert;
+  const int32_t* tile_row;
+  const int32_t* num_tiles;
+  int64_t x_stride, out_stride;
+  int pairs, experts, N, K;
+  int per_token;               // > 0: pair p reads row p / per_token of x; 0: the row of its own (sorted) place
+  int max_tiles, n_tiles;
+  uint32_t x_bytes;            // (many) what x holds
+};
+
+__device__ __forceinline__ float silu_of(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
+
+// few: workgroup = (16 outputs, expert).  The rows of the expert are found in `ids`; rows are taken 16 at a time.
+constexpr int kFewPairs = 4096;
+
+template <int kWaves, bool kGlu>
+__global__ __launch_bounds__(64 * kWaves) void moe_linear_few_kernel(const ExpertLinearArgs a) {
+  constexpr int NT = kGlu ? 2 : 1;
+  __shared__ uint16_t list[kFewPairs];
+  __shared__ int found;
+  __shared__ float4 part[kWaves][NT][64];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, i16 = lane & 15;
+  const int e = blockIdx.y;
+  if (wave == 0) {
+    int n = 0;
+    for (int base = 0; base < a.pairs; base += 64) {
+      const int p = base + lane;
+      const bool hit = p < a.pairs && a.ids[p] == e;
+      const unsigned long long hits = __ballot(hit);
+      if (hit) list[n + __popcll(hits & ((1ull << lane) - 1))] = (uint16_t)p;
+      n += __popcll(hits);
+    }
+    if (lane == 0) found = n;
+  }
+  __syncthreads();
+  const int rows = found;
+  if (rows == 0) return;
+  const int n0 = blockIdx.x * 16;                   // first output of the workgroup
+  const bf16_t* w[NT];
+#pragma unroll
+  for (int n = 0; n < NT; ++n) {
+    const int wr = kGlu ? (n0 >> 5) * 64 + (n0 & 31) + 32 * n : n0;
+    w[n] = reinterpret_cast<const bf16_t*>(a.w) + ((int64_t)e * a.N + wr + i16) * a.K;
+  }
+  for (int r0 = 0; r0 < rows; r0 += 16) {
+    const int pair = list[min(r0 + i16, rows - 1)];
+    const bf16_t* x = reinterpret_cast<const bf16_t*>(a.x) + (int64_t)(a.per_token ? pair / a.per_token : pair) * a.x_stride;
+    v4f acc[NT];
+#pragma unroll
+    for (int n = 0; n < NT; ++n) acc[n] = v4f{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int k0 = 64 * wave; k0 < a.K; k0 += 64 * kWaves) {            // a lane's 32 bytes: whole lines per row and wave
+      const int k = k0 + 16 * g;
+      uint4 xv[2], wv[NT][2];
+#pragma unroll
+      for (int half = 0; half < 2; ++half) {
+#pragma unroll
+        for (int n = 0; n < NT; ++n) wv[n][half] = load16_stream(w[n] + k + 8 * half);
+        xv[half] = *reinterpret_cast<const uint4*>(x + k + 8 * half);
+      }
+#pragma unroll
+      for (int half = 0; half < 2; ++half)
+#pragma unroll
+        for (int n = 0; n < NT; ++n) acc[n] = mfma16x16x32<bf16_t>(wv[n][half], xv[half], acc[n]);
+    }
+    // lane: row i16, outputs 4 g + r
+#pragma unroll
+    for (int n = 0; n < NT; ++n) part[wave][n][lane] = make_float4(acc[n][0], acc[n][1], acc[n][2], acc[n][3]);
+    __syncthreads();
+    if (wave == 0 && r0 + i16 < rows) {
+      float z[NT][4];
+#pragma unroll
+      for (int n = 0; n < NT; ++n) {
+        z[n][0] = z[n][1] = z[n][2] = z[n][3] = 0.f;
+#pragma unroll
+        for (int i = 0; i < kWaves; ++i) {
+          const float4 p = part[i][n][lane];
+          z[n][0] += p.x; z[n][1] += p.y; z[n][2] += p.z; z[n][3] += p.w;
+        }
+      }
+      float o[4];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o[r] = kGlu ? silu_of(z[0][r]) * z[NT - 1][r] : z[0][r];
+      bf16_t* out = reinterpret_cast<bf16_t*>(a.out) + (int64_t)pair * a.out_stride + n0 + 4 * g;
+      *reinterpret_cast<uint2*>(out) = make_uint2(pack2<bf16_t>(o[0], o[1]), pack2<bf16_t>(o[2], o[3]));
+    }
+    __syncthreads();
+  }
+}
+
+// any: workgroup = (16 outputs, expert, every gridDim.z-th 16 sorted rows), one dot product (two with the gate) per thread.
+template <typename T, bool kGlu>
+__global__ __launch_bounds__(256) void moe_linear_any_kernel(const ExpertLinearArgs a) {
+  constexpr int kStep = 64, NT = kGlu ? 2 : 1;
+  __shared__ float xs[16][kStep + 1], ws[NT][16][kStep + 1];
+  const int tid = threadIdx.x, r = tid >> 4, c = tid & 15, e = blockIdx.y, n0 = blockIdx.x * 16;
+  const int first = a.row_start[e], last = a.row_start[e + 1];
+  for (int base = first + 16 * blockIdx.z; base < last; base += 16 * gridDim.z) {
+    float acc[NT];
+#pragma unroll
+    for (int n = 0; n < NT; ++n) acc[n] = 0.f;
+    for (int k0 = 0; k0 < a.K; k0 += kStep) {
+      for (int i = tid; i < 16 * kStep; i += 256) {
+        const int rr = i / kStep, k = k0 + i % kStep, at = base + rr;
+        float xv = 0.f;
+        if (at < last && k < a.K)
+          xv = to_float(reinterpret_cast<const T*>(a.x)[(int64_t)(a.per_token ? a.sorted_pair[at] / a.per_token : at) * a.x_stride + k]);
+        xs[rr][i % kStep] = xv;
+#pragma unroll
+        for (int n = 0; n < NT; ++n) {
+          const int wr = kGlu ? ((n0 + rr) >> 5) * 64 + ((n0 + rr) & 31) + 32 * n : n0 + rr;
+          ws[n][rr][i % kStep] = wr < a.N && k < a.K ? to_float(reinterpret_cast<const T*>(a.w)[((int64_t)e * a.N + wr) * a.K + k]) : 0.f;
+        }
+      }
+      __syncthreads();
+#pragma unroll 16
+      for (int k = 0; k < kStep; ++k)
+#pragma unroll
+        for (int n = 0; n < NT; ++n) acc[n] = fmaf(xs[r][k], ws[n][c][k], acc[n]);
+      __syncthreads();
+    }
+    if (base + r < last) {
+      const float o = kGlu ? acc[0] / (1.0f + expf(-acc[0])) * acc[NT - 1] : acc[0];
+      reinterpret_cast<T*>(a.out)[(int64_t)(base + r) * a.out_stride + n0 + c] = from_float<T>(o);
+    }
+  }
+}
+
+// many: 128 sorted rows x 128 weight rows per workgroup, four waves of 64 x 64 on v_mfma_f32_32x32x16_bf16.  Weights are the
+// row operand and x the column operand, so that a lane ends with runs of four outputs of one row.  Steps of 64 along K, two
+// buffers in LDS that the copies of the next step fill during this one; a row's eight 16-byte chunks trade places by half
+// the row's number.  Consecutive workgroups of an XCD go through four row tiles for every weight tile.
+template <bool kGlu>
+__global__ __launch_bounds__(256, 2) void moe_linear_many_kernel(const ExpertLinearArgs a) {
+  constexpr int kTile = 128, kK = 64, kStage = kTile * kK * 2;       // bytes of one operand's step
+  constexpr int kTogether = 4;
+  __shared__ __attribute__((aligned(16))) char lds[4 * kStage];      // [buffer][weights, x]
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), l32 = lane & 31, hi = lane >> 5;
+  // ---- which tile ----
+  const int total = a.num_tiles[0], per = (total + 7) / 8;
+  const int xcd = blockIdx.x & 7, j = blockIdx.x >> 3;
+  const int group = j / (kTogether * a.n_tiles), in_group = j % (kTogether * a.n_tiles);
+  const int local = group * kTogether + in_group % kTogether, tile = xcd * per + local, n_tile = in_group / kTogether;
+  if (local >= per || tile >= total) return;
+  const int e = a.tile_expert[tile], row0 = a.tile_row[tile], row_end = min(row0 + kTile, a.row_start[e + 1]);
+  const int n0 = n_tile * kTile;
+
+  // ---- copies: four chunks of either operand per thread and step ----
+  const v4i w_rows = make_rsrc(reinterpret_cast<const char*>(a.w) + (int64_t)e * a.N * a.K * 2, (uint32_t)((int64_t)a.N * a.K * 2));
+  const v4i x_rows = make_rsrc(reinterpret_cast<const char*>(a.x), a.x_bytes);
+  uint32_t from_w[4], from_x[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int c = 256 * i + tid, r = c >> 3, p = (c & 7) ^ ((r >> 1) & 7);
+    from_w[i] = (uint32_t)(min(n0 + r, a.N - 1) * a.K + 8 * p) * 2u;
+    const int at = min(row0 + r, row_end - 1);
+    const uint32_t xr = (uint32_t)(a.per_token ? a.sorted_pair[at] / a.per_token : at);
+    from_x[i] = (xr * (uint32_t)a.x_stride + 8u * p) * 2u;
+  }
+  auto copy = [&](int buffer) __attribute__((always_inline)) {
+    const uint32_t base = lds_address(lds) + buffer * 2 * kStage + 1024 * wave;
+    static_for<4>([&](auto I) {
+      constexpr int i = decltype(I)::value;
+      dma16_to_lds<4096 * i>(w_rows, from_w[i], base);
+      dma16_to_lds<kStage + 4096 * i>(x_rows, from_x[i], base);
+      from_w[i] += 2 * kK;
+      from_x[i] += 2 * kK;
+    });
+  };
+  const int wn = wave & 1, wm = wave >> 1;          // the wave's half of the weight rows and of the rows
+  // places of this lane's fragments: row l32 of a 32-row block, chunk 2 st + hi
+  const int sw = (l32 >> 1) & 7;
+  const char* frag = lds + l32 * 128;
+  v16f acc[2][2];
+#pragma unroll
+  for (int n = 0; n < 2; ++n)
+#pragma unroll
+    for (int m = 0; m < 2; ++m)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) acc[n][m][r] = 0.f;
+
+  copy(0);
+  const int steps = a.K / kK;
+  for (int step = 0; step < steps; ++step) {
+    const int buffer = step & 1;
+    dma_wait_all();
+    __syncthreads();                                // this step's operands are there, the other buffer is free
+    if (step + 1 < steps) copy(buffer ^ 1);
+    const char* wb = frag + buffer * 2 * kStage + wn * 64 * 128;
+    const char* xb = frag + buffer * 2 * kStage + kStage + wm * 64 * 128;
+#pragma unroll
+    for (int st = 0; st < 4; ++st) {
+      const int p = ((2 * st + hi) ^ sw) << 4;
+      uint4 wf[2], xf[2];
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        wf[i] = *reinterpret_cast<const uint4*>(wb + i * 32 * 128 + p);
+        xf[i] = *reinterpret_cast<const uint4*>(xb + i * 32 * 128 + p);
+      }
+#pragma unroll
+      for (int n = 0; n < 2; ++n)
+#pragma unroll
+        for (int m = 0; m < 2; ++m) acc[n][m] = mfma32x32x16<bf16_t>(wf[n], xf[m], acc[n][m]);
+    }
+  }
+  // ---- lane: row l32 of a block, weight rows 8 (r / 4) + 4 hi + r % 4 ----
+#pragma unroll
+  for (int m = 0; m < 2; ++m) {
+    const int row = row0 + wm * 64 + 32 * m + l32;
+    if (row >= row_end) continue;
+    bf16_t* out = reinterpret_cast<bf16_t*>(a.out) + (int64_t)row * a.out_stride;
+#pragma unroll
+    for (int r = 0; r < 16; r += 4) {
+      if constexpr (kGlu) {
+        const int col = (n0 + wn * 64) / 2 + 2 * r + 4 * hi;
+        float o[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[i] = silu_of(acc[0][m][r + i]) * acc[1][m][r + i];
+        if (2 * col < a.N) *reinterpret_cast<uint2*>(out + col) = make_uint2(pack2<bf16_t>(o[0], o[1]), pack2<bf16_t>(o[2], o[3]));
+      } else {
+#pragma unroll
+        for (int n = 0; n < 2; ++n) {
+          const int col = n0 + wn * 64 + 32 * n + 2 * r + 4 * hi;
+          if (col < a.N)
+            *reinterpret_cast<uint2*>(out + col) = make_uint2(pack2<bf16_t>(acc[n][m][r], acc[n][m][r + 1]), pack2<bf16_t>(acc[n][m][r + 2], acc[n][m][r + 3]));
+        }
+      }
+    }
+  }
+}
+
+static int64_t max_tiles(int64_t pairs, int experts) { return (pairs + kTileRows - 1) / kTileRows + experts; }
+static int plan_blocks(int64_t pairs) { return (int)((pairs + kPlanPairs - 1) / kPlanPairs); }
+
+}  // namespace mvllm
+
+using namespace mvllm;
+
+extern "C" int mvllm_moe_route(int32_t* ids, float* weights, const float* logits, int64_t logit_row_stride,
+                               const float* correction, int64_t rows, int experts, int top, int groups, int keep,
+                               void* stream) {
+  if (rows < 0 || experts <= 0 || top <= 0 || top > experts || groups <= 0 || experts % groups != 0 || keep <= 0 || keep > groups ||
+      logit_row_stride < experts || (int64_t)keep * (experts / groups) < top)
+    return MVLLM_ERR_BAD_SHAPE;
+  if (experts > kMaxExperts || top > 64 || groups > 64 || rows > (1 << 28)) return MVLLM_ERR_UNSUPPORTED;
+  if (rows == 0) return MVLLM_OK;
+  if (!ids || !weights || !logits) return MVLLM_ERR_NULL_POINTER;
+  RouteArgs a;
+  a.ids = ids; a.weights = weights; a.z = logits; a.correction = correction; a.z_stride = logit_row_stride;
+  a.rows = (int)rows; a.experts = experts; a.top = top; a.groups = groups; a.keep = keep;
+  const dim3 grid((unsigned)((rows + 3) / 4)), block(256);
+  hipStream_t s = (hipStream_t)stream;
+  if (experts <= 64) moe_route_kernel<1><<<grid, block, 0, s>>>(a);
+  else if (experts <= 128) moe_route_kernel<2><<<grid, block, 0, s>>>(a);
+  else if (experts <= 256) moe_route_kernel<4><<<grid, block, 0, s>>>(a);
+  else moe_route_kernel<16><<<grid, block, 0, s>>>(a);
+  return launch_status();
+}
+
+extern "C" size_t mvllm_moe_plan_bytes(int64_t pairs, int experts) {
+  if (pairs <= 0 || experts <= 0) return 0;
+  return (size_t)(2 * pairs + experts + 1 + 2 * max_tiles(pairs, experts) + 1 + (int64_t)plan_blocks(pairs) * experts + 4) * sizeof(int32_t);
+}
+
+// the parts of a plan, in order
+static PlanArgs plan_parts_of(void* plan, const int32_t* ids, int64_t pairs, int experts) {
+  PlanArgs a;
+  a.ids = ids;
+  a.place = reinterpret_cast<int32_t*>(plan);
+  a.sorted_pair = a.place + pairs;
+  a.row_start = a.sorted_pair + pairs;
+  a.tile_expert = a.row_start + experts + 1;
+  a.tile_row = a.tile_expert + max_tiles(pairs, experts);
+  a.num_tiles = a.tile_row + max_tiles(pairs, experts);
+  a.hist = a.num_tiles + 1;
+  a.pairs = (int)pairs; a.experts = experts; a.blocks = plan_blocks(pairs);
+  return a;
+}
+
+extern "C" int mvllm_moe_plan(void* plan, size_t plan_bytes, const int32_t* ids, int64_t pairs, int experts, void* stream) {
+  if (pairs < 0 || experts <= 0) return MVLLM_ERR_BAD_SHAPE;
+  if (experts > kMaxExperts || pairs > (1 << 30)) return MVLLM_ERR_UNSUPPORTED;
+  if (pairs == 0) return MVLLM_OK;
+  if (!plan || !ids) return MVLLM_ERR_NULL_POINTER;
+  if (plan_bytes < mvllm_moe_plan_bytes(pairs, experts)) return MVLLM_ERR_WORKSPACE;
+  const PlanArgs a = plan_parts_of(plan, ids, pairs, experts);
+  hipStream_t s = (hipStream_t)stream;
+  moe_count_kernel<<<dim3((unsigned)a.blocks), dim3(256), 0, s>>>(a);
+  moe_place_kernel<<<dim3((unsigned)a.blocks), dim3(1024), 0, s>>>(a);
+  return launch_status();
+}
+
+extern "C" int mvllm_moe_linear(void* out, int64_t out_row_stride, const void* x, int64_t x_row_stride, const void* w,
+                                const int32_t* ids, void* plan, int64_t pairs, int experts, int N, int K, int per_token,
+                                int glu, int dtype, void* stream) {
+  if (dtype_size(dtype) == 0) return MVLLM_ERR_BAD_DTYPE;
+  if (pairs < 0 || experts <= 0 || N <= 0 || K <= 0 || per_token < 0 || x_row_stride < K || out_row_stride < (glu ? N / 2 : N)) return MVLLM_ERR_BAD_SHAPE;
+  if (dtype == MVLLM_F16 || experts > kMaxExperts || pairs > (1 << 30) || K % 64 != 0 || N % (glu ? 64 : 16) != 0 || x_row_stride % 8 != 0 ||
+      out_row_stride % 4 != 0)
+    return MVLLM_ERR_UNSUPPORTED;
+  if (pairs == 0) return MVLLM_OK;
+  if (!out || !x || !w || (!plan && !ids)) return MVLLM_ERR_NULL_POINTER;
+  if (!aligned16(out) || !aligned16(x) || !aligned16(w)) return MVLLM_ERR_MISALIGNED;
+  if (!plan && (dtype != MVLLM_BF16 || pairs > kFewPairs)) return MVLLM_ERR_UNSUPPORTED;
+  ExpertLinearArgs a = {};
+  a.out = out; a.x = x; a.w = w; a.ids = ids; a.x_stride = x_row_stride; a.out_stride = out_row_stride; a.pairs = (int)pairs;
+  a.experts = experts; a.N = N; a.K = K; a.per_token = per_token;
+  hipStream_t s = (hipStream_t)stream;
+  const int outputs = glu ? N / 2 : N;
+  if (!plan) {
+    const dim3 grid((unsigned)(outputs / 16), (unsigned)experts);
+    if (K >= 1024) {
+      if (glu) moe_linear_few_kernel<8, true><<<grid, dim3(512), 0, s>>>(a);
+      else moe_linear_few_kernel<8, false><<<grid, dim3(512), 0, s>>>(a);
+    } else {
+      if (glu) moe_linear_few_kernel<4, true><<<grid, dim3(256), 0, s>>>(a);
+      else moe_linear_few_kernel<4, false><<<grid, dim3(256), 0, s>>>(a);
+    }
+    return launch_status();
+  }
+  const PlanArgs p = plan_parts_of(plan, ids, pairs, experts);
+  a.sorted_pair = p.sorted_pair; a.row_start = p.row_start; a.tile_expert = p.tile_expert; a.tile_row = p.tile_row;
+  a.num_tiles = p.num_tiles;
+  if (dtype == MVLLM_BF16) {
+    a.max_tiles = (int)max_tiles(pairs, experts);
+    a.n_tiles = (N + 127) / 128;
+    const int64_t x_rows = per_token ? (pairs + per_token - 1) / per_token : pairs, x_bytes = ((x_rows - 1) * x_row_stride + K) * 2;
+    if (x_bytes >= (int64_t)1 << 32 || (int64_t)N * K * 2 >= (int64_t)1 << 31) return MVLLM_ERR_UNSUPPORTED;
+    a.x_bytes = (uint32_t)x_bytes;
+    const int64_t per = (a.max_tiles + 7) / 8, groups = (per + 3) / 4, blocks = 8 * groups * 4 * a.n_tiles;
+    if (blocks > 0x7fffffff) return MVLLM_ERR_BAD_SHAPE;
+    if (glu) moe_linear_many_kernel<true><<<dim3((unsigned)blocks), dim3(256), 0, s>>>(a);
+    else moe_linear_many_kernel<false><<<dim3((unsigned)blocks), dim3(256), 0, s>>>(a);
+  } else {
+    int64_t z = pairs / (16 * (int64_t)experts) + 1;
+    const dim3 grid((unsigned)(outputs / 16), (unsigned)experts, (unsigned)(z > 64 ? 64 : z));
+    if (glu) moe_linear_any_kernel<float, true><<<grid, dim3(256), 0, s>>>(a);
+    else moe_linear_any_kernel<float, false><<<grid, dim3(256), 0, s>>>(a);
+  }
+  return launch_status();
+}

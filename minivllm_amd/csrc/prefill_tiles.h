@@ -84,6 +84,10 @@ template <int LDS_IMM>   // LDS destination = lds_base + LDS_IMM: one scalar reg
 __device__ __forceinline__ void dma16_to_lds(v4i rsrc, uint32_t lane_off, uint32_t lds_base) {
   asm volatile("s_add_u32 m0, %0, %3\n\tbuffer_load_dwordx4 %1, %2, 0 offen lds" ::"s"(lds_base), "v"(lane_off), "s"(rsrc), "n"(LDS_IMM) : "scc", "m0");
 }
+// The same from a 64-bit address per lane (no bounds check).
+__device__ __forceinline__ void dma16_to_lds_from(const void* p, uint32_t lds_base) {
+  asm volatile("s_mov_b32 m0, %0\n\tglobal_load_lds_dwordx4 %1, off" ::"s"(lds_base), "v"(p) : "m0");
+}
 // Raw buffer descriptor: 48-bit base, stride 0, size in bytes, 32-bit untyped data.
 __device__ __forceinline__ v4i make_rsrc(const char* base, uint32_t bytes) {
   const uint64_t b = (uint64_t)base;

@@ -1,4 +1,4 @@
-"""Runner of models that run ragged steps and keep recurrent state (models/sokevik.py): portions of prompts and decoded
+"""Runner of models that run ragged steps and keep recurrent state (models/sokevik.py, models/niridra.py): portions of prompts and decoded
 tokens in one batch, a cache manager of its own, and the captured decode step of ``ModelRunner`` over more static buffers.
 
 Engine keys as for ``ModelRunner``; ``max_cached_blocks`` counts the blocks of each attention window's pool,
@@ -9,8 +9,7 @@ import torch
 
 from minivllm_amd.engine.hybrid_cache import HybridCacheManager
 from minivllm_amd.engine.model_runner import _DTYPES, ModelRunner
-from minivllm_amd.engine.ragged import RaggedStep, WindowStep, ragged_step
-from minivllm_amd.layers.attention import decode_workspace_bytes
+from minivllm_amd.engine.ragged import LatentStep, RaggedStep, WindowStep, ragged_step
 from minivllm_amd.layers.fused import chunk_decode_step, lm_head_sample, lm_head_sample_takes, sample_tokens
 from minivllm_amd.utils.context import reset_context, set_context
 
@@ -43,7 +42,8 @@ class HybridModelRunner(ModelRunner):
     @torch.inference_mode()
     def forward_step(self, seqs, layer_outputs=None):
         """Run every sequence's scheduled tokens; returns (hidden rows, the step)."""
-        step = ragged_step(seqs, self.model.windows, self.block_size, self.device, self.model.memory_units)
+        step = ragged_step(seqs, self.model.windows, self.block_size, self.device, self.model.memory_units,
+                           self.model.latent_views)
         set_context(step.multi_rows > 0, ragged=step)
         try:
             hidden = self.model(step.input_ids, step.positions, layer_outputs)
@@ -91,11 +91,10 @@ class HybridModelRunner(ModelRunner):
         return [self.cache_manager.blocks_for(w, longest) for w in self.model.windows]
 
     def _own_decode_workspace(self, buckets, max_blocks):
-        need = 16
+        need, widths = 16, self._table_widths()
         for layer in self.model.layer_stack:
             if layer.is_attention:
-                m, width = layer.mixer, self._table_widths()[layer.mixer.window]
-                need = max([need] + [decode_workspace_bytes(b, m.num_heads, m.head_dim, width, self.block_size) for b in buckets])
+                need = max([need] + [layer.mixer.workspace_bytes(b, widths[layer.mixer.window]) for b in buckets])
         self.decode_workspace = torch.empty(need, dtype=torch.uint8, device=self.device)
         for layer in self.model.layer_stack:
             if layer.is_attention:
@@ -114,7 +113,10 @@ class HybridModelRunner(ModelRunner):
         v = self.graph_vars
         lens, slots = [t[:bs] for t in v["chunk_lens"]], [t[:bs] for t in v["chunk_slots"]]
         tables = [t[:bs] for t in v["tables"]]
-        windows = [WindowStep(num_decode=bs, slots=s, chunk_lens=n, decode_tables=t) for s, n, t in zip(slots, lens, tables)]
+        if self.model.latent_views:
+            windows = [LatentStep(absorbed=bs, slots=s, lens=n, tables=t) for s, n, t in zip(slots, lens, tables)]
+        else:
+            windows = [WindowStep(num_decode=bs, slots=s, chunk_lens=n, decode_tables=t) for s, n, t in zip(slots, lens, tables)]
         step = RaggedStep(num_tokens=bs, num_entries=bs, num_single=bs, num_short=bs, input_ids=v["input_ids"][:bs],
                           positions=v["positions"][:bs], cu_seqlens=v["cu_seqlens"][:bs + 1], row_entry=v["row_entry"][:bs],
                           bank_in=v["banks"][:bs], bank_out=v["banks"][:bs], state_slots=v["state_slots"][:bs], windows=windows)

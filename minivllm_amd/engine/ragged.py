@@ -5,6 +5,8 @@ that goes on in a chunk whose earlier tokens are cached reads the cache (``prefi
 packed keys and values of the step (``fresh``), single tokens take the decode kernel.  Pieces are sorted in that order
 (``dst_row``), so that each kernel runs over consecutive rows.  Only the tokens of an entry's last chunk stay cached; where
 the entry also reads the chunk before, whose blocks they go to, they are stored after attention (``late_slots``).
+Layers that cache one latent per token (``LatentStep``) answer single and short entries row by row from the cache; long
+entries with a cached prefix come before those without.
 A recurrence takes single and short entries row by row and long ones in blocks of rows, cut into ``segments`` that run side
 by side where there are too few of them to fill the GPU."""
 from __future__ import annotations
@@ -35,6 +37,23 @@ class WindowStep:
 
 
 @dataclass
+class LatentStep:
+    """The step as layers see it that cache one latent per token and attend to the whole sequence."""
+    absorbed: int = 0                                 # rows of single and short entries (the first ones)
+    num_prefixed: int = 0                             # rows of long entries behind a cached prefix, next
+    num_fresh: int = 0                                # rows of long entries that start a sequence
+    slots: Optional[torch.Tensor] = None              # int64 [T]
+    lens: Optional[torch.Tensor] = None               # int64 [absorbed]: keys a row sees
+    tables: Optional[torch.Tensor] = None             # int32 [entries, width]
+    prefixed_cu_q: Optional[torch.Tensor] = None      # int32 [entries + 1]
+    prefixed_cu_k: Optional[torch.Tensor] = None
+    prefixed_max_k: int = 0
+    gather: Optional[torch.Tensor] = None             # int64 [blocks]: the prefixed entries' blocks, one after the other
+    scratch_tables: Optional[torch.Tensor] = None     # int32 [entries, width]: their places in that order
+    fresh_cu: Optional[torch.Tensor] = None
+
+
+@dataclass
 class RaggedStep:
     num_tokens: int
     num_entries: int
@@ -46,13 +65,14 @@ class RaggedStep:
     bank_in: torch.Tensor                             # int32 [entries]: banks of the short-convolution state
     bank_out: torch.Tensor
     state_slots: torch.Tensor                         # int32 [entries]
-    windows: list = field(default_factory=list)       # WindowStep per window
+    windows: list = field(default_factory=list)       # WindowStep (LatentStep) per window
     multi_rows: int = 0                               # rows of entries with more than one token
     num_short: int = 0                                # entries below LONG_ROWS (the first ones)
     segments: Optional[torch.Tensor] = None           # int32 [n, 4] of long entries: entry, first row, rows, flags
     split: bool = False                               # some long entry has more than one segment
     order: list = field(default_factory=list)         # entry e of the packing is sequence order[e] of the caller
     starts: list = field(default_factory=list)        # first packed row of the caller's sequence i
+    scratch: dict = field(default_factory=dict)       # what layers of one step share
 
 
 LONG_ROWS = 32                 # an entry of at least this many rows is long
@@ -153,11 +173,43 @@ def _window_arrays(items, window, index, block_size, cu):
     return out, counts
 
 
-def ragged_arrays(seqs, windows, block_size, memory_units=0):
+def _latent_arrays(items, index, block_size, cu, num_short):
+    """Host arrays of a LatentStep; items as for ``_window_arrays``."""
+    slots = np.empty(int(cu[-1]), dtype=np.int64)
+    pre_q, pre_k, gather, scratch, fresh = [0], [0], [], [], [0]
+    tables = [seq.group_tables[index] for _, _, seq in items]
+    for e, (p0, n, _) in enumerate(items):
+        place = np.arange(p0, p0 + n)
+        slots[cu[e]:cu[e + 1]] = np.asarray(tables[e], dtype=np.int64)[place // block_size] * block_size + place % block_size
+        if e < num_short:
+            continue
+        if p0:
+            pre_q.append(pre_q[-1] + n)
+            pre_k.append(pre_k[-1] + p0 + n)
+            used = -(-(p0 + n) // block_size)
+            scratch.append(list(range(len(gather), len(gather) + used)))
+            gather += tables[e][:used]
+        else:
+            fresh.append(fresh[-1] + n)
+    absorbed = int(cu[num_short])
+    out = dict(slots=slots, tables=_pad_tables(tables))
+    if absorbed:
+        out["lens"] = np.concatenate([np.arange(p, p + n, dtype=np.int64) + 1 for p, n, _ in items[:num_short]])
+    if scratch:
+        out.update(prefixed_cu_q=np.asarray(pre_q, dtype=np.int32), prefixed_cu_k=np.asarray(pre_k, dtype=np.int32),
+                   gather=np.asarray(gather, dtype=np.int64), scratch_tables=_pad_tables(scratch))
+    if len(fresh) > 1:
+        out["fresh_cu"] = np.asarray(fresh, dtype=np.int32)
+    counts = dict(absorbed=absorbed, num_prefixed=pre_q[-1], num_fresh=fresh[-1],
+                  prefixed_max_k=int(np.diff(pre_k).max()) if scratch else 0)
+    return out, counts
+
+
+def ragged_arrays(seqs, windows, block_size, memory_units=0, latent=False):
     """Host side of a step over ``seqs``: each runs its tokens [num_computed_tokens, + num_scheduled_tokens).  Returns
     (arrays, window arrays, window counts, facts), everything in numpy; the sequences' convolution banks flip for entries
     of more than one token."""
-    kind = [(n > 1) + (n >= LONG_ROWS) for n in (s.num_scheduled_tokens for s in seqs)]
+    kind = [((n > 1) + (n >= LONG_ROWS), s.num_computed_tokens == 0) for n, s in ((s.num_scheduled_tokens, s) for s in seqs)]
     order = sorted(range(len(seqs)), key=lambda i: kind[i])                                  # stable
     items = [(seqs[i].num_computed_tokens, seqs[i].num_scheduled_tokens, seqs[i]) for i in order]
     lens = np.asarray([n for _, n, _ in items], dtype=np.int64)
@@ -174,7 +226,9 @@ def ragged_arrays(seqs, windows, block_size, memory_units=0):
                   row_entry=np.repeat(np.arange(len(items), dtype=np.int32), lens),
                   bank_in=np.asarray(bank_in, dtype=np.int32), bank_out=np.asarray(bank_out, dtype=np.int32),
                   state_slots=np.asarray([s.state_slot for _, _, s in items], dtype=np.int32))
-    per_window = [_window_arrays(items, w, g, block_size, cu) for g, w in enumerate(windows)]
+    num_short = int((lens < LONG_ROWS).sum())
+    per_window = [_latent_arrays(items, g, block_size, cu, num_short) if latent else _window_arrays(items, w, g, block_size, cu)
+                  for g, w in enumerate(windows)]
     starts = [0] * len(seqs)
     for e, i in enumerate(order):
         starts[i] = int(cu[e])
@@ -183,13 +237,14 @@ def ragged_arrays(seqs, windows, block_size, memory_units=0):
     if segments:
         arrays["segments"] = np.asarray(segments, dtype=np.int32)
     facts = dict(num_tokens=int(cu[-1]), num_entries=len(items), num_single=singles, multi_rows=int(cu[-1]) - singles,
-                 num_short=int((lens < LONG_ROWS).sum()), split=any(not s[3] & 4 for s in segments), order=order, starts=starts)
+                 num_short=num_short, split=any(not s[3] & 4 for s in segments), order=order, starts=starts)
     return arrays, [a for a, _ in per_window], [c for _, c in per_window], facts
 
 
-def ragged_step(seqs, windows, block_size, device, memory_units=0) -> RaggedStep:
-    """The step's device tensors: one copy per integer type, every tensor a 16-byte aligned slice of it."""
-    arrays, window_arrays, counts, facts = ragged_arrays(seqs, windows, block_size, memory_units)
+def ragged_step(seqs, windows, block_size, device, memory_units=0, latent=False) -> RaggedStep:
+    """The step's device tensors: one copy per integer type, every tensor a 16-byte aligned slice of it.  ``latent``: the
+    windows' views are LatentSteps."""
+    arrays, window_arrays, counts, facts = ragged_arrays(seqs, windows, block_size, memory_units, latent)
     named = [((None, k), a) for k, a in arrays.items()]
     for g, wa in enumerate(window_arrays):
         named += [((g, k), a) for k, a in wa.items()]
@@ -207,5 +262,6 @@ def ragged_step(seqs, windows, block_size, device, memory_units=0) -> RaggedStep
         dev = host.to(device, non_blocking=True)
         for (key, a), at in zip(mine, offsets):
             placed[key] = dev[at:at + a.size].view(a.shape)
-    ws = [WindowStep(**counts[g], **{k: placed[(g, k)] for k in wa}) for g, wa in enumerate(window_arrays)]
+    view = LatentStep if latent else WindowStep
+    ws = [view(**counts[g], **{k: placed[(g, k)] for k in wa}) for g, wa in enumerate(window_arrays)]
     return RaggedStep(windows=ws, **{k: placed[(None, k)] for k in arrays}, **facts)

@@ -18,7 +18,7 @@ from minivllm_amd import _C
 
 __all__ = ["qk_norm_rope_store", "sample_tokens", "sample_tokens_into", "decode_advance", "add_rms_norm", "silu_and_mul", "linear_small_m", "linear_small_m_takes", "norm_linear_small_m", "norm_linear_small_m_takes",
            "lm_head_sample", "lm_head_sample_takes", "lm_head_sample_workspace_bytes", "norm_conv", "head_rope_store",
-           "head_unrotate_gate", "chunk_decode_step"]
+           "head_unrotate_gate", "chunk_decode_step", "stream_embed_norm", "stream_norm"]
 
 
 def _ptr(t):
@@ -517,3 +517,87 @@ def chunk_decode_step(context_lens: torch.Tensor, block_tables: torch.Tensor, ch
                                            block_tables.shape[1], int(chunk), block_size, batch,
                                            _C.current_stream_ptr(context_lens.device))
     _C.check(st, "chunk_decode_step")
+
+
+def _stream_weights(streams, hc_in, hc_out=None, hc_mix=None):
+    for name, t, shape in (("hc_in", hc_in, (streams,)), ("hc_out", hc_out, (streams,)), ("hc_mix", hc_mix, (streams, streams))):
+        if t is not None:
+            _check(t, torch.float32, shape, name)
+
+
+def stream_embed_norm(step, tokens: torch.Tensor, embed: torch.Tensor, scale: float, streams: int, gain: torch.Tensor, eps: float,
+                      hc_in: torch.Tensor | None = None, bigram: torch.Tensor | None = None, hashing: tuple = (1, 0, 0),
+                      prev_tokens: torch.Tensor | None = None, padded: int = 0):
+    """The front of a model with several residual streams: every stream starts as ``embed[token] * scale`` plus, with
+    ``bigram`` (buckets + 1, W), the row (previous token * mul_prev + token * mul_cur) mod buckets of it, ``hashing`` =
+    (buckets, mul_prev, mul_cur); a sequence's first token has row ``buckets``.  ``prev_tokens`` int64 (banks,) is the part of
+    a sequence's state that holds the token before a step's first.
+
+    Returns (rms(sum_s hc_in[s] x_s) * gain, filled up with zeros to ``padded`` columns, in embed's dtype; x float32
+    (T, streams, W))."""
+    _C.require_cuda(tokens, embed, gain, hc_in, bigram, prev_tokens)
+    rows, width = tokens.numel(), embed.shape[1]
+    padded = max(padded, width)
+    _check(tokens, torch.int64, (rows,), "tokens")
+    _check(embed, embed.dtype, embed.shape, "embed")
+    _check(gain, torch.float32, (width,), "gain")
+    _stream_weights(streams, hc_in)
+    if step.num_tokens != rows:
+        raise ValueError("the step's rows and the tokens differ")
+    if bigram is not None:
+        _check(bigram, embed.dtype, (hashing[0] + 1, width), "bigram")
+        _check(prev_tokens, torch.int64, prev_tokens.shape, "prev_tokens")
+    out = torch.empty((rows, padded), dtype=embed.dtype, device=embed.device)
+    x = torch.empty((rows, streams, width), dtype=torch.float32, device=embed.device)
+    st = _C.load().mvllm_stream_embed_norm(
+        _ptr(out), padded, _ptr(x), _ptr(embed), embed.shape[0], float(scale), _ptr(bigram), *(int(n) for n in hashing),
+        _ptr(prev_tokens), _ptr(tokens), _ptr(step.positions), _ptr(step.cu_seqlens), _ptr(step.row_entry), _ptr(step.bank_in),
+        _ptr(step.bank_out), _ptr(hc_in), _ptr(gain), float(eps), rows, streams, width, _C.dtype_code(embed.dtype),
+        _C.current_stream_ptr(embed.device))
+    _C.check(st, "stream_embed_norm")
+    return out, x
+
+
+def stream_norm(x: torch.Tensor, y, hc_out: torch.Tensor, hc_mix: torch.Tensor, gain: torch.Tensor, eps: float,
+                hc_in: torch.Tensor | None = None, scale: torch.Tensor | None = None, padded: int = 0, want_x: bool = True,
+                dtype: torch.dtype | None = None):
+    """A sublayer's result into the residual streams and the norm in front of the next one, in one launch:
+    ``x_t <- sum_s hc_mix[s, t] x_s + hc_out[t] * scale * y`` for all streams at once, in place (``want_x`` False: not kept),
+    then ``rms(sum_t hc_in[t] x_t) * gain`` (``hc_in`` None: the plain sum) with zeros up to ``padded`` columns.
+
+    x float32 (T, streams, W); y (T, >= W) with dense rows, or a mixture's unsummed results (``layers.experts.ExpertOutput``);
+    everything else float32.  Returns (the norm, x)."""
+    parts = part_row = weights = gate = None
+    if not isinstance(y, torch.Tensor):
+        parts, part_row, weights, gate, y = y.parts, y.part_row, y.weights, y.gate, y.shared
+    _C.require_cuda(x, y, parts, part_row, weights, gate, hc_out, hc_mix, gain, hc_in, scale)
+    rows, streams, width = x.shape
+    padded = max(padded, width)
+    _check(x, torch.float32, (rows, streams, width), "x")
+    _check(gain, torch.float32, (width,), "gain")
+    _stream_weights(streams, hc_in, hc_out, hc_mix)
+    if scale is not None:
+        _check(scale, torch.float32, (width,), "scale")
+    dtype = dtype or (y if y is not None else parts).dtype
+    for name, t in (("y", y), ("parts", parts)):
+        if t is not None and (t.dim() != 2 or t.dtype != dtype or t.shape[1] < width or t.stride(1) != 1):
+            raise ValueError(f"{name} must be (*, >= {width}) in {dtype} with dense rows")
+    if y is not None and y.shape[0] != rows:
+        raise ValueError("y must have one row per row of x")
+    top = 0
+    if parts is not None:
+        top = weights.shape[1]
+        _check(weights, torch.float32, (rows, top), "weights")
+        if parts.shape[0] != rows * top or (part_row is not None and (part_row.dtype != torch.int32 or part_row.numel() != rows * top
+                                                                      or not part_row.is_contiguous())):
+            raise ValueError("parts and part_row must have one row per choice")
+        if gate is not None and (gate.dtype != torch.float32 or gate.numel() != rows):
+            raise ValueError("gate must be float32, one number per row")
+    out = torch.empty((rows, padded), dtype=dtype, device=x.device)
+    st = _C.load().mvllm_stream_norm(
+        _ptr(out), padded, _ptr(x if want_x else None), _ptr(x), _ptr(y), 0 if y is None else max(y.stride(0), width), _ptr(parts),
+        0 if parts is None else max(parts.stride(0), width), _ptr(part_row), _ptr(weights), top, _ptr(gate),
+        1 if gate is None else max(gate.stride(0), 1), _ptr(scale), _ptr(hc_out), _ptr(hc_mix), _ptr(hc_in), _ptr(gain), float(eps),
+        rows, streams, width, _C.dtype_code(dtype), _C.current_stream_ptr(x.device))
+    _C.check(st, "stream_norm")
+    return out, x

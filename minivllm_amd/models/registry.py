@@ -38,7 +38,24 @@ def _sokevik_sources(config):
     return kernel_sources(config)
 
 
-DESIGNS = {"Qwen3": Design(_qwen3_runner), "Sokevik": Design(_sokevik_runner, _sokevik_normalize, _sokevik_sources)}
+def _niridra_runner(config):
+    from minivllm_amd.engine.hybrid_runner import HybridModelRunner
+    from minivllm_amd.models.niridra import NiridraForCausalLM
+    return HybridModelRunner(config, NiridraForCausalLM)
+
+
+def _niridra_normalize(config):
+    from minivllm_amd.models.niridra import engine_config
+    return engine_config(config)
+
+
+def _niridra_sources(config):
+    from minivllm_amd.models.niridra import kernel_sources
+    return kernel_sources(config)
+
+
+DESIGNS = {"Qwen3": Design(_qwen3_runner), "Sokevik": Design(_sokevik_runner, _sokevik_normalize, _sokevik_sources),
+           "Niridra": Design(_niridra_runner, _niridra_normalize, _niridra_sources)}
 
 
 def design_of(config: dict) -> Design:

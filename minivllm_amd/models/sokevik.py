@@ -138,6 +138,8 @@ class SokevikLayer(nn.Module):
 
 
 class SokevikForCausalLM(nn.Module):
+    latent_views = False                                # its attention layers cache keys and values
+
     def __init__(self, config: dict, block_size: int, dtype: torch.dtype, device: torch.device):
         super().__init__()
         self.config, self.dtype, self.device, self.block_size = config, dtype, device, block_size

@@ -35,6 +35,10 @@ def test_header_declares_expected_entry_points():
               "mvllm_prefill_paged_split_sink", "mvllm_norm_conv", "mvllm_head_rope_store", "mvllm_head_unrotate_gate",
               "mvllm_chunk_decode_step", "mvllm_gate_linear", "mvllm_mlstm_recurrent", "mvllm_mlstm_output",
               "mvllm_mlstm_chunked", "mvllm_mlstm_chunked_workspace_bytes",
+              "mvllm_stream_embed_norm", "mvllm_stream_norm", "mvllm_decay_memory_recurrent", "mvllm_decay_memory_chunked",
+              "mvllm_decay_memory_chunked_workspace_bytes", "mvllm_gated_row_norm", "mvllm_latent_norm_store",
+              "mvllm_head_linear", "mvllm_latent_decode", "mvllm_latent_decode_workspace_bytes", "mvllm_moe_route",
+              "mvllm_moe_plan", "mvllm_moe_plan_bytes", "mvllm_moe_linear",
               "mvllm_silu_and_mul", "mvllm_version", "mvllm_status_string"]:
         assert n in names
 
