@@ -38,7 +38,7 @@ def parse_args():
     ap.add_argument("--warmup", type=int, default=5)
     ap.add_argument("--seed", type=int, default=0)
     ap.add_argument("--block-size", type=int, default=16, help="block size of the headline decode workload")
-    ap.add_argument("--only", default="", help="comma list out of decode256,prefill,prefill_long,store,int8,reference_shapes,decode_small,demo_shape,head_dims,fused_qk,sampler,mfma_probe,prefill_timeline,loads_probe,engine,engine16,engine64,cpu to restrict the extras (the headline decode always runs); only when named: sokevik, the Sokevik design beside the Qwen3-style decoder, models and kernels (sokevik_kernels: kernels alone)")
+    ap.add_argument("--only", default="", help="comma list out of decode256,prefill,prefill_long,store,int8,reference_shapes,decode_small,demo_shape,head_dims,fused_qk,sampler,mfma_probe,prefill_timeline,loads_probe,engine,engine16,engine64,cpu to restrict the extras (the headline decode always runs); only when named: sokevik, the Sokevik design beside the Qwen3-style decoder, models and kernels (sokevik_kernels: kernels alone), niridra, the Niridra design beside Sokevik (niridra_kernels)")
     ap.add_argument("--no-cpu", action="store_true", help="skip the cpu_baseline leg")
     ap.add_argument("--calib-copy", action="store_true",
                     help="also launch three 1 GiB device copies (reads 1 GiB, writes 1 GiB each) so a rocprofv3 "
@@ -986,6 +986,20 @@ def bench_sokevik(args, with_models=True):
     return out
 
 
+def kernel_legs(args, res, calls):
+    """``leg(name, kernel, bytes, like, its name, its bytes, flops, its flops)`` puts a kernel's time and share of its roofline
+    (the larger of its bytes over the HBM peak and its flops over the matrix peak) beside the like kernel's into ``res``."""
+    def one(fn, b, f):
+        ms = graph_call_ms(args, fn, calls)
+        floor = max(b / (HBM_PEAK_GBS * 1e9), f / (MFMA_BF16_PEAK_TFLOPS * 1e12)) * 1e3
+        return {"us": ms * 1e3, "roofline_us": floor * 1e3, "frac": floor / ms}
+
+    def leg(name, kernel, nbytes, like, like_kernel, like_bytes, flops=0.0, like_flops=0.0):
+        mine, other = one(kernel, nbytes, flops), one(like, like_bytes, like_flops)
+        res[name] = {**mine, "like": {"name": like_kernel, **other}, "times_further": other["frac"] / mine["frac"]}
+    return leg
+
+
 def bench_sokevik_kernels(args, rows, calls):
     """Kernels at width 4096: 8192 prompt rows (8 prompts of 1024, one attention chunk each), or 64 decoded rows with 1024
     tokens in the chunk (the matrix memory and attention over 256 sequences there: their states must not fit a cache)."""
@@ -1022,13 +1036,7 @@ def bench_sokevik_kernels(args, rows, calls):
     entries = len(lengths)
     res = {}
 
-    def leg(name, kernel, nbytes, like, like_kernel, like_bytes, flops=0.0, like_flops=0.0):
-        def one(fn, b, f):
-            ms = graph_call_ms(args, fn, calls)
-            floor = max(b / (HBM_PEAK_GBS * 1e9), f / (MFMA_BF16_PEAK_TFLOPS * 1e12)) * 1e3
-            return {"us": ms * 1e3, "roofline_us": floor * 1e3, "frac": floor / ms}
-        mine, other = one(kernel, nbytes, flops), one(like, like_bytes, like_flops)
-        res[name] = {**mine, "like": {"name": like_kernel, **other}, "times_further": other["frac"] / mine["frac"]}
+    leg = kernel_legs(args, res, calls)
 
     # norm, residual, norm and short convolution | residual norm
     x, y, z = rnd(rows, width, dtype=torch.float32), rnd(rows, width), rnd(rows, width)
@@ -1100,6 +1108,200 @@ def bench_sokevik_kernels(args, rows, calls):
         gate_bytes = 64 * width * 2 + 2 * heads * width * 2
         like, like_name, gb = (lambda: linear_small_m(hh, gw)), "linear_small_m", gate_bytes + 64 * heads * 4
     leg("gate_linear", lambda: gate_linear(hh, gw, bias, heads, 15.0), gate_bytes + hh.shape[0] * heads * 8, like, like_name, gb)
+    return res
+
+
+# the same widths, heads and layers; as many feed-forward channels per token as the dense models have
+NIRIDRA_SIZES = {"w2048": dict(experts=64, top=6, ff=768, shared=1536), "w4096": dict(experts=64, top=8, ff=1280, shared=2048)}
+NIRIDRA_RANK, NIRIDRA_STREAMS = 512, 2
+
+
+def niridra_model(size):
+    """Niridra with lightning and latent-attention layers in turn (every second latent layer reads the one before it), of the
+    width, heads, memories and active feed-forward of ``sokevik_models``."""
+    z, e = SOKEVIK_SIZES[size], NIRIDRA_SIZES[size]
+    mlp = {"kind": "moe", "expert": {"ff": e["ff"]}, "shared": {"ff": e["shared"]},
+           "router": {"experts": e["experts"], "top": e["top"], "groups": {"count": 8, "keep": 4}}}
+    heads = z["width"] // SOKEVIK_VDIM
+    lightning = {"type": "lightning", "mlp": mlp, "mixer": {"heads": heads, "dim": SOKEVIK_DIM, "vdim": SOKEVIK_VDIM,
+                                                            "decay": [1.0 - 2.0 ** -(1 + 9 * h / heads) for h in range(heads)]}}
+
+    def latent(i):
+        m = {"heads": z["heads"], "dim": 128, "vdim": 128, "kv_rank": NIRIDRA_RANK, "scale": 128 ** -0.5}
+        return {"type": "latent_attention", "mlp": mlp, "mixer": m if i % 4 == 1 else {**m, "kv_from": i - 2}}
+    return {"architecture": "Niridra", "width": z["width"], "vocab": 32000, "streams": NIRIDRA_STREAMS, "norm": {"eps": 1e-6},
+            "embedding": {"scale": z["width"] ** 0.5, "bigram": {"buckets": 32003, "mul_prev": 1000003, "mul_cur": 7919}},
+            "layers": [lightning if i % 2 == 0 else latent(i) for i in range(z["layers"])]}
+
+
+def bench_niridra(args, with_models=True):
+    """The Niridra design beside Sokevik, the nearest other design (a matrix memory and attention in turn), at equal width,
+    heads, layers and active feed-forward: whole-engine throughput, and every kernel beside the like kernel."""
+    import torch
+    out = {"models": {}, "kernels": {}}
+    for size in NIRIDRA_SIZES if with_models else ():
+        for prompts, prompt_len, new in ((4, 2048, 128), (32, 512, 128), (1, 16384, 64)):
+            leg = {}
+            for name, config in (("niridra", niridra_model(size)), ("sokevik", sokevik_models(size)[0])):
+                leg[name] = engine_throughput(args, config, prompts, prompt_len, new)
+                torch.cuda.empty_cache()
+            out["models"][f"{size}_{prompts}x{prompt_len}+{new}"] = leg
+            print(f"{size} {prompts}x{prompt_len}+{new}: {leg}", file=sys.stderr, flush=True)
+    for rows, calls in ((8192, 4), (64, 20)):
+        with torch.inference_mode():
+            out["kernels"][f"{rows}_rows"] = bench_niridra_kernels(args, rows, calls)
+        torch.cuda.empty_cache()
+    return out
+
+
+def bench_niridra_kernels(args, rows, calls):
+    """Kernels at width 4096: 8192 prompt rows (8 prompts of 1024), or 64 decoded rows (memory and attention: 256 sequences of
+    1024 tokens)."""
+    import torch
+    import torch.nn.functional as F
+    from minivllm_amd.engine.hybrid_cache import HybridCacheManager
+    from minivllm_amd.engine.ragged import ragged_step
+    from minivllm_amd.engine.sequence import Sequence
+    from minivllm_amd.layers.attention import flash_attention_prefill, paged_attention_decode
+    from minivllm_amd.layers.experts import ExpertOutput, moe_linear, moe_plan, moe_route
+    from minivllm_amd.layers.fused import head_rope_store, linear_small_m, norm_conv, stream_embed_norm, stream_norm
+    from minivllm_amd.layers.latent import head_linear, latent_decode, latent_norm_store
+    from minivllm_amd.layers.recurrent import (DecayMemoryState, MlstmState, decay_memory, gate_linear, gated_row_norm, mlstm)
+
+    dev = torch.device("cuda:0")
+    gen = torch.Generator(device=dev).manual_seed(args.seed)
+    rnd = lambda *shape, dtype=torch.bfloat16: torch.randn(*shape, generator=gen, device=dev).to(dtype)
+    f32 = lambda *shape: torch.ones(*shape, device=dev)
+    prefill = rows > 64
+    width, heads_a, d, seq, bs, rank, s = 4096, 32, 128, 1024, 16, NIRIDRA_RANK, NIRIDRA_STREAMS
+    heads, dim, vdim = width // SOKEVIK_VDIM, SOKEVIK_DIM, SOKEVIK_VDIM
+    e = NIRIDRA_SIZES["w4096"]
+    experts, top, ff = e["experts"], e["top"], e["ff"]
+
+    def step_of(lengths, before, latent=True):
+        m = HybridCacheManager([0], sum(-(-(n + p) // bs) for n, p in zip(lengths, before)), bs, len(lengths))
+        seqs = []
+        for n, p0 in zip(lengths, before):
+            q = Sequence([0] * (p0 + n), block_size=bs)
+            m.allocate(q)
+            q.num_computed_tokens, q.num_scheduled_tokens = p0, n
+            seqs.append(q)
+        return ragged_step(seqs, [0], bs, dev, heads * -(-vdim // 128), latent)
+
+    lengths = [seq] * (rows // seq) if prefill else [1] * rows
+    step = step_of(lengths, [0] * len(lengths) if prefill else [seq - 1] * rows)
+    entries = len(lengths)
+    res = {}
+    leg = kernel_legs(args, res, calls)
+
+    # residual streams, norm (with the mixture's sum | embedding) | norm, residual, norm and short convolution
+    x, y = rnd(rows, s, width, dtype=torch.float32), rnd(rows, width)
+    out_w, mix, in_w, gain = f32(s), torch.eye(s, device=dev), f32(s) / s, f32(width)
+    x1 = rnd(rows, width, dtype=torch.float32)
+    one_gain, taps, state = torch.ones((), device=dev), rnd(4, width, dtype=torch.float32), torch.zeros(2 * entries + 1, 3, width, device=dev)
+    like = lambda: norm_conv(step, one_gain, 1e-6, torch.bfloat16, x=x1, y=y, post=one_gain, conv=taps, state=state)
+    like_bytes = rows * width * 12 + (1 if prefill else 2) * entries * 3 * width * 4 + 4 * width * 4
+    moved = rows * width * (8 * s + 4) + 2 * width * 4
+    leg("stream_norm", lambda: stream_norm(x, y, out_w, mix, gain, 1e-6, in_w, gain), moved, like, "norm_conv", like_bytes)
+    parts = ExpertOutput(rnd(rows * top, width), f32(rows, top) / top, None, y, rnd(rows, 1, dtype=torch.float32)[:, 0])
+    leg("stream_norm_experts", lambda: stream_norm(x, parts, out_w, mix, gain, 1e-6, in_w, gain), moved + rows * top * (2 * width + 4),
+        like, "norm_conv", like_bytes)
+    embed, bigram = rnd(32000, width), rnd(32004, width)
+    ids = torch.randint(0, 32000, (rows,), generator=gen, device=dev)
+    prev = torch.zeros(2 * entries + 1, dtype=torch.int64, device=dev)
+    leg("stream_embed_norm", lambda: stream_embed_norm(step, ids, embed, 64.0, s, gain, 1e-6, in_w, bigram, (32003, 1000003, 7919), prev),
+        rows * width * (4 + 4 * s + 2), lambda: norm_conv(step, one_gain, 1e-6, torch.bfloat16, tokens=ids, embed=embed, conv=taps, state=state),
+        "norm_conv (embedding)", rows * width * 8 + (1 if prefill else 2) * entries * 3 * width * 4)
+    del x, y, x1, parts, embed, bigram
+    # experts | dense products of as many channels per token
+    h, pairs = rnd(rows, width), rows * top
+    router = rnd(experts + 1, width)
+    logits = gate_linear(h, router, None, experts + 1, 0.0)
+    small = rnd(32, width)
+    leg("router", lambda: gate_linear(h, router, None, experts + 1, 0.0), rows * width * 2 + (experts + 1) * (width * 2 + rows * 4),
+        lambda: gate_linear(h, small, None, 16, 15.0), "gate_linear (32 columns)", rows * width * 2 + 32 * (width * 2 + rows * 4))
+    chosen, weights = moe_route(logits, None, experts, top, 8, 4)
+    for name, fn in (("moe_route", lambda: moe_route(logits, None, experts, top, 8, 4)), ("moe_plan", lambda: moe_plan(chosen, experts))):
+        if prefill or name == "moe_route":
+            res[name] = {"us": graph_call_ms(args, fn, calls) * 1e3}
+    w_up, w_down = rnd(experts, 2 * ff, width), rnd(experts, width, ff)
+    used = int(torch.unique(chosen).numel())
+    dense = top * ff
+    d_up, d_down = rnd(2 * dense, width), rnd(width, dense)
+    plan = moe_plan(chosen, experts) if prefill else None
+    act = moe_linear(h, w_up, chosen, plan, top, glu=True)
+    hid = rnd(rows, dense)
+    product, product_name = (F.linear, "library product") if prefill else (linear_small_m, "linear_small_m")
+    up_flops, down_flops = 4.0 * pairs * ff * width, 2.0 * pairs * ff * width
+    leg("moe_linear_up", lambda: moe_linear(h, w_up, chosen, plan, top, glu=True),
+        used * 2 * ff * width * 2 + rows * width * 2 + pairs * ff * 2, lambda: product(h, d_up), product_name,
+        2 * dense * width * 2 + rows * (width + 2 * dense) * 2, up_flops, up_flops)
+    leg("moe_linear_down", lambda: moe_linear(act, w_down, chosen, plan), used * ff * width * 2 + pairs * (ff + width) * 2,
+        lambda: product(hid, d_down), product_name, dense * width * 2 + rows * (width + dense) * 2, down_flops, down_flops)
+    del w_up, w_down, d_up, d_down, act, hid
+    # latents into the cache | keys and values
+    c, gain_c = rnd(rows, rank), f32(rank)
+    cache = torch.zeros(entries * seq // bs, bs, rank, dtype=torch.bfloat16, device=dev)
+    cols = (heads_a + 16) * d
+    proj, k_gain = rnd(rows, cols), f32(d)
+    kc = torch.zeros(entries * seq // bs, bs, 8, d, dtype=torch.bfloat16, device=dev)
+    vc, slots = torch.zeros_like(kc), step.windows[0].slots
+    packed = 16 if prefill else 0
+    leg("latent_norm_store", lambda: latent_norm_store(c, gain_c, 1e-6, cache, slots, need_rows=prefill),
+        rows * (rank * 2 * (3 if prefill else 2) + 8),
+        lambda: head_rope_store(proj, step.positions, heads_a, 8, d, d, d, k_gain, k_gain, 1e-6, 1.0, None, None, True, None, slots, kc, vc,
+                                need_kv=prefill),
+        "head_rope_store", rows * (2 * cols + (heads_a + packed + 16) * d * 2 + 16))
+    del proj, kc, vc, cache
+    # attention: heads' keys and values made of the latents | grouped heads; decoded rows over the latents | over keys and values
+    scale = d ** -0.5
+    if prefill:
+        q, k, v = (rnd(rows, heads_a, d) for _ in range(3))
+        kg, vg = rnd(rows, 8, d), rnd(rows, 8, d)
+        cu = step.windows[0].fresh_cu
+        flops = 4.0 * heads_a * d * entries * seq * (seq + 1) / 2
+        leg("latent_prefill", lambda: flash_attention_prefill(q, k, v, cu, scale, heads_a, heads_a, d), rows * 4 * heads_a * d * 2,
+            lambda: flash_attention_prefill(q, kg, vg, cu, scale, heads_a, 8, d), "packed prefill, 8 kv heads",
+            rows * (2 * heads_a + 16) * d * 2, flops, flops)
+        del q, k, v, kg, vg
+    else:
+        q, up = rnd(rows, heads_a, d), rnd(heads_a, rank, d)
+        down, ql = rnd(heads_a, d, rank), rnd(rows, heads_a, rank)
+        xs, flat = rnd(rows, rank), rnd(heads_a * d, rank)
+        moved = heads_a * d * rank * 2 + rows * heads_a * (d + rank) * 2
+        for name, fn in (("head_linear_k", lambda: head_linear(q, up)), ("head_linear_v", lambda: head_linear(ql, down))):
+            leg(name, fn, moved, lambda: linear_small_m(xs, flat), "linear_small_m", heads_a * d * rank * 2 + rows * (rank + heads_a * d) * 2)
+        batch = 256
+        for keys, key in ((seq, "latent_decode"), (8 * seq, "latent_decode_8k")):
+            n = batch if keys == seq else 32
+            step = step_of([1] * n, [keys - 1] * n)
+            w = step.windows[0]
+            cache, ql = rnd(n * keys // bs, bs, rank), rnd(n, heads_a, rank)
+            kc, vc, q = rnd(n * keys // bs, bs, 8, d), rnd(n * keys // bs, bs, 8, d), rnd(n, heads_a, d)
+            leg(key, lambda: latent_decode(ql, cache, w.tables, step.row_entry, w.lens, scale),
+                n * (keys * rank * 2 + 2 * heads_a * rank * 2 + 4 * keys // bs),
+                lambda: paged_attention_decode(q, kc, vc, w.tables, w.lens, scale, heads_a, 8, d, bs), "paged decode, 8 kv heads",
+                n * (keys * 16 * d * 2 + 2 * heads_a * d * 2 + 4 * keys // bs), 4.0 * n * heads_a * keys * rank, 0.0)
+            del cache, kc, vc
+        step = step_of([1] * batch, [seq - 1] * batch)
+        entries = rows = batch
+    # the matrix memory with norm and gate
+    n = heads * (2 * dim + vdim)
+    proj = rnd(rows, n + heads * vdim)
+    gates = torch.cat([rnd(rows, heads, dtype=torch.float32), F.logsigmoid(rnd(rows, heads, dtype=torch.float32) + 4)], 1).contiguous()
+    weight = f32(heads * vdim)
+    decay = DecayMemoryState.allocate(entries, [0.5 + 0.49 * i / heads for i in range(heads)], dim, vdim, dev)
+    memory = MlstmState.allocate(entries, heads, dim, vdim, dev)
+    states = (1 if prefill else 2) * entries * heads * dim * vdim * 4
+    nbytes = rows * (2 * (n + heads * vdim) + 2 * heads * vdim) + states
+    flops = rows * heads * (4.0 * dim * vdim + 64.0 * (dim + vdim)) if prefill else 0.0
+    mine = lambda st: gated_row_norm(decay_memory(st, proj, decay), weight, proj[:, n:n + heads * vdim], 1e-6)
+    other = lambda st: mlstm(st, proj, gates, n, weight, memory, 1e-6)
+    leg("decay_memory", lambda: mine(step), nbytes, lambda: other(step), "mlstm", nbytes + rows * 8 * heads, flops, flops)
+    if prefill:
+        whole = step_of([rows], [0])
+        nbytes -= (entries - 1) * heads * dim * vdim * 4
+        leg("decay_memory_one_prompt", lambda: mine(whole), nbytes, lambda: other(whole), "mlstm", nbytes + rows * 8 * heads, flops, flops)
     return res
 
 
@@ -1210,6 +1412,10 @@ def main():
         extra["sokevik"] = bench_sokevik(args)
     elif "sokevik_kernels" in only:                    # without the models, as a kernel trace wants
         extra["sokevik"] = bench_sokevik(args, with_models=False)
+    if "niridra" in only:
+        extra["niridra"] = bench_niridra(args)
+    elif "niridra_kernels" in only:
+        extra["niridra"] = bench_niridra(args, with_models=False)
 
     if "loads_only" in head:
         extra["decode_loads_only"] = head["loads_only"]

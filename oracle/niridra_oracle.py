@@ -132,3 +132,47 @@ def forward(tokens, weights, config, dtype=torch.float64, layer_outputs=None):
         if layer_outputs is not None:
             layer_outputs.append(xs.sum(0))
     return (rms(xs.sum(0), eps) * w["final.norm"]) @ w["embed"].T
+
+
+def random_weights(config, seed=0, dtype=torch.bfloat16):
+    """Checkpoint tensors of a configuration, drawn so that every gain, stream weight and correction takes part."""
+    g = torch.Generator().manual_seed(seed)
+    width, streams = config["width"], config["streams"]
+
+    def normal(*shape, std=1.0, mean=0.0):
+        return (torch.randn(shape, generator=g) * std + mean).to(dtype)
+
+    def linear(rows, columns):
+        return normal(rows, columns, std=columns ** -0.5)
+
+    w = {"embed": linear(config["vocab"], width), "final.norm": normal(width, std=0.2, mean=1.0)}
+    if config["embedding"].get("bigram"):
+        w["bigram"] = normal(config["embedding"]["bigram"]["buckets"] + 1, width, std=0.7)
+    for i, entry in enumerate(config["layers"]):
+        p, c, e = f"l{i}.", entry["mixer"], entry.get("mlp")
+        for s in ("1", "2") if e is not None else ("1",):
+            w[f"{p}norm{s}"] = normal(width, std=0.2, mean=1.0)
+            w[f"{p}ls{s}"] = normal(width, std=0.2, mean=0.7)
+            w[f"{p}hc{s}.in"] = normal(streams, std=0.3, mean=1.0 / streams)
+            w[f"{p}hc{s}.out"] = normal(streams, std=0.3, mean=1.0)
+            w[f"{p}hc{s}.mix"] = (torch.eye(streams) + torch.randn(streams, streams, generator=g) * 0.2).to(dtype)
+        m, heads = p + "mix.", c["heads"]
+        w[m + "q"] = linear(heads * c["dim"], width)
+        w[m + "o"] = linear(width, heads * c["vdim"])
+        if entry["type"] == "lightning":
+            w[m + "k"], w[m + "v"], w[m + "g"] = linear(heads * c["dim"], width), linear(heads * c["vdim"], width), linear(heads * c["vdim"], width)
+            w[m + "norm"] = normal(heads * c["vdim"], std=0.2, mean=1.0)
+        else:
+            w[m + "uk"], w[m + "uv"] = linear(heads * c["dim"], c["kv_rank"]), linear(heads * c["vdim"], c["kv_rank"])
+            if c.get("kv_from") is None:
+                w[m + "dkv"], w[m + "dkv.norm"] = linear(c["kv_rank"], width), normal(c["kv_rank"], std=0.2, mean=1.0)
+        if e is not None:
+            forms = [(f"{p}mlp.e{j}.", e["expert"]["ff"]) for j in range(e["router"]["experts"])]
+            if e.get("shared"):
+                forms.append((p + "mlp.shared.", e["shared"]["ff"]))
+                w[p + "mlp.shared.sg"] = linear(1, width)
+            for name, ff in forms:
+                w[name + "gate"], w[name + "up"], w[name + "down"] = linear(ff, width), linear(ff, width), linear(width, ff)
+            w[p + "mlp.router"] = normal(e["router"]["experts"], width, std=2 * width ** -0.5)
+            w[p + "mlp.correction"] = normal(e["router"]["experts"], std=0.5, mean=-0.3)     # choice scores of both signs
+    return w
