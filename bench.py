@@ -1215,20 +1215,19 @@ def bench_niridra_kernels(args, rows, calls):
     del x, y, x1, parts, embed, bigram
     # experts | dense products of as many channels per token
     h, pairs = rnd(rows, width), rows * top
-    router = rnd(experts + 1, width)
+    router = rnd(experts + 1, width) * width ** -0.5
     logits = gate_linear(h, router, None, experts + 1, 0.0)
     small = rnd(32, width)
     leg("router", lambda: gate_linear(h, router, None, experts + 1, 0.0), rows * width * 2 + (experts + 1) * (width * 2 + rows * 4),
         lambda: gate_linear(h, small, None, 16, 15.0), "gate_linear (32 columns)", rows * width * 2 + 32 * (width * 2 + rows * 4))
     chosen, weights = moe_route(logits, None, experts, top, 8, 4)
     for name, fn in (("moe_route", lambda: moe_route(logits, None, experts, top, 8, 4)), ("moe_plan", lambda: moe_plan(chosen, experts))):
-        if prefill or name == "moe_route":
-            res[name] = {"us": graph_call_ms(args, fn, calls) * 1e3}
+        res[name] = {"us": graph_call_ms(args, fn, calls) * 1e3}
     w_up, w_down = rnd(experts, 2 * ff, width), rnd(experts, width, ff)
     used = int(torch.unique(chosen).numel())
     dense = top * ff
     d_up, d_down = rnd(2 * dense, width), rnd(width, dense)
-    plan = moe_plan(chosen, experts) if prefill else None
+    plan = moe_plan(chosen, experts)
     act = moe_linear(h, w_up, chosen, plan, top, glu=True)
     hid = rnd(rows, dense)
     product, product_name = (F.linear, "library product") if prefill else (linear_small_m, "linear_small_m")

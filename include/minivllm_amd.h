@@ -647,8 +647,8 @@ int mvllm_latent_decode(void* out, const void* q, const void* cache, const int32
  * mvllm_moe_plan: (token, choice) pairs sorted by expert, into `plan` (mvllm_moe_plan_bytes; its first `pairs` int32 are the
  *   sorted place of every pair).
  * mvllm_moe_linear: w [experts, N, K]; glu: gate and up rows in turns of 32, result silu(gate) * up.  With a plan: row p of
- *   out is sorted place p, reading x row pair / per_token (per_token > 0) or row p.  Without (bf16, at most 4096 pairs, for
- *   the few rows of a decode step): row p of out is pair p, reading x row p / per_token or row p.  K % 64 == 0,
+ *   out is sorted place p, reading x row pair / per_token (per_token > 0) or row p.  Without (bf16, at most 512 pairs, meant
+ *   for a few): row p of out is pair p, reading x row p / per_token or row p.  K % 64 == 0,
  *   N % 16 == 0 (glu: 64), bf16 and fp32.
  */
 int mvllm_moe_route(int32_t* ids, float* weights, const float* logits, int64_t logit_row_stride, const float* correction,

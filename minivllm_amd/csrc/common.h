@@ -106,6 +106,19 @@ __device__ __forceinline__ float four_rows_sum(float x) {
   return (row(0) + row(16)) + (row(32) + row(48));
 }
 
+// The maximum over the wave, in every lane, the same way.
+__device__ __forceinline__ float wave_max_in_registers(float x) {
+  auto moved = [](float v, auto CTRL) __attribute__((always_inline)) {
+    return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), decltype(CTRL)::value, 0xf, 0xf, false));
+  };
+  x = fmaxf(x, moved(x, std::integral_constant<int, 0xB1>{}));
+  x = fmaxf(x, moved(x, std::integral_constant<int, 0x4E>{}));
+  x = fmaxf(x, moved(x, std::integral_constant<int, 0x141>{}));
+  x = fmaxf(x, moved(x, std::integral_constant<int, 0x140>{}));
+  auto row = [x](int lane) __attribute__((always_inline)) { return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(x), lane)); };
+  return fmaxf(fmaxf(row(0), row(16)), fmaxf(row(32), row(48)));
+}
+
 // 16-byte global load with the non-temporal hint: for data that is read once and should stream through the
 // caches instead of displacing what is reused (K/V cache blocks in decode).  Measured on MI355X a pure read
 // stream reaches about 7.1 TB/s with the hint against 6.0-6.5 TB/s without.

@@ -1,7 +1,7 @@
 // Gate projections of a recurrent layer: out[T, N] = act(x[T, K] W[N, K]^T + bias), N small, fp32 accumulation and fp32
 // output (a recurrence's gates enter exponentials, where a 16-bit result would be a few per cent off).  Columns below
 // `split` get a soft cap, cap * tanh(z / cap), the others logsigmoid of the same.
-//   bf16: one workgroup = 16 rows x 16 or 32 columns; its waves take 64-wide steps of K in turn on
+//   bf16: one workgroup = 16 rows x 16 to 80 columns; its waves take 64-wide steps of K in turn on
 //         v_mfma_f32_16x16x32_bf16 and meet in LDS.
 //   fp32: the same tile with one fp32 dot product per thread over K chunks staged in LDS.
 #include "common.h"
@@ -77,13 +77,14 @@ __global__ __launch_bounds__(64 * kWaves) void gate_linear_bf16_kernel(const Gat
 #pragma unroll
   for (int n = 0; n < NT; ++n) part[wave][n][lane] = make_float4(acc[n][0], acc[n][1], acc[n][2], acc[n][3]);
   __syncthreads();
-  static_assert(256 * NT <= 64 * kWaves, "one output per thread");
-  const int t = threadIdx.x, n = t >> 8, c = (t >> 4) & 15, out_row = blockIdx.x * 16 + (t & 15), out_col = (blockIdx.y * NT + n) * 16 + c;
-  if (n >= NT || out_row >= a.rows || out_col >= a.N) return;
-  float z = 0.f;
+  for (int t = threadIdx.x; t < 256 * NT; t += 64 * kWaves) {
+    const int n = t >> 8, c = (t >> 4) & 15, out_row = blockIdx.x * 16 + (t & 15), out_col = (blockIdx.y * NT + n) * 16 + c;
+    if (out_row >= a.rows || out_col >= a.N) continue;
+    float z = 0.f;
 #pragma unroll
-  for (int i = 0; i < kWaves; ++i) z += reinterpret_cast<const float*>(&part[i][n][16 * (c >> 2) + (t & 15)])[c & 3];
-  a.out[(int64_t)out_row * a.N + out_col] = gate_activation(a, z, out_col);
+    for (int i = 0; i < kWaves; ++i) z += reinterpret_cast<const float*>(&part[i][n][16 * (c >> 2) + (t & 15)])[c & 3];
+    a.out[(int64_t)out_row * a.N + out_col] = gate_activation(a, z, out_col);
+  }
 }
 
 __global__ __launch_bounds__(256) void gate_linear_f32_kernel(const GateArgs a) {
@@ -124,13 +125,17 @@ extern "C" int mvllm_gate_linear(float* out, const void* x, int64_t x_row_stride
   a.out = out; a.x = x; a.w = w; a.bias = bias; a.x_stride = x_row_stride; a.rows = (int)rows; a.N = N; a.K = K;
   a.split = split; a.cap = cap;
   const unsigned tiles = (unsigned)((rows + 15) / 16);
-  const dim3 grid(tiles, (unsigned)((N + 15) / 16)), grid2(tiles, (unsigned)((N + 31) / 32));
+  const dim3 grid(tiles, (unsigned)((N + 15) / 16));
+  auto in_tiles = [&](int n) { return dim3(tiles, (unsigned)((N + 16 * n - 1) / (16 * n))); };
   hipStream_t s = (hipStream_t)stream;
   const bool vec = K % 8 == 0 && x_row_stride % 8 == 0 && aligned16(x) && aligned16(w), full = vec && K % 64 == 0;
   if (dtype == MVLLM_F32) gate_linear_f32_kernel<<<grid, dim3(256), 0, s>>>(a);
   else if (!full) gate_linear_bf16_kernel<4, 1, false><<<grid, dim3(256), 0, s>>>(a, vec);
   else if (rows <= kFewRows) gate_linear_bf16_kernel<16, 1, true><<<grid, dim3(1024), 0, s>>>(a, vec);
   else if (N <= 16) gate_linear_bf16_kernel<8, 1, true><<<grid, dim3(512), 0, s>>>(a, vec);
-  else gate_linear_bf16_kernel<8, 2, true><<<grid2, dim3(512), 0, s>>>(a, vec);
+  else if (N <= 32) gate_linear_bf16_kernel<8, 2, true><<<in_tiles(2), dim3(512), 0, s>>>(a, vec);
+  else if (N <= 48) gate_linear_bf16_kernel<8, 3, true><<<in_tiles(3), dim3(512), 0, s>>>(a, vec);
+  else if (N <= 64) gate_linear_bf16_kernel<8, 4, true><<<in_tiles(4), dim3(512), 0, s>>>(a, vec);
+  else gate_linear_bf16_kernel<8, 5, true><<<in_tiles(5), dim3(512), 0, s>>>(a, vec);
   return launch_status();
 }

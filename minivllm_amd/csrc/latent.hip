@@ -24,6 +24,7 @@ struct LatentNormArgs {
   int64_t in_stride, num_slots;
   float eps;
   int rows, rank, padded;
+  bool vec;                 // the weight starts on 16 bytes
 };
 
 // One row per wave, 16 bytes per lane and access.
@@ -33,7 +34,19 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(const LatentNormArgs a
   const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (row >= a.rows) return;
   const T* in = reinterpret_cast<const T*>(a.in) + (int64_t)row * a.in_stride;
-  float x[NC][N], ss = 0.f;
+  const int64_t slot = a.slots ? a.slots[row] : -1;
+  float x[NC][N], w[NC][N], ss = 0.f;
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    const int at = (c * 64 + lane) * N;
+    if (at + N <= a.rank && a.vec) {
+#pragma unroll
+      for (int i = 0; i < N; i += 4) *reinterpret_cast<float4*>(&w[c][i]) = *reinterpret_cast<const float4*>(a.weight + at + i);
+    } else {
+#pragma unroll
+      for (int i = 0; i < N; ++i) w[c][i] = a.weight[min(at + i, a.rank - 1)];
+    }
+  }
 #pragma unroll
   for (int c = 0; c < NC; ++c) {
     const int at = (c * 64 + lane) * N;
@@ -47,7 +60,6 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(const LatentNormArgs a
   }
   ss = four_rows_sum(row16_sum(ss));
   const float inv = 1.0f / sqrtf(ss / (float)a.rank + a.eps);
-  const int64_t slot = a.slots ? a.slots[row] : -1;
   T* out = a.out ? reinterpret_cast<T*>(a.out) + (int64_t)row * a.padded : nullptr;
   T* cached = a.cache && slot >= 0 && slot < a.num_slots ? reinterpret_cast<T*>(a.cache) + slot * a.padded : nullptr;
 #pragma unroll
@@ -56,10 +68,10 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(const LatentNormArgs a
     if (at >= a.padded) continue;
     T v[N];
 #pragma unroll
-    for (int i = 0; i < N; ++i) v[i] = from_float<T>(at + i < a.rank ? x[c][i] * inv * a.weight[at + i] : 0.f);
-    const uint4 w = *reinterpret_cast<const uint4*>(v);
-    if (out) *reinterpret_cast<uint4*>(out + at) = w;
-    if (cached) *reinterpret_cast<uint4*>(cached + at) = w;
+    for (int i = 0; i < N; ++i) v[i] = from_float<T>(at + i < a.rank ? x[c][i] * inv * w[c][i] : 0.f);
+    const uint4 r = *reinterpret_cast<const uint4*>(v);
+    if (out) *reinterpret_cast<uint4*>(out + at) = r;
+    if (cached) *reinterpret_cast<uint4*>(cached + at) = r;
   }
 }
 
@@ -72,29 +84,70 @@ struct HeadLinearArgs {
   int rows, heads, N, K;
 };
 
-// Workgroup = 16 rows, one head, 64 outputs: a wave has 16 of them.  K a multiple of 8, N of 16.
+// Workgroup = 16 RT rows, one head.  kSplitK: 16 outputs, the waves share K and meet in LDS; otherwise 64 outputs, 16 per
+// wave.  K a multiple of 8, N of 16.  Rows and K past the end read the last ones; what they would add is multiplied by zeros
+// or not stored.
+template <int RT, bool kSplitK>
 __global__ __launch_bounds__(256) void head_linear_bf16_kernel(const HeadLinearArgs a) {
+  __shared__ float4 part[kSplitK ? 4 : 1][kSplitK ? RT : 1][kSplitK ? 64 : 1];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, g = lane >> 4, i16 = lane & 15;
-  const int h = blockIdx.y, n0 = (blockIdx.x * 4 + wave) * 16;
-  if (n0 >= a.N) return;
-  const int row = blockIdx.z * 16 + i16;
-  const bool live = row < a.rows;
-  const bf16_t* x = reinterpret_cast<const bf16_t*>(a.x) + (int64_t)(live ? row : 0) * a.x_row + (int64_t)h * a.x_head;
+  const int h = blockIdx.y, n0 = kSplitK ? blockIdx.x * 16 : (blockIdx.x * 4 + wave) * 16;
+  if (!kSplitK && n0 >= a.N) return;
+  const int row0 = blockIdx.z * 16 * RT + i16;
+  const bf16_t* x[RT];
+#pragma unroll
+  for (int t = 0; t < RT; ++t)
+    x[t] = reinterpret_cast<const bf16_t*>(a.x) + (int64_t)min(row0 + 16 * t, a.rows - 1) * a.x_row + (int64_t)h * a.x_head;
   const bf16_t* w = reinterpret_cast<const bf16_t*>(a.w) + ((int64_t)h * a.N + n0 + i16) * a.K;
-  v4f acc = {0.f, 0.f, 0.f, 0.f};
+  v4f acc[RT];
+#pragma unroll
+  for (int t = 0; t < RT; ++t) acc[t] = v4f{0.f, 0.f, 0.f, 0.f};
   const uint4 zero = make_uint4(0u, 0u, 0u, 0u);
 #pragma unroll 4
-  for (int k0 = 0; k0 < a.K; k0 += 32) {
-    const int k = k0 + 8 * g;
-    const bool has = k < a.K;
-    const uint4 wv = has ? *reinterpret_cast<const uint4*>(w + k) : zero;
-    const uint4 xv = has && live ? *reinterpret_cast<const uint4*>(x + k) : zero;
-    acc = mfma16x16x32<bf16_t>(wv, xv, acc);
+  for (int k0 = kSplitK ? 32 * wave : 0; k0 < a.K; k0 += kSplitK ? 128 : 32) {
+    const int k = min(k0 + 8 * g, a.K - 8);
+    uint4 wv = *reinterpret_cast<const uint4*>(w + k), xv[RT];
+#pragma unroll
+    for (int t = 0; t < RT; ++t) xv[t] = *reinterpret_cast<const uint4*>(x[t] + k);
+    if (k0 + 8 * g >= a.K) {
+      wv = zero;
+#pragma unroll
+      for (int t = 0; t < RT; ++t) xv[t] = zero;
+    }
+#pragma unroll
+    for (int t = 0; t < RT; ++t) acc[t] = mfma16x16x32<bf16_t>(wv, xv[t], acc[t]);
   }
-  // lane: row i16, outputs n0 + 4 g + r
-  if (!live) return;
-  bf16_t* out = reinterpret_cast<bf16_t*>(a.out) + (int64_t)row * a.out_row + (int64_t)h * a.out_head + n0 + 4 * g;
-  *reinterpret_cast<uint2*>(out) = make_uint2(pack2<bf16_t>(acc[0], acc[1]), pack2<bf16_t>(acc[2], acc[3]));
+  // lane: row i16 of a tile, outputs n0 + 4 g + r
+  auto store = [&](int t, float4 o) __attribute__((always_inline)) {
+    const int row = row0 + 16 * t;
+    if (row >= a.rows) return;
+    bf16_t* out = reinterpret_cast<bf16_t*>(a.out) + (int64_t)row * a.out_row + (int64_t)h * a.out_head + n0 + 4 * g;
+    *reinterpret_cast<uint2*>(out) = make_uint2(pack2<bf16_t>(o.x, o.y), pack2<bf16_t>(o.z, o.w));
+  };
+  if constexpr (!kSplitK) {
+#pragma unroll
+    for (int t = 0; t < RT; ++t) store(t, make_float4(acc[t][0], acc[t][1], acc[t][2], acc[t][3]));
+  } else {
+#pragma unroll
+    for (int t = 0; t < RT; ++t) part[wave][t][lane] = make_float4(acc[t][0], acc[t][1], acc[t][2], acc[t][3]);
+    __syncthreads();
+    for (int t = wave; t < RT; t += 4) {
+      float4 o = part[0][t][lane];
+#pragma unroll
+      for (int i = 1; i < 4; ++i) {
+        const float4 p = part[i][t][lane];
+        o.x += p.x; o.y += p.y; o.z += p.z; o.w += p.w;
+      }
+      store(t, o);
+    }
+  }
+}
+
+template <int RT>
+static void launch_head_linear(const HeadLinearArgs& a, hipStream_t s) {
+  const unsigned tiles = (unsigned)((a.rows + 16 * RT - 1) / (16 * RT)), heads = (unsigned)a.heads;
+  if (a.K >= 256) head_linear_bf16_kernel<RT, true><<<dim3((unsigned)(a.N / 16), heads, tiles), dim3(256), 0, s>>>(a);
+  else head_linear_bf16_kernel<RT, false><<<dim3((unsigned)((a.N + 63) / 64), heads, tiles), dim3(256), 0, s>>>(a);
 }
 
 __global__ __launch_bounds__(256) void head_linear_f32_kernel(const HeadLinearArgs a) {
@@ -170,13 +223,15 @@ __device__ __forceinline__ void store4(const LatentDecodeArgs& a, int row, int p
 // bf16: workgroup = (share, block of 16 HT heads, row), four waves; RS = padded rank / 32.  Tiles of 64 latents go to LDS
 // once, in chunks of 16 bytes whose place in a row is xor-ed with the key's low bits; wave w takes 16-head tile w % HT and
 // the key subtiles of its share w / HT.  S^T = C Q'^T (keys down the accumulator, heads across the lanes), so that the
-// weights are the operand of O^T += C^T P^T as they lie; C^T comes from the same LDS tile through the transposing loads.
+// weights are the operand of O^T += C^T P^T as they lie; C^T comes from the same LDS tile through the transposing loads.  Two
+// tiles in LDS: the next one is on its way while this one is worked on.
 template <int RS, int HT>
-__global__ __launch_bounds__(256, RS > 4 ? 2 : 3) void latent_decode_kernel(const LatentDecodeArgs a) {
+__global__ __launch_bounds__(256, RS > 8 ? 1 : RS > 4 ? 2 : 3) void latent_decode_kernel(const LatentDecodeArgs a) {
   constexpr int kShares = 4 / HT, kSub = 4 / kShares;      // key shares of a tile, 16-key subtiles of a wave
   constexpr int RC = 4 * RS, kRow = 16 * RC;               // chunks and bytes of a row
   constexpr int kXor = (RC & -RC) < 16 ? (RC & -RC) : 16;  // chunks that trade places
-  __shared__ __attribute__((aligned(16))) char lds[64 * kRow];
+  constexpr int kTile = 64 * kRow;
+  __shared__ __attribute__((aligned(16))) char lds[2 * kTile];
   __shared__ int64_t slot_of[2][64];
   __shared__ float2 ml[4][16];
   const int part = blockIdx.x, row = blockIdx.z;
@@ -212,23 +267,31 @@ __global__ __launch_bounds__(256, RS > 4 ? 2 : 3) void latent_decode_kernel(cons
     for (int j = 0; j < kCols; ++j) col_at[j] = row_b + (((2 * j + ((i16 & 3) >> 1)) ^ xb) << 4);
   }
 
-  if (tid < 64 && k0 < k1) slot_of[0][tid] = key_slot(a, table, min(k0 + tid, k1 - 1));
-  __syncthreads();
-  int flip = 0;
-  for (int base = k0; base < k1; base += 64, flip ^= 1) {
-    // ---- the tile: RS chunks per thread, straight into LDS ----
+  // a tile: RS chunks per thread, straight into LDS
+  auto copy = [&](int buffer) __attribute__((always_inline)) {
     const char* cache = reinterpret_cast<const char*>(a.cache);
 #pragma unroll
     for (int i = 0; i < RS; ++i) {
       const uint32_t c = 256u * i + (uint32_t)tid;
       const uint32_t key = c / RC, p = c % RC;
-      const char* from = cache + slot_of[flip][key] * kRow + ((p ^ (key & (kXor - 1))) << 4);
-      dma16_to_lds_from(from, lds_address(lds) + (256 * i + 64 * wave) * 16);
+      const char* from = cache + slot_of[buffer][key] * kRow + ((p ^ (key & (kXor - 1))) << 4);
+      dma16_to_lds_from(from, lds_address(lds) + buffer * kTile + (256 * i + 64 * wave) * 16);
       if (i % 4 == 3) __builtin_amdgcn_sched_barrier(0);
     }
-    if (tid < 64 && base + 64 < k1) slot_of[flip ^ 1][tid] = key_slot(a, table, min(base + 64 + tid, k1 - 1));
-    dma_wait_all();
-    __syncthreads();
+  };
+  if (tid < 128 && k0 < k1) slot_of[tid >> 6][tid & 63] = key_slot(a, table, min(k0 + tid, k1 - 1));
+  __syncthreads();
+  if (k0 < k1) copy(0);
+  dma_wait_all();
+  __syncthreads();
+  int flip = 0;
+  for (int base = k0; base < k1; base += 64, flip ^= 1) {
+    const bool more = base + 64 < k1;
+    int64_t slot_after = 0;                         // of the tile behind the next one
+    if (tid < 64 && base + 128 < k1) slot_after = key_slot(a, table, min(base + 128 + tid, k1 - 1));
+    if (more) copy(flip ^ 1);
+    __builtin_amdgcn_sched_barrier(0);
+    const int at_tile = flip * kTile;
 
     // ---- scores of the wave's subtiles ----
     v4f s[kSub];
@@ -238,7 +301,7 @@ __global__ __launch_bounds__(256, RS > 4 ? 2 : 3) void latent_decode_kernel(cons
     for (int ks = 0; ks < RS; ++ks) {
 #pragma unroll
       for (int t = 0; t < kSub; ++t)
-        s[t] = mfma16x16x32<bf16_t>(*reinterpret_cast<const uint4*>(key_at[ks % kBy] + 16 * t * kRow + 64 * (ks / kBy * kBy)), qf[ks], s[t]);
+        s[t] = mfma16x16x32<bf16_t>(*reinterpret_cast<const uint4*>(key_at[ks % kBy] + at_tile + 16 * t * kRow + 64 * (ks / kBy * kBy)), qf[ks], s[t]);
       if (ks % 4 == 3) __builtin_amdgcn_sched_barrier(0);      // operands of later steps stay in LDS until then
     }
     float most = -INFINITY;
@@ -276,7 +339,7 @@ __global__ __launch_bounds__(256, RS > 4 ? 2 : 3) void latent_decode_kernel(cons
 #pragma unroll
     for (int n = 0; n < 2 * RS; ++n) {
       auto column = [&](int t) __attribute__((always_inline)) {
-        const char* p = col_at[n % kCols] + 16 * t * kRow + 32 * (n / kCols * kCols);
+        const char* p = col_at[n % kCols] + at_tile + 16 * t * kRow + 32 * (n / kCols * kCols);
         return __builtin_bit_cast(uint2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) v4s*)p));
       };
       if constexpr (kSub == 1) {
@@ -290,7 +353,10 @@ __global__ __launch_bounds__(256, RS > 4 ? 2 : 3) void latent_decode_kernel(cons
       }
       if (n % 4 == 3) __builtin_amdgcn_sched_barrier(0);
     }
-    __syncthreads();                                // everybody is done with the tile; the next slots are there
+    __builtin_amdgcn_sched_barrier(0);
+    if (tid < 64 && base + 128 < k1) slot_of[flip][tid] = slot_after;
+    dma_wait_all();
+    __syncthreads();                                // everybody is done with the tile; the next one and its successor's slots are there
   }
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
@@ -460,15 +526,22 @@ static int launch_any(const LatentDecodeArgs& a, int rows, hipStream_t s) {
 
 constexpr int kMaxParts = 32;
 
-// Shares per row: enough workgroups for two per CU and a few rounds of them, at least two tiles of keys each.
-static int plan_parts(int rows, int heads, int64_t max_keys, int dtype) {
-  const int tiles = (heads + 15) / 16;
-  const int64_t groups = (int64_t)rows * (dtype == MVLLM_BF16 ? (tiles <= 2 ? 1 : (tiles + 3) / 4) : heads);
-  int64_t parts = (1024 + groups - 1) / groups;
-  const int64_t most = (max_keys + 127) / 128;
-  parts = parts > most ? most : parts;
-  parts = parts > kMaxParts ? kMaxParts : parts;
-  return (int)(parts < 1 ? 1 : parts);
+// Shares per row: as many as give the shortest schedule, in tiles of 64 keys (two more for a share's start and end, two for the
+// pass that joins shares), of whole rounds of the workgroups that run side by side.
+static int plan_parts(int rows, int heads, int padded, int64_t max_keys, int dtype) {
+  const int head_tiles = (heads + 15) / 16;
+  const int64_t groups = (int64_t)rows * (dtype == MVLLM_BF16 ? (head_tiles <= 2 ? 1 : (head_tiles + 3) / 4) : heads);
+  const int64_t together = 256 * (dtype != MVLLM_BF16 || padded <= 128 ? 3 : padded <= 256 ? 2 : 1), tiles = (max_keys + 63) / 64;
+  int best = 1;
+  int64_t best_time = INT64_MAX;
+  for (int parts = 1; parts <= kMaxParts && (parts == 1 || 2 * parts <= tiles); ++parts) {
+    const int64_t time = (groups * parts + together - 1) / together * ((tiles + parts - 1) / parts + 2) + (parts > 1 ? 2 : 0);
+    if (time < best_time) {
+      best = parts;
+      best_time = time;
+    }
+  }
+  return best;
 }
 
 }  // namespace mvllm
@@ -487,7 +560,7 @@ extern "C" int mvllm_latent_norm_store(void* out, const void* in, int64_t in_row
   if (!aligned16(in) || !aligned16(out) || !aligned16(cache)) return MVLLM_ERR_MISALIGNED;
   LatentNormArgs a;
   a.out = out; a.in = in; a.weight = weight; a.cache = cache; a.slots = slots; a.in_stride = in_row_stride;
-  a.num_slots = num_slots; a.eps = eps; a.rows = (int)rows; a.rank = rank; a.padded = padded;
+  a.num_slots = num_slots; a.eps = eps; a.rows = (int)rows; a.rank = rank; a.padded = padded; a.vec = aligned16(weight);
   const dim3 grid((unsigned)((rows + 3) / 4)), block(256);
   hipStream_t s = (hipStream_t)stream;
   if (dtype == MVLLM_F32) {
@@ -516,15 +589,16 @@ extern "C" int mvllm_head_linear(void* out, int64_t out_row_stride, int64_t out_
   a.out = out; a.x = x; a.w = w; a.out_row = out_row_stride; a.out_head = out_head_stride; a.x_row = x_row_stride;
   a.x_head = x_head_stride; a.rows = (int)rows; a.heads = num_heads; a.N = N; a.K = K;
   hipStream_t s = (hipStream_t)stream;
-  const unsigned row_tiles = (unsigned)((rows + 15) / 16);
-  if (dtype == MVLLM_F32) head_linear_f32_kernel<<<dim3((unsigned)((N + 15) / 16), (unsigned)num_heads, row_tiles), dim3(256), 0, s>>>(a);
-  else head_linear_bf16_kernel<<<dim3((unsigned)((N + 63) / 64), (unsigned)num_heads, row_tiles), dim3(256), 0, s>>>(a);
+  if (dtype == MVLLM_F32) head_linear_f32_kernel<<<dim3((unsigned)((N + 15) / 16), (unsigned)num_heads, (unsigned)((rows + 15) / 16)), dim3(256), 0, s>>>(a);
+  else if (rows <= 16) launch_head_linear<1>(a, s);
+  else if (rows <= 32) launch_head_linear<2>(a, s);
+  else launch_head_linear<4>(a, s);
   return launch_status();
 }
 
 extern "C" size_t mvllm_latent_decode_workspace_bytes(int rows, int num_heads, int padded, int64_t max_keys, int dtype) {
   if (rows <= 0 || num_heads <= 0 || padded <= 0 || max_keys <= 0) return 0;
-  const int parts = plan_parts(rows, num_heads, max_keys, dtype);
+  const int parts = plan_parts(rows, num_heads, padded, max_keys, dtype);
   return parts == 1 ? 0 : (size_t)rows * parts * num_heads * ((size_t)padded + 2) * sizeof(float);
 }
 
@@ -544,7 +618,7 @@ extern "C" int mvllm_latent_decode(void* out, const void* q, const void* cache, 
   a.out = out; a.q = q; a.cache = cache; a.tables = block_tables; a.row_entry = row_entry; a.lens = lens;
   a.num_blocks = num_blocks; a.table_width = table_width; a.block_size = block_size; a.heads = num_heads; a.padded = padded;
   a.scale_log2 = scale * kLog2e;
-  a.parts = plan_parts(rows, num_heads, (int64_t)table_width * block_size, dtype);
+  a.parts = plan_parts(rows, num_heads, padded, (int64_t)table_width * block_size, dtype);
   a.part_o = nullptr;
   a.part_ml = nullptr;
   if (a.parts > 1) {

@@ -2,11 +2,11 @@
 //   moe_route   scores s = sigmoid(z), choice scores s + correction; groups of neighbouring experts by the sum of their two
 //               largest choice scores, the best `keep` groups stay open; the `top` largest choice scores of those are chosen,
 //               weights s / (sum of the chosen s + 1e-20)
-//   moe_plan    (token, choice) pairs sorted by expert, and tiles of 128 sorted rows per expert
+//   moe_plan    (token, choice) pairs sorted by expert, and tiles of 128 or 256 sorted rows per expert
 //   moe_linear  out[row] = x[row] W_e^T, optionally silu(gate) * up behind it: W_e [2 F, K] with gate and up rows in turns of
 //               32, so that both halves of an output are in one lane
-// Products, by the number of rows: few (a decode step: no plan; a workgroup gathers its expert's rows itself, its waves share
-// K, weights stream once), many (bf16: 128 x 128 tiles on the matrix unit over sorted rows), any (fp32, over sorted rows).
+// Products, by the number of rows: very few (no plan; a workgroup finds its expert's rows itself, its waves share K), many (bf16: 128 x 128 or 256 x 256
+// tiles on the matrix unit over sorted rows), any (fp32, over sorted rows).
 #include "prefill_tiles.h"
 
 #pragma clang fp contract(off)
@@ -73,21 +73,23 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const RouteArgs a) {
   float my_s = 0.f, sum = 0.f;
   int my_id = 0;
   for (int k = 0; k < a.top; ++k) {
-    float best = -INFINITY, best_s = 0.f;
-    int id = 1 << 30;
+    float mine = choice[0];
 #pragma unroll
-    for (int i = 0; i < NE; ++i)
-      if (choice[i] > best) { best = choice[i]; best_s = s[i]; id = lane + 64 * i; }
+    for (int i = 1; i < NE; ++i) mine = fmaxf(mine, choice[i]);
+    const float best = wave_max_in_registers(mine);
+    int id = -1;                                    // the first expert that has it
+    float best_s = 0.f;
 #pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const float x = __shfl_xor(best, o, 64), xs = __shfl_xor(best_s, o, 64);
-      const int xi = __shfl_xor(id, o, 64);
-      if (x > best || (x == best && xi < id)) { best = x; best_s = xs; id = xi; }
+    for (int i = 0; i < NE; ++i) {
+      const unsigned long long at = __ballot(choice[i] == best);
+      if (id < 0 && at != 0ull) {
+        const int l = __builtin_amdgcn_readfirstlane(__builtin_ctzll(at));
+        id = 64 * i + l;
+        best_s = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(s[i]), l));
+        if (lane == l) choice[i] = -INFINITY;
+      }
     }
-    if (id >= E) id = 0;                            // (nothing left to choose)
-#pragma unroll
-    for (int i = 0; i < NE; ++i)
-      if (lane + 64 * i == id) choice[i] = -INFINITY;
+    if (id < 0 || id >= E) id = 0;                  // (nothing left to choose)
     sum += best_s;
     if (lane == k) { my_s = best_s; my_id = id; }
   }
@@ -98,7 +100,8 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const RouteArgs a) {
 }
 
 // ---- pairs sorted by expert ----
-constexpr int kTileRows = 128, kPlanPairs = 2048, kMaxExperts = 1024;
+constexpr int kPlanPairs = 2048, kMaxExperts = 1024;
+constexpr int kLargeTileRows = 384;      // rows per expert from which tiles are large
 
 struct PlanArgs {
   const int32_t* ids;      // [pairs]
@@ -109,7 +112,7 @@ struct PlanArgs {
   int32_t* tile_expert;    // [max tiles]
   int32_t* tile_row;       // [max tiles]: first sorted row
   int32_t* num_tiles;      // [1]
-  int pairs, experts, blocks;
+  int pairs, experts, blocks, tile_rows;
 };
 
 __global__ __launch_bounds__(256) void moe_count_kernel(const PlanArgs a) {
@@ -126,14 +129,21 @@ __global__ __launch_bounds__(1024) void moe_place_kernel(const PlanArgs a) {
   __shared__ int32_t total[kMaxExperts + 1], tiles[kMaxExperts + 1], cursor[kMaxExperts];
   const int e = threadIdx.x;
   int n = 0, mine = 0;
-  if (e < a.experts)
+  if (a.blocks == 1) {                              // counted here
+    cursor[e] = 0;
+    __syncthreads();
+    for (int p = e; p < a.pairs; p += 1024) atomicAdd(&cursor[a.ids[p]], 1);
+    __syncthreads();
+    n = cursor[e];
+    __syncthreads();
+  } else if (e < a.experts)
     for (int b = 0; b < a.blocks; ++b) {
       if (b == (int)blockIdx.x) mine = n;
       n += a.hist[(int64_t)b * a.experts + e];
     }
   // inclusive sums over the experts
   total[e + 1] = n;
-  tiles[e + 1] = (n + kTileRows - 1) / kTileRows;
+  tiles[e + 1] = (n + a.tile_rows - 1) / a.tile_rows;
   if (e == 0) total[0] = tiles[0] = 0;
   __syncthreads();
   for (int o = 1; o < 1024; o <<= 1) {
@@ -159,7 +169,7 @@ __global__ __launch_bounds__(1024) void moe_place_kernel(const PlanArgs a) {
     }
     for (int t = tiles[e]; t < tiles[e + 1]; ++t) {
       a.tile_expert[t] = e;
-      a.tile_row[t] = total[e] + (t - tiles[e]) * kTileRows;
+      a.tile_row[t] = total[e] + (t - tiles[e]) * a.tile_rows;
     }
   }
 }
@@ -184,37 +194,58 @@ struct ExpertLinearArgs {
 
 __device__ __forceinline__ float silu_of(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
 
-// few: workgroup = (16 outputs, expert).  The rows of the expert are found in `ids`; rows are taken 16 at a time.
-constexpr int kFewPairs = 4096;
+// few: workgroup = (16 kTiles outputs, expert), its waves share K.  The rows of the expert are found in `ids`; rows are taken
+// 16 at a time.
+constexpr int kFewPairs = 512;
 
-template <int kWaves, bool kGlu>
+template <int kWaves, bool kGlu, int kTiles>
 __global__ __launch_bounds__(64 * kWaves) void moe_linear_few_kernel(const ExpertLinearArgs a) {
-  constexpr int NT = kGlu ? 2 : 1;
+  constexpr int NT = kTiles * (kGlu ? 2 : 1);        // tiles of weight rows: with the gate, gate and up of an output tile in turn
   __shared__ uint16_t list[kFewPairs];
-  __shared__ int found;
+  __shared__ int found, count[kWaves];
   __shared__ float4 part[kWaves][NT][64];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, i16 = lane & 15;
   const int e = blockIdx.y;
-  if (wave == 0) {
-    int n = 0;
-    for (int base = 0; base < a.pairs; base += 64) {
-      const int p = base + lane;
-      const bool hit = p < a.pairs && a.ids[p] == e;
-      const unsigned long long hits = __ballot(hit);
-      if (hit) list[n + __popcll(hits & ((1ull << lane) - 1))] = (uint16_t)p;
-      n += __popcll(hits);
+  // the expert's pairs, in order: every wave looks through its share of the list, all loads at once
+  constexpr int kEach = (kFewPairs + 64 * kWaves - 1) / (64 * kWaves);
+  {
+    const int share = (a.pairs + 64 * kWaves - 1) / (64 * kWaves) * 64, base = wave * share;
+    int32_t id[kEach];
+#pragma unroll
+    for (int i = 0; i < kEach; ++i) {
+      const int p = base + 64 * i + lane;
+      id[i] = 64 * i < share && p < a.pairs ? a.ids[p] : -1;
     }
-    if (lane == 0) found = n;
+    int n = 0;
+#pragma unroll
+    for (int i = 0; i < kEach; ++i) n += __popcll(__ballot(id[i] == e));
+    if (lane == 0) count[wave] = n;
+    __syncthreads();
+    int at = 0, all = 0;
+#pragma unroll
+    for (int i = 0; i < kWaves; ++i) {
+      at += i < wave ? count[i] : 0;
+      all += count[i];
+    }
+    if (tid == 0) found = all;
+    if (all == 0) return;                           // (the same for every thread)
+#pragma unroll
+    for (int i = 0; i < kEach; ++i) {
+      const bool hit = id[i] == e;
+      const unsigned long long hits = __ballot(hit);
+      if (hit) list[at + __popcll(hits & ((1ull << lane) - 1))] = (uint16_t)(base + 64 * i + lane);
+      at += __popcll(hits);
+    }
   }
   __syncthreads();
   const int rows = found;
-  if (rows == 0) return;
-  const int n0 = blockIdx.x * 16;                   // first output of the workgroup
+  const int n0 = blockIdx.x * 16 * kTiles;          // first output of the workgroup
   const bf16_t* w[NT];
 #pragma unroll
   for (int n = 0; n < NT; ++n) {
-    const int wr = kGlu ? (n0 >> 5) * 64 + (n0 & 31) + 32 * n : n0;
-    w[n] = reinterpret_cast<const bf16_t*>(a.w) + ((int64_t)e * a.N + wr + i16) * a.K;
+    const int out = kGlu ? n0 + 16 * (n / 2) : n0 + 16 * n;
+    const int wr = kGlu ? (out >> 5) * 64 + (out & 31) + 32 * (n % 2) : out;
+    w[n] = reinterpret_cast<const bf16_t*>(a.w) + ((int64_t)e * a.N + min(wr + i16, a.N - 1)) * a.K;
   }
   for (int r0 = 0; r0 < rows; r0 += 16) {
     const int pair = list[min(r0 + i16, rows - 1)];
@@ -222,7 +253,7 @@ __global__ __launch_bounds__(64 * kWaves) void moe_linear_few_kernel(const Exper
     v4f acc[NT];
 #pragma unroll
     for (int n = 0; n < NT; ++n) acc[n] = v4f{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
+#pragma unroll 2
     for (int k0 = 64 * wave; k0 < a.K; k0 += 64 * kWaves) {            // a lane's 32 bytes: whole lines per row and wave
       const int k = k0 + 16 * g;
       uint4 xv[2], wv[NT][2];
@@ -241,22 +272,24 @@ __global__ __launch_bounds__(64 * kWaves) void moe_linear_few_kernel(const Exper
 #pragma unroll
     for (int n = 0; n < NT; ++n) part[wave][n][lane] = make_float4(acc[n][0], acc[n][1], acc[n][2], acc[n][3]);
     __syncthreads();
-    if (wave == 0 && r0 + i16 < rows) {
-      float z[NT][4];
+    for (int m = wave; m < kTiles; m += kWaves) {   // output tile
+      constexpr int kParts = kGlu ? 2 : 1;
+      float z[kParts][4];
 #pragma unroll
-      for (int n = 0; n < NT; ++n) {
+      for (int n = 0; n < kParts; ++n) {
         z[n][0] = z[n][1] = z[n][2] = z[n][3] = 0.f;
 #pragma unroll
         for (int i = 0; i < kWaves; ++i) {
-          const float4 p = part[i][n][lane];
+          const float4 p = part[i][m * kParts + n][lane];
           z[n][0] += p.x; z[n][1] += p.y; z[n][2] += p.z; z[n][3] += p.w;
         }
       }
       float o[4];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) o[r] = kGlu ? silu_of(z[0][r]) * z[NT - 1][r] : z[0][r];
-      bf16_t* out = reinterpret_cast<bf16_t*>(a.out) + (int64_t)pair * a.out_stride + n0 + 4 * g;
-      *reinterpret_cast<uint2*>(out) = make_uint2(pack2<bf16_t>(o[0], o[1]), pack2<bf16_t>(o[2], o[3]));
+      for (int r = 0; r < 4; ++r) o[r] = kGlu ? silu_of(z[0][r]) * z[kParts - 1][r] : z[0][r];
+      const int col = n0 + 16 * m + 4 * g;
+      bf16_t* out = reinterpret_cast<bf16_t*>(a.out) + (int64_t)pair * a.out_stride + col;
+      if (r0 + i16 < rows && col < (kGlu ? a.N / 2 : a.N)) *reinterpret_cast<uint2*>(out) = make_uint2(pack2<bf16_t>(o[0], o[1]), pack2<bf16_t>(o[2], o[3]));
     }
     __syncthreads();
   }
@@ -403,7 +436,153 @@ __global__ __launch_bounds__(256, 2) void moe_linear_many_kernel(const ExpertLin
   }
 }
 
-static int64_t max_tiles(int64_t pairs, int experts) { return (pairs + kTileRows - 1) / kTileRows + experts; }
+// many, large tiles: 256 sorted rows x 256 weight rows, four waves of 128 x 128 (a wave's accumulators fill half its SIMD's
+// registers; per flop it reads half as much of LDS as with 64 x 64).  The operands of a 16-wide step are read during the
+// products of the one before; a step's last products hide the barrier, after which the next step's operands are there and
+// more copies start: x, which other workgroups of the XCD read too, one step ahead in two buffers, the weights, which come
+// from memory, two steps ahead in three.  Together they fill the LDS.
+template <bool kGlu>
+__global__ __launch_bounds__(256, 1) void moe_linear_large_kernel(const ExpertLinearArgs a) {
+  constexpr int kTile = 256, kK = 64, kStage = kTile * kK * 2;       // bytes of one operand's step
+  constexpr int kTogether = 4;
+  __shared__ __attribute__((aligned(16))) char lds[5 * kStage];      // weights three times, x twice
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), l32 = lane & 31, hi = lane >> 5;
+  const int total = a.num_tiles[0], per = (total + 7) / 8;
+  const int xcd = blockIdx.x & 7, j = blockIdx.x >> 3;
+  const int group = j / (kTogether * a.n_tiles), in_group = j % (kTogether * a.n_tiles);
+  const int local = group * kTogether + in_group % kTogether, tile = xcd * per + local, n_tile = in_group / kTogether;
+  if (local >= per || tile >= total) return;
+  const int e = a.tile_expert[tile], row0 = a.tile_row[tile], row_end = min(row0 + kTile, a.row_start[e + 1]);
+  const int n0 = n_tile * kTile;
+
+  const v4i w_rows = make_rsrc(reinterpret_cast<const char*>(a.w) + (int64_t)e * a.N * a.K * 2, (uint32_t)((int64_t)a.N * a.K * 2));
+  const v4i x_rows = make_rsrc(reinterpret_cast<const char*>(a.x), a.x_bytes);
+  uint32_t from_w[8], from_x[8];
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const int c = 256 * i + tid, r = c >> 3, p = (c & 7) ^ ((r >> 1) & 7);
+    from_w[i] = (uint32_t)(min(n0 + r, a.N - 1) * a.K + 8 * p) * 2u;
+    const int at = min(row0 + r, row_end - 1);
+    const uint32_t xr = (uint32_t)(a.per_token ? a.sorted_pair[at] / a.per_token : at);
+    from_x[i] = (xr * (uint32_t)a.x_stride + 8u * p) * 2u;
+  }
+  constexpr int kX = 3 * kStage;                    // where x begins
+  const uint32_t lds_wave = lds_address(lds) + 1024 * wave;
+  const int steps = a.K / kK;
+  // copy i of eight of a step's operand; past the last step nothing is read (the buffer is not used again)
+  auto copy_w = [&](auto I, int step, uint32_t buffer) __attribute__((always_inline)) {
+    v4i rows = w_rows;
+    rows[2] = step < steps ? rows[2] : 0;
+    dma16_to_lds_at<4096 * decltype(I)::value>(rows, from_w[decltype(I)::value], (uint32_t)step * (2 * kK), lds_wave + buffer);
+  };
+  auto copy_x = [&](auto I, int step) __attribute__((always_inline)) {
+    v4i rows = x_rows;
+    rows[2] = step < steps ? rows[2] : 0;
+    dma16_to_lds_at<4096 * decltype(I)::value>(rows, from_x[decltype(I)::value], (uint32_t)step * (2 * kK), lds_wave + kX + (step & 1) * kStage);
+  };
+  const int wn = wave & 1, wm = wave >> 1;
+  const int sw = (l32 >> 1) & 7;
+  const char* frag = lds + l32 * 128;
+  v16f acc[4][4];
+#pragma unroll
+  for (int n = 0; n < 4; ++n)
+#pragma unroll
+    for (int m = 0; m < 4; ++m)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) acc[n][m][r] = 0.f;
+  uint4 wf[2][4], xf[2][4];
+  // where this lane's operands of the four 16-wide steps lie in a buffer
+  uint32_t place[4];
+#pragma unroll
+  for (int st = 0; st < 4; ++st) place[st] = ((2 * st + hi) ^ sw) << 4;
+  const char* w_frag = frag + wn * (128 * 128);
+  const char* x_frag = frag + wm * (128 * 128) + kX;
+  // The products of a 16-wide step one by one; after each of them one of the next step's reads (every kEvery-th from product
+  // kFirst on, those that are needed first come first) and whatever `also` does: the matrix unit must not wait for a queue of
+  // reads or copies.
+  auto products = [&](auto SET, auto FIRST, auto EVERY, const char* wb, const char* xb, auto&& also) __attribute__((always_inline)) {
+    constexpr int set = decltype(SET)::value, next = set ^ 1, kFirst = decltype(FIRST)::value, kEvery = decltype(EVERY)::value;
+    static_for<16>([&](auto I) {
+      constexpr int i = decltype(I)::value;
+      acc[i / 4][i % 4] = mfma32x32x16<bf16_t>(wf[set][i / 4], xf[set][i % 4], acc[i / 4][i % 4]);
+      also(I);
+      if constexpr (i >= kFirst && (i - kFirst) % kEvery == 0 && (i - kFirst) / kEvery < 8) {
+        constexpr int j = (i - kFirst) / kEvery;
+        if constexpr (j >= 1 && j <= 4) xf[next][j - 1] = *reinterpret_cast<const uint4*>(xb + (j - 1) * 32 * 128);
+        else wf[next][j == 0 ? 0 : j - 4] = *reinterpret_cast<const uint4*>(wb + (j == 0 ? 0 : j - 4) * 32 * 128);
+      }
+      __builtin_amdgcn_sched_barrier(0);
+    });
+  };
+  constexpr std::integral_constant<int, 0> c0{};
+  constexpr std::integral_constant<int, 1> c1{};
+  constexpr std::integral_constant<int, 2> c2{};
+  constexpr std::integral_constant<int, 4> c4{};
+  auto nothing = [](auto) {};
+
+  static_for<8>([&](auto I) {
+    copy_w(I, 0, 0);
+    copy_x(I, 0);
+    copy_w(I, 1, kStage);
+  });
+  dma_wait_all();
+  __syncthreads();
+  static_for<8>([&](auto I) { copy_x(I, 1); });
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    wf[0][i] = *reinterpret_cast<const uint4*>(w_frag + place[0] + i * 32 * 128);
+    xf[0][i] = *reinterpret_cast<const uint4*>(x_frag + place[0] + i * 32 * 128);
+  }
+  uint32_t w_at = 0;                                // the weights' buffer of this step, in bytes
+  for (int step = 0; step < steps; ++step) {
+    const uint32_t w_next = w_at == 2 * kStage ? 0 : w_at + kStage, w_free = w_at == 0 ? 2 * kStage : w_at - kStage;
+    const char* wb = w_frag + w_at;
+    const char* xb = x_frag + (step & 1) * kStage;
+    // the weights two steps ahead, into the buffer that the step before this one has left
+    products(c0, c1, c2, wb + place[1], xb + place[1], [&](auto I) {
+      constexpr int i = decltype(I)::value;
+      if constexpr (i % 2 == 0) copy_w(std::integral_constant<int, i / 2>{}, step + 2, w_free);
+    });
+    products(c1, c1, c2, wb + place[2], xb + place[2], nothing);
+    products(c0, c1, c2, wb + place[3], xb + place[3], nothing);
+    // the next step's operands have to be there before its first reads, and this step's have been read: then x two steps
+    // ahead follows into its buffer.  What may be in flight until then are the eight copies of weights from above.
+    products(c1, c4, c1, w_frag + w_next + place[0], x_frag + ((step & 1) ^ 1) * kStage + place[0], [&](auto I) {
+      constexpr int i = decltype(I)::value;
+      if constexpr (i == 3) {
+        dma_wait_but<8>();
+        workgroup_barrier();
+      }
+      if constexpr (i >= 8) copy_x(std::integral_constant<int, i - 8>{}, step + 2);
+    });
+    w_at = w_next;
+  }
+  dma_wait_all();                                   // (copies past the last step)
+  // ---- lane: row l32 of a block, weight rows 8 (r / 4) + 4 hi + r % 4; halves of the wave trade runs of four, so that a lane
+  // stores eight outputs in a row ----
+#pragma unroll
+  for (int m = 0; m < 4; ++m) {
+    const int row = row0 + wm * 128 + 32 * m + l32;
+    bf16_t* out = reinterpret_cast<bf16_t*>(a.out) + (int64_t)min(row, row_end - 1) * a.out_stride;
+#pragma unroll
+    for (int n = 0; n < (kGlu ? 2 : 4); ++n) {
+#pragma unroll
+      for (int r = 0; r < 16; r += 8) {
+        float o[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) o[i] = kGlu ? silu_of(acc[2 * n][m][r + i]) * acc[2 * n + 1][m][r + i] : acc[n][m][r + i];
+        const auto x = __builtin_amdgcn_permlane32_swap(pack2<bf16_t>(o[0], o[1]), pack2<bf16_t>(o[4], o[5]), false, false);
+        const auto y = __builtin_amdgcn_permlane32_swap(pack2<bf16_t>(o[2], o[3]), pack2<bf16_t>(o[6], o[7]), false, false);
+        const int col = (kGlu ? (n0 + wn * 128) / 2 : n0 + wn * 128) + 32 * n + 2 * r + 8 * hi;
+        if (row < row_end && col < (kGlu ? a.N / 2 : a.N)) *reinterpret_cast<uint4*>(out + col) = make_uint4(x[0], y[0], x[1], y[1]);
+      }
+    }
+  }
+}
+
+// Rows of a tile: large ones where experts have enough rows on average to fill them.
+static int tile_rows(int64_t pairs, int experts) { return pairs >= kLargeTileRows * (int64_t)experts ? 256 : 128; }
+static int64_t max_tiles(int64_t pairs, int experts) { return (pairs + tile_rows(pairs, experts) - 1) / tile_rows(pairs, experts) + experts; }
 static int plan_blocks(int64_t pairs) { return (int)((pairs + kPlanPairs - 1) / kPlanPairs); }
 
 }  // namespace mvllm
@@ -448,6 +627,7 @@ static PlanArgs plan_parts_of(void* plan, const int32_t* ids, int64_t pairs, int
   a.num_tiles = a.tile_row + max_tiles(pairs, experts);
   a.hist = a.num_tiles + 1;
   a.pairs = (int)pairs; a.experts = experts; a.blocks = plan_blocks(pairs);
+  a.tile_rows = tile_rows(pairs, experts);
   return a;
 }
 
@@ -459,7 +639,7 @@ extern "C" int mvllm_moe_plan(void* plan, size_t plan_bytes, const int32_t* ids,
   if (plan_bytes < mvllm_moe_plan_bytes(pairs, experts)) return MVLLM_ERR_WORKSPACE;
   const PlanArgs a = plan_parts_of(plan, ids, pairs, experts);
   hipStream_t s = (hipStream_t)stream;
-  moe_count_kernel<<<dim3((unsigned)a.blocks), dim3(256), 0, s>>>(a);
+  if (a.blocks > 1) moe_count_kernel<<<dim3((unsigned)a.blocks), dim3(256), 0, s>>>(a);
   moe_place_kernel<<<dim3((unsigned)a.blocks), dim3(1024), 0, s>>>(a);
   return launch_status();
 }
@@ -482,13 +662,13 @@ extern "C" int mvllm_moe_linear(void* out, int64_t out_row_stride, const void* x
   hipStream_t s = (hipStream_t)stream;
   const int outputs = glu ? N / 2 : N;
   if (!plan) {
-    const dim3 grid((unsigned)(outputs / 16), (unsigned)experts);
-    if (K >= 1024) {
-      if (glu) moe_linear_few_kernel<8, true><<<grid, dim3(512), 0, s>>>(a);
-      else moe_linear_few_kernel<8, false><<<grid, dim3(512), 0, s>>>(a);
+    const unsigned n32 = (unsigned)((outputs + 31) / 32), n64 = (unsigned)((outputs + 63) / 64), n_experts = (unsigned)experts;
+    if (K >= 2048) {
+      if (glu) moe_linear_few_kernel<8, true, 2><<<dim3(n32, n_experts), dim3(512), 0, s>>>(a);
+      else moe_linear_few_kernel<8, false, 4><<<dim3(n64, n_experts), dim3(512), 0, s>>>(a);
     } else {
-      if (glu) moe_linear_few_kernel<4, true><<<grid, dim3(256), 0, s>>>(a);
-      else moe_linear_few_kernel<4, false><<<grid, dim3(256), 0, s>>>(a);
+      if (glu) moe_linear_few_kernel<4, true, 2><<<dim3(n32, n_experts), dim3(256), 0, s>>>(a);
+      else moe_linear_few_kernel<4, false, 4><<<dim3(n64, n_experts), dim3(256), 0, s>>>(a);
     }
     return launch_status();
   }
@@ -497,13 +677,17 @@ extern "C" int mvllm_moe_linear(void* out, int64_t out_row_stride, const void* x
   a.num_tiles = p.num_tiles;
   if (dtype == MVLLM_BF16) {
     a.max_tiles = (int)max_tiles(pairs, experts);
-    a.n_tiles = (N + 127) / 128;
+    a.n_tiles = (N + p.tile_rows - 1) / p.tile_rows;
+    if (p.tile_rows == 256 && out_row_stride % 8 != 0) return MVLLM_ERR_UNSUPPORTED;
     const int64_t x_rows = per_token ? (pairs + per_token - 1) / per_token : pairs, x_bytes = ((x_rows - 1) * x_row_stride + K) * 2;
     if (x_bytes >= (int64_t)1 << 32 || (int64_t)N * K * 2 >= (int64_t)1 << 31) return MVLLM_ERR_UNSUPPORTED;
     a.x_bytes = (uint32_t)x_bytes;
     const int64_t per = (a.max_tiles + 7) / 8, groups = (per + 3) / 4, blocks = 8 * groups * 4 * a.n_tiles;
     if (blocks > 0x7fffffff) return MVLLM_ERR_BAD_SHAPE;
-    if (glu) moe_linear_many_kernel<true><<<dim3((unsigned)blocks), dim3(256), 0, s>>>(a);
+    if (p.tile_rows == 256) {
+      if (glu) moe_linear_large_kernel<true><<<dim3((unsigned)blocks), dim3(256), 0, s>>>(a);
+      else moe_linear_large_kernel<false><<<dim3((unsigned)blocks), dim3(256), 0, s>>>(a);
+    } else if (glu) moe_linear_many_kernel<true><<<dim3((unsigned)blocks), dim3(256), 0, s>>>(a);
     else moe_linear_many_kernel<false><<<dim3((unsigned)blocks), dim3(256), 0, s>>>(a);
   } else {
     int64_t z = pairs / (16 * (int64_t)experts) + 1;

@@ -84,6 +84,11 @@ template <int LDS_IMM>   // LDS destination = lds_base + LDS_IMM: one scalar reg
 __device__ __forceinline__ void dma16_to_lds(v4i rsrc, uint32_t lane_off, uint32_t lds_base) {
   asm volatile("s_add_u32 m0, %0, %3\n\tbuffer_load_dwordx4 %1, %2, 0 offen lds" ::"s"(lds_base), "v"(lane_off), "s"(rsrc), "n"(LDS_IMM) : "scc", "m0");
 }
+// The same with one more offset for all lanes (it counts in the bounds check).
+template <int LDS_IMM>
+__device__ __forceinline__ void dma16_to_lds_at(v4i rsrc, uint32_t lane_off, uint32_t wave_off, uint32_t lds_base) {
+  asm volatile("s_add_u32 m0, %0, %4\n\tbuffer_load_dwordx4 %1, %2, %3 offen lds" ::"s"(lds_base), "v"(lane_off), "s"(rsrc), "s"(wave_off), "n"(LDS_IMM) : "scc", "m0");
+}
 // The same from a 64-bit address per lane (no bounds check).
 __device__ __forceinline__ void dma16_to_lds_from(const void* p, uint32_t lds_base) {
   asm volatile("s_mov_b32 m0, %0\n\tglobal_load_lds_dwordx4 %1, off" ::"s"(lds_base), "v"(p) : "m0");
@@ -99,6 +104,11 @@ __device__ __forceinline__ v4i make_rsrc(const char* base, uint32_t bytes) {
   return r;
 }
 __device__ __forceinline__ void dma_wait_all() { asm volatile("s_waitcnt vmcnt(0)" ::: "memory"); }
+// All but the N newest copies (nothing else of the wave may be in flight: loads count too).
+template <int N>
+__device__ __forceinline__ void dma_wait_but() { asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory"); }
+// A barrier that leaves copies in flight (__syncthreads waits for every one): this wave's LDS reads are complete.
+__device__ __forceinline__ void workgroup_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 __device__ __forceinline__ uint32_t lds_address(const void* p) {
   return (uint32_t)(uintptr_t)(const __attribute__((address_space(3))) void*)p;
 }

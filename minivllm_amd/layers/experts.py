@@ -17,8 +17,7 @@ from minivllm_amd.utils.padding import pad_to, round_up
 
 __all__ = ["ExpertOutput", "ExpertPlan", "SparseExperts", "moe_route", "moe_plan", "moe_linear", "interleave_gate_up"]
 
-FEW_PAIRS = 4096           # (token, choice) pairs the products take without a plan ...
-FEW_ROWS = 32              # ... while an expert has at most that many rows on average
+FEW_PAIRS = 16             # (token, choice) pairs up to which the products run without a plan
 
 
 def _ptr(t):
@@ -149,7 +148,7 @@ class SparseExperts(nn.Module):
         ids, weights = moe_route(logits, self.correction, self.experts, self.top, self.groups, self.keep)
         pairs = ids.numel()
         plan = None
-        if h.dtype != torch.bfloat16 or pairs > FEW_PAIRS or pairs > FEW_ROWS * self.experts:
+        if h.dtype != torch.bfloat16 or pairs > FEW_PAIRS:
             plan = moe_plan(ids, self.experts)
         act = moe_linear(h, self.gate_up, ids, plan, self.top, glu=True)
         parts = moe_linear(act, self.down, ids, plan)

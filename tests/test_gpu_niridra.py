@@ -15,7 +15,7 @@ from minivllm_amd.layers.experts import ExpertOutput, SparseExperts, interleave_
 from minivllm_amd.layers.fused import stream_embed_norm, stream_norm
 from minivllm_amd.layers.latent import head_linear, latent_decode, latent_norm_store, latent_width
 from minivllm_amd.layers.mixers import DecayMemory, LatentAttention
-from minivllm_amd.layers.recurrent import DecayMemoryState, decay_memory, gated_row_norm
+from minivllm_amd.layers.recurrent import DecayMemoryState, decay_memory, gate_linear, gated_row_norm
 from minivllm_amd.models.niridra import NiridraForCausalLM, engine_config
 from minivllm_amd.sampling_parameters import SamplingParams
 from niridra_cases import CONFIGS, config, latent_layer, lightning_layer, moe
@@ -430,6 +430,15 @@ def test_latent_attention_single_keys_in_every_path(dtype):
 
 
 # ---- mixture of experts ----
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("rows", [5, 600])
+@pytest.mark.parametrize("n,k", [(11, 128), (40, 64), (61, 192), (65, 1024), (81, 320), (200, 128)])
+def test_router_logits(dtype, rows, n, k):
+    """Any number of experts beside the shared expert's gate."""
+    x, w = torch.randn(rows, k, generator=gen(n)).to(dtype), (torch.randn(n, k, generator=gen(k)) * k ** -0.5).to(dtype)
+    assert row_rel(gate_linear(x.to(DEV), w.to(DEV), None, n, 0.0), x.double() @ w.double().T) < 1e-5
+
+
 ROUTERS = [(10, 3, 2, 1), (12, 5, 3, 2), (5, 1, 1, 1), (64, 6, 8, 3), (128, 8, 16, 4), (200, 9, 4, 2), (1000, 12, 50, 7), (6, 6, 1, 1), (16, 2, 16, 3), (7, 4, 7, 5)]
 
 
@@ -462,11 +471,12 @@ def test_moe_plan(rows, top, experts):
 
 
 @pytest.mark.parametrize("rows,top,experts,n,k", [(1, 1, 1, 64, 64), (5, 3, 10, 80, 128), (64, 8, 16, 272, 1088), (170, 2, 3, 128, 320), (700, 3, 7, 336, 192),
-                                                  (40, 6, 6, 1024, 64), (1500, 4, 30, 64, 576)])
+                                                  (40, 6, 6, 1024, 64), (1500, 4, 30, 64, 576), (1300, 2, 4, 336, 192), (2100, 1, 3, 1040, 64),
+                                                  (1100, 3, 5, 80, 704)])
 @pytest.mark.parametrize("path", ["few", "many", "any"])
 def test_moe_linear(rows, top, experts, n, k, path):
     """Both products of an expert over unsorted pairs and over a plan; rows of experts in any number, also none."""
-    if path == "few" and rows * top > 4096:
+    if path == "few" and rows * top > 512:
         pytest.skip("more pairs than the unsorted form takes")
     dtype, g = torch.float32 if path == "any" else torch.bfloat16, gen(n + k)
     f = -(-n // 64) * 64
