@@ -1,10 +1,11 @@
 """Metadata of a ragged step: entries of any length (portions of prompts beside single decoded tokens) in one packed batch.
 
-Rows are packed entry by entry: entries of one token first, then short ones, then long ones.  Attention sees a row's entry cut at chunk borders: the piece
-that goes on in a chunk whose earlier tokens are cached reads the cache (``prefixed``), pieces that start a chunk read the
-packed keys and values of the step (``fresh``), single tokens take the decode kernel.  Pieces are sorted in that order
-(``dst_row``), so that each kernel runs over consecutive rows.  Only the tokens of an entry's last chunk stay cached; where
-the entry also reads the chunk before, whose blocks they go to, they are stored after attention (``late_slots``).
+Rows are packed entry by entry: entries of one token first, then short ones, then long ones.  Attention sees a row's entry
+cut at chunk borders: the piece that goes on in a chunk whose earlier tokens are cached reads the cache (``prefixed``),
+pieces that start a chunk read the packed keys and values of the step (``fresh``), single tokens take the decode kernel.
+Pieces are sorted in that order (``dst_row``), so that each kernel runs over consecutive rows.  Only the tokens of an entry's
+last chunk stay cached; where the entry also reads the chunk before, whose blocks they go to, they are stored after
+attention (``late_slots``).
 Layers that cache one latent per token (``LatentStep``) answer single and short entries row by row from the cache; long
 entries with a cached prefix come before those without.
 A recurrence takes single and short entries row by row and long ones in blocks of rows, cut into ``segments`` that run side
