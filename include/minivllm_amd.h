@@ -659,6 +659,84 @@ int mvllm_moe_linear(void* out, int64_t out_row_stride, const void* x, int64_t x
                      const int32_t* ids, void* plan, int64_t pairs, int experts, int N, int K, int per_token, int glu,
                      int dtype, void* stream);
 
+/*
+ * ... and for models whose router is a softmax and whose experts have a clamped gate:
+ * mvllm_moe_route_softmax: s = softmax(z) over experts + identity outputs, choice = s + correction, weights = s (renormalize:
+ *   s / (sum + 1e-20)).  The last `identity` outputs stand for no expert: their id is -1, and the plan leaves such pairs out
+ *   (their place is -1, their rows of the products are not written).
+ * mvllm_moe_linear_clamped: mvllm_moe_linear with g' sigmoid(alpha g') (u' + shift) behind it, g' = min(g, limit), u' = u clamped
+ *   to +-limit.
+ * mvllm_gated_unit: the same of dense rows: in [rows, in_row_stride] = g [width] | u [width], out [rows, out_row_stride].
+ * mvllm_stream_norm_identity: mvllm_stream_norm whose choices with ids < 0 (int32 [rows, top]) read row t of `self`
+ *   [rows, self_row_stride] instead of a row of parts.
+ */
+int mvllm_moe_route_softmax(int32_t* ids, float* weights, const float* logits, int64_t logit_row_stride,
+                            const float* correction, int64_t rows, int experts, int identity, int top, int renormalize,
+                            void* stream);
+int mvllm_moe_linear_clamped(void* out, int64_t out_row_stride, const void* x, int64_t x_row_stride, const void* w,
+                             const int32_t* ids, void* plan, int64_t pairs, int experts, int N, int K, int per_token,
+                             float alpha, float limit, float shift, int dtype, void* stream);
+int mvllm_gated_unit(void* out, int64_t out_row_stride, const void* in, int64_t in_row_stride, int64_t rows, int width,
+                     float alpha, float limit, float shift, int dtype, void* stream);
+int mvllm_stream_norm_identity(void* out, int64_t out_row_stride, float* x_out, const float* x, const void* y,
+                               int64_t y_row_stride, const void* parts, int64_t part_row_stride, const int32_t* part_row,
+                               const float* weights, int top, const int32_t* ids, const void* self,
+                               int64_t self_row_stride, const float* gate, int64_t gate_row_stride, const float* scale,
+                               const float* hc_out, const float* hc_mix, const float* hc_in, const float* gain, float eps,
+                               int64_t rows, int streams, int width, int dtype, void* stream);
+
+/*
+ * Windowed attention over rows that are keys and values at once, or over keys in two parts with values of their own
+ * (csrc/window_prefill.hip, csrc/window_decode.hip).  A query sees the `window` keys up to its own (0: all of them);
+ *     score = scale * t(p) * q . k - slopes[h] * distance,   t(p) = 1 + temp_coef ln(floor((p + 1) / temp_every) + 1)
+ * (slopes fp32 [H] or NULL; temp_every 0: t = 1), out = softmax . v, times sigmoid(gate) where gate is not NULL (head h's
+ * columns at h * gate_head_stride).  Strides are in elements; bf16 and fp32.
+ * mvllm_window_prefill: entries of packed queries (cu_q) over packed keys (cu_k); query i of an entry stands at key
+ *   (keys - queries) + i.  q: head h at h * q_head_stride, [dim | rot]; k: kv head g at g * k_head_stride, [dim]; k2 [rot], shared
+ *   by all heads, or NULL with rot 0; v like k, or NULL: the values are the keys.  positions int64 [total_q] (t only).  Tiled in
+ *   bf16 for dim 32, 64, 96, 128, 192, 256, with k2 and v for rot 32 and 64 (no slopes); else dim and rot up to 512.
+ * mvllm_window_decode: single query rows over a paged cache [num_blocks, block_size, kv heads, padded] (padded a multiple of 32)
+ *   whose rows are keys and, their first `values` columns (padded, or 512 of 576), values.  lens int64 [rows]: position + 1;
+ *   ring > 0: token p lies at place p mod ring of its entry's table (ring >= window + the most rows an entry has in a call - 1),
+ *   0: at place p.  Everything else as for mvllm_latent_decode.
+ * mvllm_latent_rope_store: mvllm_latent_norm_store with a part behind the latent, columns rot_col .. rot_col + rot of a row, that is
+ *   not normed; its first rot_dims columns turn by rot_table fp32 [max_position, rot_dims / 2, 2] (cos, sin) in pairs (2i, 2i + 1) if
+ *   interleaved, else (i, i + rot_dims / 2).  out_rows int64 [rows] (< 0: none) or NULL: rows of `out`.  in2 != NULL: a second plain
+ *   norm in the same launch, out2 [rows, padded2] = rms(in2[:rank2]) * weight2.
+ * mvllm_head_rope: the same rotation of columns x_col .. x_col + rot of every head of x, in place; the first `first_rows` rows go to
+ *   columns out_col .. out_col + out_width of first_out instead, zeros behind the part.
+ * mvllm_copy_rows: row src_rows[t] of src to row dst_rows[t] of dst and dst2_rows[t] of dst2 (indices int64, negative ones are
+ *   skipped, NULL: row t; dst or dst2 NULL: none); rows a multiple of 16 bytes.
+ */
+int mvllm_window_prefill(void* out, int64_t out_row_stride, int64_t out_head_stride, const void* q, int64_t q_row_stride,
+                         int64_t q_head_stride, const void* k, int64_t k_row_stride, int64_t k_head_stride, const void* k2,
+                         int64_t k2_row_stride, const void* v, int64_t v_row_stride, int64_t v_head_stride, const void* gate,
+                         int64_t gate_row_stride, int64_t gate_head_stride, const int32_t* cu_q, const int32_t* cu_k,
+                         const int64_t* positions, const float* slopes, int num_seqs, int64_t total_q, int num_heads,
+                         int num_kv_heads, int dim, int rot, int window, float scale, float temp_coef, float temp_every,
+                         int dtype, void* stream);
+size_t mvllm_window_decode_workspace_bytes(int rows, int num_heads, int num_kv_heads, int padded, int values, int64_t max_keys,
+                                           int dtype);
+int mvllm_window_decode(void* out, int64_t out_row_stride, int64_t out_head_stride, const void* q, int64_t q_row_stride,
+                        int64_t q_head_stride, const void* cache, const int32_t* block_tables, int table_width,
+                        const int32_t* row_entry, const int64_t* lens, const float* slopes, const void* gate,
+                        int64_t gate_row_stride, int64_t gate_head_stride, int rows, int num_heads, int num_kv_heads,
+                        int padded, int values, int block_size, int64_t num_blocks, int window, int ring, float scale,
+                        float temp_coef, float temp_every, int dtype, void* workspace, size_t workspace_bytes, void* stream);
+int mvllm_latent_rope_store(void* out, const int64_t* out_rows, const void* in, int64_t in_row_stride, const float* weight,
+                            float eps, const float* rot_table, int rot_col, int rot, int rot_dims, int interleaved,
+                            int64_t max_position, const int64_t* positions, void* cache, int64_t num_slots,
+                            const int64_t* slots, void* out2, const void* in2, int64_t in2_row_stride, const float* weight2,
+                            int rank2, int padded2, int64_t rows, int rank, int padded, int dtype, void* stream);
+int mvllm_head_rope(void* x, int64_t x_row_stride, int64_t x_head_stride, int x_col, void* first_out, int64_t out_row_stride,
+                    int64_t out_head_stride, int out_col, int out_width, int64_t first_rows, const float* table, int rot,
+                    int rot_dims, int interleaved, int64_t max_position, const int64_t* positions, int64_t rows, int num_heads,
+                    int dtype, void* stream);
+int mvllm_copy_rows(void* dst, int64_t dst_row_stride, int64_t dst_count, const int64_t* dst_rows, void* dst2,
+                    int64_t dst2_row_stride, int64_t dst2_count, const int64_t* dst2_rows, const void* src,
+                    int64_t src_row_stride, int64_t src_count, const int64_t* src_rows, int64_t rows, int width, int dtype,
+                    void* stream);
+
 #ifdef __cplusplus
 }
 #endif

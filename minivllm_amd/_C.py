@@ -118,6 +118,28 @@ SIGNATURES = {
     "mvllm_moe_linear": (c_int, [c_void_p, c_int64, c_void_p, c_int64] + [c_void_p] * 3 + [c_int64] + [c_int] * 6 + [c_void_p]),
     "mvllm_mlstm_output": (c_int, [c_void_p] * 5 + [c_int64, c_float] + [c_void_p] * 5 + [c_int64, c_int, c_int, c_int,
                                                                                       c_void_p]),
+    "mvllm_moe_route_softmax": (c_int, [c_void_p] * 3 + [c_int64, c_void_p, c_int64] + [c_int] * 4 + [c_void_p]),
+    "mvllm_moe_linear_clamped": (c_int, [c_void_p, c_int64, c_void_p, c_int64] + [c_void_p] * 3 + [c_int64] + [c_int] *
+          4 + [c_float] * 3 + [c_int, c_void_p]),
+    "mvllm_gated_unit": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int] + [c_float] * 3 + [c_int,
+          c_void_p]),
+    "mvllm_stream_norm_identity": (c_int, [c_void_p, c_int64] + [c_void_p] * 3 + [c_int64, c_void_p, c_int64, c_void_p,
+          c_void_p, c_int, c_void_p, c_void_p, c_int64, c_void_p, c_int64] + [c_void_p] * 5 + [c_float, c_int64] + [c_int] * 3
+          + [c_void_p]),
+    "mvllm_window_prefill": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_int64, c_int64, c_void_p, c_int64, c_int64,
+          c_void_p, c_int64, c_void_p, c_int64, c_int64, c_void_p, c_int64, c_int64] + [c_void_p] * 4 + [c_int, c_int64] +
+          [c_int] * 5 + [c_float] * 3 + [c_int, c_void_p]),
+    "mvllm_window_decode_workspace_bytes": (c_size_t, [c_int] * 5 + [c_int64, c_int]),
+    "mvllm_window_decode": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_int] +
+          [c_void_p] * 4 + [c_int64, c_int64] + [c_int] * 6 + [c_int64, c_int, c_int] + [c_float] * 3 + [c_int, c_void_p,
+          c_size_t, c_void_p]),
+    "mvllm_latent_rope_store": (c_int, [c_void_p] * 3 + [c_int64, c_void_p, c_float, c_void_p] + [c_int] * 4 + [c_int64,
+          c_void_p, c_void_p, c_int64] + [c_void_p] * 3 + [c_int64, c_void_p, c_int, c_int, c_int64] + [c_int] * 3 +
+          [c_void_p]),
+    "mvllm_head_rope": (c_int, [c_void_p, c_int64, c_int64, c_int, c_void_p, c_int64, c_int64, c_int, c_int, c_int64,
+          c_void_p] + [c_int] * 3 + [c_int64, c_void_p, c_int64, c_int, c_int, c_void_p]),
+    "mvllm_copy_rows": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_void_p, c_void_p,
+          c_int64, c_int64, c_void_p, c_int64, c_int, c_int, c_void_p]),
 }
 
 

@@ -2,6 +2,8 @@
 //   x, y = input.chunk(2, dim=-1);  out = silu(x) * y
 // Rounding follows the two tensor operations: silu(x) = x / (1 + exp(-x)) in fp32 rounded to the element type,
 // then the product in fp32 rounded again.  One launch, 16-byte accesses, rows of the GEMM output as they lie.
+// mvllm_gated_unit: min(x, limit) * sigmoid(alpha min(x, limit)) * (clamp(y, +-limit) + shift), x and y the halves of a row:
+//   a clamped gated unit (limit infinite, alpha 1, shift 0: silu(x) * y in one rounding)
 #include "common.h"
 
 #pragma clang fp contract(off)
@@ -58,6 +60,28 @@ __global__ __launch_bounds__(kActThreads) void silu_and_mul_kernel(T* __restrict
   }
 }
 
+// One rounding; rows of both sides with strides.
+template <typename T>
+__global__ __launch_bounds__(kActThreads) void gated_unit_kernel(T* __restrict__ out, const T* __restrict__ in, int64_t rows, int width,
+                                                                 int64_t in_stride, int64_t out_stride, float alpha, float limit, float shift) {
+  constexpr int N = Act8<T>::N;
+  const int per_row = width / N;
+  const int64_t total = rows * per_row;
+  for (int64_t i = (int64_t)blockIdx.x * kActThreads + threadIdx.x; i < total; i += (int64_t)gridDim.x * kActThreads) {
+    const int64_t r = i / per_row;
+    const int c = (int)(i - r * per_row) * N;
+    float a[8], b[8], y[8];
+    Act8<T>::load(in + r * in_stride + c, a);
+    Act8<T>::load(in + r * in_stride + width + c, b);
+#pragma unroll
+    for (int e = 0; e < N; ++e) {
+      const float g = fminf(a[e], limit), u = fminf(fmaxf(b[e], -limit), limit);
+      y[e] = g / (1.0f + expf(-alpha * g)) * (u + shift);
+    }
+    Act8<T>::store(out + r * out_stride + c, y);
+  }
+}
+
 }  // namespace mvllm
 
 using namespace mvllm;
@@ -82,5 +106,23 @@ extern "C" int mvllm_silu_and_mul(void* out, const void* in, int64_t rows, int w
     case MVLLM_BF16: silu_and_mul_kernel<bf16_t><<<grid, block, 0, s>>>((bf16_t*)out, (const bf16_t*)in, rows, width, in_row_stride); break;
     default: silu_and_mul_kernel<f16_t><<<grid, block, 0, s>>>((f16_t*)out, (const f16_t*)in, rows, width, in_row_stride); break;
   }
+  return launch_status();
+}
+
+extern "C" int mvllm_gated_unit(void* out, int64_t out_row_stride, const void* in, int64_t in_row_stride, int64_t rows,
+                                int width, float alpha, float limit, float shift, int dtype, void* stream) {
+  const int esize = dtype_size(dtype);
+  if (esize == 0) return MVLLM_ERR_BAD_DTYPE;
+  if (rows < 0 || width <= 0 || in_row_stride < 2 * (int64_t)width || out_row_stride < width || !(limit >= 0.f)) return MVLLM_ERR_BAD_SHAPE;
+  const int n = 16 / esize;
+  if (dtype == MVLLM_F16 || width % n != 0 || in_row_stride % n != 0 || out_row_stride % n != 0) return MVLLM_ERR_UNSUPPORTED;
+  if (rows == 0) return MVLLM_OK;
+  if (!out || !in) return MVLLM_ERR_NULL_POINTER;
+  if (!aligned16(out) || !aligned16(in)) return MVLLM_ERR_MISALIGNED;
+  const int64_t blocks = (rows * (width / n) + kActThreads - 1) / kActThreads;
+  const dim3 grid((unsigned)(blocks > 65536 ? 65536 : blocks)), block(kActThreads);
+  hipStream_t s = (hipStream_t)stream;
+  if (dtype == MVLLM_F32) gated_unit_kernel<float><<<grid, block, 0, s>>>((float*)out, (const float*)in, rows, width, in_row_stride, out_row_stride, alpha, limit, shift);
+  else gated_unit_kernel<bf16_t><<<grid, block, 0, s>>>((bf16_t*)out, (const bf16_t*)in, rows, width, in_row_stride, out_row_stride, alpha, limit, shift);
   return launch_status();
 }

@@ -5,10 +5,11 @@
 // That is the form for decoded tokens and short portions; long portions make keys and values of the latents (a matrix
 // product) and run the prefill kernels.
 //   latent_norm_store   c = rms(row) * weight, packed and into the cache
+//   latent_rope_store   the same with a rotated part behind the latent, and another norm (the queries' latent) beside it
 //   head_linear         out[t, h] = W_h x[t, h]
 //   latent_decode       one query row per (row, block of heads, share of the keys); latent_merge joins the shares
 // The rank is padded to a multiple of 32 with zeros; scores, weights and sums are fp32.
-#include "prefill_tiles.h"
+#include "latent_decode.h"
 
 #pragma clang fp contract(off)
 
@@ -16,25 +17,43 @@ namespace mvllm {
 
 // ---- norm and store ----
 struct LatentNormArgs {
-  void* out;                // [T, padded] or null
+  void* out;                // [*, padded] or null
+  const int64_t* out_rows;  // [T]: row of `out` (< 0: none), or null: row t
   const void* in;           // [T, in_stride]
   const float* weight;      // [rank]
   void* cache;              // [num_slots, padded] or null
   const int64_t* slots;     // [T], < 0: not stored
-  int64_t in_stride, num_slots;
+  const float2* rot_table;  // [max_position, rot_dims / 2] (cos, sin) or null
+  const int64_t* positions; // [T]
+  int64_t in_stride, num_slots, max_position;
   float eps;
   int rows, rank, padded;
+  int rot_col, rot, rot_dims, interleaved;   // columns rot_col .. rot_col + rot are not normed; their first rot_dims turn
   bool vec;                 // the weight starts on 16 bytes
 };
 
-// One row per wave, 16 bytes per lane and access.
+// Column `d` of the rotated part of a row, its partner read from memory; pairs (2i, 2i + 1) or (i, i + dims / 2).
+template <typename T>
+__device__ __forceinline__ float turned_column(const LatentNormArgs& a, const T* part, const float2* cs, float own, int d) {
+  if (d >= a.rot_dims) return own;
+  const int half = a.rot_dims / 2;
+  const bool low = a.interleaved ? (d & 1) == 0 : d < half;
+  const int pair = a.interleaved ? d >> 1 : low ? d : d - half, other = a.interleaved ? d ^ 1 : low ? d + half : d - half;
+  const float2 c = cs[pair];
+  const float p = to_float(part[other]);
+  return low ? own * c.x - p * c.y : own * c.x + p * c.y;
+}
+
+// One row per wave, 16 bytes per lane and access; blockIdx.y: which of two norms.
 template <typename T, int NC>
-__global__ __launch_bounds__(256) void latent_norm_kernel(const LatentNormArgs a) {
+__global__ __launch_bounds__(256) void latent_norm_kernel(const LatentNormArgs first, const LatentNormArgs second) {
   constexpr int N = 16 / (int)sizeof(T);
+  const LatentNormArgs& a = blockIdx.y == 0 ? first : second;
   const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (row >= a.rows) return;
   const T* in = reinterpret_cast<const T*>(a.in) + (int64_t)row * a.in_stride;
   const int64_t slot = a.slots ? a.slots[row] : -1;
+  const int64_t out_row = a.out_rows ? a.out_rows[row] : row;
   float x[NC][N], w[NC][N], ss = 0.f;
 #pragma unroll
   for (int c = 0; c < NC; ++c) {
@@ -47,6 +66,9 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(const LatentNormArgs a
       for (int i = 0; i < N; ++i) w[c][i] = a.weight[min(at + i, a.rank - 1)];
     }
   }
+  const bool turns = a.rot_table != nullptr;
+  const float2* cs = nullptr;
+  if (turns) cs = a.rot_table + min(max(a.positions[row], (int64_t)0), a.max_position - 1) * (a.rot_dims / 2);
 #pragma unroll
   for (int c = 0; c < NC; ++c) {
     const int at = (c * 64 + lane) * N;
@@ -57,10 +79,15 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(const LatentNormArgs a
       x[c][i] = at + i < a.rank ? to_float(v[i]) : 0.f;
       ss = fmaf(x[c][i], x[c][i], ss);
     }
+    if (turns && at + N > a.rot_col && at < a.rot_col + a.rot) {         // (the parts start on multiples of N: all or none)
+#pragma unroll
+      for (int i = 0; i < N; ++i)
+        if (at + i < a.rot_col + a.rot) x[c][i] = turned_column(a, in + a.rot_col, cs, to_float(v[i]), at + i - a.rot_col);
+    }
   }
   ss = four_rows_sum(row16_sum(ss));
   const float inv = 1.0f / sqrtf(ss / (float)a.rank + a.eps);
-  T* out = a.out ? reinterpret_cast<T*>(a.out) + (int64_t)row * a.padded : nullptr;
+  T* out = a.out && out_row >= 0 ? reinterpret_cast<T*>(a.out) + out_row * a.padded : nullptr;
   T* cached = a.cache && slot >= 0 && slot < a.num_slots ? reinterpret_cast<T*>(a.cache) + slot * a.padded : nullptr;
 #pragma unroll
   for (int c = 0; c < NC; ++c) {
@@ -68,11 +95,21 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(const LatentNormArgs a
     if (at >= a.padded) continue;
     T v[N];
 #pragma unroll
-    for (int i = 0; i < N; ++i) v[i] = from_float<T>(at + i < a.rank ? x[c][i] * inv * w[c][i] : 0.f);
+    for (int i = 0; i < N; ++i) v[i] = from_float<T>(at + i < a.rank ? x[c][i] * inv * w[c][i] : x[c][i]);
     const uint4 r = *reinterpret_cast<const uint4*>(v);
     if (out) *reinterpret_cast<uint4*>(out + at) = r;
     if (cached) *reinterpret_cast<uint4*>(cached + at) = r;
   }
+}
+
+template <typename T>
+static void launch_latent_norm(const LatentNormArgs& a, const LatentNormArgs& b, bool two, hipStream_t s) {
+  const dim3 grid((unsigned)((a.rows + 3) / 4), two ? 2 : 1), block(256);
+  const int widest = two && b.padded > a.padded ? b.padded : a.padded;
+  constexpr int kFew = sizeof(T) == 4 ? 2 : 1;
+  if (widest <= 512) latent_norm_kernel<T, kFew><<<grid, block, 0, s>>>(a, b);
+  else if (widest <= 1024) latent_norm_kernel<T, 2 * kFew><<<grid, block, 0, s>>>(a, b);
+  else latent_norm_kernel<T, 4 * kFew><<<grid, block, 0, s>>>(a, b);
 }
 
 // ---- a matrix per head ----
@@ -173,377 +210,6 @@ __global__ __launch_bounds__(256) void head_linear_f32_kernel(const HeadLinearAr
   if (row < a.rows && col < a.N) reinterpret_cast<float*>(a.out)[(int64_t)row * a.out_row + (int64_t)h * a.out_head + col] = acc;
 }
 
-// ---- attention of single rows over the cache ----
-struct LatentDecodeArgs {
-  void* out;                 // [rows, H, padded]
-  const void* q;             // [rows, H, padded]
-  const void* cache;         // [num_blocks, block_size, padded]
-  const int32_t* tables;     // [entries, table_width]
-  const int32_t* row_entry;  // [rows]
-  const int64_t* lens;       // [rows]: keys the row sees
-  float* part_o;             // [rows, parts, H, padded] (parts > 1)
-  float2* part_ml;           // [rows, parts, H]: maximum (base 2), sum
-  int64_t num_blocks;
-  int table_width, block_size, heads, padded, parts;
-  float scale_log2;
-};
-
-// Keys of share `part`: whole tiles of 64, all shares of a row as even as that allows.
-__device__ __forceinline__ void key_share(const LatentDecodeArgs& a, int row, int part, int& k0, int& k1) {
-  const int64_t most = (int64_t)a.table_width * a.block_size;
-  const int n = (int)min(max(a.lens[row], (int64_t)0), most);
-  const int tiles = (n + 63) / 64, per = (tiles + a.parts - 1) / a.parts;
-  k0 = min(part * per * 64, n);
-  k1 = min(k0 + per * 64, n);
-}
-
-// Cache row of key `at` of the entry.
-__device__ __forceinline__ int64_t key_slot(const LatentDecodeArgs& a, const int32_t* table, int at) {
-  const int b = at / a.block_size;
-  const int64_t block = min(max((int64_t)table[b], (int64_t)0), a.num_blocks - 1);
-  return block * a.block_size + (at - b * a.block_size);
-}
-
-// Results of a share: the answer itself when there is one share only, otherwise partial sums.
-template <typename T>
-__device__ __forceinline__ void store4(const LatentDecodeArgs& a, int row, int part, int h, int col, const float* o, float inv) {
-  if (a.parts == 1) {
-    T* p = reinterpret_cast<T*>(a.out) + ((int64_t)row * a.heads + h) * a.padded + col;
-    T v[4];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) v[i] = from_float<T>(o[i] * inv);
-    if constexpr (sizeof(T) == 4) *reinterpret_cast<uint4*>(p) = *reinterpret_cast<const uint4*>(v);
-    else *reinterpret_cast<uint2*>(p) = *reinterpret_cast<const uint2*>(v);
-  } else {
-    float* p = a.part_o + (((int64_t)row * a.parts + part) * a.heads + h) * a.padded + col;
-    *reinterpret_cast<float4*>(p) = make_float4(o[0], o[1], o[2], o[3]);
-  }
-}
-
-// bf16: workgroup = (share, block of 16 HT heads, row), four waves; RS = padded rank / 32.  Tiles of 64 latents go to LDS
-// once, in chunks of 16 bytes whose place in a row is xor-ed with the key's low bits; wave w takes 16-head tile w % HT and
-// the key subtiles of its share w / HT.  S^T = C Q'^T (keys down the accumulator, heads across the lanes), so that the
-// weights are the operand of O^T += C^T P^T as they lie; C^T comes from the same LDS tile through the transposing loads.  Two
-// tiles in LDS: the next one is on its way while this one is worked on.
-template <int RS, int HT>
-__global__ __launch_bounds__(256, RS > 8 ? 1 : RS > 4 ? 2 : 3) void latent_decode_kernel(const LatentDecodeArgs a) {
-  constexpr int kShares = 4 / HT, kSub = 4 / kShares;      // key shares of a tile, 16-key subtiles of a wave
-  constexpr int RC = 4 * RS, kRow = 16 * RC;               // chunks and bytes of a row
-  constexpr int kXor = (RC & -RC) < 16 ? (RC & -RC) : 16;  // chunks that trade places
-  constexpr int kTile = 64 * kRow;
-  __shared__ __attribute__((aligned(16))) char lds[2 * kTile];
-  __shared__ int64_t slot_of[2][64];
-  __shared__ float2 ml[4][16];
-  const int part = blockIdx.x, row = blockIdx.z;
-  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), g = lane >> 4, i16 = lane & 15;
-  const int ht = wave % HT, share = wave / HT;
-  const int h = (blockIdx.y * HT + ht) * 16 + i16;         // this lane's head (as column)
-  int k0, k1;
-  key_share(a, row, part, k0, k1);
-  const int32_t* table = a.tables + (int64_t)a.row_entry[row] * a.table_width;
-
-  uint4 qf[RS];
-  {
-    const bf16_t* q = reinterpret_cast<const bf16_t*>(a.q) + ((int64_t)row * a.heads + min(h, a.heads - 1)) * (32 * RS) + 8 * g;
-#pragma unroll
-    for (int ks = 0; ks < RS; ++ks) qf[ks] = *reinterpret_cast<const uint4*>(q + 32 * ks);
-  }
-  v4f o[2 * RS];
-#pragma unroll
-  for (int n = 0; n < 2 * RS; ++n) o[n] = v4f{0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, l = 0.f;
-
-  // places in LDS: only the low bits of a chunk's number depend on the lane
-  constexpr int kBy = kXor / 4 > 0 ? kXor / 4 : 1, kCols = kXor / 2;
-  const char* key_at[kBy];                         // chunk 4 b + g of key 16 (first subtile) + i16
-  const char* col_at[kCols];                       // column group j of key 4 g + i16 / 4 of the first subtile
-  {
-    const char* row_a = lds + (16 * share * kSub + i16) * kRow;
-    const char* row_b = lds + (16 * share * kSub + 4 * g + (i16 >> 2)) * kRow + 8 * (i16 & 1);
-    const int xa = i16 & (kXor - 1), xb = (4 * g + (i16 >> 2)) & (kXor - 1);
-#pragma unroll
-    for (int b = 0; b < kBy; ++b) key_at[b] = row_a + (((4 * b + g) ^ xa) << 4);
-#pragma unroll
-    for (int j = 0; j < kCols; ++j) col_at[j] = row_b + (((2 * j + ((i16 & 3) >> 1)) ^ xb) << 4);
-  }
-
-  // a tile: RS chunks per thread, straight into LDS
-  auto copy = [&](int buffer) __attribute__((always_inline)) {
-    const char* cache = reinterpret_cast<const char*>(a.cache);
-#pragma unroll
-    for (int i = 0; i < RS; ++i) {
-      const uint32_t c = 256u * i + (uint32_t)tid;
-      const uint32_t key = c / RC, p = c % RC;
-      const char* from = cache + slot_of[buffer][key] * kRow + ((p ^ (key & (kXor - 1))) << 4);
-      dma16_to_lds_from(from, lds_address(lds) + buffer * kTile + (256 * i + 64 * wave) * 16);
-      if (i % 4 == 3) __builtin_amdgcn_sched_barrier(0);
-    }
-  };
-  if (tid < 128 && k0 < k1) slot_of[tid >> 6][tid & 63] = key_slot(a, table, min(k0 + tid, k1 - 1));
-  __syncthreads();
-  if (k0 < k1) copy(0);
-  dma_wait_all();
-  __syncthreads();
-  int flip = 0;
-  for (int base = k0; base < k1; base += 64, flip ^= 1) {
-    const bool more = base + 64 < k1;
-    int64_t slot_after = 0;                         // of the tile behind the next one
-    if (tid < 64 && base + 128 < k1) slot_after = key_slot(a, table, min(base + 128 + tid, k1 - 1));
-    if (more) copy(flip ^ 1);
-    __builtin_amdgcn_sched_barrier(0);
-    const int at_tile = flip * kTile;
-
-    // ---- scores of the wave's subtiles ----
-    v4f s[kSub];
-#pragma unroll
-    for (int t = 0; t < kSub; ++t) s[t] = v4f{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int ks = 0; ks < RS; ++ks) {
-#pragma unroll
-      for (int t = 0; t < kSub; ++t)
-        s[t] = mfma16x16x32<bf16_t>(*reinterpret_cast<const uint4*>(key_at[ks % kBy] + at_tile + 16 * t * kRow + 64 * (ks / kBy * kBy)), qf[ks], s[t]);
-      if (ks % 4 == 3) __builtin_amdgcn_sched_barrier(0);      // operands of later steps stay in LDS until then
-    }
-    float most = -INFINITY;
-#pragma unroll
-    for (int t = 0; t < kSub; ++t)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int at = base + 16 * (share * kSub + t) + 4 * g + r;
-        s[t][r] = at < k1 ? s[t][r] * a.scale_log2 : -INFINITY;
-        most = fmaxf(most, s[t][r]);
-      }
-    most = fmaxf(most, __shfl_xor(most, 16, 64));
-    most = fmaxf(most, __shfl_xor(most, 32, 64));
-    // the running maximum moves only when it grows by more than 2^8 (or from nothing): weights stay below that
-    if (__any(most > m + 8.f || (m == -INFINITY && most > -INFINITY))) {
-      const float m_new = fmaxf(m, most);
-      const float keep = m == -INFINITY ? 0.f : fast_exp2(m - m_new);
-      m = m_new;
-      l *= keep;
-#pragma unroll
-      for (int n = 0; n < 2 * RS; ++n) o[n] *= keep;
-    }
-    uint2 w[kSub];
-#pragma unroll
-    for (int t = 0; t < kSub; ++t) {
-      float p[4];
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        p[r] = m == -INFINITY ? 0.f : fast_exp2(s[t][r] - m);
-        l += p[r];
-      }
-      w[t] = make_uint2(pack2<bf16_t>(p[0], p[1]), pack2<bf16_t>(p[2], p[3]));
-    }
-    // ---- O^T += C^T P^T: 16 columns of the latents at a time ----
-#pragma unroll
-    for (int n = 0; n < 2 * RS; ++n) {
-      auto column = [&](int t) __attribute__((always_inline)) {
-        const char* p = col_at[n % kCols] + at_tile + 16 * t * kRow + 32 * (n / kCols * kCols);
-        return __builtin_bit_cast(uint2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) v4s*)p));
-      };
-      if constexpr (kSub == 1) {
-        o[n] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(__builtin_bit_cast(v4s, column(0)), __builtin_bit_cast(v4s, w[0]), o[n], 0, 0, 0);
-      } else {
-#pragma unroll
-        for (int t = 0; t < kSub; t += 2) {
-          const uint2 c0 = column(t), c1 = column(t + 1);
-          o[n] = mfma16x16x32<bf16_t>(make_uint4(c0.x, c0.y, c1.x, c1.y), make_uint4(w[t].x, w[t].y, w[t + 1].x, w[t + 1].y), o[n]);
-        }
-      }
-      if (n % 4 == 3) __builtin_amdgcn_sched_barrier(0);
-    }
-    __builtin_amdgcn_sched_barrier(0);
-    if (tid < 64 && base + 128 < k1) slot_of[flip][tid] = slot_after;
-    dma_wait_all();
-    __syncthreads();                                // everybody is done with the tile; the next one and its successor's slots are there
-  }
-  l += __shfl_xor(l, 16, 64);
-  l += __shfl_xor(l, 32, 64);
-
-  // ---- the shares of a head tile meet in LDS, one after the other ----
-  if constexpr (kShares > 1) {
-    float4* box = reinterpret_cast<float4*>(lds) + ht * 2 * RS * 64;
-    for (int other = 1; other < kShares; ++other) {
-      if (share == other) {
-#pragma unroll
-        for (int n = 0; n < 2 * RS; ++n) box[n * 64 + lane] = make_float4(o[n][0], o[n][1], o[n][2], o[n][3]);
-        if (g == 0) ml[ht][i16] = make_float2(m, l);
-      }
-      __syncthreads();
-      if (share == 0) {
-        const float2 x = ml[ht][i16];
-        const float m_new = fmaxf(m, x.x);
-        const float mine = m == -INFINITY ? 0.f : fast_exp2(m - m_new), theirs = x.x == -INFINITY ? 0.f : fast_exp2(x.x - m_new);
-#pragma unroll
-        for (int n = 0; n < 2 * RS; ++n) {
-          const float4 b = box[n * 64 + lane];
-          o[n] = v4f{o[n][0] * mine + b.x * theirs, o[n][1] * mine + b.y * theirs, o[n][2] * mine + b.z * theirs, o[n][3] * mine + b.w * theirs};
-          if (n % 4 == 3) __builtin_amdgcn_sched_barrier(0);
-        }
-        l = l * mine + x.y * theirs;
-        m = m_new;
-      }
-      __syncthreads();
-    }
-  }
-  if (share != 0 || h >= a.heads) return;
-  const float inv = l > 0.f ? 1.0f / l : 0.f;
-  if (a.parts > 1 && g == 0) a.part_ml[((int64_t)row * a.parts + part) * a.heads + h] = make_float2(m, l);
-  if (a.parts > 1 && m == -INFINITY) return;                // the merge reads nothing of it
-#pragma unroll
-  for (int n = 0; n < 2 * RS; ++n) {
-    const float x[4] = {o[n][0], o[n][1], o[n][2], o[n][3]};
-    store4<bf16_t>(a, row, part, h, 16 * n + 4 * g, x, inv);
-  }
-}
-
-// Any type and rank up to 64 NE: workgroup = (share, head, row); a wave takes every fourth key, its lanes the columns.
-template <typename T, int NE>
-__global__ __launch_bounds__(256) void latent_decode_any_kernel(const LatentDecodeArgs a) {
-  __shared__ float part_o[4][64 * NE];
-  __shared__ float2 ml[4];
-  const int part = blockIdx.x, h = blockIdx.y, row = blockIdx.z;
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  int k0, k1;
-  key_share(a, row, part, k0, k1);
-  const int32_t* table = a.tables + (int64_t)a.row_entry[row] * a.table_width;
-  const T* q_row = reinterpret_cast<const T*>(a.q) + ((int64_t)row * a.heads + h) * a.padded;
-  float q[NE], o[NE];
-#pragma unroll
-  for (int i = 0; i < NE; ++i) {
-    const int c = lane + 64 * i;
-    q[i] = c < a.padded ? to_float(q_row[c]) * a.scale_log2 : 0.f;
-    o[i] = 0.f;
-  }
-  float m = -INFINITY, l = 0.f;
-  constexpr int kTogether = NE > 8 ? 2 : 4;
-  for (int base = k0 + wave * kTogether; base < k1; base += 4 * kTogether) {
-    float c[kTogether][NE], s[kTogether];
-#pragma unroll
-    for (int j = 0; j < kTogether; ++j) {
-      const T* p = reinterpret_cast<const T*>(a.cache) + key_slot(a, table, min(base + j, k1 - 1)) * a.padded;
-      s[j] = 0.f;
-#pragma unroll
-      for (int i = 0; i < NE; ++i) {
-        c[j][i] = lane + 64 * i < a.padded ? to_float(p[lane + 64 * i]) : 0.f;
-        s[j] = fmaf(q[i], c[j][i], s[j]);
-      }
-    }
-    float m_new = m;
-#pragma unroll
-    for (int j = 0; j < kTogether; ++j) {
-      s[j] = base + j < k1 ? wave_sum(s[j]) : -INFINITY;
-      m_new = fmaxf(m_new, s[j]);
-    }
-    const float keep = exp2f(m - m_new);            // from nothing: exp2(-inf) = 0
-    m = m_new;
-    l *= keep;
-#pragma unroll
-    for (int i = 0; i < NE; ++i) o[i] *= keep;
-#pragma unroll
-    for (int j = 0; j < kTogether; ++j) {
-      const float p = exp2f(s[j] - m);
-      l += p;
-#pragma unroll
-      for (int i = 0; i < NE; ++i) o[i] = fmaf(p, c[j][i], o[i]);
-    }
-  }
-#pragma unroll
-  for (int i = 0; i < NE; ++i) part_o[wave][lane + 64 * i] = o[i];
-  if (lane == 0) ml[wave] = make_float2(m, l);
-  __syncthreads();
-  float m_all = -INFINITY, l_all = 0.f, w[4];
-#pragma unroll
-  for (int i = 0; i < 4; ++i) m_all = fmaxf(m_all, ml[i].x);
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    w[i] = ml[i].x == -INFINITY ? 0.f : exp2f(ml[i].x - m_all);
-    l_all = fmaf(w[i], ml[i].y, l_all);
-  }
-  const float inv = l_all > 0.f ? 1.0f / l_all : 0.f;
-  if (a.parts > 1 && threadIdx.x == 0) a.part_ml[((int64_t)row * a.parts + part) * a.heads + h] = make_float2(m_all, l_all);
-  for (int c = 4 * threadIdx.x; c < a.padded; c += 1024) {
-    float x[4];
-#pragma unroll
-    for (int e = 0; e < 4; ++e)
-      x[e] = w[0] * part_o[0][c + e] + w[1] * part_o[1][c + e] + w[2] * part_o[2][c + e] + w[3] * part_o[3][c + e];
-    store4<T>(a, row, part, h, c, x, inv);
-  }
-}
-
-// Joins the shares of a (row, head): one wave each, four columns per lane and step.
-template <typename T>
-__global__ __launch_bounds__(256) void latent_merge_kernel(const LatentDecodeArgs a, int rows) {
-  const int64_t item = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-  const int lane = threadIdx.x & 63;
-  if (item >= (int64_t)rows * a.heads) return;
-  const int64_t row = item / a.heads;
-  const int h = (int)(item - row * a.heads);
-  // lane p has the maximum and sum of share p (at most 64 shares)
-  float2 x = make_float2(-INFINITY, 0.f);
-  if (lane < a.parts) x = a.part_ml[(row * a.parts + lane) * a.heads + h];
-  const float m = wave_max(x.x);
-  const float w = x.x == -INFINITY ? 0.f : exp2f(x.x - m);
-  const float l = wave_sum(w * x.y);
-  const float f = l > 0.f ? w / l : 0.f;
-  for (int c = 4 * lane; c < a.padded; c += 256) {
-    float o[4] = {0.f, 0.f, 0.f, 0.f};
-    for (int p = 0; p < a.parts; ++p) {
-      const float g = __shfl(f, p, 64);
-      if (g == 0.f) continue;                       // empty shares have left nothing (uniform over the wave)
-      const float4 v = *reinterpret_cast<const float4*>(a.part_o + ((row * a.parts + p) * a.heads + h) * a.padded + c);
-      o[0] = fmaf(g, v.x, o[0]); o[1] = fmaf(g, v.y, o[1]); o[2] = fmaf(g, v.z, o[2]); o[3] = fmaf(g, v.w, o[3]);
-    }
-    T v[4];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) v[i] = from_float<T>(o[i]);
-    T* out = reinterpret_cast<T*>(a.out) + (row * a.heads + h) * a.padded + c;
-    if constexpr (sizeof(T) == 4) *reinterpret_cast<uint4*>(out) = *reinterpret_cast<const uint4*>(v);
-    else *reinterpret_cast<uint2*>(out) = *reinterpret_cast<const uint2*>(v);
-  }
-}
-
-template <int RS>
-static int launch_decode(const LatentDecodeArgs& a, int rows, hipStream_t s) {
-  const int tiles = (a.heads + 15) / 16;
-  const dim3 block(256);
-  if (tiles == 1) latent_decode_kernel<RS, 1><<<dim3((unsigned)a.parts, 1, (unsigned)rows), block, 0, s>>>(a);
-  else if (tiles == 2) latent_decode_kernel<RS, 2><<<dim3((unsigned)a.parts, 1, (unsigned)rows), block, 0, s>>>(a);
-  else latent_decode_kernel<RS, 4><<<dim3((unsigned)a.parts, (unsigned)((tiles + 3) / 4), (unsigned)rows), block, 0, s>>>(a);
-  return launch_status();
-}
-
-template <typename T>
-static int launch_any(const LatentDecodeArgs& a, int rows, hipStream_t s) {
-  const dim3 grid((unsigned)a.parts, (unsigned)a.heads, (unsigned)rows), block(256);
-  if (a.padded <= 128) latent_decode_any_kernel<T, 2><<<grid, block, 0, s>>>(a);
-  else if (a.padded <= 512) latent_decode_any_kernel<T, 8><<<grid, block, 0, s>>>(a);
-  else if (a.padded <= 1024) latent_decode_any_kernel<T, 16><<<grid, block, 0, s>>>(a);
-  else latent_decode_any_kernel<T, 32><<<grid, block, 0, s>>>(a);
-  return launch_status();
-}
-
-constexpr int kMaxParts = 32;
-
-// Shares per row: as many as give the shortest schedule, in tiles of 64 keys (two more for a share's start and end, two for the
-// pass that joins shares), of whole rounds of the workgroups that run side by side.
-static int plan_parts(int rows, int heads, int padded, int64_t max_keys, int dtype) {
-  const int head_tiles = (heads + 15) / 16;
-  const int64_t groups = (int64_t)rows * (dtype == MVLLM_BF16 ? (head_tiles <= 2 ? 1 : (head_tiles + 3) / 4) : heads);
-  const int64_t together = 256 * (dtype != MVLLM_BF16 || padded <= 128 ? 3 : padded <= 256 ? 2 : 1), tiles = (max_keys + 63) / 64;
-  int best = 1;
-  int64_t best_time = INT64_MAX;
-  for (int parts = 1; parts <= kMaxParts && (parts == 1 || 2 * parts <= tiles); ++parts) {
-    const int64_t time = (groups * parts + together - 1) / together * ((tiles + parts - 1) / parts + 2) + (parts > 1 ? 2 : 0);
-    if (time < best_time) {
-      best = parts;
-      best_time = time;
-    }
-  }
-  return best;
-}
-
 }  // namespace mvllm
 
 using namespace mvllm;
@@ -558,18 +224,40 @@ extern "C" int mvllm_latent_norm_store(void* out, const void* in, int64_t in_row
   if (rows == 0) return MVLLM_OK;
   if (!in || !weight || (!out && !cache) || (cache && !slots)) return MVLLM_ERR_NULL_POINTER;
   if (!aligned16(in) || !aligned16(out) || !aligned16(cache)) return MVLLM_ERR_MISALIGNED;
-  LatentNormArgs a;
+  LatentNormArgs a = {};
   a.out = out; a.in = in; a.weight = weight; a.cache = cache; a.slots = slots; a.in_stride = in_row_stride;
   a.num_slots = num_slots; a.eps = eps; a.rows = (int)rows; a.rank = rank; a.padded = padded; a.vec = aligned16(weight);
-  const dim3 grid((unsigned)((rows + 3) / 4)), block(256);
-  hipStream_t s = (hipStream_t)stream;
-  if (dtype == MVLLM_F32) {
-    if (padded <= 512) latent_norm_kernel<float, 2><<<grid, block, 0, s>>>(a);
-    else latent_norm_kernel<float, 8><<<grid, block, 0, s>>>(a);
-  } else {
-    if (padded <= 512) latent_norm_kernel<bf16_t, 1><<<grid, block, 0, s>>>(a);
-    else latent_norm_kernel<bf16_t, 4><<<grid, block, 0, s>>>(a);
-  }
+  if (dtype == MVLLM_F32) launch_latent_norm<float>(a, a, false, (hipStream_t)stream);
+  else launch_latent_norm<bf16_t>(a, a, false, (hipStream_t)stream);
+  return launch_status();
+}
+
+extern "C" int mvllm_latent_rope_store(void* out, const int64_t* out_rows, const void* in, int64_t in_row_stride,
+                                       const float* weight, float eps, const float* rot_table, int rot_col, int rot,
+                                       int rot_dims, int interleaved, int64_t max_position, const int64_t* positions,
+                                       void* cache, int64_t num_slots, const int64_t* slots, void* out2, const void* in2,
+                                       int64_t in2_row_stride, const float* weight2, int rank2, int padded2, int64_t rows,
+                                       int rank, int padded, int dtype, void* stream) {
+  const int esize = dtype_size(dtype);
+  if (esize == 0) return MVLLM_ERR_BAD_DTYPE;
+  if (rows < 0 || rank <= 0 || padded < rank || padded % 32 != 0 || in_row_stride < padded || rot < 0 || rot_dims < 0 || rot_dims > rot ||
+      rot_dims % 2 != 0 || (rot > 0 && (rot_col < rank || rot_col % 8 != 0 || rot_col + rot > padded || max_position <= 0)) ||
+      (in2 && (rank2 <= 0 || padded2 < rank2 || padded2 % 32 != 0 || in2_row_stride < padded2)))
+    return MVLLM_ERR_BAD_SHAPE;
+  if (dtype == MVLLM_F16 || padded > 2048 || padded2 > 2048 || rows > (1 << 30) || (in_row_stride * esize) % 16 != 0 || (in2_row_stride * esize) % 16 != 0)
+    return MVLLM_ERR_UNSUPPORTED;
+  if (rows == 0) return MVLLM_OK;
+  if (!in || !weight || (cache && !slots) || (rot > 0 && (!rot_table || !positions)) || (in2 && (!weight2 || !out2))) return MVLLM_ERR_NULL_POINTER;
+  if (!aligned16(in) || !aligned16(out) || !aligned16(cache) || !aligned16(in2) || !aligned16(out2)) return MVLLM_ERR_MISALIGNED;
+  LatentNormArgs a = {}, b = {};
+  a.out = out; a.out_rows = out_rows; a.in = in; a.weight = weight; a.cache = cache; a.slots = slots;
+  a.rot_table = rot > 0 ? reinterpret_cast<const float2*>(rot_table) : nullptr; a.positions = positions; a.in_stride = in_row_stride;
+  a.num_slots = num_slots; a.max_position = max_position; a.eps = eps; a.rows = (int)rows; a.rank = rank; a.padded = padded;
+  a.rot_col = rot_col; a.rot = rot; a.rot_dims = rot_dims; a.interleaved = interleaved; a.vec = aligned16(weight);
+  b.out = out2; b.in = in2; b.weight = weight2; b.in_stride = in2_row_stride; b.eps = eps; b.rows = (int)rows; b.rank = rank2;
+  b.padded = padded2; b.vec = aligned16(weight2);
+  if (dtype == MVLLM_F32) launch_latent_norm<float>(a, b, in2 != nullptr, (hipStream_t)stream);
+  else launch_latent_norm<bf16_t>(a, b, in2 != nullptr, (hipStream_t)stream);
   return launch_status();
 }
 
@@ -598,7 +286,7 @@ extern "C" int mvllm_head_linear(void* out, int64_t out_row_stride, int64_t out_
 
 extern "C" size_t mvllm_latent_decode_workspace_bytes(int rows, int num_heads, int padded, int64_t max_keys, int dtype) {
   if (rows <= 0 || num_heads <= 0 || padded <= 0 || max_keys <= 0) return 0;
-  const int parts = plan_parts(rows, num_heads, padded, max_keys, dtype);
+  const int parts = plan_parts(rows, num_heads, 1, padded, max_keys, dtype);
   return parts == 1 ? 0 : (size_t)rows * parts * num_heads * ((size_t)padded + 2) * sizeof(float);
 }
 
@@ -614,11 +302,12 @@ extern "C" int mvllm_latent_decode(void* out, const void* q, const void* cache, 
   if (rows == 0) return MVLLM_OK;
   if (!out || !q || !cache || !block_tables || !row_entry || !lens) return MVLLM_ERR_NULL_POINTER;
   if (!aligned16(out) || !aligned16(q) || !aligned16(cache)) return MVLLM_ERR_MISALIGNED;
-  LatentDecodeArgs a;
+  LatentDecodeArgs a = {};
   a.out = out; a.q = q; a.cache = cache; a.tables = block_tables; a.row_entry = row_entry; a.lens = lens;
   a.num_blocks = num_blocks; a.table_width = table_width; a.block_size = block_size; a.heads = num_heads; a.padded = padded;
+  a.kv_heads = 1; a.values = padded; a.q_head = a.out_head = padded; a.q_row = a.out_row = (int64_t)num_heads * padded;
   a.scale_log2 = scale * kLog2e;
-  a.parts = plan_parts(rows, num_heads, padded, (int64_t)table_width * block_size, dtype);
+  a.parts = plan_parts(rows, num_heads, 1, padded, (int64_t)table_width * block_size, dtype);
   a.part_o = nullptr;
   a.part_ml = nullptr;
   if (a.parts > 1) {
@@ -627,23 +316,5 @@ extern "C" int mvllm_latent_decode(void* out, const void* q, const void* cache, 
     a.part_o = reinterpret_cast<float*>(workspace);
     a.part_ml = reinterpret_cast<float2*>(a.part_o + (int64_t)rows * a.parts * num_heads * padded);
   }
-  hipStream_t s = (hipStream_t)stream;
-  int st;
-  if (dtype == MVLLM_F32) st = launch_any<float>(a, rows, s);
-  else switch (padded) {
-    case 32: st = launch_decode<1>(a, rows, s); break;
-    case 64: st = launch_decode<2>(a, rows, s); break;
-    case 96: st = launch_decode<3>(a, rows, s); break;
-    case 128: st = launch_decode<4>(a, rows, s); break;
-    case 192: st = launch_decode<6>(a, rows, s); break;
-    case 256: st = launch_decode<8>(a, rows, s); break;
-    case 384: st = launch_decode<12>(a, rows, s); break;
-    case 512: st = launch_decode<16>(a, rows, s); break;
-    default: st = launch_any<bf16_t>(a, rows, s);
-  }
-  if (st != MVLLM_OK || a.parts == 1) return st;
-  const dim3 grid((unsigned)(((int64_t)rows * num_heads + 3) / 4)), block(256);
-  if (dtype == MVLLM_F32) latent_merge_kernel<float><<<grid, block, 0, s>>>(a, rows);
-  else latent_merge_kernel<bf16_t><<<grid, block, 0, s>>>(a, rows);
-  return launch_status();
+  return launch_decode<false>(a, rows, dtype, (hipStream_t)stream);
 }

@@ -1,9 +1,10 @@
 // Mixture of experts: the router's choice, the rows sorted by expert, and the experts' products.
 //   moe_route   scores s = sigmoid(z), choice scores s + correction; groups of neighbouring experts by the sum of their two
 //               largest choice scores, the best `keep` groups stay open; the `top` largest choice scores of those are chosen,
-//               weights s / (sum of the chosen s + 1e-20)
+//               weights s / (sum of the chosen s + 1e-20); or s = softmax(z), the weights s as they are; the last outputs may
+//               stand for no expert but for the input itself: their id is -1
 //   moe_plan    (token, choice) pairs sorted by expert, and tiles of 128 or 256 sorted rows per expert
-//   moe_linear  out[row] = x[row] W_e^T, optionally silu(gate) * up behind it: W_e [2 F, K] with gate and up rows in turns of
+//   moe_linear  out[row] = x[row] W_e^T, optionally silu(gate) * up or its clamped form behind it: W_e [2 F, K] with gate and up rows in turns of
 //               32, so that both halves of an output are in one lane
 // Products, by the number of rows: very few (no plan; a workgroup finds its expert's rows itself, its waves share K), many (bf16: 128 x 128 or 256 x 256
 // tiles on the matrix unit over sorted rows), any (fp32, over sorted rows).
@@ -21,6 +22,8 @@ struct RouteArgs {
   const float* correction; // [E] or null
   int64_t z_stride;
   int rows, experts, top, groups, keep;
+  int identity;            // of the experts: the last ones, whose output is their input
+  bool softmax, renormalize;
 };
 
 // One token per wave; lane l has experts l, l + 64, ...
@@ -38,9 +41,28 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const RouteArgs a) {
     s[i] = 0.f;
     choice[i] = -INFINITY;
     if (live && e < E) {
-      s[i] = 1.0f / (1.0f + expf(-a.z[(int64_t)row * a.z_stride + e]));
-      choice[i] = s[i] + (a.correction ? a.correction[e] : 0.f);
+      const float z = a.z[(int64_t)row * a.z_stride + e];
+      s[i] = a.softmax ? z : 1.0f / (1.0f + expf(-z));
     }
+  }
+  if (a.softmax) {
+    float most = -INFINITY, sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < NE; ++i) most = fmaxf(most, lane + 64 * i < E ? s[i] : -INFINITY);
+    most = wave_max_in_registers(most);
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      s[i] = lane + 64 * i < E ? expf(s[i] - most) : 0.f;
+      sum += s[i];
+    }
+    sum = four_rows_sum(row16_sum(sum));
+#pragma unroll
+    for (int i = 0; i < NE; ++i) s[i] /= sum;
+  }
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const int e = lane + 64 * i;
+    if (live && e < E) choice[i] = s[i] + (a.correction ? a.correction[e] : 0.f);
     choice_of[wave][e] = choice[i];
   }
   if (a.groups > 1) {
@@ -94,8 +116,8 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const RouteArgs a) {
     if (lane == k) { my_s = best_s; my_id = id; }
   }
   if (live && lane < a.top) {
-    a.ids[(int64_t)row * a.top + lane] = my_id;
-    a.weights[(int64_t)row * a.top + lane] = my_s / (sum + 1e-20f);
+    a.ids[(int64_t)row * a.top + lane] = my_id < E - a.identity ? my_id : -1;
+    a.weights[(int64_t)row * a.top + lane] = a.renormalize ? my_s / (sum + 1e-20f) : my_s;
   }
 }
 
@@ -120,7 +142,10 @@ __global__ __launch_bounds__(256) void moe_count_kernel(const PlanArgs a) {
   for (int e = threadIdx.x; e < a.experts; e += 256) count[e] = 0;
   __syncthreads();
   const int end = min((int)(blockIdx.x + 1) * kPlanPairs, a.pairs);
-  for (int p = blockIdx.x * kPlanPairs + threadIdx.x; p < end; p += 256) atomicAdd(&count[a.ids[p]], 1);
+  for (int p = blockIdx.x * kPlanPairs + threadIdx.x; p < end; p += 256) {
+    const int id = a.ids[p];
+    if (id >= 0) atomicAdd(&count[id], 1);
+  }
   __syncthreads();
   for (int e = threadIdx.x; e < a.experts; e += 256) a.hist[(int64_t)blockIdx.x * a.experts + e] = count[e];
 }
@@ -132,7 +157,10 @@ __global__ __launch_bounds__(1024) void moe_place_kernel(const PlanArgs a) {
   if (a.blocks == 1) {                              // counted here
     cursor[e] = 0;
     __syncthreads();
-    for (int p = e; p < a.pairs; p += 1024) atomicAdd(&cursor[a.ids[p]], 1);
+    for (int p = e; p < a.pairs; p += 1024) {
+      const int id = a.ids[p];
+      if (id >= 0) atomicAdd(&cursor[id], 1);
+    }
     __syncthreads();
     n = cursor[e];
     __syncthreads();
@@ -157,7 +185,12 @@ __global__ __launch_bounds__(1024) void moe_place_kernel(const PlanArgs a) {
   __syncthreads();
   const int end = min((int)(blockIdx.x + 1) * kPlanPairs, a.pairs);
   for (int p = blockIdx.x * kPlanPairs + threadIdx.x; p < end; p += 1024) {
-    const int at = atomicAdd(&cursor[a.ids[p]], 1);
+    const int id = a.ids[p];
+    if (id < 0) {                                   // no expert's: nobody computes or reads it
+      a.place[p] = -1;
+      continue;
+    }
+    const int at = atomicAdd(&cursor[id], 1);
     a.sorted_pair[at] = p;
     a.place[p] = at;
   }
@@ -190,15 +223,25 @@ struct ExpertLinearArgs {
   int per_token;               // > 0: pair p reads row p / per_token of x; 0: the row of its own (sorted) place
   int max_tiles, n_tiles;
   uint32_t x_bytes;            // (many) what x holds
+  float alpha, limit, shift;   // of kClampedGlu
 };
 
-__device__ __forceinline__ float silu_of(float z) { return z * __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
+enum { kNoGlu = 0, kSiluGlu = 1, kClampedGlu = 2 };
+
+// silu(g) * u, or with g' = min(g, limit) and u' = u within +-limit: g' sigmoid(alpha g') (u' + shift)
+template <int kGlu> __device__ __forceinline__ float glu_of(const ExpertLinearArgs& a, float g, float u) {
+  if constexpr (kGlu == kClampedGlu) {
+    g = fminf(g, a.limit);
+    return g * __builtin_amdgcn_rcpf(1.0f + __expf(-a.alpha * g)) * (fminf(fmaxf(u, -a.limit), a.limit) + a.shift);
+  }
+  return g * __builtin_amdgcn_rcpf(1.0f + __expf(-g)) * u;
+}
 
 // few: workgroup = (16 kTiles outputs, expert), its waves share K.  The rows of the expert are found in `ids`; rows are taken
 // 16 at a time.
 constexpr int kFewPairs = 512;
 
-template <int kWaves, bool kGlu, int kTiles>
+template <int kWaves, int kGlu, int kTiles>
 __global__ __launch_bounds__(64 * kWaves) void moe_linear_few_kernel(const ExpertLinearArgs a) {
   constexpr int NT = kTiles * (kGlu ? 2 : 1);        // tiles of weight rows: with the gate, gate and up of an output tile in turn
   __shared__ uint16_t list[kFewPairs];
@@ -286,7 +329,7 @@ __global__ __launch_bounds__(64 * kWaves) void moe_linear_few_kernel(const Exper
       }
       float o[4];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) o[r] = kGlu ? silu_of(z[0][r]) * z[kParts - 1][r] : z[0][r];
+      for (int r = 0; r < 4; ++r) o[r] = kGlu ? glu_of<kGlu>(a, z[0][r], z[kParts - 1][r]) : z[0][r];
       const int col = n0 + 16 * m + 4 * g;
       bf16_t* out = reinterpret_cast<bf16_t*>(a.out) + (int64_t)pair * a.out_stride + col;
       if (r0 + i16 < rows && col < (kGlu ? a.N / 2 : a.N)) *reinterpret_cast<uint2*>(out) = make_uint2(pack2<bf16_t>(o[0], o[1]), pack2<bf16_t>(o[2], o[3]));
@@ -296,7 +339,7 @@ __global__ __launch_bounds__(64 * kWaves) void moe_linear_few_kernel(const Exper
 }
 
 // any: workgroup = (16 outputs, expert, every gridDim.z-th 16 sorted rows), one dot product (two with the gate) per thread.
-template <typename T, bool kGlu>
+template <typename T, int kGlu>
 __global__ __launch_bounds__(256) void moe_linear_any_kernel(const ExpertLinearArgs a) {
   constexpr int kStep = 64, NT = kGlu ? 2 : 1;
   __shared__ float xs[16][kStep + 1], ws[NT][16][kStep + 1];
@@ -327,7 +370,12 @@ __global__ __launch_bounds__(256) void moe_linear_any_kernel(const ExpertLinearA
       __syncthreads();
     }
     if (base + r < last) {
-      const float o = kGlu ? acc[0] / (1.0f + expf(-acc[0])) * acc[NT - 1] : acc[0];
+      float o = acc[0];
+      if constexpr (kGlu == kSiluGlu) o = acc[0] / (1.0f + expf(-acc[0])) * acc[NT - 1];
+      if constexpr (kGlu == kClampedGlu) {
+        const float z = fminf(acc[0], a.limit);
+        o = z / (1.0f + expf(-a.alpha * z)) * (fminf(fmaxf(acc[NT - 1], -a.limit), a.limit) + a.shift);
+      }
       reinterpret_cast<T*>(a.out)[(int64_t)(base + r) * a.out_stride + n0 + c] = from_float<T>(o);
     }
   }
@@ -337,7 +385,7 @@ __global__ __launch_bounds__(256) void moe_linear_any_kernel(const ExpertLinearA
 // row operand and x the column operand, so that a lane ends with runs of four outputs of one row.  Steps of 64 along K, two
 // buffers in LDS that the copies of the next step fill during this one; a row's eight 16-byte chunks trade places by half
 // the row's number.  Consecutive workgroups of an XCD go through four row tiles for every weight tile.
-template <bool kGlu>
+template <int kGlu>
 __global__ __launch_bounds__(256, 2) void moe_linear_many_kernel(const ExpertLinearArgs a) {
   constexpr int kTile = 128, kK = 64, kStage = kTile * kK * 2;       // bytes of one operand's step
   constexpr int kTogether = 4;
@@ -422,7 +470,7 @@ __global__ __launch_bounds__(256, 2) void moe_linear_many_kernel(const ExpertLin
         const int col = (n0 + wn * 64) / 2 + 2 * r + 4 * hi;
         float o[4];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) o[i] = silu_of(acc[0][m][r + i]) * acc[1][m][r + i];
+        for (int i = 0; i < 4; ++i) o[i] = glu_of<kGlu>(a, acc[0][m][r + i], acc[1][m][r + i]);
         if (2 * col < a.N) *reinterpret_cast<uint2*>(out + col) = make_uint2(pack2<bf16_t>(o[0], o[1]), pack2<bf16_t>(o[2], o[3]));
       } else {
 #pragma unroll
@@ -441,7 +489,7 @@ __global__ __launch_bounds__(256, 2) void moe_linear_many_kernel(const ExpertLin
 // products of the one before; a step's last products hide the barrier, after which the next step's operands are there and
 // more copies start: x, which other workgroups of the XCD read too, one step ahead in two buffers, the weights, which come
 // from memory, two steps ahead in three.  Together they fill the LDS.
-template <bool kGlu>
+template <int kGlu>
 __global__ __launch_bounds__(256, 1) void moe_linear_large_kernel(const ExpertLinearArgs a) {
   constexpr int kTile = 256, kK = 64, kStage = kTile * kK * 2;       // bytes of one operand's step
   constexpr int kTogether = 4;
@@ -570,7 +618,10 @@ __global__ __launch_bounds__(256, 1) void moe_linear_large_kernel(const ExpertLi
       for (int r = 0; r < 16; r += 8) {
         float o[8];
 #pragma unroll
-        for (int i = 0; i < 8; ++i) o[i] = kGlu ? silu_of(acc[2 * n][m][r + i]) * acc[2 * n + 1][m][r + i] : acc[n][m][r + i];
+        for (int i = 0; i < 8; ++i) {
+          if constexpr (kGlu) o[i] = glu_of<kGlu>(a, acc[2 * n][m][r + i], acc[2 * n + 1][m][r + i]);
+          else o[i] = acc[n][m][r + i];
+        }
         const auto x = __builtin_amdgcn_permlane32_swap(pack2<bf16_t>(o[0], o[1]), pack2<bf16_t>(o[4], o[5]), false, false);
         const auto y = __builtin_amdgcn_permlane32_swap(pack2<bf16_t>(o[2], o[3]), pack2<bf16_t>(o[6], o[7]), false, false);
         const int col = (kGlu ? (n0 + wn * 128) / 2 : n0 + wn * 128) + 32 * n + 2 * r + 8 * hi;
@@ -589,25 +640,41 @@ static int plan_blocks(int64_t pairs) { return (int)((pairs + kPlanPairs - 1) / 
 
 using namespace mvllm;
 
+static int route(RouteArgs a, int64_t rows, void* stream) {
+  if (rows < 0 || a.experts <= 0 || a.top <= 0 || a.top > a.experts || a.groups <= 0 || a.experts % a.groups != 0 || a.keep <= 0 ||
+      a.keep > a.groups || a.z_stride < a.experts || (int64_t)a.keep * (a.experts / a.groups) < a.top || a.identity < 0 || a.identity > a.experts)
+    return MVLLM_ERR_BAD_SHAPE;
+  if (a.experts > kMaxExperts || a.top > 64 || a.groups > 64 || rows > (1 << 28)) return MVLLM_ERR_UNSUPPORTED;
+  if (rows == 0) return MVLLM_OK;
+  if (!a.ids || !a.weights || !a.z) return MVLLM_ERR_NULL_POINTER;
+  a.rows = (int)rows;
+  const dim3 grid((unsigned)((rows + 3) / 4)), block(256);
+  hipStream_t s = (hipStream_t)stream;
+  if (a.experts <= 64) moe_route_kernel<1><<<grid, block, 0, s>>>(a);
+  else if (a.experts <= 128) moe_route_kernel<2><<<grid, block, 0, s>>>(a);
+  else if (a.experts <= 256) moe_route_kernel<4><<<grid, block, 0, s>>>(a);
+  else moe_route_kernel<16><<<grid, block, 0, s>>>(a);
+  return launch_status();
+}
+
 extern "C" int mvllm_moe_route(int32_t* ids, float* weights, const float* logits, int64_t logit_row_stride,
                                const float* correction, int64_t rows, int experts, int top, int groups, int keep,
                                void* stream) {
-  if (rows < 0 || experts <= 0 || top <= 0 || top > experts || groups <= 0 || experts % groups != 0 || keep <= 0 || keep > groups ||
-      logit_row_stride < experts || (int64_t)keep * (experts / groups) < top)
-    return MVLLM_ERR_BAD_SHAPE;
-  if (experts > kMaxExperts || top > 64 || groups > 64 || rows > (1 << 28)) return MVLLM_ERR_UNSUPPORTED;
-  if (rows == 0) return MVLLM_OK;
-  if (!ids || !weights || !logits) return MVLLM_ERR_NULL_POINTER;
-  RouteArgs a;
+  RouteArgs a = {};
   a.ids = ids; a.weights = weights; a.z = logits; a.correction = correction; a.z_stride = logit_row_stride;
-  a.rows = (int)rows; a.experts = experts; a.top = top; a.groups = groups; a.keep = keep;
-  const dim3 grid((unsigned)((rows + 3) / 4)), block(256);
-  hipStream_t s = (hipStream_t)stream;
-  if (experts <= 64) moe_route_kernel<1><<<grid, block, 0, s>>>(a);
-  else if (experts <= 128) moe_route_kernel<2><<<grid, block, 0, s>>>(a);
-  else if (experts <= 256) moe_route_kernel<4><<<grid, block, 0, s>>>(a);
-  else moe_route_kernel<16><<<grid, block, 0, s>>>(a);
-  return launch_status();
+  a.experts = experts; a.top = top; a.groups = groups; a.keep = keep; a.renormalize = true;
+  return route(a, rows, stream);
+}
+
+extern "C" int mvllm_moe_route_softmax(int32_t* ids, float* weights, const float* logits, int64_t logit_row_stride,
+                                       const float* correction, int64_t rows, int experts, int identity, int top,
+                                       int renormalize, void* stream) {
+  if (experts < 0 || identity < 0 || experts > kMaxExperts || identity > kMaxExperts) return MVLLM_ERR_BAD_SHAPE;
+  RouteArgs a = {};
+  a.ids = ids; a.weights = weights; a.z = logits; a.correction = correction; a.z_stride = logit_row_stride;
+  a.experts = experts + identity; a.identity = identity; a.top = top; a.groups = 1; a.keep = 1; a.softmax = true;
+  a.renormalize = renormalize != 0;
+  return route(a, rows, stream);
 }
 
 extern "C" size_t mvllm_moe_plan_bytes(int64_t pairs, int experts) {
@@ -644,9 +711,16 @@ extern "C" int mvllm_moe_plan(void* plan, size_t plan_bytes, const int32_t* ids,
   return launch_status();
 }
 
-extern "C" int mvllm_moe_linear(void* out, int64_t out_row_stride, const void* x, int64_t x_row_stride, const void* w,
-                                const int32_t* ids, void* plan, int64_t pairs, int experts, int N, int K, int per_token,
-                                int glu, int dtype, void* stream) {
+// f(a kGlu as a constant)
+template <typename F> static void with_glu(int glu, F f) {
+  if (glu == kClampedGlu) f(std::integral_constant<int, kClampedGlu>{});
+  else if (glu == kSiluGlu) f(std::integral_constant<int, kSiluGlu>{});
+  else f(std::integral_constant<int, kNoGlu>{});
+}
+
+static int expert_linear(void* out, int64_t out_row_stride, const void* x, int64_t x_row_stride, const void* w,
+                         const int32_t* ids, void* plan, int64_t pairs, int experts, int N, int K, int per_token,
+                         int glu, float alpha, float limit, float shift, int dtype, void* stream) {
   if (dtype_size(dtype) == 0) return MVLLM_ERR_BAD_DTYPE;
   if (pairs < 0 || experts <= 0 || N <= 0 || K <= 0 || per_token < 0 || x_row_stride < K || out_row_stride < (glu ? N / 2 : N)) return MVLLM_ERR_BAD_SHAPE;
   if (dtype == MVLLM_F16 || experts > kMaxExperts || pairs > (1 << 30) || K % 64 != 0 || N % (glu ? 64 : 16) != 0 || x_row_stride % 8 != 0 ||
@@ -658,18 +732,17 @@ extern "C" int mvllm_moe_linear(void* out, int64_t out_row_stride, const void* x
   if (!plan && (dtype != MVLLM_BF16 || pairs > kFewPairs)) return MVLLM_ERR_UNSUPPORTED;
   ExpertLinearArgs a = {};
   a.out = out; a.x = x; a.w = w; a.ids = ids; a.x_stride = x_row_stride; a.out_stride = out_row_stride; a.pairs = (int)pairs;
-  a.experts = experts; a.N = N; a.K = K; a.per_token = per_token;
+  a.experts = experts; a.N = N; a.K = K; a.per_token = per_token; a.alpha = alpha; a.limit = limit; a.shift = shift;
   hipStream_t s = (hipStream_t)stream;
   const int outputs = glu ? N / 2 : N;
   if (!plan) {
     const unsigned n32 = (unsigned)((outputs + 31) / 32), n64 = (unsigned)((outputs + 63) / 64), n_experts = (unsigned)experts;
-    if (K >= 2048) {
-      if (glu) moe_linear_few_kernel<8, true, 2><<<dim3(n32, n_experts), dim3(512), 0, s>>>(a);
-      else moe_linear_few_kernel<8, false, 4><<<dim3(n64, n_experts), dim3(512), 0, s>>>(a);
-    } else {
-      if (glu) moe_linear_few_kernel<4, true, 2><<<dim3(n32, n_experts), dim3(256), 0, s>>>(a);
-      else moe_linear_few_kernel<4, false, 4><<<dim3(n64, n_experts), dim3(256), 0, s>>>(a);
-    }
+    with_glu(glu, [&](auto G) {
+      constexpr int kGlu = decltype(G)::value, kTiles = kGlu ? 2 : 4;
+      const dim3 grid(kGlu ? n32 : n64, n_experts);
+      if (K >= 2048) moe_linear_few_kernel<8, kGlu, kTiles><<<grid, dim3(512), 0, s>>>(a);
+      else moe_linear_few_kernel<4, kGlu, kTiles><<<grid, dim3(256), 0, s>>>(a);
+    });
     return launch_status();
   }
   const PlanArgs p = plan_parts_of(plan, ids, pairs, experts);
@@ -684,16 +757,30 @@ extern "C" int mvllm_moe_linear(void* out, int64_t out_row_stride, const void* x
     a.x_bytes = (uint32_t)x_bytes;
     const int64_t per = (a.max_tiles + 7) / 8, groups = (per + 3) / 4, blocks = 8 * groups * 4 * a.n_tiles;
     if (blocks > 0x7fffffff) return MVLLM_ERR_BAD_SHAPE;
-    if (p.tile_rows == 256) {
-      if (glu) moe_linear_large_kernel<true><<<dim3((unsigned)blocks), dim3(256), 0, s>>>(a);
-      else moe_linear_large_kernel<false><<<dim3((unsigned)blocks), dim3(256), 0, s>>>(a);
-    } else if (glu) moe_linear_many_kernel<true><<<dim3((unsigned)blocks), dim3(256), 0, s>>>(a);
-    else moe_linear_many_kernel<false><<<dim3((unsigned)blocks), dim3(256), 0, s>>>(a);
+    const bool large = p.tile_rows == 256;
+    with_glu(glu, [&](auto G) {
+      constexpr int kGlu = decltype(G)::value;
+      if (large) moe_linear_large_kernel<kGlu><<<dim3((unsigned)blocks), dim3(256), 0, s>>>(a);
+      else moe_linear_many_kernel<kGlu><<<dim3((unsigned)blocks), dim3(256), 0, s>>>(a);
+    });
   } else {
     int64_t z = pairs / (16 * (int64_t)experts) + 1;
     const dim3 grid((unsigned)(outputs / 16), (unsigned)experts, (unsigned)(z > 64 ? 64 : z));
-    if (glu) moe_linear_any_kernel<float, true><<<grid, dim3(256), 0, s>>>(a);
-    else moe_linear_any_kernel<float, false><<<grid, dim3(256), 0, s>>>(a);
+    with_glu(glu, [&](auto G) { moe_linear_any_kernel<float, decltype(G)::value><<<grid, dim3(256), 0, s>>>(a); });
   }
   return launch_status();
+}
+
+extern "C" int mvllm_moe_linear(void* out, int64_t out_row_stride, const void* x, int64_t x_row_stride, const void* w,
+                                const int32_t* ids, void* plan, int64_t pairs, int experts, int N, int K, int per_token,
+                                int glu, int dtype, void* stream) {
+  return expert_linear(out, out_row_stride, x, x_row_stride, w, ids, plan, pairs, experts, N, K, per_token, glu ? kSiluGlu : kNoGlu,
+                       0.f, 0.f, 0.f, dtype, stream);
+}
+
+extern "C" int mvllm_moe_linear_clamped(void* out, int64_t out_row_stride, const void* x, int64_t x_row_stride, const void* w,
+                                        const int32_t* ids, void* plan, int64_t pairs, int experts, int N, int K,
+                                        int per_token, float alpha, float limit, float shift, int dtype, void* stream) {
+  return expert_linear(out, out_row_stride, x, x_row_stride, w, ids, plan, pairs, experts, N, K, per_token, kClampedGlu, alpha, limit,
+                       shift, dtype, stream);
 }

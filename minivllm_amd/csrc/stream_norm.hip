@@ -3,7 +3,8 @@
 //     x'_t = sum_s mix[s, t] x_s + out[t] * y'           (all streams at once from the old ones, fp32)
 //     h    = rms(sum_t in[t] x'_t) * gain                (what the next sublayer reads; no `in`: the plain sum)
 // The sublayer's result is one row y, or what a mixture of experts leaves behind: the sum of `top` rows of `parts` with fp32
-// weights, and a row of a shared expert times the sigmoid of one number.  At the front of the model the streams start as
+// weights (a choice that is no expert counts with the row the mixture read), and a row of a shared expert times the sigmoid of
+// one number.  At the front of the model the streams start as
 // scaled embedding rows, with a second table indexed by a hash of the token and the one before it:
 //     e = embed[token] * embed_scale + bigram[(prev * mul_prev + token * mul_cur) mod buckets]
 // (a sequence's first token: row `buckets`).  The token before an entry's first row is part of the sequence's state.
@@ -24,6 +25,8 @@ struct StreamNormArgs {
   const void* parts;          // [*, part_stride] element type
   const int32_t* part_row;    // [T, top] rows of `parts`, or null: row t * top + k
   const float* weights;       // [T, top]
+  const int32_t* ids;         // [T, top] or null: a negative one stands for the mixture's input ...
+  const void* self;           // ... [T, self_stride] element type
   const float* gate;          // [T, gate_stride]: one logit per row for y, or null
   const float* scale;         // [W] or null
   const float* hc_out;        // [S]
@@ -41,7 +44,7 @@ struct StreamNormArgs {
   const int32_t* bank_in;     // [entries]
   const int32_t* bank_out;    // [entries]
   int64_t vocab, buckets, mul_prev, mul_cur;
-  int64_t out_stride, y_stride, part_stride, gate_stride;
+  int64_t out_stride, y_stride, part_stride, gate_stride, self_stride;
   float embed_scale, eps;
   int width, top;
 };
@@ -135,7 +138,9 @@ __global__ __launch_bounds__(kMaxThreads) void stream_norm_kernel(const StreamNo
           const int64_t from = a.part_row ? (int64_t)a.part_row[at] : at;
           const float w = a.weights[at];
           float p[VEC];
-          Chunk<T, VEC>::load(reinterpret_cast<const T*>(a.parts) + from * a.part_stride + chan[c], p);
+          const bool own = a.ids && a.ids[at] < 0;
+          const T* p_row = own ? reinterpret_cast<const T*>(a.self) + row * a.self_stride : reinterpret_cast<const T*>(a.parts) + from * a.part_stride;
+          Chunk<T, VEC>::load(p_row + chan[c], p);
 #pragma unroll
           for (int i = 0; i < VEC; ++i) sum[i] = fmaf(w, p[i], sum[i]);
         }
@@ -187,7 +192,7 @@ template <typename T, int S, int MODE>
 static int launch_stream_norm(const StreamNormArgs& a, int rows, hipStream_t stream) {
   const int n = sizeof(T) == 4 ? 4 : 8;            // rows of the element type start on 8 or 16 bytes
   const bool vec = a.width % 4 == 0 && (a.out_stride * (int64_t)sizeof(T)) % n == 0 && (a.y_stride * (int64_t)sizeof(T)) % n == 0 &&
-                   (a.part_stride * (int64_t)sizeof(T)) % n == 0 && aligned16(a.out) && aligned16(a.x_out) && aligned16(a.x) &&
+                   (a.part_stride * (int64_t)sizeof(T)) % n == 0 && (a.self_stride * (int64_t)sizeof(T)) % n == 0 && aligned16(a.self) && aligned16(a.out) && aligned16(a.x_out) && aligned16(a.x) &&
                    aligned16(a.y) && aligned16(a.parts) && aligned16(a.scale) && aligned16(a.gain) && aligned16(a.embed) && aligned16(a.bigram);
   const int chunks = vec ? a.width / 4 : a.width;
   // few rows: short threads; many: 256 threads with several chunks each, so that a row's loads overlap
@@ -257,26 +262,38 @@ extern "C" int mvllm_stream_embed_norm(void* out, int64_t out_row_stride, float*
                             : launch_streams<bf16_t, kFromEmbedding>(a, (int)rows, streams, s);
 }
 
-extern "C" int mvllm_stream_norm(void* out, int64_t out_row_stride, float* x_out, const float* x, const void* y,
-                                 int64_t y_row_stride, const void* parts, int64_t part_row_stride,
-                                 const int32_t* part_row, const float* weights, int top, const float* gate,
-                                 int64_t gate_row_stride, const float* scale, const float* hc_out, const float* hc_mix,
-                                 const float* hc_in, const float* gain, float eps, int64_t rows, int streams, int width,
-                                 int dtype, void* stream) {
+extern "C" int mvllm_stream_norm_identity(void* out, int64_t out_row_stride, float* x_out, const float* x, const void* y,
+                                          int64_t y_row_stride, const void* parts, int64_t part_row_stride,
+                                          const int32_t* part_row, const float* weights, int top, const int32_t* ids,
+                                          const void* self, int64_t self_row_stride, const float* gate,
+                                          int64_t gate_row_stride, const float* scale, const float* hc_out,
+                                          const float* hc_mix, const float* hc_in, const float* gain, float eps,
+                                          int64_t rows, int streams, int width, int dtype, void* stream) {
   const int st = check_common(out, out_row_stride, gain, rows, streams, width, dtype);
   if (st != MVLLM_OK) return st;
-  if ((y && y_row_stride < width) || (parts && (part_row_stride < width || top <= 0)) || (gate && gate_row_stride <= 0)) return MVLLM_ERR_BAD_SHAPE;
+  if ((y && y_row_stride < width) || (parts && (part_row_stride < width || top <= 0)) || (gate && gate_row_stride <= 0) || (ids && self_row_stride < width)) return MVLLM_ERR_BAD_SHAPE;
   if (rows == 0) return MVLLM_OK;
-  if (!x || !hc_out || !hc_mix || (!y && !parts) || (parts && !weights)) return MVLLM_ERR_NULL_POINTER;
+  if (!x || !hc_out || !hc_mix || (!y && !parts) || (parts && !weights) || (ids && !self)) return MVLLM_ERR_NULL_POINTER;
   StreamNormArgs a = {};
   a.out = out; a.out_stride = out_row_stride; a.x_out = x_out; a.x = x; a.y = y; a.y_stride = y_row_stride; a.parts = parts;
   a.part_stride = part_row_stride; a.part_row = part_row; a.weights = weights; a.top = top; a.gate = gate;
   a.gate_stride = gate_row_stride; a.scale = scale; a.hc_out = hc_out; a.hc_mix = hc_mix; a.hc_in = hc_in; a.gain = gain;
-  a.eps = eps; a.width = width;
+  a.eps = eps; a.width = width; a.ids = ids; a.self = self; a.self_stride = self_row_stride;
   hipStream_t s = (hipStream_t)stream;
   if (parts)
     return dtype == MVLLM_F32 ? launch_streams<float, kFromExperts>(a, (int)rows, streams, s)
                               : launch_streams<bf16_t, kFromExperts>(a, (int)rows, streams, s);
   return dtype == MVLLM_F32 ? launch_streams<float, kFromRow>(a, (int)rows, streams, s)
                             : launch_streams<bf16_t, kFromRow>(a, (int)rows, streams, s);
+}
+
+extern "C" int mvllm_stream_norm(void* out, int64_t out_row_stride, float* x_out, const float* x, const void* y,
+                                 int64_t y_row_stride, const void* parts, int64_t part_row_stride,
+                                 const int32_t* part_row, const float* weights, int top, const float* gate,
+                                 int64_t gate_row_stride, const float* scale, const float* hc_out, const float* hc_mix,
+                                 const float* hc_in, const float* gain, float eps, int64_t rows, int streams, int width,
+                                 int dtype, void* stream) {
+  return mvllm_stream_norm_identity(out, out_row_stride, x_out, x, y, y_row_stride, parts, part_row_stride, part_row, weights, top,
+                                    nullptr, nullptr, 0, gate, gate_row_stride, scale, hc_out, hc_mix, hc_in, gain, eps, rows, streams,
+                                    width, dtype, stream);
 }

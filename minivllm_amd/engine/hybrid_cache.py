@@ -3,7 +3,7 @@
 
 A window of ``size`` is chunked attention: a token sees the earlier tokens of its own chunk only, so a sequence needs the
 blocks of one chunk, and the next chunk overwrites them; token ``p`` lies at place ``p mod size`` of the table.  Window 0
-keeps everything.  Blocks come from the block pools of ``BlockManager``; prefixes are not shared (a recurrent state
+keeps everything.  A sliding window (engine/windows.py) is a ring of places in the same way.  Blocks come from the block pools of ``BlockManager``; prefixes are not shared (a recurrent state
 cannot be entered in the middle), so the pools are used without hashes.
 
 Same interface towards the scheduler as ``BlockManager``."""
@@ -13,18 +13,20 @@ from collections import deque
 
 from minivllm_amd.engine.block_manager import BlockManager
 from minivllm_amd.engine.sequence import Sequence
+from minivllm_amd.engine.windows import places
 
 
 class HybridCacheManager:
-    def __init__(self, windows: list[int], num_blocks: int, block_size: int, num_slots: int):
+    def __init__(self, windows: list, num_blocks: int, block_size: int, num_slots: int):
         self.windows = list(windows)
         self.block_size = block_size
         self.num_slots = num_slots
         self.pools = [BlockManager(num_blocks, block_size) for _ in self.windows]
         self.free_slots: deque[int] = deque(range(num_slots))
 
-    def blocks_for(self, window: int, tokens: int) -> int:
-        return -(-(min(tokens, window) if window else tokens) // self.block_size)
+    def blocks_for(self, window, tokens: int) -> int:
+        most = places(window)
+        return -(-(min(tokens, most) if most else tokens) // self.block_size)
 
     def _missing(self, seq: Sequence) -> list[int]:
         held = seq.group_tables or [[] for _ in self.windows]

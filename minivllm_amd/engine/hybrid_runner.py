@@ -1,4 +1,4 @@
-"""Runner of models that run ragged steps and keep recurrent state (models/sokevik.py, models/niridra.py): portions of
+"""Runner of models that run ragged steps and keep recurrent state (models/sokevik.py, models/niridra.py, models/fevosun.py): portions of
 prompts and decoded tokens in one batch, a cache manager of its own, and the captured decode step of ``ModelRunner`` over
 more static buffers.
 
@@ -10,7 +10,8 @@ import torch
 
 from minivllm_amd.engine.hybrid_cache import HybridCacheManager
 from minivllm_amd.engine.model_runner import _DTYPES, ModelRunner
-from minivllm_amd.engine.ragged import LatentStep, RaggedStep, WindowStep, ragged_step
+from minivllm_amd.engine.ragged import LatentStep, RaggedStep, RingStep, WindowStep, ragged_step
+from minivllm_amd.engine.windows import SlidingWindow, places
 from minivllm_amd.layers.fused import chunk_decode_step, lm_head_sample, lm_head_sample_takes, sample_tokens
 from minivllm_amd.utils.context import reset_context, set_context
 
@@ -114,19 +115,24 @@ class HybridModelRunner(ModelRunner):
         v = self.graph_vars
         lens, slots = [t[:bs] for t in v["chunk_lens"]], [t[:bs] for t in v["chunk_slots"]]
         tables = [t[:bs] for t in v["tables"]]
-        if self.model.latent_views:
-            windows = [LatentStep(absorbed=bs, slots=s, lens=n, tables=t) for s, n, t in zip(slots, lens, tables)]
-        else:
-            windows = [WindowStep(num_decode=bs, slots=s, chunk_lens=n, decode_tables=t) for s, n, t in zip(slots, lens, tables)]
+
+        def view(w, s, n, t):
+            if isinstance(w, SlidingWindow):
+                return RingStep(absorbed=bs, slots=s, lens=v["context_lens"][:bs], tables=t)
+            if self.model.latent_views:
+                return LatentStep(absorbed=bs, slots=s, lens=n, tables=t)
+            return WindowStep(num_decode=bs, slots=s, chunk_lens=n, decode_tables=t)
+
+        windows = [view(*of) for of in zip(self.model.windows, slots, lens, tables)]
         step = RaggedStep(num_tokens=bs, num_entries=bs, num_single=bs, num_short=bs, input_ids=v["input_ids"][:bs],
                           positions=v["positions"][:bs], cu_seqlens=v["cu_seqlens"][:bs + 1], row_entry=v["row_entry"][:bs],
                           bank_in=v["banks"][:bs], bank_out=v["banks"][:bs], state_slots=v["state_slots"][:bs], windows=windows)
         set_context(False, ragged=step)
 
         def prepare():
-            # where the rows' tokens lie in their chunks follows from the context lengths the step before left behind
+            # where the rows' tokens lie in their chunks (rings) follows from the context lengths the step before left behind
             for w, t, n, s in zip(self.model.windows, tables, lens, slots):
-                chunk_decode_step(v["context_lens"][:bs], t, w, self.block_size, n, s)
+                chunk_decode_step(v["context_lens"][:bs], t, places(w), self.block_size, n, s)
         return prepare
 
     def _fill_decode_buffers(self, seqs, gbs):

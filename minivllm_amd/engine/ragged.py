@@ -8,6 +8,8 @@ last chunk stay cached; where the entry also reads the chunk before, whose block
 attention (``late_slots``).
 Layers that cache one latent per token (``LatentStep``) answer single and short entries row by row from the cache; long
 entries with a cached prefix come before those without.
+Layers with a sliding window (``RingStep``) answer single and short entries row by row from their ring; long entries bring the
+last tokens of their past with them, taken out of the ring before the new ones go in.
 A recurrence takes single and short entries row by row and long ones in blocks of rows, cut into ``segments`` that run side
 by side where there are too few of them to fill the GPU."""
 from __future__ import annotations
@@ -17,6 +19,8 @@ from typing import Optional
 
 import numpy as np
 import torch
+
+from minivllm_amd.engine.windows import LONG_ROWS, SlidingWindow
 
 
 @dataclass
@@ -55,6 +59,23 @@ class LatentStep:
 
 
 @dataclass
+class RingStep:
+    """The step as layers with a sliding window see it: new tokens go to ``slots`` of the ring; rows of long entries find their
+    keys in a packed order, every entry's past in front of its own."""
+    absorbed: int = 0                                 # rows of single and short entries (the first ones)
+    num_long: int = 0                                 # rows of long entries, next
+    num_keys: int = 0                                 # packed keys of the long entries
+    slots: Optional[torch.Tensor] = None              # int64 [T], -1: overwritten by a later row of the step
+    lens: Optional[torch.Tensor] = None               # int64 [absorbed]: position + 1
+    tables: Optional[torch.Tensor] = None             # int32 [entries, width]
+    cu_q: Optional[torch.Tensor] = None               # int32 [long entries + 1]
+    cu_k: Optional[torch.Tensor] = None
+    key_rows: Optional[torch.Tensor] = None           # int64 [T]: packed place of a row's own key, -1 for absorbed rows
+    past_slots: Optional[torch.Tensor] = None         # int64 [n]: where the past of the long entries lies (None: no past) ...
+    past_rows: Optional[torch.Tensor] = None          # ... and its packed places
+
+
+@dataclass
 class RaggedStep:
     num_tokens: int
     num_entries: int
@@ -66,7 +87,7 @@ class RaggedStep:
     bank_in: torch.Tensor                             # int32 [entries]: banks of the short-convolution state
     bank_out: torch.Tensor
     state_slots: torch.Tensor                         # int32 [entries]
-    windows: list = field(default_factory=list)       # WindowStep (LatentStep) per window
+    windows: list = field(default_factory=list)       # WindowStep (LatentStep, RingStep) per window
     multi_rows: int = 0                               # rows of entries with more than one token
     num_short: int = 0                                # entries below LONG_ROWS (the first ones)
     segments: Optional[torch.Tensor] = None           # int32 [n, 4] of long entries: entry, first row, rows, flags
@@ -76,7 +97,6 @@ class RaggedStep:
     scratch: dict = field(default_factory=dict)       # what layers of one step share
 
 
-LONG_ROWS = 32                 # an entry of at least this many rows is long
 BLOCK_ROWS = 64                # rows per block of a recurrence's block form: segments are whole blocks
 FILL_WORKGROUPS = 512          # segments are made shorter until there are this many workgroups ...
 MIN_SEGMENT_ROWS = 256         # ... but not shorter than this
@@ -206,6 +226,40 @@ def _latent_arrays(items, index, block_size, cu, num_short):
     return out, counts
 
 
+def _ring_arrays(items, window, index, block_size, cu, num_short):
+    """Host arrays of a RingStep; items as for ``_window_arrays``."""
+    total = int(cu[-1])
+    slots, key_rows = np.full(total, -1, dtype=np.int64), np.full(total, -1, dtype=np.int64)
+    cu_q, cu_k, past_slots, past_rows = [0], [0], [], []
+    for e, (p0, n, seq) in enumerate(items):
+        table = np.asarray(seq.group_tables[index], dtype=np.int64)
+
+        def slots_of(positions):
+            place = positions % window.places if window.places else positions
+            return table[place // block_size] * block_size + place % block_size
+
+        stay = min(n, window.places) if window.places else n
+        slots[cu[e + 1] - stay:cu[e + 1]] = slots_of(np.arange(p0 + n - stay, p0 + n))
+        if e < num_short:
+            continue
+        past = min(p0, window.size - 1) if window.size else p0
+        if past:
+            past_slots.append(slots_of(np.arange(p0 - past, p0)))
+            past_rows.append(cu_k[-1] + np.arange(past))
+        key_rows[cu[e]:cu[e + 1]] = cu_k[-1] + past + np.arange(n)
+        cu_q.append(cu_q[-1] + n)
+        cu_k.append(cu_k[-1] + past + n)
+    absorbed = int(cu[num_short])
+    out = dict(slots=slots, tables=_pad_tables([seq.group_tables[index] for _, _, seq in items]))
+    if absorbed:
+        out["lens"] = np.concatenate([np.arange(p, p + n, dtype=np.int64) + 1 for p, n, _ in items[:num_short]])
+    if len(cu_q) > 1:
+        out.update(cu_q=np.asarray(cu_q, dtype=np.int32), cu_k=np.asarray(cu_k, dtype=np.int32), key_rows=key_rows)
+    if past_slots:
+        out.update(past_slots=np.concatenate(past_slots), past_rows=np.concatenate(past_rows).astype(np.int64))
+    return out, dict(absorbed=absorbed, num_long=cu_q[-1], num_keys=cu_k[-1])
+
+
 def ragged_arrays(seqs, windows, block_size, memory_units=0, latent=False):
     """Host side of a step over ``seqs``: each runs its tokens [num_computed_tokens, + num_scheduled_tokens).  Returns
     (arrays, window arrays, window counts, facts), everything in numpy; the sequences' convolution banks flip for entries
@@ -228,7 +282,8 @@ def ragged_arrays(seqs, windows, block_size, memory_units=0, latent=False):
                   bank_in=np.asarray(bank_in, dtype=np.int32), bank_out=np.asarray(bank_out, dtype=np.int32),
                   state_slots=np.asarray([s.state_slot for _, _, s in items], dtype=np.int32))
     num_short = int((lens < LONG_ROWS).sum())
-    per_window = [_latent_arrays(items, g, block_size, cu, num_short) if latent else _window_arrays(items, w, g, block_size, cu)
+    per_window = [_ring_arrays(items, w, g, block_size, cu, num_short) if isinstance(w, SlidingWindow) else
+                  _latent_arrays(items, g, block_size, cu, num_short) if latent else _window_arrays(items, w, g, block_size, cu)
                   for g, w in enumerate(windows)]
     starts = [0] * len(seqs)
     for e, i in enumerate(order):
@@ -244,7 +299,7 @@ def ragged_arrays(seqs, windows, block_size, memory_units=0, latent=False):
 
 def ragged_step(seqs, windows, block_size, device, memory_units=0, latent=False) -> RaggedStep:
     """The step's device tensors: one copy per integer type, every tensor a 16-byte aligned slice of it.  ``latent``: the
-    windows' views are LatentSteps."""
+    views of windows that are plain numbers are LatentSteps."""
     arrays, window_arrays, counts, facts = ragged_arrays(seqs, windows, block_size, memory_units, latent)
     named = [((None, k), a) for k, a in arrays.items()]
     for g, wa in enumerate(window_arrays):
@@ -263,6 +318,6 @@ def ragged_step(seqs, windows, block_size, device, memory_units=0, latent=False)
         dev = host.to(device, non_blocking=True)
         for (key, a), at in zip(mine, offsets):
             placed[key] = dev[at:at + a.size].view(a.shape)
-    view = LatentStep if latent else WindowStep
-    ws = [view(**counts[g], **{k: placed[(g, k)] for k in wa}) for g, wa in enumerate(window_arrays)]
+    views = [RingStep if isinstance(w, SlidingWindow) else LatentStep if latent else WindowStep for w in windows]
+    ws = [views[g](**counts[g], **{k: placed[(g, k)] for k in wa}) for g, wa in enumerate(window_arrays)]
     return RaggedStep(windows=ws, **{k: placed[(None, k)] for k in arrays}, **facts)

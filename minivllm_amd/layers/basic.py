@@ -92,15 +92,26 @@ def rotary_pair_table(base: float, dims: int, max_position: int, scaling: dict |
     """float32 (max_position, dims / 2, 2): cos and sin of position * base^(-2 i / dims), angles in double precision.
 
     ``scaling`` (``factor``, ``low``, ``high``, ``original``) stretches the slow pairs: wavelengths beyond original / low
-    by ``factor``, those below original / high not at all, a blend linear in original / wavelength between them."""
+    by ``factor``, those below original / high not at all, a blend linear in original / wavelength between them.  With
+    ``fast`` and ``slow`` instead (YaRN) the blend is linear in the pair's number, between the pairs that turn ``fast`` and
+    ``slow`` times over the original context, and cos and sin are multiplied by 0.1 ln(factor) + 1."""
     freq = float(base) ** (-torch.arange(0, dims, 2, dtype=torch.float64) / dims)
-    if scaling is not None:
+    amplitude = 1.0
+    if scaling is not None and "fast" in scaling:
+        def pair_of(turns):
+            return dims * math.log(scaling["original"] / (2 * math.pi * turns)) / (2 * math.log(base))
+
+        lo, hi = max(math.floor(pair_of(scaling["fast"])), 0), min(math.ceil(pair_of(scaling["slow"])), dims - 1)
+        stretch = ((torch.arange(dims // 2, dtype=torch.float64) - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+        freq = freq / scaling["factor"] * stretch + freq * (1.0 - stretch)
+        amplitude = 0.1 * math.log(scaling["factor"]) + 1.0
+    elif scaling is not None:
         turns = scaling["original"] * freq / (2 * math.pi)                 # of a pair over the original context
         keep = ((turns - scaling["low"]) / (scaling["high"] - scaling["low"])).clamp(0.0, 1.0) if (
             scaling["high"] != scaling["low"]) else (turns > scaling["high"]).double()
         freq = (1.0 - keep) * freq / scaling["factor"] + keep * freq
     angle = torch.outer(torch.arange(max_position, dtype=torch.float64), freq)
-    return torch.stack([angle.cos(), angle.sin()], dim=-1).float().contiguous()
+    return (torch.stack([angle.cos(), angle.sin()], dim=-1) * amplitude).float().contiguous()
 
 
 class SiluAndMul(nn.Module):

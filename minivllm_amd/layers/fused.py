@@ -12,13 +12,15 @@ LM-head output, with the Exp(1) noise drawn inside the kernel (Philox4x32-10) or
 """
 from __future__ import annotations
 
+import math
+
 import torch
 
 from minivllm_amd import _C
 
 __all__ = ["qk_norm_rope_store", "sample_tokens", "sample_tokens_into", "decode_advance", "add_rms_norm", "silu_and_mul", "linear_small_m", "linear_small_m_takes", "norm_linear_small_m", "norm_linear_small_m_takes",
            "lm_head_sample", "lm_head_sample_takes", "lm_head_sample_workspace_bytes", "norm_conv", "head_rope_store",
-           "head_unrotate_gate", "chunk_decode_step", "stream_embed_norm", "stream_norm"]
+           "head_unrotate_gate", "chunk_decode_step", "stream_embed_norm", "stream_norm", "gated_unit"]
 
 
 def _ptr(t):
@@ -252,6 +254,24 @@ def silu_and_mul(x: torch.Tensor) -> torch.Tensor:
         st = lib.mvllm_silu_and_mul(_ptr(out), _ptr(x), rows, two_w // 2, stride, _C.dtype_code(x.dtype),
                                     _C.current_stream_ptr(x.device))
         _C.check(st, "silu_and_mul")
+    return out
+
+
+def gated_unit(x: torch.Tensor, out: torch.Tensor | None = None, alpha: float = 1.0, limit: float = math.inf,
+               shift: float = 0.0) -> torch.Tensor:
+    """g sigmoid(alpha g) (u + shift) of the halves of x's rows, g at most ``limit`` and u within +-``limit``; rows of x and
+    ``out`` may be strided.  By default silu(g) * u, rounded once."""
+    _C.require_cuda(x, out)
+    rows, width = x.shape[0], x.shape[1] // 2
+    if x.dim() != 2 or x.shape[1] % 2 or x.stride(1) != 1:
+        raise ValueError("x must be (rows, 2 * width) with dense rows")
+    if out is None:
+        out = torch.empty((rows, width), dtype=x.dtype, device=x.device)
+    if tuple(out.shape) != (rows, width) or out.dtype != x.dtype or out.stride(1) != 1:
+        raise ValueError(f"out must be ({rows}, {width}) in x's dtype with dense rows")
+    st = _C.load().mvllm_gated_unit(_ptr(out), out.stride(0) if rows > 1 else width, _ptr(x), x.stride(0) if rows > 1 else 2 * width, rows,
+                                    width, float(alpha), float(limit), float(shift), _C.dtype_code(x.dtype), _C.current_stream_ptr(x.device))
+    _C.check(st, "gated_unit")
     return out
 
 
@@ -567,10 +587,10 @@ def stream_norm(x: torch.Tensor, y, hc_out: torch.Tensor, hc_mix: torch.Tensor, 
 
     x float32 (T, streams, W); y (T, >= W) with dense rows, or a mixture's unsummed results (``layers.experts.ExpertOutput``);
     everything else float32.  Returns (the norm, x)."""
-    parts = part_row = weights = gate = None
+    parts = part_row = weights = gate = ids = own = None
     if not isinstance(y, torch.Tensor):
-        parts, part_row, weights, gate, y = y.parts, y.part_row, y.weights, y.gate, y.shared
-    _C.require_cuda(x, y, parts, part_row, weights, gate, hc_out, hc_mix, gain, hc_in, scale)
+        parts, part_row, weights, gate, ids, own, y = y.parts, y.part_row, y.weights, y.gate, y.ids, y.inputs, y.shared
+    _C.require_cuda(x, y, parts, part_row, weights, gate, ids, own, hc_out, hc_mix, gain, hc_in, scale)
     rows, streams, width = x.shape
     padded = max(padded, width)
     _check(x, torch.float32, (rows, streams, width), "x")
@@ -593,11 +613,15 @@ def stream_norm(x: torch.Tensor, y, hc_out: torch.Tensor, hc_mix: torch.Tensor, 
             raise ValueError("parts and part_row must have one row per choice")
         if gate is not None and (gate.dtype != torch.float32 or gate.numel() != rows):
             raise ValueError("gate must be float32, one number per row")
+        if ids is not None:
+            _check(ids, torch.int32, (rows, top), "ids")
+            if own.dtype != dtype or own.dim() != 2 or own.shape[0] != rows or own.shape[1] < width or own.stride(1) != 1:
+                raise ValueError(f"inputs must be ({rows}, >= {width}) in {dtype} with dense rows")
     out = torch.empty((rows, padded), dtype=dtype, device=x.device)
-    st = _C.load().mvllm_stream_norm(
+    st = _C.load().mvllm_stream_norm_identity(
         _ptr(out), padded, _ptr(x if want_x else None), _ptr(x), _ptr(y), 0 if y is None else max(y.stride(0), width), _ptr(parts),
-        0 if parts is None else max(parts.stride(0), width), _ptr(part_row), _ptr(weights), top, _ptr(gate),
-        1 if gate is None else max(gate.stride(0), 1), _ptr(scale), _ptr(hc_out), _ptr(hc_mix), _ptr(hc_in), _ptr(gain), float(eps),
+        0 if parts is None else max(parts.stride(0), width), _ptr(part_row), _ptr(weights), top, _ptr(ids),
+        _ptr(own), 0 if own is None else max(own.stride(0), width), _ptr(gate), 1 if gate is None else max(gate.stride(0), 1), _ptr(scale), _ptr(hc_out), _ptr(hc_mix), _ptr(hc_in), _ptr(gain), float(eps),
         rows, streams, width, _C.dtype_code(dtype), _C.current_stream_ptr(x.device))
     _C.check(st, "stream_norm")
     return out, x

@@ -2,7 +2,8 @@
 memories.
 
 ``RaggedAttention`` runs a step's pieces through the framework's decode, paged-prefill and packed-prefill kernels,
-``LatentAttention`` through the latent decode and the same prefill kernels; ``MatrixMemory`` runs it through the mLSTM
+``LatentAttention`` through the latent decode and the same prefill kernels, ``SharedKeyAttention`` and ``RotaryLatentAttention``
+through the windowed kernels; ``MatrixMemory`` runs it through the mLSTM
 recurrence, ``DecayMemory`` through the one with constant decays.  ``RaggedAttention`` and the memories take the packed
 projection of the step's rows and return what the output projection reads.  Caches and states are assigned from outside, as
 for ``layers.attention.Attention``."""
@@ -20,7 +21,10 @@ from minivllm_amd.layers.fused import head_rope_store, head_unrotate_gate
 from minivllm_amd.layers.basic import Linear
 from minivllm_amd.layers.latent import (head_linear, latent_decode, latent_decode_workspace_bytes, latent_norm_store,
                                         latent_width)
+from minivllm_amd.layers.window import (copy_rows, head_rope, head_size, latent_layout, latent_rope_store, shared_part_size,
+                                        window_decode, window_decode_workspace_bytes, window_prefill)
 from minivllm_amd.layers.recurrent import DecayMemoryState, MlstmState, decay_memory, gate_linear, gated_row_norm, mlstm
+from minivllm_amd.engine.windows import SlidingWindow
 from minivllm_amd.utils.padding import pad_heads, pad_to, round_up
 
 LOG2E = math.log2(math.e)
@@ -188,3 +192,153 @@ class LatentAttention(nn.Module):
             k, v = (F.linear(rows[b:], w).view(-1, heads, d) for w in (self.up_k, self.up_v))
             flash_attention_prefill(q[b:], k, v, view.fresh_cu, *shape, out=o[b:])
         return self.out(o.view(t, heads * d))
+
+
+def distance_slopes(heads: int) -> torch.Tensor:
+    """2^(-8 (h + 1) / heads) of head h, float32."""
+    return (2.0 ** (-8.0 * torch.arange(1, heads + 1, dtype=torch.float64) / heads)).float()
+
+
+class SharedKeyAttention(nn.Module):
+    """Grouped softmax attention in a sliding window whose values are the keys, without a rotation: ``slopes`` times the distance is
+    taken off a score, ``temperature`` = (coef, every) makes scores grow with the query's position, a gate per channel follows.
+
+    It works between two projections that it may share with other sublayers: ``forward`` reads columns q | k | gate of ``proj`` and
+    writes ``out`` (T, H * head_dim).  ``sizes``: columns it needs of both; ``window``: index into the step's windows."""
+
+    def __init__(self, num_heads, num_kv_heads, dim, scale, window, view: SlidingWindow, block_size, dtype, temperature=(0.0, 0),
+                 slopes=None, gated=True):
+        super().__init__()
+        self.num_heads, self.num_kv_heads, self.dim, self.scale = num_heads, num_kv_heads, dim, scale
+        self.window, self.view, self.block_size, self.dtype = window, view, block_size, dtype
+        self.temperature, self.slopes, self.gated = temperature, slopes, gated
+        d = self.head_dim = head_size(dim)
+        self.q_size, self.k_size = num_heads * d, num_kv_heads * d
+        self.sizes = (self.q_size + self.k_size + (self.q_size if gated else 0), self.q_size)
+        self.cache = torch.tensor([])                                     # (blocks, block_size, G, head_dim)
+        self.decode_workspace = None
+
+    def load(self, get, matrix, inputs):
+        """``get(name)``: checkpoint tensor, ``matrix(t)``: on the device in the model's type.  Returns this sublayer's rows of the
+        projection in front of it and its columns of the one behind."""
+        d, rows = self.head_dim, [("q", self.num_heads), ("k", self.num_kv_heads)] + [("g", self.num_heads)] * self.gated
+        front = torch.cat([pad_heads(matrix(get(n)), h, d, inputs) for n, h in rows])
+        if self.slopes is not None:
+            self.slopes = self.slopes.to(front.device)
+        return front, pad_heads(matrix(get("o")).t().contiguous(), self.num_heads, d).t()
+
+    def allocate(self, num_blocks, device):
+        self.cache = torch.zeros(num_blocks, self.block_size, self.num_kv_heads, self.head_dim, dtype=self.dtype, device=device)
+
+    def workspace_bytes(self, batch, table_width):
+        return window_decode_workspace_bytes(batch, self.num_heads, self.num_kv_heads, self.head_dim, self.head_dim,
+                                             table_width * self.block_size, self.dtype)
+
+    def forward(self, h, proj, out, step):
+        view, heads, groups, d = step.windows[self.window], self.num_heads, self.num_kv_heads, self.head_dim
+        a = view.absorbed
+        q, k, o = proj[:, :self.q_size].unflatten(-1, (heads, d)), proj[:, self.q_size:self.q_size + self.k_size], out.unflatten(-1, (heads, d))
+        gate = proj[:, self.q_size + self.k_size:self.sizes[0]].unflatten(-1, (heads, d)) if self.gated else None
+        cut = lambda t, *rows: None if t is None else t[slice(*rows)]
+        places, keys, key_rows, cu_k = self.cache.view(-1, self.k_size), None, None, view.cu_q
+        if view.past_slots is not None:                                   # the past comes out of the ring before the new keys go in
+            keys, key_rows, cu_k = torch.empty((view.num_keys, self.k_size), dtype=k.dtype, device=k.device), view.key_rows, view.cu_k
+            copy_rows(places, keys, view.past_rows, view.past_slots)
+        copy_rows(k, places, view.slots, None, keys, key_rows)
+        how = dict(slopes=self.slopes, temperature=self.temperature)
+        if a:
+            window_decode(o[:a], q[:a], self.cache, view.tables, step.row_entry, view.lens, self.scale, self.view.size, self.view.places,
+                          gate=cut(gate, 0, a), workspace=self.decode_workspace, **how)
+        if view.num_long:
+            keys = k[a:] if keys is None else keys
+            window_prefill(o[a:], q[a:], keys.unflatten(-1, (groups, d)), view.cu_q, cu_k, self.scale, self.view.size,
+                           gate=cut(gate, a, None), positions=step.positions[a:], **how)
+
+
+class RotaryLatentAttention(nn.Module):
+    """Softmax attention in a sliding window over keys and values made of one cached latent per token, with a rotated part of the
+    keys beside it that all heads share.  Queries come from the input, or from a normed latent of their own (``q_rank``).
+
+    Single rows and short entries are answered from the latents (queries through the heads' key matrices, results through their
+    value matrices), for long entries keys and values are made of them.  It works between two projections like
+    ``SharedKeyAttention``: columns q (or the queries' latent) | latent | rotated part.  ``table``: float32
+    (max_position, dims / 2, 2), assigned from outside."""
+
+    def __init__(self, num_heads, dim, rot_dim, vdim, rank, scale, window, view: SlidingWindow, block_size, dtype, eps, interleaved,
+                 q_rank=0, small_rows=0):
+        super().__init__()
+        self.num_heads, self.dim, self.rot_dim, self.vdim, self.rank, self.scale = num_heads, dim, rot_dim, vdim, rank, scale
+        self.window, self.view, self.block_size, self.dtype, self.eps = window, view, block_size, dtype, eps
+        self.interleaved, self.q_rank = interleaved, q_rank
+        d, self.rot_size = head_size(dim, vdim), shared_part_size(rot_dim)
+        self.head_dim, self.q_dim = d, d + self.rot_size
+        self.rot_column, self.latent_width, self.values = latent_layout(rank, rot_dim)
+        self.q_size = num_heads * self.q_dim
+        self.q_columns = round_up(q_rank, 64) if q_rank else self.q_size
+        self.sizes = (self.q_columns + self.latent_width, num_heads * d)
+        if q_rank:
+            with torch.device("meta"):
+                self.up_q = Linear(self.q_columns, self.q_size, bias=False, small_rows=small_rows)
+        self.table = None
+        self.cache = torch.tensor([])                                     # (blocks, block_size, 1, latent_width)
+        self.decode_workspace = None
+
+    @torch.no_grad()
+    def load(self, get, matrix, inputs):
+        """As ``SharedKeyAttention.load``."""
+        heads, d, r = self.num_heads, self.head_dim, self.rot_dim
+
+        def query_rows(t, columns):                                       # (H * (dim + rot_dim), n): both parts filled up
+            t = matrix(t)
+            w = t.new_zeros(heads, self.q_dim, columns)
+            of = t.view(heads, self.dim + r, -1)
+            w[:, :self.dim, :t.shape[1]], w[:, d:d + r, :t.shape[1]] = of[:, :self.dim], of[:, self.dim:]
+            return w.view(heads * self.q_dim, columns)
+
+        down = matrix(get("dkv"))
+        latent = down.new_zeros(self.latent_width, inputs)
+        latent[:self.rank, :down.shape[1]], latent[self.rot_column:self.rot_column + r, :down.shape[1]] = down[:self.rank], down[self.rank:]
+        f32 = lambda name: get(name).to(device=down.device, dtype=torch.float32).contiguous()
+        self.norm_weight, self.q_norm_weight = f32("dkv.norm"), None
+        if self.q_rank:
+            self.q_norm_weight = f32("dq.norm")
+            self.up_q.weight = nn.Parameter(query_rows(get("uq"), self.q_columns), requires_grad=False)
+            first = pad_to(matrix(get("dq")), self.q_columns, inputs)
+        else:
+            first = query_rows(get("q"), inputs)
+        uk, uv = (pad_heads(matrix(get(n)), heads, d, self.rot_column) for n in ("uk", "uv"))       # (H * D, latent columns)
+        self.up_kv = torch.cat([uk, uv])
+        self.absorb_k = uk.view(heads, d, -1).transpose(1, 2).contiguous()
+        self.absorb_v = pad_to(uv, None, self.values)[:, :self.values].contiguous().view(heads, d, self.values)
+        return torch.cat([first, latent]), pad_heads(matrix(get("o")).t().contiguous(), heads, d).t()
+
+    def allocate(self, num_blocks, device):
+        self.cache = torch.zeros(num_blocks, self.block_size, 1, self.latent_width, dtype=self.dtype, device=device)
+
+    def workspace_bytes(self, batch, table_width):
+        return window_decode_workspace_bytes(batch, self.num_heads, 1, self.latent_width, self.values, table_width * self.block_size, self.dtype)
+
+    def forward(self, h, proj, out, step):
+        view, heads, d, w, rot = step.windows[self.window], self.num_heads, self.head_dim, self.latent_width, self.rot_column
+        t, a, new = proj.shape[0], view.absorbed, lambda *shape: torch.empty(shape, dtype=proj.dtype, device=proj.device)
+        cache, rows, key_rows = self.cache.view(-1, self.block_size, w), None, None
+        if view.num_long:
+            rows, key_rows = new(view.num_keys, w), view.key_rows
+            if view.past_slots is not None:                               # out of the ring before the new latents go in
+                copy_rows(cache.view(-1, w), rows, view.past_rows, view.past_slots)
+        first, latents = proj[:, :self.q_columns], proj[:, self.q_columns:self.sizes[0]]
+        c_q = latent_rope_store(latents, self.norm_weight, self.eps, rot, self.rot_dim, self.table, step.positions, self.interleaved,
+                                cache, view.slots, rows, key_rows, first if self.q_rank else None, self.q_norm_weight)
+        q = (self.up_q(c_q) if self.q_rank else first).unflatten(-1, (heads, self.q_dim))
+        x = new(a, heads, w) if a else None
+        head_rope(q, d, self.rot_dim, self.table, step.positions, self.interleaved, x, rot, a)
+        o = out.unflatten(-1, (heads, d))
+        if a:
+            y = new(a, heads, self.values)
+            head_linear(q[:a, :, :d], self.absorb_k, out=x[:, :, :rot])
+            window_decode(y, x, self.cache, view.tables, step.row_entry, view.lens, self.scale, self.view.size, self.view.places,
+                          workspace=self.decode_workspace)
+            head_linear(y, self.absorb_v, out=o[:a])
+        if view.num_long:
+            k, v = F.linear(rows[:, :rot], self.up_kv).unflatten(-1, (2, heads, d)).unbind(1)
+            window_prefill(o[a:], q[a:], k, view.cu_q, view.cu_k, self.scale, self.view.size, k2=rows[:, rot:rot + self.rot_size], v=v)

@@ -54,8 +54,25 @@ def _niridra_sources(config):
     return kernel_sources(config)
 
 
+def _fevosun_runner(config):
+    from minivllm_amd.engine.hybrid_runner import HybridModelRunner
+    from minivllm_amd.models.fevosun import FevosunForCausalLM
+    return HybridModelRunner(config, FevosunForCausalLM)
+
+
+def _fevosun_normalize(config):
+    from minivllm_amd.models.fevosun import engine_config
+    return engine_config(config)
+
+
+def _fevosun_sources(config):
+    from minivllm_amd.models.fevosun import kernel_sources
+    return kernel_sources(config)
+
+
 DESIGNS = {"Qwen3": Design(_qwen3_runner), "Sokevik": Design(_sokevik_runner, _sokevik_normalize, _sokevik_sources),
-           "Niridra": Design(_niridra_runner, _niridra_normalize, _niridra_sources)}
+           "Niridra": Design(_niridra_runner, _niridra_normalize, _niridra_sources),
+           "Fevosun": Design(_fevosun_runner, _fevosun_normalize, _fevosun_sources)}
 
 
 def design_of(config: dict) -> Design:

@@ -39,6 +39,8 @@ def test_header_declares_expected_entry_points():
               "mvllm_decay_memory_chunked_workspace_bytes", "mvllm_gated_row_norm", "mvllm_latent_norm_store",
               "mvllm_head_linear", "mvllm_latent_decode", "mvllm_latent_decode_workspace_bytes", "mvllm_moe_route",
               "mvllm_moe_plan", "mvllm_moe_plan_bytes", "mvllm_moe_linear",
+              "mvllm_moe_route_softmax", "mvllm_moe_linear_clamped", "mvllm_gated_unit", "mvllm_stream_norm_identity", "mvllm_window_prefill",
+              "mvllm_window_decode_workspace_bytes", "mvllm_window_decode", "mvllm_latent_rope_store", "mvllm_head_rope", "mvllm_copy_rows",
               "mvllm_silu_and_mul", "mvllm_version", "mvllm_status_string"]:
         assert n in names
 
