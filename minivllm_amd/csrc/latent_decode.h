@@ -391,15 +391,17 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const LatentDecodeArg
   const float w = x.x == -INFINITY ? 0.f : exp2f(x.x - m);
   const float l = wave_sum(w * x.y);
   const float f = l > 0.f ? w / l : 0.f;
-  for (int c = 4 * lane; c < a.values; c += 256) {
+  for (int c0 = 0; c0 < a.values; c0 += 256) {      // every lane goes round as often: the shares' factors come from all of them
+    const int c = c0 + 4 * lane;
+    const bool mine = c < a.values;
     float o[4] = {0.f, 0.f, 0.f, 0.f};
     for (int p = 0; p < a.parts; ++p) {
       const float g = __shfl(f, p, 64);
       if (g == 0.f) continue;                       // empty shares have left nothing (uniform over the wave)
-      const float4 v = *reinterpret_cast<const float4*>(a.part_o + ((row * a.parts + p) * a.heads + h) * a.values + c);
+      const float4 v = *reinterpret_cast<const float4*>(a.part_o + ((row * a.parts + p) * a.heads + h) * a.values + (mine ? c : 0));
       o[0] = fmaf(g, v.x, o[0]); o[1] = fmaf(g, v.y, o[1]); o[2] = fmaf(g, v.z, o[2]); o[3] = fmaf(g, v.w, o[3]);
     }
-    finish4<T, kWindowed>(a, row, h, c, o);
+    if (mine) finish4<T, kWindowed>(a, row, h, c, o);
   }
 }
 

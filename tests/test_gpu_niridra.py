@@ -317,6 +317,15 @@ def test_latent_decode(dtype, padded, heads):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("padded", [32, 64, 96])
+def test_latent_decode_joins_many_shares_of_narrow_rows(dtype, padded):
+    """More shares than the pass that joins them has lanes with columns."""
+    q, cache, tables, entry, lengths, rows = latent_case(padded, [5000, 3, 2049], 2, padded, dtype, 16)
+    got = latent_decode(q.to(DEV), cache.to(DEV), tables.to(DEV), entry.to(DEV), lengths.to(DEV), 0.2)
+    assert row_rel(got, latent_reference(q, rows, 0.2)) < tol(dtype, 1e-5, 1.5e-2)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("padded,heads", [(96, 4), (512, 32), (160, 3)])
 def test_latent_decode_finds_single_keys(dtype, padded, heads):
     """One score stands out: first and last keys, both sides of page and tile borders, far back; one past the end never."""
