@@ -38,7 +38,7 @@ def parse_args():
     ap.add_argument("--warmup", type=int, default=5)
     ap.add_argument("--seed", type=int, default=0)
     ap.add_argument("--block-size", type=int, default=16, help="block size of the headline decode workload")
-    ap.add_argument("--only", default="", help="comma list out of decode256,prefill,prefill_long,store,int8,reference_shapes,decode_small,demo_shape,head_dims,fused_qk,sampler,mfma_probe,prefill_timeline,loads_probe,engine,engine16,engine64,cpu to restrict the extras (the headline decode always runs); only when named: sokevik, the Sokevik design beside the Qwen3-style decoder, models and kernels (sokevik_kernels: kernels alone), niridra, the Niridra design beside Sokevik (niridra_kernels)")
+    ap.add_argument("--only", default="", help="comma list out of decode256,prefill,prefill_long,store,int8,reference_shapes,decode_small,demo_shape,head_dims,fused_qk,sampler,mfma_probe,prefill_timeline,loads_probe,engine,engine16,engine64,cpu to restrict the extras (the headline decode always runs); only when named: sokevik, the Sokevik design beside the Qwen3-style decoder, models and kernels (sokevik_kernels: kernels alone), niridra, the Niridra design beside Sokevik (niridra_kernels), fevosun, the Fevosun design beside Niridra (fevosun_kernels)")
     ap.add_argument("--no-cpu", action="store_true", help="skip the cpu_baseline leg")
     ap.add_argument("--calib-copy", action="store_true",
                     help="also launch three 1 GiB device copies (reads 1 GiB, writes 1 GiB each) so a rocprofv3 "
@@ -1304,6 +1304,184 @@ def bench_niridra_kernels(args, rows, calls):
     return res
 
 
+
+FEVOSUN_WINDOW, FEVOSUN_ROT, FEVOSUN_IDENTITY = 1024, 64, 8
+
+
+def fevosun_model(size):
+    """Fevosun with its three mixers in turn (attention every second layer), of the width, heads, layers, latents and experts of
+    ``niridra_model``, some identity experts beside them."""
+    z, e = SOKEVIK_SIZES[size], NIRIDRA_SIZES[size]
+    mlp = {"kind": "moe", "expert": {"ff": e["ff"], "limit": 7.0}, "shared": {"ff": e["shared"], "limit": 7.0},
+           "router": {"experts": e["experts"], "identity": FEVOSUN_IDENTITY, "top": e["top"]}}
+    mask, rot = {"size": FEVOSUN_WINDOW}, {"base": 1e6, "dims": FEVOSUN_ROT}
+    attention = {"type": "attention", "mlp": mlp, "mixer": {"heads": z["heads"], "kv_heads": z["kv"], "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                                                            "mask": mask, "q_temp": {"coef": 0.1, "every": 8192}}}
+    m = {"heads": z["heads"], "dim": 128, "rot_dim": FEVOSUN_ROT, "vdim": 128, "kv_rank": NIRIDRA_RANK, "scale": 192 ** -0.5, "mask": mask}
+    yarn = {**rot, "scaling": {"factor": 8.0, "fast": 32.0, "slow": 1.0, "original": 4096}}
+    latents = [{"type": "latent_attention", "mlp": mlp, "mixer": {**m, "rot": yarn}},
+               {"type": "latent_attention_2", "mlp": mlp, "mixer": {**m, "rot": rot, "q_rank": 3 * z["width"] // 8}}]
+    return {"architecture": "Fevosun", "width": z["width"], "vocab": 32000, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+            "layers": [attention if i % 2 == 0 else latents[i // 2 % 2] for i in range(z["layers"])]}
+
+
+def bench_fevosun(args, with_models=True):
+    """The Fevosun design beside Niridra, the nearest other design (latents and mixtures of experts), at equal width, heads, layers
+    and experts: whole-engine throughput, and every kernel beside the like kernel."""
+    import torch
+    out = {"models": {}, "kernels": {}}
+    for size in NIRIDRA_SIZES if with_models else ():
+        for prompts, prompt_len, new in ((4, 2048, 128), (32, 512, 128), (1, 16384, 64)):
+            leg = {}
+            for name, config in (("fevosun", fevosun_model(size)), ("niridra", niridra_model(size))):
+                leg[name] = engine_throughput(args, config, prompts, prompt_len, new)
+                torch.cuda.empty_cache()
+            out["models"][f"{size}_{prompts}x{prompt_len}+{new}"] = leg
+            print(f"{size} {prompts}x{prompt_len}+{new}: {leg}", file=sys.stderr, flush=True)
+    for rows, calls in ((8192, 4), (64, 20)):
+        with torch.inference_mode():
+            out["kernels"][f"{rows}_rows"] = bench_fevosun_kernels(args, rows, calls)
+        torch.cuda.empty_cache()
+    return out
+
+
+def bench_fevosun_kernels(args, rows, calls):
+    """Kernels at width 4096: 8192 prompt rows (8 prompts of 1024, or one), or 64 decoded rows (attention: 256 sequences of 1024
+    tokens in the window)."""
+    import torch
+    from minivllm_amd.engine.hybrid_cache import HybridCacheManager
+    from minivllm_amd.engine.ragged import ragged_step
+    from minivllm_amd.engine.sequence import Sequence
+    from minivllm_amd.engine.windows import SlidingWindow
+    from minivllm_amd.layers.attention import flash_attention_prefill, paged_attention_decode, store_kvcache
+    from minivllm_amd.layers.basic import rotary_pair_table
+    from minivllm_amd.layers.experts import ExpertOutput, moe_linear, moe_plan, moe_route, moe_route_softmax
+    from minivllm_amd.layers.fused import gated_unit, head_rope_store, silu_and_mul, stream_norm
+    from minivllm_amd.layers.latent import latent_decode, latent_norm_store
+    from minivllm_amd.layers.mixers import distance_slopes
+    from minivllm_amd.layers.window import copy_rows, head_rope, latent_layout, latent_rope_store, window_decode, window_prefill
+
+    dev = torch.device("cuda:0")
+    gen = torch.Generator(device=dev).manual_seed(args.seed)
+    rnd = lambda *shape, dtype=torch.bfloat16: torch.randn(*shape, generator=gen, device=dev).to(dtype)
+    f32 = lambda *shape: torch.ones(*shape, device=dev)
+    prefill = rows > 64
+    width, hq, hkv, d, rot, rank, window, bs = 4096, 32, 8, 128, FEVOSUN_ROT, NIRIDRA_RANK, FEVOSUN_WINDOW, 16
+    e = NIRIDRA_SIZES["w4096"]
+    experts, top, ff, shared = e["experts"], e["top"], e["ff"], e["shared"]
+    view = SlidingWindow(window)
+
+    def step_of(lengths, before):
+        m = HybridCacheManager([view], sum(-(-min(n + p, view.places) // bs) for n, p in zip(lengths, before)), bs, len(lengths))
+        seqs = []
+        for n, p0 in zip(lengths, before):
+            q = Sequence([0] * (p0 + n), block_size=bs)
+            m.allocate(q)
+            q.num_computed_tokens, q.num_scheduled_tokens = p0, n
+            seqs.append(q)
+        return ragged_step(seqs, [view], bs, dev), sum(len(p.blocks) for p in m.pools)
+
+    lengths = [window] * (rows // window) if prefill else [1] * rows
+    step, blocks = step_of(lengths, [0] * len(lengths) if prefill else [window - 1] * rows)
+    res = {}
+    leg = kernel_legs(args, res, calls)
+    scale, slopes = d ** -0.5, distance_slopes(hq).to(dev)
+    rot_column, latent_width, values = latent_layout(rank, rot)
+
+    # ---- attention ----
+    if prefill:
+        pairs = sum(n * (n + 1) // 2 for n in lengths)
+        cu = step.windows[0].cu_q
+        q, k, gate, out = rnd(rows, hq, d), rnd(rows, hkv, d), rnd(rows, hq, d), torch.empty(rows, hq, d, dtype=torch.bfloat16, device=dev)
+        vg, flops = rnd(rows, hkv, d), 4.0 * hq * d * pairs
+        like = lambda: flash_attention_prefill(q, k, vg, cu, scale, hq, hkv, d)
+        like_bytes, moved = rows * (2 * hq + 2 * hkv) * d * 2, rows * (3 * hq + hkv) * d * 2
+        run = lambda c: window_prefill(out, q, k, c, c, scale, window, gate=gate, slopes=slopes, positions=step.positions, temperature=(0.1, 8192))
+        leg("window_prefill", lambda: run(cu), moved, like, "packed prefill, 8 kv heads", like_bytes, flops, flops)
+        whole = torch.tensor([0, rows], dtype=torch.int32, device=dev)
+        seen = window * (window + 1) // 2 + (rows - window) * window
+        leg("window_prefill_one_prompt", lambda: run(whole), moved, like, "packed prefill, 8 kv heads", like_bytes, 4.0 * hq * d * seen, flops)
+        qr, k1, k2, v, vl = rnd(rows, hq, d + rot), rnd(rows, hq, d), rnd(rows, rot), rnd(rows, hq, d), rnd(rows, hq, d)
+        parts = lambda c: window_prefill(out, qr, k1, c, c, 192 ** -0.5, window, k2=k2, v=v)
+        moved, like_bytes = rows * (hq * (4 * d + rot) + rot) * 2, rows * 4 * hq * d * 2
+        like = lambda: flash_attention_prefill(q, k1, vl, cu, scale, hq, hq, d)
+        leg("window_prefill_latents", lambda: parts(cu), moved, like, "packed prefill, 32 kv heads", like_bytes, 2.0 * hq * (2 * d + rot) * pairs, flops)
+        leg("window_prefill_latents_one_prompt", lambda: parts(whole), moved, like, "packed prefill, 32 kv heads", like_bytes,
+            2.0 * hq * (2 * d + rot) * seen, flops)
+        del q, k, gate, out, vg, qr, k1, k2, v, vl
+    else:
+        for name, tokens, batch in (("", window, 256), ("_16_rows", window, 16)):
+            st, n = step_of([1] * batch, [tokens - 1] * batch)
+            w = st.windows[0]
+            ring, gate, q = rnd(n, bs, hkv, d), rnd(batch, hq, d), rnd(batch, hq, d)
+            kc, vc = rnd(batch * tokens // bs, bs, hkv, d), rnd(batch * tokens // bs, bs, hkv, d)
+            plain, lens = w.tables[:, :tokens // bs].contiguous() % (batch * tokens // bs), w.lens
+            out = torch.empty(batch, hq, d, dtype=torch.bfloat16, device=dev)
+            leg("window_decode" + name, lambda: window_decode(out, q, ring, w.tables, st.row_entry, lens, scale, window, view.places, gate=gate, slopes=slopes,
+                                                               temperature=(0.1, 8192)),
+                batch * (tokens * hkv * d * 2 + 3 * hq * d * 2 + 4 * tokens // bs),
+                lambda: paged_attention_decode(q, kc, vc, plain, lens, scale, hq, hkv, d, bs), "paged decode, 8 kv heads",
+                batch * (tokens * 2 * hkv * d * 2 + 2 * hq * d * 2 + 4 * tokens // bs))
+            del kc, vc, ring
+            cache, x = rnd(n, bs, 1, latent_width), rnd(batch, hq, latent_width)
+            y, x2, cache2 = torch.empty(batch, hq, values, dtype=torch.bfloat16, device=dev), rnd(batch, hq, rank), rnd(n, bs, rank)
+            # the absorbed products are arithmetic too: 2 H (width + values) flop per key
+            leg("window_decode_latents" + name, lambda: window_decode(y, x, cache, w.tables, st.row_entry, lens, scale, window, view.places),
+                batch * (tokens * latent_width * 2 + hq * (latent_width + values) * 2),
+                lambda: latent_decode(x2, cache2, w.tables, st.row_entry, lens, scale), "latent_decode",
+                batch * (tokens * rank * 2 + 2 * hq * rank * 2), 2.0 * batch * tokens * hq * (latent_width + values), 4.0 * batch * tokens * hq * rank)
+            del cache, x, y, x2, cache2
+    # ---- around attention: latents and keys into the ring, rotated queries ----
+    table, slots = rotary_pair_table(1e6, rot, 2048).to(dev), step.windows[0].slots
+    c, c0, gain = rnd(rows, latent_width), rnd(rows, rank), f32(rank)
+    cache, cache0 = torch.zeros(blocks, bs, latent_width, dtype=torch.bfloat16, device=dev), torch.zeros(blocks, bs, rank, dtype=torch.bfloat16, device=dev)
+    packed = torch.empty(rows, latent_width, dtype=torch.bfloat16, device=dev) if prefill else None
+    key_rows = step.windows[0].key_rows
+    copies = 3 if prefill else 2
+    leg("latent_rope_store", lambda: latent_rope_store(c, gain, 1e-6, rot_column, rot, table, step.positions, False, cache, slots, packed, key_rows),
+        rows * (latent_width * 2 * copies + 8), lambda: latent_norm_store(c0, gain, 1e-6, cache0, slots, need_rows=prefill), "latent_norm_store",
+        rows * (rank * 2 * copies + 8))
+    q = rnd(rows, hq, d + rot)
+    first = 0 if prefill else rows
+    x = torch.empty(rows, hq, latent_width, dtype=torch.bfloat16, device=dev) if first else None
+    cols = (hq + 2 * hkv) * d
+    proj, kc = rnd(rows, cols), torch.zeros(blocks, bs, hkv, d, dtype=torch.bfloat16, device=dev)
+    vc = torch.zeros_like(kc)
+    leg("head_rope", lambda: head_rope(q, d, rot, table, step.positions, False, x, rot_column, first), rows * hq * rot * 4,
+        lambda: head_rope_store(proj, step.positions, hq, hkv, d, d, d, None, None, 1e-6, 1.0, None, None, True, None, slots, kc, vc, need_kv=False),
+        "head_rope_store", rows * (2 * cols + (hq + 2 * hkv) * d * 2 + 16))
+    keys = proj[:, hq * d:hq * d + hkv * d]
+    kd, vd = rnd(rows, hkv, d), rnd(rows, hkv, d)
+    leg("copy_rows", lambda: copy_rows(keys, kc.view(-1, hkv * d), slots), rows * (2 * hkv * d * 2 + 8),
+        lambda: store_kvcache(kd, vd, kc, vc, slots, bs), "store_kvcache", rows * (4 * hkv * d * 2 + 8))
+    del c, c0, cache, cache0, q, x, proj, kc, vc
+    # ---- feed-forwards and residual ----
+    act = rnd(rows, 2 * shared)
+    wide = torch.empty(rows, hq * d + shared, dtype=torch.bfloat16, device=dev)
+    leg("gated_unit", lambda: gated_unit(act, wide[:, hq * d:], 1.702, 7.0, 1.0), rows * shared * 6, lambda: silu_and_mul(act), "silu_and_mul", rows * shared * 6)
+    h, y = rnd(rows, width), rnd(rows, width)
+    logits = rnd(rows, experts + FEVOSUN_IDENTITY, dtype=torch.float32)
+    correction = torch.zeros(experts + FEVOSUN_IDENTITY, device=dev)
+    plain_logits, plain_correction = logits[:, :experts].contiguous(), torch.zeros(experts, device=dev)
+    leg("moe_route_softmax", lambda: moe_route_softmax(logits, correction, experts, FEVOSUN_IDENTITY, top), rows * (4 * (experts + FEVOSUN_IDENTITY) + 8 * top),
+        lambda: moe_route(plain_logits, plain_correction, experts, top, 8, 4), "moe_route", rows * (4 * experts + 8 * top))
+    ids, weights = moe_route_softmax(logits, correction, experts, FEVOSUN_IDENTITY, top)
+    plain_ids, _ = moe_route(plain_logits, plain_correction, experts, top, 8, 4)
+    plan, plain_plan = moe_plan(ids, experts), moe_plan(plain_ids, experts)
+    w_up, pairs, all_pairs = rnd(experts, 2 * ff, width), int((ids >= 0).sum()), rows * top
+    used = [int(torch.unique(t[t >= 0]).numel()) for t in (ids, plain_ids)]
+    leg("moe_linear_clamped", lambda: moe_linear(h, w_up, ids, plan, top, glu=(1.702, 7.0, 1.0)), used[0] * 2 * ff * width * 2 + rows * width * 2 + pairs * ff * 2,
+        lambda: moe_linear(h, w_up, plain_ids, plain_plan, top, glu=True), "moe_linear", used[1] * 2 * ff * width * 2 + rows * width * 2 + all_pairs * ff * 2,
+        4.0 * pairs * ff * width, 4.0 * all_pairs * ff * width)
+    del w_up
+    one, gains, xs = f32(1), f32(width), rnd(rows, 1, width, dtype=torch.float32)
+    parts = rnd(all_pairs, width)
+    mine, plain = ExpertOutput(parts, weights, plan.place, y, None, ids, h), ExpertOutput(parts, weights, plain_plan.place, y)
+    moved = rows * width * 12 + 4 * width
+    leg("stream_norm_identity", lambda: stream_norm(xs, mine, one, one[None], gains, 1e-6), moved + all_pairs * (2 * width + 12),
+        lambda: stream_norm(xs, plain, one, one[None], gains, 1e-6), "stream_norm (experts)", moved + all_pairs * (2 * width + 8))
+    return res
+
 def summary_of(line):
     """The figures of every quantity the metric names, in a few hundred characters, for the end of the JSON line."""
     ex = line["extra"]
@@ -1415,6 +1593,10 @@ def main():
         extra["niridra"] = bench_niridra(args)
     elif "niridra_kernels" in only:
         extra["niridra"] = bench_niridra(args, with_models=False)
+    if "fevosun" in only:
+        extra["fevosun"] = bench_fevosun(args)
+    elif "fevosun_kernels" in only:
+        extra["fevosun"] = bench_fevosun(args, with_models=False)
 
     if "loads_only" in head:
         extra["decode_loads_only"] = head["loads_only"]

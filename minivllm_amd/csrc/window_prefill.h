@@ -8,9 +8,11 @@
 //
 // bf16 (tiles): workgroup = 4 waves = one kv head x HPW of its query heads x 32-row query tiles; 64-key tiles in LDS, two
 // buffers, filled by copies that run during the other one's products; Sᵀ = K Qᵀ, Oᵀ += Vᵀ Pᵀ on v_mfma_f32_32x32x16_bf16, one
-// query row per lane (as in prefill_mfma.h).  Values that are the keys are read from the keys' tile.  The distance bias is one
-// more 16-dim step of the first product: the keys' side holds a key's place in its tile and the tile's distance (small integers,
-// exact), the queries' side the slope as a sum of three bf16 numbers; what is constant for a row drops out of the softmax.
+// query row per lane (as in prefill_mfma.h).  Values that are the keys are read from the keys' tile.  The first product has one
+// more 16-dim step, whose operands are made in registers: against ones on the keys' side the row's negated running maximum as a
+// sum of three bf16 numbers (scores leave the matrix unit as exp2 arguments, and the accumulators start from nothing), and for
+// the distance bias, against a key's place in its tile and the tile's distance (small integers, exact), the slope in the same
+// way; what is constant for a row drops out of the softmax.
 #pragma once
 #include "prefill_tiles.h"
 
@@ -57,6 +59,19 @@ template <int RC> struct Chunks {
 };
 
 constexpr int kWinKeys = 64;       // keys per tile
+
+// Copies of a part of a tile, a quarter per wave, 1 KB per instruction.  Where rows divide an instruction the four waves take
+// turns, so that a lane's place in a row repeats every sixteen rows: copy i starts from offset i % kStarts and goes on by whole
+// rows, which is one number for all lanes.
+template <int RC> struct Copies {
+  static constexpr int kCount = RC / 4;
+  static constexpr bool kEven = 64 % RC == 0;
+  static constexpr int kRows = kEven ? 256 / RC : 0;                          // rows the four waves copy at once
+  static constexpr int kStarts = !kEven ? kCount : kRows >= 16 ? 1 : 16 / kRows;
+  static __device__ __forceinline__ int chunk(int i, int wave, int lane) { return (kEven ? 4 * i + wave : wave * kCount + i) * 64 + lane; }
+  static constexpr int lds(int i) { return (kEven ? 4 * i : i) * 1024; }      // behind the wave's first
+  static constexpr int kWave = (kEven ? 1 : kCount) * 1024;
+};
 constexpr int kWinRows = 32;       // query rows per wave
 
 // KS1, KS2: 16-dim steps of the two parts of the keys; TD: 32-dim blocks of the values; SHARED: values are the keys (the form
@@ -98,23 +113,26 @@ __global__ __launch_bounds__(256, KS1 > 8 ? 1 : 2) void window_prefill_kernel(co
   const int j_first = max(0, pos0 - W + 1) / kWinKeys, j_last = min(pos0 + kWinRows - 1, kv_len - 1) / kWinKeys;
   const int wg_first = max(0, cached + row0 - W + 1) / kWinKeys, wg_last = (cached + min(row0 + BM, seq_len) - 1) / kWinKeys;
 
-  // ---- copies: a quarter of every part of a tile per wave, 1 KB per instruction ----
-  constexpr int n1 = RC1 / 4, n2 = KS2 > 0 ? RC2 / 4 : 0, nv = SHARED ? 0 : RCV / 4;
-  uint32_t off1[n1], off2[n2 > 0 ? n2 : 1], offv[nv > 0 ? nv : 1];
+  // ---- copies ----
+  using C1 = Copies<RC1>;
+  using C2 = Copies<RC2>;
+  using CV = Copies<RCV>;
+  constexpr int n1 = C1::kCount, n2 = KS2 > 0 ? C2::kCount : 0, nv = SHARED ? 0 : CV::kCount;
+  uint32_t off1[C1::kStarts], off2[C2::kStarts], offv[CV::kStarts];
   const uint32_t row1 = (uint32_t)(a.k_row * 2), row2 = (uint32_t)(a.k2_row * 2), rowv = (uint32_t)(a.v_row * 2);
 #pragma unroll
-  for (int i = 0; i < n1; ++i) {
-    const int c = (wave * n1 + i) * 64 + lane, row = c / RC1;
+  for (int i = 0; i < C1::kStarts; ++i) {
+    const int c = C1::chunk(i, wave, lane), row = c / RC1;
     off1[i] = (uint32_t)row * row1 + (uint32_t)(((c % RC1) ^ swz1(row)) << 4);
   }
 #pragma unroll
-  for (int i = 0; i < n2; ++i) {
-    const int c = (wave * n2 + i) * 64 + lane, row = c / RC2;
+  for (int i = 0; i < C2::kStarts; ++i) {
+    const int c = C2::chunk(i, wave, lane), row = c / RC2;
     off2[i] = (uint32_t)row * row2 + (uint32_t)(((c % RC2) ^ Chunks<RC2>::keys(row)) << 4);
   }
 #pragma unroll
-  for (int i = 0; i < nv; ++i) {
-    const int c = (wave * nv + i) * 64 + lane, row = c / RCV;
+  for (int i = 0; i < CV::kStarts; ++i) {
+    const int c = CV::chunk(i, wave, lane), row = c / RCV;
     offv[i] = (uint32_t)row * rowv + (uint32_t)(((c % RCV) ^ swzv(row)) << 4);
   }
   const char* k_base = reinterpret_cast<const char*>(a.k) + ((int64_t)k_start * a.k_row + (int64_t)g * a.k_head) * 2;
@@ -137,9 +155,15 @@ __global__ __launch_bounds__(256, KS1 > 8 ? 1 : 2) void window_prefill_kernel(co
   auto copy = [&](const Source& s, auto C, int buffer) __attribute__((always_inline)) {
     constexpr int c = decltype(C)::value;
     const uint32_t base = lds_base + (uint32_t)(buffer * kBuffer);
-    if constexpr (c < n1) dma16_to_lds<c * 1024>(s.k, off1[c], base + (uint32_t)(wave * n1 * 1024));
-    else if constexpr (c < n1 + n2) dma16_to_lds<kTile1 + (c - n1) * 1024>(s.k2, off2[c - n1], base + (uint32_t)(wave * n2 * 1024));
-    else dma16_to_lds<kTile1 + kTile2 + (c - n1 - n2) * 1024>(s.v, offv[c - n1 - n2], base + (uint32_t)(wave * nv * 1024));
+    auto go = [&](auto PART, auto I, auto REGION, v4i rsrc, const uint32_t* off, uint32_t row_bytes) __attribute__((always_inline)) {
+      using P = decltype(PART);
+      constexpr int i = decltype(I)::value, behind = P::kEven ? i / P::kStarts * P::kStarts * P::kRows : 0;       // rows behind the start
+      dma16_to_lds_at<decltype(REGION)::value + P::lds(i)>(rsrc, off[i % P::kStarts], (uint32_t)behind * row_bytes, base + (uint32_t)(wave * P::kWave));
+    };
+    using std::integral_constant;
+    if constexpr (c < n1) go(C1{}, integral_constant<int, c>{}, integral_constant<int, 0>{}, s.k, off1, row1);
+    else if constexpr (c < n1 + n2) go(C2{}, integral_constant<int, c - n1>{}, integral_constant<int, kTile1>{}, s.k2, off2, row2);
+    else go(CV{}, integral_constant<int, c - n1 - n2>{}, integral_constant<int, kTile1 + kTile2>{}, s.v, offv, rowv);
   };
   constexpr int kCopies = n1 + n2 + nv;
   {
@@ -165,64 +189,66 @@ __global__ __launch_bounds__(256, KS1 > 8 ? 1 : 2) void window_prefill_kernel(co
   }
 #pragma unroll
   for (int ks = 0; ks < KS1 + KS2; ++ks) asm volatile("" ::"v"(qf[ks].x), "v"(qf[ks].w));   // retired before the copies are counted
-  // the bias step: slope times (place in the tile - 64 * tiles up to the wave's last one)
-  uint4 q_bias = make_uint4(0u, 0u, 0u, 0u);
+  // the further step: lanes of the first half hold the slope times (place in the tile - 64 * tiles up to the wave's last one),
+  // the others the running maximum
+  uint4 q_more = make_uint4(0u, 0u, 0u, 0u);
   if constexpr (SHARED) {
     const float s = a.slopes ? a.slopes[h] * kLog2e : 0.f;
     const float s0 = to_float(from_float<bf16_t>(s)), s1 = to_float(from_float<bf16_t>(s - s0)), s2 = s - s0 - s1;
     if (hi == 0)
-      q_bias = make_uint4(pack2<bf16_t>(s0, s1), pack2<bf16_t>(s2, -64.f * s0), pack2<bf16_t>(-64.f * s1, -64.f * s2),
+      q_more = make_uint4(pack2<bf16_t>(s0, s1), pack2<bf16_t>(s2, -64.f * s0), pack2<bf16_t>(-64.f * s1, -64.f * s2),
                           pack2<bf16_t>(-16384.f * s0, -16384.f * s1));
-    else q_bias.x = pack2<bf16_t>(-16384.f * s2, 0.f);
   }
+  const uint32_t ones = hi ? 0x3f803f80u : 0u;       // keys' side of the maximum: 1, 1, 1
 
-  v16f o[TD], neg_m;
+  v16f o[TD];
 #pragma unroll
   for (int td = 0; td < TD; ++td)
 #pragma unroll
     for (int r = 0; r < 16; ++r) o[td][r] = 0.f;
-  // running maximum of the lane's row, negated, as the C operand of the scores' first product (prefill_mfma.h)
-#pragma unroll
-  for (int r = 0; r < 16; ++r) neg_m[r] = 0.f;
+  float m = 0.f;                                     // running maximum of the lane's row
   bool fresh = true;                                 // the row has seen no key yet
   float l = 0.f;
 
-  // ---- places of this lane's operands in a buffer ----
-  constexpr int kOffs1 = Chunks<RC1>::kBits / 2, kOffs2 = Chunks<RC2>::kBits / 2, kOffsV = Chunks<RCV>::kBits / 4;
-  int k_off[kOffs1], k2_off[kOffs2], v_off[kOffsV];
-#pragma unroll
-  for (int i = 0; i < kOffs1; ++i) k_off[i] = l32 * kRow1 + (((2 * i + hi) ^ swz1(l32)) << 4);
-#pragma unroll
-  for (int i = 0; i < kOffs2; ++i) k2_off[i] = kTile1 + l32 * kRow2 + (((2 * i + hi) ^ Chunks<RC2>::keys(l32)) << 4);
-  const int i16 = lane & 15, half = (lane >> 4) & 1, v_row = 4 * hi + (i16 >> 2);
-#pragma unroll
-  for (int i = 0; i < kOffsV; ++i)
-    v_off[i] = (SHARED ? 0 : kTile1 + kTile2) + v_row * kRowV + (((4 * i + 2 * half + ((i16 & 3) >> 1)) ^ swzv(v_row)) << 4) + ((i16 & 1) << 3);
+  // ---- places of this lane's operands in a buffer: chunks of one row differ by an xor (and whole groups of chunks) ----
+  constexpr int kGroup1 = Chunks<RC1>::kBits, kGroup2 = Chunks<RC2>::kBits, kGroupV = Chunks<RCV>::kBits;
+  auto lds16 = [](uint32_t at) __attribute__((always_inline)) { return *reinterpret_cast<const __attribute__((address_space(3))) u32x4*>(at); };
 
   auto tile_step = [&](int j, auto MASKED, int buffer, bool prefetch) __attribute__((always_inline)) {
     constexpr bool masked = decltype(MASKED)::value;
     const Source next = source(j + 1, prefetch);
-    const char* buf = lds + buffer * kBuffer;
+    // worked out anew for every tile: kept, they would be the registers that do not fit
+    int ln = lane;
+    asm volatile("" : "+v"(ln));
+    const int l32 = ln & 31, hi = ln >> 5, i16 = ln & 15, half = (ln >> 4) & 1, v_row = 4 * hi + (i16 >> 2);
+    const uint32_t base = lds_base + (uint32_t)(buffer * kBuffer);
+    const uint32_t k_at = base + l32 * kRow1 + ((hi ^ swz1(l32)) << 4);
+    const uint32_t k2_at = base + kTile1 + l32 * kRow2 + ((hi ^ Chunks<RC2>::keys(l32)) << 4);
+    const uint32_t v_at = base + (SHARED ? 0 : kTile1 + kTile2) + v_row * kRowV + (((2 * half + ((i16 & 3) >> 1)) ^ swzv(v_row)) << 4) + ((i16 & 1) << 3);
     v16f s[2];
+    const v16f nothing = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
     if constexpr (SHARED) {
       const int tt = j_last - j;
       const float t0 = (float)(tt & 255), t1 = (float)(tt >> 8);
 #pragma unroll
       for (int tk = 0; tk < 2; ++tk) {
         const float at = (float)(l32 + 32 * tk);
-        const uint4 kb = hi == 0 ? make_uint4(pack2<bf16_t>(at, at), pack2<bf16_t>(at, t0), pack2<bf16_t>(t0, t0), pack2<bf16_t>(t1, t1))
-                                 : make_uint4(pack2<bf16_t>(t1, 0.f), 0u, 0u, 0u);
-        s[tk] = mfma32x32x16<bf16_t>(kb, q_bias, neg_m);
+        const uint4 k_more = make_uint4(hi ? ones : pack2<bf16_t>(at, at), hi ? ones & 0xffffu : pack2<bf16_t>(at, t0), pack2<bf16_t>(t0, t0), pack2<bf16_t>(t1, t1));
+        s[tk] = mfma32x32x16<bf16_t>(k_more, q_more, nothing);
       }
+    } else {
+      const uint4 k_more = make_uint4(ones, ones & 0xffffu, 0u, 0u);
+      s[0] = mfma32x32x16<bf16_t>(k_more, q_more, nothing);
+      s[1] = mfma32x32x16<bf16_t>(k_more, q_more, nothing);
     }
     // ---- scores: fragments one step ahead of the products, a copy of the next tile behind every step ----
     constexpr int KS = KS1 + KS2;
     auto k_frag = [&](auto K, int tk) __attribute__((always_inline)) {
-      constexpr int ks = decltype(K)::value;
-      if constexpr (ks < KS1)
-        return *reinterpret_cast<const uint4*>(buf + k_off[ks % kOffs1] + (ks / kOffs1) * (Chunks<RC1>::kBits * 16) + tk * 32 * kRow1);
-      else
-        return *reinterpret_cast<const uint4*>(buf + k2_off[(ks - KS1) % kOffs2] + ((ks - KS1) / kOffs2) * (Chunks<RC2>::kBits * 16) + tk * 32 * kRow2);
+      constexpr int ks = decltype(K)::value, k2 = ks - KS1;
+      u32x4 x;
+      if constexpr (ks < KS1) x = lds16((k_at ^ (32u * (ks % (kGroup1 / 2)))) + 16 * kGroup1 * (ks / (kGroup1 / 2)) + tk * 32 * kRow1);
+      else x = lds16((k2_at ^ (32u * (k2 % (kGroup2 / 2)))) + 16 * kGroup2 * (k2 / (kGroup2 / 2)) + tk * 32 * kRow2);
+      return make_uint4(x[0], x[1], x[2], x[3]);
     };
     uint4 kf[2][2];
 #pragma unroll
@@ -235,7 +261,7 @@ __global__ __launch_bounds__(256, KS1 > 8 ? 1 : 2) void window_prefill_kernel(co
         __builtin_amdgcn_sched_barrier(0);
       }
 #pragma unroll
-      for (int tk = 0; tk < 2; ++tk) s[tk] = mfma32x32x16<bf16_t>(kf[ks & 1][tk], qf[ks], !SHARED && ks == 0 ? neg_m : s[tk]);
+      for (int tk = 0; tk < 2; ++tk) s[tk] = mfma32x32x16<bf16_t>(kf[ks & 1][tk], qf[ks], s[tk]);
       if constexpr (ks < kCopies) copy(next, K, buffer ^ 1);
     });
     if constexpr (KS < kCopies)
@@ -269,9 +295,9 @@ __global__ __launch_bounds__(256, KS1 > 8 ? 1 : 2) void window_prefill_kernel(co
       for (int td = 0; td < TD; ++td)
 #pragma unroll
         for (int r = 0; r < 16; ++r) o[td][r] *= alpha;
-      const float nm = neg_m[0] - d;
-#pragma unroll
-      for (int r = 0; r < 16; ++r) neg_m[r] = nm;
+      m += d;
+      const float m0 = to_float(from_float<bf16_t>(m)), m1 = to_float(from_float<bf16_t>(m - m0)), m2 = m - m0 - m1;
+      if (hi) q_more = make_uint4(pack2<bf16_t>(-m0, -m1), pack2<bf16_t>(-m2, 0.f), 0u, 0u);
 #pragma unroll
       for (int tk = 0; tk < 2; ++tk)
 #pragma unroll
@@ -295,12 +321,11 @@ __global__ __launch_bounds__(256, KS1 > 8 ? 1 : 2) void window_prefill_kernel(co
       uint4 vf[TD];
 #pragma unroll
       for (int td = 0; td < TD; ++td) {
-        const int at = v_off[td % kOffsV];
-        constexpr int kGroup = Chunks<RCV>::kBits * 16;
-        const char* p0 = buf + at + (td / kOffsV) * kGroup + 16 * step * kRowV;
-        const char* p1 = buf + (SHARED ? at ^ 32 : at) + (td / kOffsV) * kGroup + (16 * step + 8) * kRowV;
-        const uint2 a0 = __builtin_bit_cast(uint2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) v4s*)p0));
-        const uint2 a1 = __builtin_bit_cast(uint2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) v4s*)p1));
+        const uint32_t at = (v_at ^ (64u * (td % (kGroupV / 4)))) + 16 * kGroupV * (td / (kGroupV / 4));
+        auto turned = [](uint32_t p) __attribute__((always_inline)) {
+          return __builtin_bit_cast(uint2, __builtin_amdgcn_ds_read_tr16_b64_v4i16(reinterpret_cast<__attribute__((address_space(3))) v4s*>(p)));
+        };
+        const uint2 a0 = turned(at + 16 * step * kRowV), a1 = turned((SHARED ? at ^ 32u : at) + (16 * step + 8) * kRowV);
         vf[td] = make_uint4(a0.x, a0.y, a1.x, a1.y);
       }
 #pragma unroll
