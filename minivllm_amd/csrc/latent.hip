@@ -54,6 +54,8 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(const LatentNormArgs f
   const T* in = reinterpret_cast<const T*>(a.in) + (int64_t)row * a.in_stride;
   const int64_t slot = a.slots ? a.slots[row] : -1;
   const int64_t out_row = a.out_rows ? a.out_rows[row] : row;
+  const bool turns = a.rot_table != nullptr;
+  const int64_t pos = turns ? a.positions[row] : 0;
   float x[NC][N], w[NC][N], ss = 0.f;
 #pragma unroll
   for (int c = 0; c < NC; ++c) {
@@ -61,14 +63,12 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(const LatentNormArgs f
     if (at + N <= a.rank && a.vec) {
 #pragma unroll
       for (int i = 0; i < N; i += 4) *reinterpret_cast<float4*>(&w[c][i]) = *reinterpret_cast<const float4*>(a.weight + at + i);
-    } else {
+    } else if (at < a.rank) {
 #pragma unroll
       for (int i = 0; i < N; ++i) w[c][i] = a.weight[min(at + i, a.rank - 1)];
     }
   }
-  const bool turns = a.rot_table != nullptr;
-  const float2* cs = nullptr;
-  if (turns) cs = a.rot_table + min(max(a.positions[row], (int64_t)0), a.max_position - 1) * (a.rot_dims / 2);
+  const float2* cs = turns ? a.rot_table + min(max(pos, (int64_t)0), a.max_position - 1) * (a.rot_dims / 2) : nullptr;
 #pragma unroll
   for (int c = 0; c < NC; ++c) {
     const int at = (c * 64 + lane) * N;

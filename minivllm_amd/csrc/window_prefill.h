@@ -14,7 +14,7 @@
 // the distance bias, against a key's place in its tile and the tile's distance (small integers, exact), the slope in the same
 // way; what is constant for a row drops out of the softmax.
 #pragma once
-#include "prefill_tiles.h"
+#include "prefill_mfma.h"
 
 #pragma clang fp contract(off)
 
@@ -33,7 +33,7 @@ struct WindowPrefillArgs {
   const float* slopes;        // [heads] or null
   int64_t out_row, out_head, q_row, q_head, k_row, k_head, k2_row, v_row, v_head, gate_row, gate_head;
   int64_t total_q;
-  int num_seqs, heads, kv_heads, dim, rot, window, hpw, tiles_x, heads_y;
+  int num_seqs, heads, kv_heads, dim, rot, window, hpw, tiles_x, heads_y, band_bits, band_shift;
   float scale_log2, temp_coef, temp_every;
 };
 
@@ -87,15 +87,22 @@ __global__ __launch_bounds__(256, KS1 > 8 ? 1 : 2) void window_prefill_kernel(co
   auto swz1 = [](int row) __attribute__((always_inline)) { return SHARED ? Chunks<RC1>::both(row) : Chunks<RC1>::keys(row); };
   auto swzv = [](int row) __attribute__((always_inline)) { return SHARED ? Chunks<RCV>::both(row) : Chunks<RCV>::values(row); };
 
-  // ---- work item: (head slice, query tile), tiles of a sequence one after the other; runs of 32 on one XCD ----
-  constexpr unsigned kRun = 32;
-  const unsigned id = blockIdx.x, slot = id >> 3, xcd = id & 7, round = slot / kRun;
-  const unsigned item = (round * 8 + ((xcd + round) & 7)) * kRun + slot % kRun;
-  if (item >= (unsigned)a.tiles_x * (unsigned)a.heads_y) return;
-  const int item_y = __builtin_amdgcn_readfirstlane((int)(item / (unsigned)a.tiles_x));
+  // ---- work item: (head slice, query tile), dealt as in prefill_mfma.h ----
+  const unsigned id = blockIdx.x, slot = id >> 3, xcd = id & 7, round = slot / kXcdChunk;
+  const unsigned item = (round * 8 + ((xcd + round) & 7)) * kXcdChunk + slot % kXcdChunk;
   const int BM = kWinRows * (4 / a.hpw);
-  int seq_start, seq_len, row0, seq;
-  if (!locate_tile(a.cu_q, a.num_seqs, a.tiles_x - 1 - (int)(item % (unsigned)a.tiles_x), BM, seq_start, seq_len, row0, seq)) return;
+  int seq_start, seq_len, row0, seq, item_y;
+  if (a.num_seqs <= 64) {
+    const bool found = a.hpw == 4 ? locate_banded<kWinRows>(a.cu_q, a.num_seqs, item, a.heads_y, a.band_bits, a.band_shift, seq_start, seq_len, row0, seq, item_y)
+                     : a.hpw == 2 ? locate_banded<2 * kWinRows>(a.cu_q, a.num_seqs, item, a.heads_y, a.band_bits, a.band_shift, seq_start, seq_len, row0, seq, item_y)
+                                  : locate_banded<4 * kWinRows>(a.cu_q, a.num_seqs, item, a.heads_y, a.band_bits, a.band_shift, seq_start, seq_len, row0, seq, item_y);
+    if (!found) return;
+  } else {
+    if (item >= (unsigned)a.tiles_x * (unsigned)a.heads_y) return;
+    item_y = (int)(item / (unsigned)a.tiles_x);
+    if (!locate_tile(a.cu_q, a.num_seqs, a.tiles_x - 1 - (int)(item % (unsigned)a.tiles_x), BM, seq_start, seq_len, row0, seq)) return;
+  }
+  item_y = __builtin_amdgcn_readfirstlane(item_y);
   seq_start = __builtin_amdgcn_readfirstlane(seq_start);
   seq_len = __builtin_amdgcn_readfirstlane(seq_len);
   row0 = __builtin_amdgcn_readfirstlane(row0);
@@ -288,7 +295,7 @@ __global__ __launch_bounds__(256, KS1 > 8 ? 1 : 2) void window_prefill_kernel(co
     mx = fmaxf(max3(mx, s[0][14], s[1][14]), mx1);
     mx = max_with_lane_xor32(mx);                    // relative to the running maximum
     const bool grow = fresh ? mx > -INFINITY : mx > 8.f;
-    if (__any(grow)) {
+    if (KS1 > 8 ? __builtin_expect(__any(grow), 0) : __any(grow)) {
       const float d = grow ? mx : 0.f, alpha = fresh ? 1.f : fast_exp2(-d);
       l *= alpha;
 #pragma unroll
@@ -346,8 +353,8 @@ __global__ __launch_bounds__(256, KS1 > 8 ? 1 : 2) void window_prefill_kernel(co
       continue;
     }
     const bool whole = j * kWinKeys > pos0 + kWinRows - 1 - W && j * kWinKeys + kWinKeys - 1 <= pos0;
-    if (whole) tile_step(j, std::false_type{}, buffer, more);
-    else tile_step(j, std::true_type{}, buffer, more);
+    if (KS1 <= 8 && whole) tile_step(j, std::false_type{}, buffer, more);
+    else tile_step(j, std::true_type{}, buffer, more);      // (the large heads: one copy of the step, whose registers then stay put)
   }
 
   // ---- normalise, turn through LDS, store whole rows ----
@@ -389,9 +396,12 @@ static int launch_window_prefill(const WindowPrefillArgs& a, hipStream_t s) {
   const int group = a.heads / a.kv_heads;
   b.hpw = group % 4 == 0 ? 4 : group % 2 == 0 ? 2 : 1;
   const int bm = kWinRows * (4 / b.hpw);
-  b.tiles_x = (int)(a.total_q / bm + a.num_seqs);
+  b.band_shift = band_shift_for(a.total_q, a.num_seqs, bm, false);
+  b.tiles_x = (int)(a.total_q / bm + (a.num_seqs <= 64 ? (int64_t)a.num_seqs << b.band_shift : a.num_seqs));
   b.heads_y = a.kv_heads * (group / b.hpw);
-  const int64_t items = (int64_t)b.tiles_x * b.heads_y, span = 8 * 32, blocks = (items + span - 1) / span * span;
+  b.band_bits = 1;
+  while (((int64_t)1 << b.band_bits) <= a.total_q / (bm << b.band_shift) + 1) ++b.band_bits;
+  const int64_t items = (int64_t)b.tiles_x * b.heads_y, span = 8 * (int64_t)kXcdChunk, blocks = (items + span - 1) / span * span;
   if (blocks > 0x7fffffff) return MVLLM_ERR_UNSUPPORTED;
   window_prefill_kernel<KS1, KS2, TD, SHARED><<<dim3((unsigned)blocks), dim3(256), 0, s>>>(b);
   return launch_status();
