@@ -96,7 +96,7 @@ class FevosunLayer(nn.Module):
             return t.to(device=device, dtype=dtype).contiguous()
 
         get = lambda name: tensors[prefix + name]
-        self.gain = 1.0 + get("norm1").to(device=device, dtype=torch.float32)           # stored around zero
+        self.gain = 1.0 + get("norm1").to(device=device, dtype=torch.float32)           # the checkpoint holds gain - 1
         rows, columns = self.mixer.load(lambda name: get("mix." + name), matrix, self.inputs)
         rows, columns = [rows], [columns]
         if self.dense_names:

@@ -15,7 +15,7 @@ def rms(x, eps):
 
 
 def shifted_norm(x, w, eps):
-    """A norm whose weight is stored around zero."""
+    """The norm's gain is one more than its stored weight."""
     return rms(x, eps) * (1 + w)
 
 
@@ -91,8 +91,8 @@ def attention(h, w, p, cfg):
 
 
 def latent_attention(h, w, p, cfg, eps, interleaved):
-    """Heads over keys and values made of one normed latent per token, plus one rotated key part for all heads; queries come
-    from h, or (``dq`` present) from a normed latent of their own."""
+    """Heads over keys and values made of one normed latent per token, beside a rotated part of the keys that the heads
+    have in common; queries come from h, or (``dq`` present) from a normed latent of their own."""
     n, heads, d, r, rank = h.shape[0], cfg["heads"], cfg["dim"], cfg["rot_dim"], cfg["kv_rank"]
     if p + "dq" in w:
         q = (rms(h @ w[p + "dq"].T, eps) * w[p + "dq.norm"]) @ w[p + "uq"].T

@@ -92,7 +92,7 @@ def test_caches_are_allocated_per_layer():
 def test_sizes_that_kernels_step_in():
     assert [head_size(n) for n in (1, 32, 33, 96, 97, 200, 256, 257)] == [32, 32, 64, 96, 128, 256, 256, 288]
     assert [shared_part_size(n) for n in (2, 32, 34, 64, 66)] == [32, 32, 64, 64, 96]
-    assert latent_layout(96, 16) == (96, 128, 128) and latent_layout(512, 64) == (512, 576, 512) and latent_layout(500, 64) == (512, 576, 512)
+    assert latent_layout(80, 10) == (80, 128, 128) and latent_layout(512, 64) == (512, 576, 512) and latent_layout(500, 64) == (512, 576, 512)
     assert latent_layout(150, 20) == (160, 192, 192) and latent_layout(600, 64) == (608, 672, 672)
     with pytest.raises(ValueError):
         head_size(600)
