@@ -522,6 +522,21 @@ int mvllm_head_rope_store(void* q_out, void* k_out, void* v_out, const void* pro
                           int vdim, int head_dim, int dtype, void* stream);
 
 /*
+ * mvllm_head_rope_store with other norms, added up in `norms`: 1: q and k over all heads of a row at once (gain_q fp32 [Hq dim],
+ * gain_k [Hkv dim]) in front of the rotation; 2: q and k of every head divided by their root mean square behind it; 4: values
+ * divided by theirs (behind a rotation, if there is one).  head_scale fp32 [Hq] or NULL: a further factor of q.  kv_row int64
+ * [rows] or NULL: rows of k_out and v_out (< 0: none).  kv_head_stride: elements between the heads of a row of k_out, v_out and
+ * the caches (with v_cache = k_cache + head_dim and twice head_dim, a key and its value are neighbours).
+ */
+int mvllm_head_norm_rope_store(void* q_out, void* k_out, void* v_out, const int64_t* kv_row, const void* proj,
+                               int64_t proj_row_stride, const float* gain_q, const float* gain_k, int norms, float eps,
+                               float q_scale, const float* head_scale, const float* rot_table, int rot_dims,
+                               const float* v_table, int interleaved, int64_t max_position, const int64_t* positions,
+                               const int32_t* dst_row, const int64_t* slots, void* k_cache, void* v_cache, int kv_head_stride,
+                               int64_t num_slots, int64_t rows, int num_heads, int num_kv_heads, int dim, int vdim,
+                               int head_dim, int dtype, void* stream);
+
+/*
  * Behind attention over rotated values: out[t, h, :vdim] = rotate(o[dst_row[t], h], -position) * sigmoid(gate[t, h]).
  * o [*, Hq, head_dim]; gate [rows, gate_row_stride] dtype, Hq values per row, or NULL; v_table as above or NULL.
  */
@@ -690,15 +705,19 @@ int mvllm_stream_norm_identity(void* out, int64_t out_row_stride, float* x_out, 
  * (csrc/window_prefill.hip, csrc/window_decode.hip).  A query sees the `window` keys up to its own (0: all of them);
  *     score = scale * t(p) * q . k - slopes[h] * distance,   t(p) = 1 + temp_coef ln(floor((p + 1) / temp_every) + 1)
  * (slopes fp32 [H] or NULL; temp_every 0: t = 1), out = softmax . v, times sigmoid(gate) where gate is not NULL (head h's
- * columns at h * gate_head_stride).  Strides are in elements; bf16 and fp32.
+ * columns at h * gate_head_stride; stride 1: one number for all of a head's columns).  Strides are in elements; bf16 and fp32.
  * mvllm_window_prefill: entries of packed queries (cu_q) over packed keys (cu_k); query i of an entry stands at key
  *   (keys - queries) + i.  q: head h at h * q_head_stride, [dim | rot]; k: kv head g at g * k_head_stride, [dim]; k2 [rot], shared
  *   by all heads, or NULL with rot 0; v like k, or NULL: the values are the keys.  positions int64 [total_q] (t only).  Tiled in
- *   bf16 for dim 32, 64, 96, 128, 192, 256, with k2 and v for rot 32 and 64 (no slopes); else dim and rot up to 512.
+ *   bf16 for dim 32, 64, 96, 128, 192, 256: without v, with v alone (no slopes), and with v and k2 for rot 32 and 64 (no slopes);
+ *   else dim and rot up to 512.
  * mvllm_window_decode: single query rows over a paged cache [num_blocks, block_size, kv heads, padded] (padded a multiple of 32)
  *   whose rows are keys and, their first `values` columns (padded, or 512 of 576), values.  lens int64 [rows]: position + 1;
  *   ring > 0: token p lies at place p mod ring of its entry's table (ring >= window + the most rows an entry has in a call - 1),
  *   0: at place p.  Everything else as for mvllm_latent_decode.
+ * mvllm_window_decode_split: the same over rows of `keys` columns of a key and behind them `values` of its value (multiples of 32;
+ *   tiled in bf16 where both are one of the widths of the tiled prefill).  Workspace: mvllm_window_decode_workspace_bytes with
+ *   padded = keys + values.
  * mvllm_latent_rope_store: mvllm_latent_norm_store with a part behind the latent, columns rot_col .. rot_col + rot of a row, that is
  *   not normed; its first rot_dims columns turn by rot_table fp32 [max_position, rot_dims / 2, 2] (cos, sin) in pairs (2i, 2i + 1) if
  *   interleaved, else (i, i + rot_dims / 2).  out_rows int64 [rows] (< 0: none) or NULL: rows of `out`.  in2 != NULL: a second plain
@@ -723,6 +742,12 @@ int mvllm_window_decode(void* out, int64_t out_row_stride, int64_t out_head_stri
                         int64_t gate_row_stride, int64_t gate_head_stride, int rows, int num_heads, int num_kv_heads,
                         int padded, int values, int block_size, int64_t num_blocks, int window, int ring, float scale,
                         float temp_coef, float temp_every, int dtype, void* workspace, size_t workspace_bytes, void* stream);
+int mvllm_window_decode_split(void* out, int64_t out_row_stride, int64_t out_head_stride, const void* q, int64_t q_row_stride,
+                              int64_t q_head_stride, const void* cache, const int32_t* block_tables, int table_width,
+                              const int32_t* row_entry, const int64_t* lens, const float* slopes, const void* gate,
+                              int64_t gate_row_stride, int64_t gate_head_stride, int rows, int num_heads, int num_kv_heads,
+                              int keys, int values, int block_size, int64_t num_blocks, int window, int ring, float scale,
+                              float temp_coef, float temp_every, int dtype, void* workspace, size_t workspace_bytes, void* stream);
 int mvllm_latent_rope_store(void* out, const int64_t* out_rows, const void* in, int64_t in_row_stride, const float* weight,
                             float eps, const float* rot_table, int rot_col, int rot, int rot_dims, int interleaved,
                             int64_t max_position, const int64_t* positions, void* cache, int64_t num_slots,
@@ -736,6 +761,48 @@ int mvllm_copy_rows(void* dst, int64_t dst_row_stride, int64_t dst_count, const 
                     int64_t dst2_row_stride, int64_t dst2_count, const int64_t* dst2_rows, const void* src,
                     int64_t src_row_stride, int64_t src_count, const int64_t* src_rows, int64_t rows, int width, int dtype,
                     void* stream);
+
+/*
+ * out = gelu(in), z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))); rows of `width` numbers (a multiple of 16 bytes), strides in
+ * elements.  mvllm_linear_small_m_gelu: mvllm_linear_small_m with it behind the bias, rounded once.
+ */
+int mvllm_gelu_tanh(void* out, int64_t out_row_stride, const void* in, int64_t in_row_stride, int64_t rows, int width, int dtype,
+                    void* stream);
+int mvllm_linear_small_m_gelu(void* out, const void* x, const void* w, const void* bias, int64_t x_row_stride, int M, int N, int K,
+                              int dtype, void* stream);
+
+/*
+ * Between the sublayers of a decoder that norms what they return (csrc/post_norm.hip): x_out = x + norm(y) * gain (fp32
+ * [rows, width]; may be x itself, or NULL), out = x_out, or norm(x_out) * final_gain where that is not NULL, in dtype, zeros from
+ * `width` to out_row_stride.  norm divides by sqrt(mean of squares + eps), with `centred` after taking the mean off.
+ * mvllm_embed_rows: x_out = embed[token] * scale, out = x_out.
+ */
+int mvllm_post_norm(void* out, int64_t out_row_stride, float* x_out, const float* x, const void* y, int64_t y_row_stride,
+                    const float* gain, const float* final_gain, float eps, int centred, int64_t rows, int width, int dtype,
+                    void* stream);
+int mvllm_embed_rows(void* out, int64_t out_row_stride, float* x_out, const void* embed, int64_t vocab, float scale,
+                     const int64_t* tokens, int64_t rows, int width, int dtype, void* stream);
+
+/*
+ * Attention whose heads' scores are mixed before the softmax (csrc/talk.h): s_h = sum_g talk[h, g] q_g . k, with an optional sink
+ * per head (one more exp(sink) in the denominator).  Queries carry the score scale and log2 e: scores are exponents of two as
+ * they come.  q [rows, H, dim] contiguous, talk fp32 [H, H], sinks fp32 [H] or NULL, out: head h at h * out_head_stride.
+ * mvllm_talk_prefill: pieces of packed queries (cu_q); keys and values [*, Hkv, dim], packed (cu_k: more keys than queries in front,
+ *   NULL: as many) or, with block_tables, a paged cache [num_blocks, block_size, Hkv, dim].  out_rows int32 [total_q] or NULL: rows
+ *   of out.
+ * mvllm_talk_decode: single rows over the cache, lens int64 [rows] keys each, a table per row; the workspace holds partial results.
+ * bf16 and fp32; H up to 64, H * dim up to 16384.  Tiled in bf16 for dim 32, 64, 96, 128 and up to 8 kv heads (prefill: up to 8
+ * groups of four heads that share one, and talk rounded to bf16).
+ */
+int mvllm_talk_prefill(void* out, int64_t out_row_stride, int64_t out_head_stride, const int32_t* out_rows, const void* q,
+                       const void* k, const void* v, const int32_t* cu_q, const int32_t* cu_k, const int32_t* block_tables,
+                       int table_width, int block_size, int64_t num_blocks, const float* talk, const float* sinks, int num_seqs,
+                       int64_t total_q, int num_heads, int num_kv_heads, int dim, int dtype, void* stream);
+size_t mvllm_talk_decode_workspace_bytes(int rows, int num_heads, int num_kv_heads, int dim, int64_t max_keys, int dtype);
+int mvllm_talk_decode(void* out, int64_t out_row_stride, int64_t out_head_stride, const void* q, const void* k_cache,
+                      const void* v_cache, const int32_t* block_tables, int table_width, const int64_t* lens, const float* talk,
+                      const float* sinks, int rows, int num_heads, int num_kv_heads, int dim, int block_size, int64_t num_blocks,
+                      int dtype, void* workspace, size_t workspace_bytes, void* stream);
 
 #ifdef __cplusplus
 }

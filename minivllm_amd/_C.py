@@ -140,6 +140,23 @@ SIGNATURES = {
           c_void_p] + [c_int] * 3 + [c_int64, c_void_p, c_int64, c_int, c_int, c_void_p]),
     "mvllm_copy_rows": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_void_p, c_void_p,
           c_int64, c_int64, c_void_p, c_int64, c_int, c_int, c_void_p]),
+    "mvllm_head_norm_rope_store": (c_int, [c_void_p] * 5 + [c_int64, c_void_p, c_void_p, c_int, c_float, c_float,
+          c_void_p, c_void_p, c_int, c_void_p, c_int, c_int64] + [c_void_p] * 5 + [c_int, c_int64, c_int64] + [c_int]
+          * 6 + [c_void_p]),
+    "mvllm_window_decode_split": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_int64, c_int64, c_void_p, c_void_p,
+          c_int] + [c_void_p] * 4 + [c_int64, c_int64] + [c_int] * 6 + [c_int64, c_int, c_int] + [c_float] * 3 +
+          [c_int, c_void_p, c_size_t, c_void_p]),
+    "mvllm_gelu_tanh": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int, c_int, c_void_p]),
+    "mvllm_linear_small_m_gelu": (c_int, [c_void_p] * 4 + [c_int64] + [c_int] * 4 + [c_void_p]),
+    "mvllm_post_norm": (c_int, [c_void_p, c_int64] + [c_void_p] * 3 + [c_int64, c_void_p, c_void_p, c_float, c_int,
+          c_int64, c_int, c_int, c_void_p]),
+    "mvllm_embed_rows": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_float, c_void_p, c_int64, c_int,
+          c_int, c_void_p]),
+    "mvllm_talk_prefill": (c_int, [c_void_p, c_int64, c_int64] + [c_void_p] * 7 + [c_int, c_int, c_int64, c_void_p,
+          c_void_p, c_int, c_int64] + [c_int] * 4 + [c_void_p]),
+    "mvllm_talk_decode_workspace_bytes": (c_size_t, [c_int] * 4 + [c_int64, c_int]),
+    "mvllm_talk_decode": (c_int, [c_void_p, c_int64, c_int64] + [c_void_p] * 4 + [c_int] + [c_void_p] * 3 + [c_int] *
+          5 + [c_int64, c_int, c_void_p, c_size_t, c_void_p]),
 }
 
 

@@ -23,7 +23,8 @@ PROBE_SOURCES = ["mfma_probe.hip"]
 SOURCES = ["capi.hip", "store_kvcache.hip", "paged_decode.hip", "prefill_varlen.hip", "prefill_other_dims.hip", "prefill_half_step_dims.hip", "prefill_pingpong.hip", "prefill_staged.hip", "prefill_split.hip", "prefill_f32.hip", "qk_norm_rope_store.hip", "sampler.hip",
            "rms_norm.hip", "activation.hip", "linear_small.hip", "norm_conv.hip", "head_rope.hip", "gate_linear.hip", "mlstm.hip", "mlstm_chunk.hip",
            "decay_memory.hip", "latent.hip", "moe.hip", "stream_norm.hip", "ring_rows.hip", "window_prefill.hip",
-           "window_prefill_latent.hip", "window_decode.hip"]
+           "window_prefill_latent.hip", "window_prefill_heads.hip", "window_decode.hip", "window_decode_split.hip", "post_norm.hip",
+           "talk.hip", "talk_prefill.hip", "talk_decode.hip"]
 
 HIPCC_FLAGS = [
     "--offload-arch=gfx950",

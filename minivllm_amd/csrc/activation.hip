@@ -4,6 +4,7 @@
 // then the product in fp32 rounded again.  One launch, 16-byte accesses, rows of the GEMM output as they lie.
 // mvllm_gated_unit: min(x, limit) * sigmoid(alpha min(x, limit)) * (clamp(y, +-limit) + shift), x and y the halves of a row:
 //   a clamped gated unit (limit infinite, alpha 1, shift 0: silu(x) * y in one rounding)
+// mvllm_gelu_tanh: the tanh form of gelu (common.h), rows of both sides with strides
 #include "common.h"
 
 #pragma clang fp contract(off)
@@ -82,6 +83,23 @@ __global__ __launch_bounds__(kActThreads) void gated_unit_kernel(T* __restrict__
   }
 }
 
+template <typename T>
+__global__ __launch_bounds__(kActThreads) void gelu_tanh_kernel(T* __restrict__ out, const T* __restrict__ in, int64_t rows, int width,
+                                                                int64_t in_stride, int64_t out_stride) {
+  constexpr int N = Act8<T>::N;
+  const int per_row = width / N;
+  const int64_t total = rows * per_row;
+  for (int64_t i = (int64_t)blockIdx.x * kActThreads + threadIdx.x; i < total; i += (int64_t)gridDim.x * kActThreads) {
+    const int64_t r = i / per_row;
+    const int c = (int)(i - r * per_row) * N;
+    float z[8], y[8];
+    Act8<T>::load(in + r * in_stride + c, z);
+#pragma unroll
+    for (int e = 0; e < N; ++e) y[e] = gelu_tanh(z[e]);
+    Act8<T>::store(out + r * out_stride + c, y);
+  }
+}
+
 }  // namespace mvllm
 
 using namespace mvllm;
@@ -124,5 +142,23 @@ extern "C" int mvllm_gated_unit(void* out, int64_t out_row_stride, const void* i
   hipStream_t s = (hipStream_t)stream;
   if (dtype == MVLLM_F32) gated_unit_kernel<float><<<grid, block, 0, s>>>((float*)out, (const float*)in, rows, width, in_row_stride, out_row_stride, alpha, limit, shift);
   else gated_unit_kernel<bf16_t><<<grid, block, 0, s>>>((bf16_t*)out, (const bf16_t*)in, rows, width, in_row_stride, out_row_stride, alpha, limit, shift);
+  return launch_status();
+}
+
+extern "C" int mvllm_gelu_tanh(void* out, int64_t out_row_stride, const void* in, int64_t in_row_stride, int64_t rows, int width,
+                               int dtype, void* stream) {
+  const int esize = dtype_size(dtype);
+  if (esize == 0) return MVLLM_ERR_BAD_DTYPE;
+  if (rows < 0 || width <= 0 || in_row_stride < width || out_row_stride < width) return MVLLM_ERR_BAD_SHAPE;
+  const int n = 16 / esize;
+  if (dtype == MVLLM_F16 || width % n != 0 || in_row_stride % n != 0 || out_row_stride % n != 0) return MVLLM_ERR_UNSUPPORTED;
+  if (rows == 0) return MVLLM_OK;
+  if (!out || !in) return MVLLM_ERR_NULL_POINTER;
+  if (!aligned16(out) || !aligned16(in)) return MVLLM_ERR_MISALIGNED;
+  const int64_t blocks = (rows * (width / n) + kActThreads - 1) / kActThreads;
+  const dim3 grid((unsigned)(blocks > 65536 ? 65536 : blocks)), block(kActThreads);
+  hipStream_t s = (hipStream_t)stream;
+  if (dtype == MVLLM_F32) gelu_tanh_kernel<float><<<grid, block, 0, s>>>((float*)out, (const float*)in, rows, width, in_row_stride, out_row_stride);
+  else gelu_tanh_kernel<bf16_t><<<grid, block, 0, s>>>((bf16_t*)out, (const bf16_t*)in, rows, width, in_row_stride, out_row_stride);
   return launch_status();
 }

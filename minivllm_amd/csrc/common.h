@@ -145,6 +145,12 @@ __device__ __forceinline__ void store4_stream(void* p, uint32_t v) {
 
 __device__ __forceinline__ float fast_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
 
+// z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), with the tanh as an exponential: (1 + tanh u) / 2 = 1 / (1 + exp(-2 u)).
+__device__ __forceinline__ float gelu_tanh(float z) {
+  const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
+  return z / (1.f + expf(-2.f * u));
+}
+
 // A softmax denominator l, counted in units of 2^m, with one further term exp(sink): a learned number per query head
 // that has neither key nor value.  A row that saw no key (m = -inf) keeps its zero.
 __device__ __forceinline__ float add_sink(float l, float m, float sink) {

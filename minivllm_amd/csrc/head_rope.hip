@@ -9,6 +9,10 @@
 //     v           = rotate(v, pos) with a table of its own        [*, G, D]   packed (v_out) and / or cache slot
 //   D >= max(dim, vdim) is the head size the attention kernels run at: dims past dim / vdim are written as zeros.
 //   dst = dst_row[t] (null: t) reorders the rows for attention, which runs over groups of rows.
+// mvllm_head_norm_rope_store: the same with other norms: q and k over all heads of a row at once (a workgroup per row),
+// q and k divided by their root mean square behind the rotation, values divided by theirs; a factor per query head; packed
+// keys and values at rows of their own; any distance between the heads of a key or value row (so that a key and its
+// value may be neighbours).
 // mvllm_head_unrotate_gate: attention output rows [*, H, D] ->
 //     out[t, h * vdim + d] = rotate(o[dst_row[t], h], -pos)[d] * sigmoid(gate[t, h])
 // Sixteen lanes own one head vector, eight consecutive dims per lane and step (in long batches four heads of a row, which
@@ -111,33 +115,48 @@ struct HeadRopeArgs {
   void* k_out;             // [*, G, D] or null
   void* v_out;
   const void* proj;        // [T, proj_stride]: q at 0, k at H dim, v at (H + G) dim
-  const float* gain_q;     // [dim] or null (no norm)
-  const float* gain_k;
+  const float* gain_q;     // [dim], with kNormRows [H dim], or null (no norm)
+  const float* gain_k;     // [dim], with kNormRows [G dim]
+  const float* head_scale; // [H] or null: further factor of q
   const float2* rot_table;    // [max_position, rot / 2] (cos, sin) or null
   const float2* v_table;      // [max_position, vdim / 2] or null
   const int64_t* positions;   // [T]
   const int32_t* dst_row;     // [T] or null
+  const int64_t* kv_row;      // [T] or null (dst): rows of k_out and v_out, negative: none
   const int64_t* slots;       // [T] or null
-  void* k_cache;              // [slots, G, D]
+  void* k_cache;              // [slots, G, kv_head]: heads in the first D
   void* v_cache;
   int64_t proj_stride;
   int64_t max_position;
   int64_t num_slots;
   int64_t rows;
   int heads, kv_heads, dim, vdim, D, rot;
-  int interleaved;
+  int interleaved, norms, kv_head;
   float eps, q_scale;
 };
 
+enum { kNormRows = 1, kNormTurned = 2, kNormValues = 4 };
+constexpr int kMaxRowParts = 64;
+
+// Sum of squares over the sixteen lanes of a head.
+template <int kSteps> __device__ __forceinline__ float head_squares(const float (&x)[kSteps][8]) {
+  float ss = 0.f;
+#pragma unroll
+  for (int s = 0; s < kSteps; ++s)
+#pragma unroll
+    for (int i = 0; i < 8; ++i) ss = fmaf(x[s][i], x[s][i], ss);
+  return row16_sum(ss);
+}
+
 // Sixteen lanes take kUnits heads of one row that turn by the same table (q and k heads, or v heads), so that the row's
-// angles are read once for all of them; kSteps steps of 128 dims.
-template <typename T, int kSteps, int kUnits>
-__global__ __launch_bounds__(256) void head_rope_store_kernel(const HeadRopeArgs a, unsigned parts_qk, unsigned parts) {
-  const unsigned item = blockIdx.x * (256 / kLanes) + threadIdx.x / kLanes;
+// angles are read once for all of them; kSteps steps of 128 dims.  kRow: the workgroup is one row, normed as a whole.
+template <typename T, int kSteps, int kUnits, bool kRow>
+__global__ __launch_bounds__(kRow ? 16 * kMaxRowParts : 256) void head_rope_store_kernel(const HeadRopeArgs a, unsigned parts_qk, unsigned parts) {
+  const unsigned item = kRow ? threadIdx.x / kLanes : blockIdx.x * (256 / kLanes) + threadIdx.x / kLanes;
   const int li = threadIdx.x % kLanes;
-  const bool live = item < (unsigned)a.rows * parts;
-  const int64_t t = live ? item / parts : 0;
-  const unsigned part = live ? item - (unsigned)t * parts : 0;
+  const bool live = item < (kRow ? parts : (unsigned)a.rows * parts);
+  const int64_t t = kRow ? (int64_t)blockIdx.x : live ? item / parts : 0;
+  const unsigned part = !live ? 0 : kRow ? item : item - (unsigned)t * parts;
   const bool is_v = part >= parts_qk;
   const int u0 = (int)(is_v ? part - parts_qk : part) * kUnits;        // first head: q and k heads counted through, or v heads
   const int count = live ? min(kUnits, (is_v ? a.kv_heads : a.heads + a.kv_heads) - u0) : 0;
@@ -157,8 +176,30 @@ __global__ __launch_bounds__(256) void head_rope_store_kernel(const HeadRopeArgs
   pos = pos < 0 ? 0 : pos >= a.max_position ? a.max_position - 1 : pos;
   const int rot = is_v ? (a.v_table ? a.vdim : 0) : (a.rot_table ? a.rot : 0);
   const float2* cs = rot == 0 ? nullptr : (is_v ? a.v_table : a.rot_table) + pos * (rot / 2);
-  const int64_t dst = a.dst_row ? a.dst_row[t] : t;
+  const int64_t dst = a.dst_row ? a.dst_row[t] : t, kv_dst = a.kv_row ? a.kv_row[t] : dst;
   const int64_t own_slot = a.slots ? a.slots[t] : -1;
+  float row_scale[2] = {1.f, 1.f};                                     // of q and of k
+  if constexpr (kRow) {
+    __shared__ float squares[2][kMaxRowParts];
+    float mine[2] = {0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < kUnits; ++j) {
+      const float ss = head_squares(x[j]);                             // heads that are not there are zeros
+      if (!is_v) mine[u0 + j >= a.heads] += ss;
+    }
+    if (li == 0) {
+      squares[0][item] = live ? mine[0] : 0.f;
+      squares[1][item] = live ? mine[1] : 0.f;
+    }
+    __syncthreads();
+    const unsigned groups = blockDim.x / kLanes;
+#pragma unroll
+    for (int w = 0; w < 2; ++w) {
+      float ss = 0.f;
+      for (unsigned i = li; i < groups; i += kLanes) ss += squares[w][i];
+      row_scale[w] = 1.0f / sqrtf(row16_sum(ss) / (float)((w == 0 ? a.heads : a.kv_heads) * n) + a.eps);
+    }
+  }
   float2 angle[kSteps][4];                                             // of the lane's pairs (interleaved layout)
 #pragma unroll
   for (int s = 0; s < kSteps; ++s) load_angles(angle[s], cs, 8 * (li + kLanes * s), a.interleaved ? rot : 0);
@@ -166,46 +207,57 @@ __global__ __launch_bounds__(256) void head_rope_store_kernel(const HeadRopeArgs
   for (int j = 0; j < kUnits; ++j) {
     const int u = u0 + j;
     const bool is_q = !is_v && u < a.heads;
+    const int head = is_q || is_v ? u : u - a.heads;
     const float* gain = is_v ? nullptr : is_q ? a.gain_q : a.gain_k;
     float scale = 1.f;
-    if (gain) {                                                        // the same for the sixteen lanes
-      float ss = 0.f;
-#pragma unroll
-      for (int s = 0; s < kSteps; ++s)
-#pragma unroll
-        for (int i = 0; i < 8; ++i) ss = fmaf(x[j][s][i], x[j][s][i], ss);
-      scale = 1.0f / sqrtf(row16_sum(ss) / (float)n + a.eps);
+    if constexpr (kRow) {
+      scale = row_scale[is_q ? 0 : 1];
+      if (gain && j < count) gain += (int64_t)head * a.dim;
+    } else if (gain) {                                                 // the same for the sixteen lanes
+      scale = 1.0f / sqrtf(head_squares(x[j]) / (float)n + a.eps);
     }
+    // what follows the rotation; a rotation by unequal angles keeps a head's squares only up to the table's amplitude
+    const bool unit = is_v ? (a.norms & kNormValues) != 0 : (a.norms & kNormTurned) != 0;
+    if (j < count) {
+#pragma unroll
+      for (int s = 0; s < kSteps; ++s) {
+        const int d0 = 8 * (li + kLanes * s);
+        if (d0 >= a.D) continue;
+        float* v = x[j][s];
+        if (gain) {
+          float g[8];
+          load8(gain + d0, max(min(8, n - d0), 0), g);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) v[i] = v[i] * scale * g[i];
+        }
+        if (d0 < rot) {
+          if (a.interleaved) {
+            turn_pairs(v, angle[s], 1.f);
+          } else {
+            float partner[8];
+            load_partner(src + j * n, gain, scale, d0, rot, partner);
+            turn_halves(v, partner, d0, rot, cs, 1.f);
+          }
+        }
+      }
+    }
+    float factor = unit ? 1.0f / sqrtf(head_squares(x[j]) / (float)n + a.eps) : 1.f;
     if (j >= count) continue;
-    const int head = is_q || is_v ? u : u - a.heads, groups = is_q ? a.heads : a.kv_heads;
+    if (is_q) factor *= a.head_scale ? a.q_scale * a.head_scale[head] : a.q_scale;
     T* packed = reinterpret_cast<T*>(is_q ? a.q_out : is_v ? a.v_out : a.k_out);
-    if (packed) packed += (dst * groups + head) * a.D;
+    if (packed && is_q) packed += (dst * a.heads + head) * a.D;
+    else if (packed) packed = kv_dst < 0 ? nullptr : packed + (kv_dst * a.kv_heads + head) * a.kv_head;
     const int64_t slot = is_q ? -1 : own_slot;
     T* cached = nullptr;
-    if (slot >= 0 && slot < a.num_slots) cached = reinterpret_cast<T*>(is_v ? a.v_cache : a.k_cache) + (slot * a.kv_heads + head) * a.D;
+    if (slot >= 0 && slot < a.num_slots) cached = reinterpret_cast<T*>(is_v ? a.v_cache : a.k_cache) + (slot * a.kv_heads + head) * a.kv_head;
 #pragma unroll
     for (int s = 0; s < kSteps; ++s) {
       const int d0 = 8 * (li + kLanes * s);
       if (d0 >= a.D) continue;
       float* v = x[j][s];
-      if (gain) {
-        float g[8];
-        load8(gain + d0, max(min(8, n - d0), 0), g);
+      if (is_q || unit) {
 #pragma unroll
-        for (int i = 0; i < 8; ++i) v[i] = v[i] * scale * g[i];
-      }
-      if (d0 < rot) {
-        if (a.interleaved) {
-          turn_pairs(v, angle[s], 1.f);
-        } else {
-          float partner[8];
-          load_partner(src + j * n, gain, scale, d0, rot, partner);
-          turn_halves(v, partner, d0, rot, cs, 1.f);
-        }
-      }
-      if (is_q) {
-#pragma unroll
-        for (int i = 0; i < 8; ++i) v[i] *= a.q_scale;
+        for (int i = 0; i < 8; ++i) v[i] *= factor;
       }
       const int m = min(8, a.D - d0);
       if (packed) store8(packed + d0, m, v);
@@ -315,6 +367,56 @@ template <typename F> static void with_steps(int head_dim, int64_t rows, F f) {
   else f(integral_constant<int, 1>{}, integral_constant<int, kRowUnits>{});
 }
 
+extern "C" int mvllm_head_norm_rope_store(void* q_out, void* k_out, void* v_out, const int64_t* kv_row, const void* proj,
+                                          int64_t proj_row_stride, const float* gain_q, const float* gain_k, int norms, float eps,
+                                          float q_scale, const float* head_scale, const float* rot_table, int rot_dims,
+                                          const float* v_table, int interleaved, int64_t max_position, const int64_t* positions,
+                                          const int32_t* dst_row, const int64_t* slots, void* k_cache, void* v_cache,
+                                          int kv_head_stride, int64_t num_slots, int64_t rows, int num_heads, int num_kv_heads,
+                                          int dim, int vdim, int head_dim, int dtype, void* stream) {
+  if (dtype_size(dtype) == 0) return MVLLM_ERR_BAD_DTYPE;
+  if (rows < 0 || num_heads <= 0 || num_kv_heads <= 0 || num_heads % num_kv_heads != 0 || dim <= 0 || vdim <= 0 ||
+      head_dim < dim || head_dim < vdim || rot_dims < 0 || rot_dims > dim || rot_dims % 2 != 0 || kv_head_stride < head_dim ||
+      (v_table && vdim % 2 != 0) || max_position <= 0 || num_slots < 0 || norms < 0 || norms > 7 ||
+      ((norms & kNormRows) && (!gain_q || !gain_k)) || proj_row_stride < (int64_t)num_heads * dim + (int64_t)num_kv_heads * (dim + vdim))
+    return MVLLM_ERR_BAD_SHAPE;
+  if (dtype == MVLLM_F16 || head_dim > 8 * kLanes * kMaxSteps || rows > ((int64_t)1 << 31) / (num_heads + 2 * (int64_t)num_kv_heads))
+    return MVLLM_ERR_UNSUPPORTED;
+  if (rows == 0) return MVLLM_OK;
+  if (!q_out || !proj || !positions || (slots && (!k_cache || !v_cache)) || (rot_dims && !rot_table)) return MVLLM_ERR_NULL_POINTER;
+  HeadRopeArgs a;
+  a.q_out = q_out; a.k_out = k_out; a.v_out = v_out; a.proj = proj; a.gain_q = gain_q; a.gain_k = gain_k; a.head_scale = head_scale;
+  a.rot_table = rot_dims ? reinterpret_cast<const float2*>(rot_table) : nullptr;
+  a.v_table = reinterpret_cast<const float2*>(v_table);
+  a.positions = positions; a.dst_row = dst_row; a.kv_row = kv_row; a.slots = slots; a.k_cache = k_cache; a.v_cache = v_cache;
+  a.proj_stride = proj_row_stride; a.max_position = max_position; a.num_slots = num_slots; a.rows = rows;
+  a.heads = num_heads; a.kv_heads = num_kv_heads; a.dim = dim; a.vdim = vdim; a.D = head_dim; a.rot = rot_dims;
+  a.interleaved = interleaved; a.norms = norms; a.kv_head = kv_head_stride; a.eps = eps; a.q_scale = q_scale;
+  int st = MVLLM_OK;
+  auto launch = [&](auto STEPS, auto UNITS) {
+    constexpr int kSteps = decltype(STEPS)::value, kUnits = decltype(UNITS)::value;
+    const unsigned parts_qk = (unsigned)(num_heads + num_kv_heads + kUnits - 1) / kUnits, parts = parts_qk + (unsigned)(num_kv_heads + kUnits - 1) / kUnits;
+    hipStream_t s = (hipStream_t)stream;
+    if (norms & kNormRows) {
+      if (parts > (unsigned)kMaxRowParts) {
+        st = MVLLM_ERR_UNSUPPORTED;
+        return;
+      }
+      const dim3 grid((unsigned)rows), block((parts * kLanes + 63) / 64 * 64);
+      if (dtype == MVLLM_F32) head_rope_store_kernel<float, kSteps, kUnits, true><<<grid, block, 0, s>>>(a, parts_qk, parts);
+      else head_rope_store_kernel<bf16_t, kSteps, kUnits, true><<<grid, block, 0, s>>>(a, parts_qk, parts);
+    } else {
+      const dim3 grid(head_blocks(rows * parts));
+      if (dtype == MVLLM_F32) head_rope_store_kernel<float, kSteps, kUnits, false><<<grid, dim3(256), 0, s>>>(a, parts_qk, parts);
+      else head_rope_store_kernel<bf16_t, kSteps, kUnits, false><<<grid, dim3(256), 0, s>>>(a, parts_qk, parts);
+    }
+  };
+  // more heads than one per sixteen lanes can take side by side: several each, whatever the number of rows
+  const bool wide = (norms & kNormRows) && num_heads + 2 * num_kv_heads > kMaxRowParts;
+  with_steps(head_dim, wide ? (int64_t)kManyRows : rows, launch);
+  return st != MVLLM_OK ? st : launch_status();
+}
+
 extern "C" int mvllm_head_rope_store(void* q_out, void* k_out, void* v_out, const void* proj, int64_t proj_row_stride,
                                      const float* gain_q, const float* gain_k, float eps, float q_scale,
                                      const float* rot_table, int rot_dims, const float* v_table, int interleaved,
@@ -322,32 +424,9 @@ extern "C" int mvllm_head_rope_store(void* q_out, void* k_out, void* v_out, cons
                                      const int64_t* slots, void* k_cache, void* v_cache, int64_t num_slots, int64_t rows,
                                      int num_heads, int num_kv_heads, int dim, int vdim, int head_dim, int dtype,
                                      void* stream) {
-  if (dtype_size(dtype) == 0) return MVLLM_ERR_BAD_DTYPE;
-  if (rows < 0 || num_heads <= 0 || num_kv_heads <= 0 || num_heads % num_kv_heads != 0 || dim <= 0 || vdim <= 0 ||
-      head_dim < dim || head_dim < vdim || rot_dims < 0 || rot_dims > dim || rot_dims % 2 != 0 ||
-      (v_table && vdim % 2 != 0) || max_position <= 0 || num_slots < 0 ||
-      proj_row_stride < (int64_t)num_heads * dim + (int64_t)num_kv_heads * (dim + vdim))
-    return MVLLM_ERR_BAD_SHAPE;
-  if (dtype == MVLLM_F16 || head_dim > 8 * kLanes * kMaxSteps || rows > ((int64_t)1 << 31) / (num_heads + 2 * (int64_t)num_kv_heads))
-    return MVLLM_ERR_UNSUPPORTED;
-  if (rows == 0) return MVLLM_OK;
-  if (!q_out || !proj || !positions || (slots && (!k_cache || !v_cache)) || (rot_dims && !rot_table)) return MVLLM_ERR_NULL_POINTER;
-  HeadRopeArgs a;
-  a.q_out = q_out; a.k_out = k_out; a.v_out = v_out; a.proj = proj; a.gain_q = gain_q; a.gain_k = gain_k;
-  a.rot_table = rot_dims ? reinterpret_cast<const float2*>(rot_table) : nullptr;
-  a.v_table = reinterpret_cast<const float2*>(v_table);
-  a.positions = positions; a.dst_row = dst_row; a.slots = slots; a.k_cache = k_cache; a.v_cache = v_cache;
-  a.proj_stride = proj_row_stride; a.max_position = max_position; a.num_slots = num_slots; a.rows = rows;
-  a.heads = num_heads; a.kv_heads = num_kv_heads; a.dim = dim; a.vdim = vdim; a.D = head_dim; a.rot = rot_dims;
-  a.interleaved = interleaved; a.eps = eps; a.q_scale = q_scale;
-  with_steps(head_dim, rows, [&](auto STEPS, auto UNITS) {
-    constexpr int kSteps = decltype(STEPS)::value, kUnits = decltype(UNITS)::value;
-    const unsigned parts_qk = (unsigned)(num_heads + num_kv_heads + kUnits - 1) / kUnits, parts = parts_qk + (unsigned)(num_kv_heads + kUnits - 1) / kUnits;
-    const dim3 grid(head_blocks(rows * parts));
-    if (dtype == MVLLM_F32) head_rope_store_kernel<float, kSteps, kUnits><<<grid, dim3(256), 0, (hipStream_t)stream>>>(a, parts_qk, parts);
-    else head_rope_store_kernel<bf16_t, kSteps, kUnits><<<grid, dim3(256), 0, (hipStream_t)stream>>>(a, parts_qk, parts);
-  });
-  return launch_status();
+  return mvllm_head_norm_rope_store(q_out, k_out, v_out, nullptr, proj, proj_row_stride, gain_q, gain_k, 0, eps, q_scale, nullptr,
+                                    rot_table, rot_dims, v_table, interleaved, max_position, positions, dst_row, slots, k_cache,
+                                    v_cache, head_dim, num_slots, rows, num_heads, num_kv_heads, dim, vdim, head_dim, dtype, stream);
 }
 
 extern "C" int mvllm_head_unrotate_gate(void* out, const void* o, const void* gate, int64_t gate_row_stride,

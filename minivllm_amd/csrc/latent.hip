@@ -305,7 +305,7 @@ extern "C" int mvllm_latent_decode(void* out, const void* q, const void* cache, 
   LatentDecodeArgs a = {};
   a.out = out; a.q = q; a.cache = cache; a.tables = block_tables; a.row_entry = row_entry; a.lens = lens;
   a.num_blocks = num_blocks; a.table_width = table_width; a.block_size = block_size; a.heads = num_heads; a.padded = padded;
-  a.kv_heads = 1; a.values = padded; a.q_head = a.out_head = padded; a.q_row = a.out_row = (int64_t)num_heads * padded;
+  a.kv_heads = 1; a.values = a.row = padded; a.q_head = a.out_head = padded; a.q_row = a.out_row = (int64_t)num_heads * padded;
   a.scale_log2 = scale * kLog2e;
   a.parts = plan_parts(rows, num_heads, 1, padded, (int64_t)table_width * block_size, dtype);
   a.part_o = nullptr;

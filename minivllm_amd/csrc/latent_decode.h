@@ -1,6 +1,6 @@
 // Attention of single query rows over a paged cache whose rows are keys and values at once (latents, or keys that are their
-// own values): the kernels of latent.hip and window_decode.hip.  The windowed form adds kv heads, a ring of places, a
-// distance bias, a query temperature and an output gate.
+// own values), or hold a key and behind it a value: the kernels of latent.hip and window_decode.hip.  The windowed form adds
+// kv heads, a ring of places, a distance bias, a query temperature and an output gate.
 #pragma once
 #include "prefill_tiles.h"
 
@@ -11,7 +11,7 @@ namespace mvllm {
 struct LatentDecodeArgs {
   void* out;                 // [rows, H, value columns] with strides
   const void* q;             // [rows, H, padded] with strides
-  const void* cache;         // [num_blocks, block_size, kv_heads, padded]
+  const void* cache;         // [num_blocks, block_size, kv_heads, row]: keys in the first `padded` columns
   const int32_t* tables;     // [entries, table_width]
   const int32_t* row_entry;  // [rows]
   const int64_t* lens;       // [rows]: keys the row sees
@@ -20,14 +20,17 @@ struct LatentDecodeArgs {
   int64_t num_blocks;
   int64_t q_row, q_head, out_row, out_head;      // elements
   int table_width, block_size, heads, kv_heads, padded, values, parts;
+  int row, value_col;        // columns of a cached row; where its values start (0: they are the keys)
   float scale_log2;
   // the windowed form
   const float* slopes;       // [H] or null: slope * distance is taken off a score (natural units)
-  const void* gate;          // [rows, gate_row], head h's columns at h * gate_head, or null: the result times sigmoid(gate)
+  const void* gate;          // [rows, gate_row], head h's columns at h * gate_head (1: one number for all), or null: the result
+                             // times sigmoid(gate)
   int64_t gate_row, gate_head;
   int window;                // keys nearer than this are seen; 0: all
   int ring;                  // token p lies at place p mod ring of the table; 0: at place p
   float temp_coef, temp_every;       // scores times 1 + coef ln(floor((p + 1) / every) + 1); every 0: not
+  const float* sinks;        // [H] or null (the merge only): one more exp(sink) in a row's denominator
 };
 
 // Factor of the scores of a query at position p.
@@ -79,9 +82,11 @@ __device__ __forceinline__ void finish4(const LatentDecodeArgs& a, int64_t row, 
   T* p = reinterpret_cast<T*>(a.out) + row * a.out_row + h * a.out_head + col;
   T v[4];
   if (kWindowed && a.gate) {
-    const T* gate = reinterpret_cast<const T*>(a.gate) + row * a.gate_row + h * a.gate_head + col;
+    const bool one = a.gate_head == 1;
+    const T* gate = reinterpret_cast<const T*>(a.gate) + row * a.gate_row + h * a.gate_head + (one ? 0 : col);
     T g[4];
-    if constexpr (sizeof(T) == 4) *reinterpret_cast<uint4*>(g) = *reinterpret_cast<const uint4*>(gate);
+    if (one) g[0] = g[1] = g[2] = g[3] = *gate;
+    else if constexpr (sizeof(T) == 4) *reinterpret_cast<uint4*>(g) = *reinterpret_cast<const uint4*>(gate);
     else *reinterpret_cast<uint2*>(g) = *reinterpret_cast<const uint2*>(gate);
 #pragma unroll
     for (int i = 0; i < 4; ++i) v[i] = from_float<T>(o[i] / (1.f + expf(-to_float(g[i]))));
@@ -105,15 +110,16 @@ __device__ __forceinline__ void store4(const LatentDecodeArgs& a, int row, int p
 }
 
 // bf16: workgroup = (share, kv head and block of 16 HT of its heads, row), four waves; RS = padded rank / 32, VS = value
-// columns / 32 (the first ones of a row).  Tiles of 64 latents go to LDS
+// columns / 32 (the first ones of a row, or with SPLIT the ones behind the key).  Tiles of 64 latents go to LDS
 // once, in chunks of 16 bytes whose place in a row is xor-ed with the key's low bits; wave w takes 16-head tile w % HT and
 // the key subtiles of its share w / HT.  S^T = C Q'^T (keys down the accumulator, heads across the lanes), so that the
 // weights are the operand of O^T += C^T P^T as they lie; C^T comes from the same LDS tile through the transposing loads.  Two
 // tiles in LDS: the next one is on its way while this one is worked on.
-template <int RS, int VS, int HT, bool kWindowed>
-__global__ __launch_bounds__(256, RS > 8 ? 1 : RS > 4 ? 2 : 3) void latent_decode_kernel(const LatentDecodeArgs a) {
+template <int RS, int VS, int HT, bool kWindowed, bool SPLIT = false>
+__global__ __launch_bounds__(256, RS + SPLIT * VS > 8 ? 1 : RS + SPLIT * VS > 4 ? 2 : 3) void latent_decode_kernel(const LatentDecodeArgs a) {
   constexpr int kShares = 4 / HT, kSub = 4 / kShares;      // key shares of a tile, 16-key subtiles of a wave
-  constexpr int RC = 4 * RS, kRow = 16 * RC;               // chunks and bytes of a row
+  constexpr int RB = RS + SPLIT * VS, VC = SPLIT ? 2 * RS : 0;     // 32-column blocks of a row; 16-column groups before its values
+  constexpr int RC = 4 * RB, kRow = 16 * RC;               // chunks and bytes of a row
   constexpr int kXor = (RC & -RC) < 16 ? (RC & -RC) : 16;  // chunks that trade places
   constexpr int kTile = 64 * kRow;
   __shared__ __attribute__((aligned(16))) char lds[2 * kTile];
@@ -158,11 +164,11 @@ __global__ __launch_bounds__(256, RS > 8 ? 1 : RS > 4 ? 2 : 3) void latent_decod
     for (int j = 0; j < kCols; ++j) col_at[j] = row_b + (((2 * j + ((i16 & 3) >> 1)) ^ xb) << 4);
   }
 
-  // a tile: RS chunks per thread, straight into LDS
+  // a tile: RB chunks per thread, straight into LDS
   auto copy = [&](int buffer) __attribute__((always_inline)) {
     const char* cache = reinterpret_cast<const char*>(a.cache) + kv * (int64_t)kRow;
 #pragma unroll
-    for (int i = 0; i < RS; ++i) {
+    for (int i = 0; i < RB; ++i) {
       const uint32_t c = 256u * i + (uint32_t)tid;
       const uint32_t key = c / RC, p = c % RC;
       const char* from = cache + slot_of[buffer][key] * cache_row + ((p ^ (key & (kXor - 1))) << 4);
@@ -235,7 +241,7 @@ __global__ __launch_bounds__(256, RS > 8 ? 1 : RS > 4 ? 2 : 3) void latent_decod
 #pragma unroll
     for (int n = 0; n < 2 * VS; ++n) {
       auto column = [&](int t) __attribute__((always_inline)) {
-        const char* p = col_at[n % kCols] + at_tile + 16 * t * kRow + 32 * (n / kCols * kCols);
+        const char* p = col_at[(n + VC) % kCols] + at_tile + 16 * t * kRow + 32 * ((n + VC) / kCols * kCols);
         return __builtin_bit_cast(uint2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) v4s*)p));
       };
       if constexpr (kSub == 1) {
@@ -319,15 +325,22 @@ __global__ __launch_bounds__(256) void latent_decode_any_kernel(const LatentDeco
   constexpr int kTogether = NE > 8 ? 2 : 4;
   for (int base = k0 + wave * kTogether; base < k1; base += 4 * kTogether) {
     float c[kTogether][NE], s[kTogether];
+    const T* from[kTogether];
 #pragma unroll
     for (int j = 0; j < kTogether; ++j) {
-      const T* p = reinterpret_cast<const T*>(a.cache) + (key_slot(a, table, min(base + j, k1 - 1)) * kv_heads + kv) * a.padded;
+      const T* p = from[j] = reinterpret_cast<const T*>(a.cache) + (key_slot(a, table, min(base + j, k1 - 1)) * kv_heads + kv) * a.row;
       s[j] = 0.f;
 #pragma unroll
       for (int i = 0; i < NE; ++i) {
         c[j][i] = lane + 64 * i < a.padded ? to_float(p[lane + 64 * i]) : 0.f;
         s[j] = fmaf(q[i], c[j][i], s[j]);
       }
+    }
+    if (kWindowed && a.value_col > 0) {             // the values behind the keys take their place
+#pragma unroll
+      for (int j = 0; j < kTogether; ++j)
+#pragma unroll
+        for (int i = 0; i < NE; ++i) c[j][i] = lane + 64 * i < a.values ? to_float(from[j][a.value_col + lane + 64 * i]) : 0.f;
     }
     float m_new = m;
 #pragma unroll
@@ -389,7 +402,8 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const LatentDecodeArg
   if (lane < a.parts) x = a.part_ml[(row * a.parts + lane) * a.heads + h];
   const float m = wave_max(x.x);
   const float w = x.x == -INFINITY ? 0.f : exp2f(x.x - m);
-  const float l = wave_sum(w * x.y);
+  float l = wave_sum(w * x.y);
+  if (a.sinks) l = add_sink(l, m, a.sinks[h]);
   const float f = l > 0.f ? w / l : 0.f;
   for (int c0 = 0; c0 < a.values; c0 += 256) {      // every lane goes round as often: the shares' factors come from all of them
     const int c = c0 + 4 * lane;
@@ -405,33 +419,41 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const LatentDecodeArg
   }
 }
 
-template <int RS, int VS, bool kWindowed>
+template <int RS, int VS, bool kWindowed, bool SPLIT = false>
 static int launch_decode_as(const LatentDecodeArgs& a, int rows, hipStream_t s) {
   const int tiles = (a.heads / a.kv_heads + 15) / 16;
   const dim3 block(256);
   auto grid = [&](int per) { return dim3((unsigned)a.parts, (unsigned)(a.kv_heads * ((tiles + per - 1) / per)), (unsigned)rows); };
-  if (tiles == 1) latent_decode_kernel<RS, VS, 1, kWindowed><<<grid(1), block, 0, s>>>(a);
-  else if (tiles == 2) latent_decode_kernel<RS, VS, 2, kWindowed><<<grid(2), block, 0, s>>>(a);
-  else latent_decode_kernel<RS, VS, 4, kWindowed><<<grid(4), block, 0, s>>>(a);
+  if (tiles == 1) latent_decode_kernel<RS, VS, 1, kWindowed, SPLIT><<<grid(1), block, 0, s>>>(a);
+  else if (tiles == 2) latent_decode_kernel<RS, VS, 2, kWindowed, SPLIT><<<grid(2), block, 0, s>>>(a);
+  else latent_decode_kernel<RS, VS, 4, kWindowed, SPLIT><<<grid(4), block, 0, s>>>(a);
   return launch_status();
 }
 
 template <typename T, bool kWindowed>
 static int launch_any(const LatentDecodeArgs& a, int rows, hipStream_t s) {
   const dim3 grid((unsigned)a.parts, (unsigned)a.heads, (unsigned)rows), block(256);
-  if (a.padded <= 128) latent_decode_any_kernel<T, 2, kWindowed><<<grid, block, 0, s>>>(a);
-  else if (a.padded <= 512) latent_decode_any_kernel<T, 8, kWindowed><<<grid, block, 0, s>>>(a);
-  else if (a.padded <= 1024) latent_decode_any_kernel<T, 16, kWindowed><<<grid, block, 0, s>>>(a);
+  const int widest = max(a.padded, a.values);
+  if (widest <= 128) latent_decode_any_kernel<T, 2, kWindowed><<<grid, block, 0, s>>>(a);
+  else if (widest <= 512) latent_decode_any_kernel<T, 8, kWindowed><<<grid, block, 0, s>>>(a);
+  else if (widest <= 1024) latent_decode_any_kernel<T, 16, kWindowed><<<grid, block, 0, s>>>(a);
   else latent_decode_any_kernel<T, 32, kWindowed><<<grid, block, 0, s>>>(a);
   return launch_status();
 }
 
+// Rows of a key and a value of the same width (window_decode_split.hip), or kNotBuilt.
+constexpr int kNotBuilt = 1 << 30;
+int launch_decode_split(const LatentDecodeArgs& a, int rows, hipStream_t s);
+
 // Width 576 may be 512 value columns and 64 that only the scores read; every other width is read as values whole.
 template <bool kWindowed>
 static int launch_decode(const LatentDecodeArgs& a, int rows, int dtype, hipStream_t s) {
-  int st;
+  int st = kNotBuilt;
   if (dtype == MVLLM_F32) st = launch_any<float, kWindowed>(a, rows, s);
-  else switch (a.padded) {
+  else if (a.value_col > 0) {
+    if constexpr (kWindowed) st = launch_decode_split(a, rows, s);
+    if (st == kNotBuilt) st = launch_any<bf16_t, kWindowed>(a, rows, s);
+  } else switch (a.padded) {
     case 32: st = launch_decode_as<1, 1, kWindowed>(a, rows, s); break;
     case 64: st = launch_decode_as<2, 2, kWindowed>(a, rows, s); break;
     case 96: st = launch_decode_as<3, 3, kWindowed>(a, rows, s); break;

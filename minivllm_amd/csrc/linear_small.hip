@@ -34,6 +34,7 @@ struct LinearArgs {
   void* residual_out;     // [M, K] contiguous: x + residual in the element type; must not alias x or residual
   const float* gamma;     // [K]
   float eps;
+  int gelu;               // plain product only: the result through the tanh form of gelu
 };
 
 // silu(g) * u with the roundings of the two tensor operations (activation.hip): silu in fp32 rounded to T, then the
@@ -226,7 +227,13 @@ __global__ __launch_bounds__(64 * W) void linear_small_kernel(const LinearArgs a
     const int m = m0 + 16 * mt + col;
     T r4[4];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) r4[r] = from_float<T>(s[r] + b4[r]);
+    for (int r = 0; r < 4; ++r) s[r] += b4[r];
+    if (!NORM && !GLU && a.gelu) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) s[r] = gelu_tanh(s[r]);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) r4[r] = from_float<T>(s[r]);
     if constexpr (GLU) {
       // classes 0, 1 hold the gate columns, classes 2, 3 the up columns that meet them 32 lanes further on
       const uint2 mine = *reinterpret_cast<const uint2*>(r4);
@@ -363,16 +370,27 @@ static int linear_check(const void* out, const void* x, const void* w, const voi
 
 using namespace mvllm;
 
-extern "C" int mvllm_linear_small_m(void* out, const void* x, const void* w, const void* bias, int64_t x_row_stride,
-                                    int M, int N, int K, int dtype, void* stream) {
+static int linear_plain(void* out, const void* x, const void* w, const void* bias, int64_t x_row_stride, int M, int N, int K,
+                        int gelu, int dtype, void* stream) {
   const int bad = linear_check(out, x, w, bias, x_row_stride, M, N, K, dtype);
   if (bad || M == 0) return bad;
   LinearArgs a{};
   a.out = out; a.x = x; a.w = w; a.bias = bias; a.x_row_stride = x_row_stride; a.M = M; a.N = N; a.K = K;
+  a.gelu = gelu;
   a.cols = linear_cols(N, true);
   a.row_tiles = linear_row_tiles(M);
   return dtype == MVLLM_BF16 ? launch_linear_fused<bf16_t>(a, false, (hipStream_t)stream)
                              : launch_linear_fused<f16_t>(a, false, (hipStream_t)stream);
+}
+
+extern "C" int mvllm_linear_small_m(void* out, const void* x, const void* w, const void* bias, int64_t x_row_stride,
+                                    int M, int N, int K, int dtype, void* stream) {
+  return linear_plain(out, x, w, bias, x_row_stride, M, N, K, 0, dtype, stream);
+}
+
+extern "C" int mvllm_linear_small_m_gelu(void* out, const void* x, const void* w, const void* bias, int64_t x_row_stride,
+                                         int M, int N, int K, int dtype, void* stream) {
+  return linear_plain(out, x, w, bias, x_row_stride, M, N, K, 1, dtype, stream);
 }
 
 extern "C" int mvllm_linear_small_m_plan(int M, int N, int K, int norm, int glu, int dtype, int* waves) {

@@ -26,7 +26,7 @@ struct WindowPrefillArgs {
   const void* k;              // [total_k, k_row], kv head g at g * k_head: [dim]
   const void* k2;             // [total_k, k2_row]: [rot] or null
   const void* v;              // [total_k, v_row], kv head g at g * v_head: [dim], or null: the keys
-  const void* gate;           // [total_q, gate_row], head h at h * gate_head, or null
+  const void* gate;           // [total_q, gate_row], head h at h * gate_head (1: one number for all its columns), or null
   const int32_t* cu_q;        // [num_seqs + 1]
   const int32_t* cu_k;        // [num_seqs + 1]
   const int64_t* positions;   // [total_q] (temperature)
@@ -379,7 +379,14 @@ __global__ __launch_bounds__(256, KS1 > 8 ? 1 : 2) void window_prefill_kernel(co
     if (r0 + row >= seq_len) continue;
     const int64_t t = (int64_t)seq_start + r0 + row;
     if (a.gate) {
-      const uint4 gw = *reinterpret_cast<const uint4*>(reinterpret_cast<const bf16_t*>(a.gate) + t * a.gate_row + (int64_t)h * a.gate_head + 8 * p);
+      const bf16_t* gate = reinterpret_cast<const bf16_t*>(a.gate) + t * a.gate_row + (int64_t)h * a.gate_head;
+      uint4 gw;
+      if (a.gate_head == 1) {
+        const uint32_t two = (uint32_t)gate->bits * 0x10001u;
+        gw = make_uint4(two, two, two, two);
+      } else {
+        gw = *reinterpret_cast<const uint4*>(gate + 8 * p);
+      }
       auto gated = [](uint32_t x, uint32_t y) __attribute__((always_inline)) {
         auto sig = [](float z) __attribute__((always_inline)) { return __builtin_amdgcn_rcpf(1.f + __expf(-z)); };
         return pack2<bf16_t>(lo_to_float<bf16_t>(x) * sig(lo_to_float<bf16_t>(y)), hi_to_float<bf16_t>(x) * sig(hi_to_float<bf16_t>(y)));
@@ -410,5 +417,7 @@ static int launch_window_prefill(const WindowPrefillArgs& a, hipStream_t s) {
 constexpr int kNoTiles = 1 << 30;      // no tiled kernel is built for the sizes
 // keys of two parts and values of their own (window_prefill_latent.hip), or kNoTiles
 int launch_window_prefill_parts(const WindowPrefillArgs& a, hipStream_t stream);
+// keys of one part and values of their own (window_prefill_heads.hip), or kNoTiles
+int launch_window_prefill_heads(const WindowPrefillArgs& a, hipStream_t stream);
 
 }  // namespace mvllm

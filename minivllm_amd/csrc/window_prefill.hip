@@ -67,7 +67,7 @@ __global__ __launch_bounds__(256) void window_prefill_any_kernel(const WindowPre
     const int c = lane + 64 * i;
     if (c >= a.dim) continue;
     float x = o[i] * inv;
-    if (a.gate) x /= 1.f + expf(-to_float(reinterpret_cast<const T*>(a.gate)[t * a.gate_row + (int64_t)h * a.gate_head + c]));
+    if (a.gate) x /= 1.f + expf(-to_float(reinterpret_cast<const T*>(a.gate)[t * a.gate_row + (int64_t)h * a.gate_head + (a.gate_head == 1 ? 0 : c)]));
     out[c] = from_float<T>(x);
   }
 }
@@ -97,6 +97,7 @@ static int launch_shared(const WindowPrefillArgs& a, hipStream_t s) {
 }
 
 __attribute__((weak)) int launch_window_prefill_parts(const WindowPrefillArgs&, hipStream_t) { return kNoTiles; }
+__attribute__((weak)) int launch_window_prefill_heads(const WindowPrefillArgs&, hipStream_t) { return kNoTiles; }
 
 }  // namespace mvllm
 
@@ -113,7 +114,7 @@ extern "C" int mvllm_window_prefill(void* out, int64_t out_row_stride, int64_t o
   if (dtype_size(dtype) == 0) return MVLLM_ERR_BAD_DTYPE;
   if (num_seqs < 0 || total_q < 0 || num_heads <= 0 || num_kv_heads <= 0 || num_heads % num_kv_heads != 0 || dim <= 0 || rot < 0 ||
       window < 0 || (k2 == nullptr) != (rot == 0) || q_head_stride < dim + rot || out_head_stride < dim || k_row_stride < dim ||
-      (v && v_row_stride < dim) || (k2 && k2_row_stride < rot) || (gate && gate_head_stride < dim) || !(temp_every >= 0.f))
+      (v && v_row_stride < dim) || (k2 && k2_row_stride < rot) || (gate && gate_head_stride != 1 && gate_head_stride < dim) || !(temp_every >= 0.f))
     return MVLLM_ERR_BAD_SHAPE;
   if (dtype == MVLLM_F16 || num_heads > 65535 || total_q > ((int64_t)1 << 30)) return MVLLM_ERR_UNSUPPORTED;
   if (num_seqs == 0 || total_q == 0) return MVLLM_OK;
@@ -126,12 +127,13 @@ extern "C" int mvllm_window_prefill(void* out, int64_t out_row_stride, int64_t o
   a.kv_heads = num_kv_heads; a.dim = dim; a.rot = rot; a.window = window; a.scale_log2 = scale * kLog2e;
   a.temp_coef = temp_coef; a.temp_every = temp_every;
   hipStream_t s = (hipStream_t)stream;
+  const bool one_gate = gate_head_stride == 1;       // read number by number
   const int64_t strides[] = {out_row_stride, out_head_stride, q_row_stride, q_head_stride, k_row_stride, k_head_stride, k2_row_stride,
-                             v_row_stride, v_head_stride, gate_row_stride, gate_head_stride};
-  bool tiles = dtype == MVLLM_BF16 && aligned16(out) && aligned16(q) && aligned16(k) && aligned16(k2) && aligned16(v) && aligned16(gate) &&
-               k_row_stride < (1 << 24) && k2_row_stride < (1 << 24) && v_row_stride < (1 << 24) && (v == nullptr) == (k2 == nullptr) && !(v && slopes);
+                             v_row_stride, v_head_stride, one_gate ? 0 : gate_row_stride, one_gate ? 0 : gate_head_stride};
+  bool tiles = dtype == MVLLM_BF16 && aligned16(out) && aligned16(q) && aligned16(k) && aligned16(k2) && aligned16(v) && (one_gate || aligned16(gate)) &&
+               k_row_stride < (1 << 24) && k2_row_stride < (1 << 24) && v_row_stride < (1 << 24) && (v || !k2) && !(v && slopes);
   for (int64_t x : strides) tiles = tiles && x % 8 == 0;
-  const int st = !tiles ? kNoTiles : v ? launch_window_prefill_parts(a, s) : launch_shared(a, s);
+  const int st = !tiles ? kNoTiles : k2 ? launch_window_prefill_parts(a, s) : v ? launch_window_prefill_heads(a, s) : launch_shared(a, s);
   if (st != kNoTiles) return st;
   return dtype == MVLLM_F32 ? launch_any<float>(a, s) : launch_any<bf16_t>(a, s);
 }

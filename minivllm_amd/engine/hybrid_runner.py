@@ -1,5 +1,5 @@
-"""Runner of models that run ragged steps and keep recurrent state (models/sokevik.py, models/niridra.py, models/fevosun.py): portions of
-prompts and decoded tokens in one batch, a cache manager of its own, and the captured decode step of ``ModelRunner`` over
+"""Runner of models that run ragged steps and keep recurrent state (models/sokevik.py, models/niridra.py, models/fevosun.py,
+models/lenuzen.py): portions of prompts and decoded tokens in one batch, a cache manager of its own, and the captured decode step of ``ModelRunner`` over
 more static buffers.
 
 Engine keys as for ``ModelRunner``; ``max_cached_blocks`` counts the blocks of each attention window's pool,

@@ -30,6 +30,7 @@ class WindowStep:
     num_prefixed: int = 0                             # rows of pieces with a cached prefix
     num_fresh: int = 0
     dst_row: Optional[torch.Tensor] = None            # int32 [T], None: rows stay in order
+    src_row: Optional[torch.Tensor] = None            # int32 [T], the way back, None: rows stay in order
     slots: Optional[torch.Tensor] = None              # int64 [T], stored before attention (-1: not)
     late_slots: Optional[torch.Tensor] = None         # int64 [T] in dst_row order, stored after attention, or None
     chunk_lens: Optional[torch.Tensor] = None         # int64 [num_decode]
@@ -178,6 +179,7 @@ def _window_arrays(items, window, index, block_size, cu):
     out = dict(slots=slots)
     if not sorted_as_packed:
         out["dst_row"] = dst
+        out["src_row"] = order.astype(np.int32)
     if any_late:
         out["late_slots"] = late[order]
     if single:

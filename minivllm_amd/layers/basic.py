@@ -10,7 +10,7 @@ import torch
 import torch.nn as nn
 import torch.nn.functional as F
 
-from minivllm_amd.layers.fused import add_rms_norm, linear_small_m, linear_small_m_takes, silu_and_mul
+from minivllm_amd.layers.fused import add_rms_norm, gelu_tanh, linear_small_m, linear_small_m_takes, silu_and_mul
 
 
 class Linear(nn.Linear):
@@ -21,10 +21,12 @@ class Linear(nn.Linear):
         super().__init__(in_features, out_features, bias=bias)
         self.small_rows = small_rows
 
-    def forward(self, x):
+    def forward(self, x, gelu: bool = False):
+        """``gelu``: the result through the tanh form of gelu."""
         if self.small_rows and linear_small_m_takes(x, self.weight, self.small_rows):
-            return linear_small_m(x, self.weight, self.bias)
-        return F.linear(x, self.weight, self.bias)
+            return linear_small_m(x, self.weight, self.bias, gelu)
+        y = F.linear(x, self.weight, self.bias)
+        return gelu_tanh(y, out=y) if gelu else y
 
 
 class RMSNorm(nn.Module):

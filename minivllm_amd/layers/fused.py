@@ -20,7 +20,8 @@ from minivllm_amd import _C
 
 __all__ = ["qk_norm_rope_store", "sample_tokens", "sample_tokens_into", "decode_advance", "add_rms_norm", "silu_and_mul", "linear_small_m", "linear_small_m_takes", "norm_linear_small_m", "norm_linear_small_m_takes",
            "lm_head_sample", "lm_head_sample_takes", "lm_head_sample_workspace_bytes", "norm_conv", "head_rope_store",
-           "head_unrotate_gate", "chunk_decode_step", "stream_embed_norm", "stream_norm", "gated_unit"]
+           "head_unrotate_gate", "chunk_decode_step", "stream_embed_norm", "stream_norm", "gated_unit", "gelu_tanh", "post_norm",
+           "embed_rows"]
 
 
 def _ptr(t):
@@ -275,6 +276,19 @@ def gated_unit(x: torch.Tensor, out: torch.Tensor | None = None, alpha: float = 
     return out
 
 
+def gelu_tanh(x: torch.Tensor, out: torch.Tensor | None = None) -> torch.Tensor:
+    """The tanh form of gelu of x's rows (strided; ``out`` may be x itself)."""
+    _C.require_cuda(x, out)
+    rows, width = x.shape
+    out = torch.empty((rows, width), dtype=x.dtype, device=x.device) if out is None else out
+    if tuple(out.shape) != (rows, width) or out.dtype != x.dtype or out.stride(1) != 1 or x.stride(1) != 1:
+        raise ValueError(f"x and out must be ({rows}, {width}) in one dtype with dense rows")
+    st = _C.load().mvllm_gelu_tanh(_ptr(out), out.stride(0) if rows > 1 else width, _ptr(x), x.stride(0) if rows > 1 else width, rows,
+                                   width, _C.dtype_code(x.dtype), _C.current_stream_ptr(x.device))
+    _C.check(st, "gelu_tanh")
+    return out
+
+
 def linear_small_m_takes(x: torch.Tensor, weight: torch.Tensor, max_rows: int = 64) -> bool:
     """Whether ``linear_small_m`` is built for this call: at most 64 rows, bf16 / fp16 on the GPU, N a multiple of 16,
     K a multiple of 512, rows of x dense."""
@@ -284,11 +298,12 @@ def linear_small_m_takes(x: torch.Tensor, weight: torch.Tensor, max_rows: int = 
             and x.data_ptr() % 16 == 0)
 
 
-def linear_small_m(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None = None) -> torch.Tensor:
+def linear_small_m(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None = None, gelu: bool = False) -> torch.Tensor:
     """``F.linear(x, weight, bias)`` for the few rows of a decode step (the reference's projections,
     models/qwen3.py:90-94, 118, 121-160, are library GEMMs): one HIP launch in which every wave asks for its whole
     share of the weights at once, so the call costs about one memory round trip.  x (M <= 64, K), weight (N, K)
-    contiguous, bias (N,) or None, all in one 16-bit dtype; fp32 accumulation.  Returns (M, N)."""
+    contiguous, bias (N,) or None, all in one 16-bit dtype; fp32 accumulation.  ``gelu``: the result through the tanh form
+    of gelu, rounded once.  Returns (M, N)."""
     _C.require_cuda(x, weight, bias)
     if x.dim() != 2 or weight.dim() != 2 or weight.shape[1] != x.shape[1]:
         raise ValueError(f"x (M, K) and weight (N, K) expected, got {tuple(x.shape)} and {tuple(weight.shape)}")
@@ -299,8 +314,10 @@ def linear_small_m(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | N
     m, k = x.shape
     n = weight.shape[0]
     out = torch.empty(m, n, dtype=x.dtype, device=x.device)
-    st = _C.load().mvllm_linear_small_m(_ptr(out), _ptr(x), _ptr(weight), _ptr(bias), x.stride(0) if m > 1 else k,
-                                        m, n, k, _C.dtype_code(x.dtype), _C.current_stream_ptr(x.device))
+    lib = _C.load()
+    st = (lib.mvllm_linear_small_m_gelu if gelu else lib.mvllm_linear_small_m)(
+        _ptr(out), _ptr(x), _ptr(weight), _ptr(bias), x.stride(0) if m > 1 else k, m, n, k, _C.dtype_code(x.dtype),
+        _C.current_stream_ptr(x.device))
     _C.check(st, "linear_small_m")
     return out
 
@@ -456,21 +473,31 @@ def head_rope_store(proj: torch.Tensor, positions: torch.Tensor, num_heads: int,
                     eps: float = 1e-6, q_scale: float = 1.0, rot_table: torch.Tensor | None = None,
                     v_table: torch.Tensor | None = None, interleaved: bool = True, dst_row: torch.Tensor | None = None,
                     slots: torch.Tensor | None = None, k_cache: torch.Tensor | None = None,
-                    v_cache: torch.Tensor | None = None, need_kv: bool = True):
-    """Per-head norms, rotary embedding, rotated values and the cache store of packed projection rows [q | k | v | ...].
+                    v_cache: torch.Tensor | None = None, need_kv: bool = True, row_norm: bool = False, unit_qk: bool = False,
+                    unit_v: bool = False, head_scale: torch.Tensor | None = None, kv_cache: torch.Tensor | None = None,
+                    kv_out: torch.Tensor | None = None, kv_rows: torch.Tensor | None = None):
+    """Norms, rotary embedding, rotated values and the cache store of packed projection rows [q | k | v | ...].
 
     ``rot_table`` float32 (max_position, rot_dims / 2, 2) and ``v_table`` (max_position, vdim / 2, 2) hold (cos, sin) per
     pair; ``interleaved`` pairs dims 2i and 2i + 1, otherwise the halves.  Heads leave ``head_dim`` wide, zeros past
-    ``dim`` / ``vdim``; row t goes to row ``dst_row[t]`` of the packed results.  Returns (q, k, v), k and v None unless
-    ``need_kv``."""
-    _C.require_cuda(proj, positions, gain_q, gain_k, rot_table, v_table, dst_row, slots, k_cache, v_cache)
+    ``dim`` / ``vdim``; row t goes to row ``dst_row[t]`` of the packed results.  Gains norm every head, with ``row_norm`` all
+    heads of a row at once (gains of that many numbers); ``unit_qk`` / ``unit_v``: every head of q and k behind the rotation /
+    of v over its root mean square; ``head_scale`` float32 (num_heads,): a further factor of q.  Returns (q, k, v), k and v None
+    unless ``need_kv``.
+
+    With ``kv_cache`` (blocks, block_size, num_kv_heads, 2 head_dim) a key and its value are neighbours; ``kv_out`` (n,
+    num_kv_heads, 2 head_dim) takes them packed at rows ``kv_rows`` int64 (negative: none; None: t).  Returns q."""
+    _C.require_cuda(proj, positions, gain_q, gain_k, rot_table, v_table, dst_row, slots, k_cache, v_cache, head_scale, kv_cache,
+                    kv_out, kv_rows)
     rows = proj.shape[0]
     if proj.dim() != 2 or (proj.shape[1] > 1 and proj.stride(1) != 1) or proj.shape[1] < num_heads * dim + num_kv_heads * (dim + vdim):
         raise ValueError("proj must be (T, >= q + k + v columns) with dense rows")
     _check(positions, torch.int64, (rows,), "positions")
     for name, g in (("gain_q", gain_q), ("gain_k", gain_k)):
         if g is not None:
-            _check(g, torch.float32, (dim,), name)
+            _check(g, torch.float32, (dim * (1 if not row_norm else num_heads if name == "gain_q" else num_kv_heads),), name)
+    if head_scale is not None:
+        _check(head_scale, torch.float32, (num_heads,), "head_scale")
     tables = [t for t in (rot_table, v_table) if t is not None]
     max_position = min((t.shape[0] for t in tables), default=1 << 62)
     rot = 0 if rot_table is None else 2 * rot_table.shape[1]
@@ -482,20 +509,39 @@ def head_rope_store(proj: torch.Tensor, positions: torch.Tensor, num_heads: int,
     num_slots = 0
     if slots is not None:
         _check(slots, torch.int64, (rows,), "slots")
-        for name, c in (("k_cache", k_cache), ("v_cache", v_cache)):
-            _check(c, proj.dtype, (*c.shape[:2], num_kv_heads, head_dim), name)
-        num_slots = min(k_cache.shape[0] * k_cache.shape[1], v_cache.shape[0] * v_cache.shape[1])
+        for name, c, d in (("kv_cache", kv_cache, 2 * head_dim),) if kv_cache is not None else (
+                ("k_cache", k_cache, head_dim), ("v_cache", v_cache, head_dim)):
+            _check(c, proj.dtype, (*c.shape[:2], num_kv_heads, d), name)
+            num_slots = min(num_slots or c.shape[0] * c.shape[1], c.shape[0] * c.shape[1])
     q = torch.empty((rows, num_heads, head_dim), dtype=proj.dtype, device=proj.device)
-    k = torch.empty((rows, num_kv_heads, head_dim), dtype=proj.dtype, device=proj.device) if need_kv else None
-    v = torch.empty_like(k) if need_kv else None
-    st = _C.load().mvllm_head_rope_store(
-        _ptr(q), _ptr(k), _ptr(v), _ptr(proj), proj.stride(0) if rows > 1 else proj.shape[1], _ptr(gain_q), _ptr(gain_k),
-        float(eps), float(q_scale), _ptr(rot_table), rot, _ptr(v_table), int(interleaved), max_position, _ptr(positions),
-        _ptr(dst_row), _ptr(slots), _ptr(k_cache if slots is not None else None), _ptr(v_cache if slots is not None else None),
-        num_slots, rows, num_heads, num_kv_heads, dim, vdim, head_dim, _C.dtype_code(proj.dtype),
-        _C.current_stream_ptr(proj.device))
+    k = v = None
+    behind = head_dim * proj.element_size()
+    if kv_cache is not None:
+        caches = (kv_cache.data_ptr(), kv_cache.data_ptr() + behind) if slots is not None else (0, 0)
+        packed = (0, 0)
+        if kv_out is not None:
+            _check(kv_out, proj.dtype, (kv_out.shape[0], num_kv_heads, 2 * head_dim), "kv_out")
+            if kv_rows is None and kv_out.shape[0] < rows:
+                raise ValueError("kv_out has fewer rows than proj")
+            packed = (kv_out.data_ptr(), kv_out.data_ptr() + behind)
+        if kv_rows is not None:
+            _check(kv_rows, torch.int64, (rows,), "kv_rows")
+        if dst_row is not None:
+            raise ValueError("kv_rows instead of dst_row")
+    else:
+        if need_kv:
+            k = torch.empty((rows, num_kv_heads, head_dim), dtype=proj.dtype, device=proj.device)
+            v = torch.empty_like(k)
+        caches = (_ptr(k_cache), _ptr(v_cache)) if slots is not None else (0, 0)
+        packed, kv_rows = (_ptr(k), _ptr(v)), None
+    st = _C.load().mvllm_head_norm_rope_store(
+        _ptr(q), *packed, _ptr(kv_rows), _ptr(proj), proj.stride(0) if rows > 1 else proj.shape[1], _ptr(gain_q), _ptr(gain_k),
+        int(row_norm) + 2 * int(unit_qk) + 4 * int(unit_v), float(eps), float(q_scale), _ptr(head_scale), _ptr(rot_table), rot,
+        _ptr(v_table), int(interleaved), max_position, _ptr(positions), _ptr(dst_row), _ptr(slots), *caches,
+        head_dim * (1 if kv_cache is None else 2), num_slots, rows, num_heads, num_kv_heads, dim, vdim, head_dim,
+        _C.dtype_code(proj.dtype), _C.current_stream_ptr(proj.device))
     _C.check(st, "head_rope_store")
-    return q, k, v
+    return q if kv_cache is not None else (q, k, v)
 
 
 def head_unrotate_gate(o: torch.Tensor, positions: torch.Tensor, vdim: int, gate: torch.Tensor | None = None,
@@ -624,4 +670,42 @@ def stream_norm(x: torch.Tensor, y, hc_out: torch.Tensor, hc_mix: torch.Tensor, 
         _ptr(own), 0 if own is None else max(own.stride(0), width), _ptr(gate), 1 if gate is None else max(gate.stride(0), 1), _ptr(scale), _ptr(hc_out), _ptr(hc_mix), _ptr(hc_in), _ptr(gain), float(eps),
         rows, streams, width, _C.dtype_code(dtype), _C.current_stream_ptr(x.device))
     _C.check(st, "stream_norm")
+    return out, x
+
+
+def embed_rows(tokens: torch.Tensor, embed: torch.Tensor, scale: float, padded: int = 0):
+    """The front of a model whose sublayers read the residual itself: (embed[token] * scale in embed's dtype, zeros up to
+    ``padded`` columns; the same in float32)."""
+    _C.require_cuda(tokens, embed)
+    rows, width = tokens.numel(), embed.shape[1]
+    padded = max(padded, width)
+    _check(tokens, torch.int64, (rows,), "tokens")
+    _check(embed, embed.dtype, embed.shape, "embed")
+    out = torch.empty((rows, padded), dtype=embed.dtype, device=embed.device)
+    x = torch.empty((rows, width), dtype=torch.float32, device=embed.device)
+    st = _C.load().mvllm_embed_rows(_ptr(out), padded, _ptr(x), _ptr(embed), embed.shape[0], float(scale), _ptr(tokens), rows, width,
+                                    _C.dtype_code(embed.dtype), _C.current_stream_ptr(embed.device))
+    _C.check(st, "embed_rows")
+    return out, x
+
+
+def post_norm(x: torch.Tensor, y: torch.Tensor, gain: torch.Tensor, eps: float, centred: bool = True,
+              final_gain: torch.Tensor | None = None, padded: int = 0, want_x: bool = True):
+    """``x + norm(y) * gain`` into x (float32 (T, W), in place unless ``want_x`` is False), norm with the mean taken off
+    (``centred``) or not.  Returns (what is read next, x): the new x in y's dtype with zeros up to ``padded`` columns, or with
+    ``final_gain`` its norm times that."""
+    _C.require_cuda(x, y, gain, final_gain)
+    rows, width = x.shape
+    padded = max(padded, width)
+    _check(x, torch.float32, (rows, width), "x")
+    for name, g in (("gain", gain), ("final_gain", final_gain)):
+        if g is not None:
+            _check(g, torch.float32, (width,), name)
+    if y.dim() != 2 or y.shape[0] != rows or y.shape[1] < width or y.stride(1) != 1:
+        raise ValueError(f"y must be ({rows}, >= {width}) with dense rows")
+    out = torch.empty((rows, padded), dtype=y.dtype, device=y.device)
+    st = _C.load().mvllm_post_norm(_ptr(out), padded, _ptr(x if want_x else None), _ptr(x), _ptr(y), max(y.stride(0), width), _ptr(gain),
+                                   _ptr(final_gain), float(eps), int(centred), rows, width, _C.dtype_code(y.dtype),
+                                   _C.current_stream_ptr(y.device))
+    _C.check(st, "post_norm")
     return out, x

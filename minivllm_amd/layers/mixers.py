@@ -2,9 +2,9 @@
 memories.
 
 ``RaggedAttention`` runs a step's pieces through the framework's decode, paged-prefill and packed-prefill kernels,
-``LatentAttention`` through the latent decode and the same prefill kernels, ``SharedKeyAttention`` and ``RotaryLatentAttention``
-through the windowed kernels; ``MatrixMemory`` runs it through the mLSTM
-recurrence, ``DecayMemory`` through the one with constant decays.  ``RaggedAttention`` and the memories take the packed
+``LatentAttention`` through the latent decode and the same prefill kernels, ``SharedKeyAttention``, ``RotaryLatentAttention`` and
+``UnitHeadAttention`` through the windowed kernels, ``TalkingAttention`` through the ones that mix heads' scores;
+``MatrixMemory`` runs it through the mLSTM recurrence, ``DecayMemory`` through the one with constant decays.  ``RaggedAttention`` and the memories take the packed
 projection of the step's rows and return what the output projection reads.  Caches and states are assigned from outside, as
 for ``layers.attention.Attention``."""
 from __future__ import annotations
@@ -21,6 +21,7 @@ from minivllm_amd.layers.fused import head_rope_store, head_unrotate_gate
 from minivllm_amd.layers.basic import Linear
 from minivllm_amd.layers.latent import (head_linear, latent_decode, latent_decode_workspace_bytes, latent_norm_store,
                                         latent_width)
+from minivllm_amd.layers.talk import talk_decode, talk_decode_workspace_bytes, talk_head_size, talk_prefill
 from minivllm_amd.layers.window import (copy_rows, head_rope, head_size, latent_layout, latent_rope_store, shared_part_size,
                                         window_decode, window_decode_workspace_bytes, window_prefill)
 from minivllm_amd.layers.recurrent import DecayMemoryState, MlstmState, decay_memory, gate_linear, gated_row_norm, mlstm
@@ -342,3 +343,130 @@ class RotaryLatentAttention(nn.Module):
         if view.num_long:
             k, v = F.linear(rows[:, :rot], self.up_kv).unflatten(-1, (2, heads, d)).unbind(1)
             window_prefill(o[a:], q[a:], k, view.cu_q, view.cu_k, self.scale, self.view.size, k2=rows[:, rot:rot + self.rot_size], v=v)
+
+
+class _HeadsAttention(nn.Module):
+    """Grouped heads between projections of their own: rows q | k | v | (a gate per head) in front, heads side by side behind.
+    Heads are ``head_dim`` wide behind the front projection, zeros past ``dim`` / ``vdim``.  ``table``: float32 (max_position,
+    dims / 2, 2) or None, assigned from outside; ``window``: index into the step's windows."""
+
+    def __init__(self, width, num_heads, num_kv_heads, dim, vdim, head_dim, scale, window, block_size, dtype, eps, interleaved, bias,
+                 gated, small_rows):
+        super().__init__()
+        self.num_heads, self.num_kv_heads, self.dim, self.vdim, self.head_dim = num_heads, num_kv_heads, dim, vdim, head_dim
+        self.window, self.block_size, self.dtype, self.eps, self.interleaved = window, block_size, dtype, eps, interleaved
+        self.scale, self.gated = scale, gated
+        self.gate_col = num_heads * dim + num_kv_heads * (dim + vdim)
+        self.out_size = num_heads * head_dim
+        with torch.device("meta"):
+            self.proj = Linear(width, round_up(self.gate_col + (num_heads if gated else 0), 16), bias=bias, small_rows=small_rows)
+            self.out = Linear(self.out_size, width, bias=False, small_rows=small_rows)
+        self.table = None
+        self.decode_workspace = None
+
+    @torch.no_grad()
+    def load(self, get, matrix, inputs):
+        """``get(name)``: checkpoint tensor, ``matrix(t)``: on the device in the model's type; ``inputs``: columns of h."""
+        p, total = lambda t: nn.Parameter(t.contiguous(), requires_grad=False), self.proj.out_features
+        self.proj.weight = p(pad_to(torch.cat([matrix(get(n)) for n in ("q", "k", "v") + ("g",) * self.gated]), total, inputs))
+        if self.proj.bias is not None:
+            self.proj.bias = p(F.pad(torch.cat([matrix(get(n + ".b")) for n in ("q", "k", "v")]), (0, total - self.gate_col)))
+        self.out.weight = p(pad_heads(matrix(get("o")).t().contiguous(), self.num_heads, self.head_dim).t())
+        self.f32 = lambda name: get(name).to(device=self.out.weight.device, dtype=torch.float32).contiguous()
+
+    def heads(self, proj, step, **how):
+        # log2 e goes into q with the scale, in fp32, as in RaggedAttention
+        return head_rope_store(proj, step.positions, self.num_heads, self.num_kv_heads, self.dim, self.vdim, self.head_dim,
+                               eps=self.eps, q_scale=self.scale * LOG2E, rot_table=self.table, interleaved=self.interleaved, **how)
+
+
+class UnitHeadAttention(_HeadsAttention):
+    """Softmax attention in a sliding window over heads of unit root mean square: rotated queries and keys (``unit_qk``), values
+    (``unit_v``), with a learned factor per head on the scores and a sigmoid gate per head on the results.  A cached row holds a
+    key and behind it its value."""
+
+    def __init__(self, width, num_heads, num_kv_heads, dim, vdim, scale, window, view: SlidingWindow, block_size, dtype, eps,
+                 interleaved=True, unit_qk=True, unit_v=True, bias=True, gated=True, small_rows=0):
+        super().__init__(width, num_heads, num_kv_heads, dim, vdim, head_size(dim, vdim), scale, window, block_size, dtype, eps,
+                         interleaved, bias, gated, small_rows)
+        self.view, self.unit_qk, self.unit_v = view, unit_qk, unit_v
+        self.cache = torch.tensor([])                                     # (blocks, block_size, G, 2 * head_dim)
+        self.head_scale = None
+
+    def load(self, get, matrix, inputs):
+        super().load(get, matrix, inputs)
+        self.head_scale = self.f32("temp")
+
+    def allocate(self, num_blocks, device):
+        self.cache = torch.zeros(num_blocks, self.block_size, self.num_kv_heads, 2 * self.head_dim, dtype=self.dtype, device=device)
+
+    def workspace_bytes(self, batch, table_width):
+        return window_decode_workspace_bytes(batch, self.num_heads, self.num_kv_heads, 2 * self.head_dim, self.head_dim,
+                                             table_width * self.block_size, self.dtype)
+
+    def forward(self, h, step):
+        view, d, a = step.windows[self.window], self.head_dim, step.windows[self.window].absorbed
+        proj = self.proj(h)
+        keys = None
+        if view.num_long:
+            keys = torch.empty((view.num_keys, self.num_kv_heads, 2 * d), dtype=proj.dtype, device=proj.device)
+            if view.past_slots is not None:                               # out of the ring before the new ones go in
+                copy_rows(self.cache.view(-1, keys[0].numel()), keys.flatten(1), view.past_rows, view.past_slots)
+        q = self.heads(proj, step, unit_qk=self.unit_qk, unit_v=self.unit_v, head_scale=self.head_scale, kv_cache=self.cache,
+                       slots=view.slots, kv_out=keys, kv_rows=view.key_rows)
+        gate = proj[:, self.gate_col:self.gate_col + self.num_heads] if self.gated else None
+        cut = lambda *rows: None if gate is None else gate[slice(*rows)]
+        o = torch.empty_like(q)
+        if a:
+            window_decode(o[:a], q[:a], self.cache, view.tables, step.row_entry, view.lens, 1.0 / LOG2E, self.view.size, self.view.places,
+                          gate=cut(0, a), workspace=self.decode_workspace)
+        if view.num_long:
+            window_prefill(o[a:], q[a:], keys[..., :d], view.cu_q, view.cu_k, 1.0 / LOG2E, self.view.size, v=keys[..., d:], gate=cut(a, None))
+        return self.out(o.flatten(1))
+
+
+class TalkingAttention(_HeadsAttention):
+    """Chunked attention whose heads' scores are mixed before the softmax (``talk``), with a sink; queries and keys are normed over
+    all heads of a row at once, then rotated."""
+
+    def __init__(self, width, num_heads, num_kv_heads, dim, vdim, scale, window, block_size, dtype, eps, interleaved=True, sink=None,
+                 small_rows=0):
+        super().__init__(width, num_heads, num_kv_heads, dim, vdim, talk_head_size(dim, vdim), scale, window, block_size, dtype, eps,
+                         interleaved, False, False, small_rows)
+        if num_heads > 64 or self.out_size > 16384:
+            raise ValueError(f"{num_heads} heads of {self.head_dim}: at most 64 and 16384 columns together")
+        self.sink = sink                                                  # one number for all heads, or None
+        self.k_cache = self.v_cache = torch.tensor([])                    # (blocks, block_size, G, head_dim)
+
+    def load(self, get, matrix, inputs):
+        super().load(get, matrix, inputs)
+        self.gain_q, self.gain_k, self.talk = (self.f32(n) for n in ("q.norm", "k.norm", "talk"))
+        self.sinks = None if self.sink is None else torch.full((self.num_heads,), float(self.sink), device=self.talk.device)
+
+    def allocate(self, num_blocks, device):
+        shape = (num_blocks, self.block_size, self.num_kv_heads, self.head_dim)
+        self.k_cache, self.v_cache = (torch.zeros(shape, dtype=self.dtype, device=device) for _ in range(2))
+
+    def workspace_bytes(self, batch, table_width):
+        return talk_decode_workspace_bytes(batch, self.num_heads, self.num_kv_heads, self.head_dim, table_width * self.block_size, self.dtype)
+
+    def forward(self, h, step):
+        w = step.windows[self.window]
+        a, b = w.num_decode, w.num_decode + w.num_prefixed
+        q, k, v = self.heads(self.proj(h), step, gain_q=self.gain_q, gain_k=self.gain_k, row_norm=True, dst_row=w.dst_row, slots=w.slots,
+                             k_cache=self.k_cache, v_cache=self.v_cache, need_kv=w.num_fresh > 0 or w.late_slots is not None)
+        o = torch.empty_like(q)
+        if a:
+            talk_decode(o[:a], q[:a], self.k_cache, self.v_cache, w.decode_tables, w.chunk_lens, self.talk, self.sinks, self.decode_workspace)
+
+        def prefill(lo, hi, *keys, **how):                                # results go back to where the rows came from
+            where = dict(out=o, out_rows=w.src_row[lo:hi]) if w.src_row is not None else dict(out=o[lo:hi])
+            talk_prefill(q=q[lo:hi], k=keys[0], v=keys[1], talk=self.talk, sinks=self.sinks, **where, **how)
+
+        if b > a:
+            prefill(a, b, self.k_cache, self.v_cache, cu_q=w.prefixed_cu_q, cu_k=w.prefixed_cu_k, block_tables=w.prefixed_tables)
+        if w.num_fresh:
+            prefill(b, q.shape[0], k[b:], v[b:], cu_q=w.fresh_cu)
+        if w.late_slots is not None:
+            store_kvcache(k, v, self.k_cache, self.v_cache, w.late_slots, self.block_size)
+        return self.out(o.flatten(1))

@@ -1,4 +1,4 @@
-"""Operators of windowed attention whose cached rows are keys and values at once, or make both.
+"""Operators of windowed attention whose cached rows are keys and values at once, make both, or hold both side by side.
 
 All of it calls libminivllm_amd.so on the current torch stream; tensors are read and written where projections leave and take
 them (dense rows, any row stride)."""
@@ -141,6 +141,15 @@ def _heads(name, t, like, rows, heads, least):
     return _stride(t, 0, heads * t.shape[2]), _stride(t, 1, t.shape[2])
 
 
+def _gate(t, like, rows, heads, least):
+    """Strides of a gate: one number per column, or (rows, heads) one per head (head stride 1)."""
+    if t is None or t.dim() == 3:
+        return _heads("gate", t, like, rows, heads, least)
+    if t.dim() != 2 or t.shape[0] < rows or t.shape[1] != heads or t.dtype != like.dtype or (heads > 1 and t.stride(1) != 1):
+        raise ValueError(f"gate must be ({rows}, {heads}) in {like.dtype} with dense rows, got {t.dtype} {tuple(t.shape)}")
+    return _stride(t, 0, heads), 1
+
+
 def _floats(name, t, n):
     if t is not None and (t.dtype != torch.float32 or t.numel() != n or not t.is_contiguous()):
         raise ValueError(f"{name} must be contiguous float32 ({n},)")
@@ -152,7 +161,7 @@ def window_prefill(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, cu_q: to
     """Entries of packed queries q (T, H, dim + rot) over packed keys k (K, G, dim), k2 (K, rot) shared by all heads, values v like k
     (None: the keys), into out (T, H, dim).  Query i of an entry stands at key (keys - queries) + i and sees ``window`` keys up to it
     (0: all); ``slopes`` times the distance is taken off a score, ``temperature`` = (coef, every) makes scores grow with
-    ``positions``, ``gate`` (T, H, dim) multiplies the result with its sigmoid."""
+    ``positions``, ``gate`` (T, H, dim), or (T, H) for one number per head, multiplies the result with its sigmoid."""
     _C.require_cuda(out, q, k, cu_q, cu_k, k2, v, gate, slopes, positions)
     t, heads = q.shape[:2]
     keys, groups, dim = k.shape
@@ -167,7 +176,7 @@ def window_prefill(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, cu_q: to
     st = _C.load().mvllm_window_prefill(
         _ptr(out), *_heads("out", out, q, t, heads, dim), _ptr(q), *_heads("q", q, q, t, heads, dim + rot), _ptr(k),
         *_heads("k", k, q, keys, groups, dim), _ptr(k2), 0 if k2 is None else _stride(k2, 0, rot), _ptr(v),
-        *_heads("v", v, q, keys, groups, dim), _ptr(gate), *_heads("gate", gate, q, t, heads, dim), _ptr(cu_q), _ptr(cu_k),
+        *_heads("v", v, q, keys, groups, dim), _ptr(gate), *_gate(gate, q, t, heads, dim), _ptr(cu_q), _ptr(cu_k),
         _ptr(positions), _ptr(slopes), cu_q.numel() - 1, t, heads, groups, dim, rot, int(window), float(scale),
         float(temperature[0]), float(temperature[1]), _C.dtype_code(q.dtype), _C.current_stream_ptr(q.device))
     _C.check(st, "window_prefill")
@@ -182,12 +191,14 @@ def window_decode(out: torch.Tensor, q: torch.Tensor, cache: torch.Tensor, block
                   lens: torch.Tensor, scale: float, window: int, ring: int, gate: torch.Tensor | None = None,
                   slopes: torch.Tensor | None = None, temperature: tuple = (0.0, 0), workspace: torch.Tensor | None = None) -> None:
     """Single query rows q (rows, H, width) over ``cache`` (blocks, block_size, G, width), whose rows are keys and, in their first
-    columns, values: out (rows, H, width, or 512 of 576).  ``lens`` int64 (rows,): position + 1; ``ring``: token p lies at place
+    columns, values: out (rows, H, width, or 512 of 576).  Cached rows wider than q hold a value of out's width behind the key.
+    ``lens`` int64 (rows,): position + 1; ``ring``: token p lies at place
     p mod ring of row ``row_entry[row]`` of ``block_tables`` (0: at place p).  Everything else as in ``window_prefill``."""
     _C.require_cuda(out, q, cache, block_tables, row_entry, lens, gate, slopes, workspace)
     rows, heads, width = q.shape
-    if cache.dim() != 4 or cache.shape[3] != width or cache.dtype != q.dtype or not cache.is_contiguous():
-        raise ValueError(f"cache must be contiguous (blocks, block_size, kv heads, {width}) in q's dtype")
+    split = cache.dim() == 4 and cache.shape[3] > width
+    if cache.dim() != 4 or cache.shape[3] != width + split * out.shape[2] or cache.dtype != q.dtype or not cache.is_contiguous():
+        raise ValueError(f"cache must be contiguous (blocks, block_size, kv heads, {width} or that and the values' width) in q's dtype")
     if block_tables.dtype != torch.int32 or block_tables.dim() != 2 or not block_tables.is_contiguous():
         raise ValueError("block_tables must be contiguous int32 (entries, width)")
     if row_entry.dtype != torch.int32 or row_entry.numel() < rows or not row_entry.is_contiguous():
@@ -195,12 +206,13 @@ def window_decode(out: torch.Tensor, q: torch.Tensor, cache: torch.Tensor, block
     _index(lens, rows, "lens")
     _floats("slopes", slopes, heads)
     groups, block_size, values, most = cache.shape[2], cache.shape[1], out.shape[2], block_tables.shape[1]
-    need = window_decode_workspace_bytes(rows, heads, groups, width, values, most * block_size, q.dtype)
+    need = window_decode_workspace_bytes(rows, heads, groups, cache.shape[3], values, most * block_size, q.dtype)
     if need and (workspace is None or workspace.numel() < need):
         workspace = torch.empty(need, dtype=torch.uint8, device=q.device)
-    st = _C.load().mvllm_window_decode(
+    lib = _C.load()
+    st = (lib.mvllm_window_decode_split if split else lib.mvllm_window_decode)(
         _ptr(out), *_heads("out", out, q, rows, heads, 1), _ptr(q), *_heads("q", q, q, rows, heads, width), _ptr(cache),
-        _ptr(block_tables), most, _ptr(row_entry), _ptr(lens), _ptr(slopes), _ptr(gate), *_heads("gate", gate, q, rows, heads, values),
+        _ptr(block_tables), most, _ptr(row_entry), _ptr(lens), _ptr(slopes), _ptr(gate), *_gate(gate, q, rows, heads, values),
         rows, heads, groups, width, values, block_size, cache.shape[0], int(window), int(ring), float(scale), float(temperature[0]),
         float(temperature[1]), _C.dtype_code(q.dtype), _ptr(workspace), 0 if workspace is None else workspace.numel(),
         _C.current_stream_ptr(q.device))

@@ -70,9 +70,26 @@ def _fevosun_sources(config):
     return kernel_sources(config)
 
 
+def _lenuzen_runner(config):
+    from minivllm_amd.engine.hybrid_runner import HybridModelRunner
+    from minivllm_amd.models.lenuzen import LenuzenForCausalLM
+    return HybridModelRunner(config, LenuzenForCausalLM)
+
+
+def _lenuzen_normalize(config):
+    from minivllm_amd.models.lenuzen import engine_config
+    return engine_config(config)
+
+
+def _lenuzen_sources(config):
+    from minivllm_amd.models.lenuzen import kernel_sources
+    return kernel_sources(config)
+
+
 DESIGNS = {"Qwen3": Design(_qwen3_runner), "Sokevik": Design(_sokevik_runner, _sokevik_normalize, _sokevik_sources),
            "Niridra": Design(_niridra_runner, _niridra_normalize, _niridra_sources),
-           "Fevosun": Design(_fevosun_runner, _fevosun_normalize, _fevosun_sources)}
+           "Fevosun": Design(_fevosun_runner, _fevosun_normalize, _fevosun_sources),
+           "Lenuzen": Design(_lenuzen_runner, _lenuzen_normalize, _lenuzen_sources)}
 
 
 def design_of(config: dict) -> Design:

@@ -41,6 +41,8 @@ def test_header_declares_expected_entry_points():
               "mvllm_moe_plan", "mvllm_moe_plan_bytes", "mvllm_moe_linear",
               "mvllm_moe_route_softmax", "mvllm_moe_linear_clamped", "mvllm_gated_unit", "mvllm_stream_norm_identity", "mvllm_window_prefill",
               "mvllm_window_decode_workspace_bytes", "mvllm_window_decode", "mvllm_latent_rope_store", "mvllm_head_rope", "mvllm_copy_rows",
+              "mvllm_head_norm_rope_store", "mvllm_window_decode_split", "mvllm_gelu_tanh", "mvllm_linear_small_m_gelu",
+              "mvllm_post_norm", "mvllm_embed_rows", "mvllm_talk_prefill", "mvllm_talk_decode", "mvllm_talk_decode_workspace_bytes",
               "mvllm_silu_and_mul", "mvllm_version", "mvllm_status_string"]:
         assert n in names
 
