@@ -38,7 +38,7 @@ def parse_args():
     ap.add_argument("--warmup", type=int, default=5)
     ap.add_argument("--seed", type=int, default=0)
     ap.add_argument("--block-size", type=int, default=16, help="block size of the headline decode workload")
-    ap.add_argument("--only", default="", help="comma list out of decode256,prefill,prefill_long,store,int8,reference_shapes,decode_small,demo_shape,head_dims,fused_qk,sampler,mfma_probe,prefill_timeline,loads_probe,engine,engine16,engine64,cpu to restrict the extras (the headline decode always runs); only when named: sokevik, the Sokevik design beside the Qwen3-style decoder, models and kernels (sokevik_kernels: kernels alone), niridra, the Niridra design beside Sokevik (niridra_kernels), fevosun, the Fevosun design beside Niridra (fevosun_kernels)")
+    ap.add_argument("--only", default="", help="comma list out of decode256,prefill,prefill_long,store,int8,reference_shapes,decode_small,demo_shape,head_dims,fused_qk,sampler,mfma_probe,prefill_timeline,loads_probe,engine,engine16,engine64,cpu to restrict the extras (the headline decode always runs); only when named: sokevik, the Sokevik design beside the Qwen3-style decoder, models and kernels (sokevik_kernels: kernels alone), niridra, the Niridra design beside Sokevik (niridra_kernels), fevosun, the Fevosun design beside Niridra (fevosun_kernels), lenuzen, the Lenuzen design beside the Qwen3-style decoder (lenuzen_kernels)")
     ap.add_argument("--no-cpu", action="store_true", help="skip the cpu_baseline leg")
     ap.add_argument("--calib-copy", action="store_true",
                     help="also launch three 1 GiB device copies (reads 1 GiB, writes 1 GiB each) so a rocprofv3 "
@@ -1482,6 +1482,144 @@ def bench_fevosun_kernels(args, rows, calls):
         lambda: stream_norm(xs, plain, one, one[None], gains, 1e-6), "stream_norm (experts)", moved + all_pairs * (2 * width + 8))
     return res
 
+
+LENUZEN_WINDOW = 1024                                      # of the sliding windows and of the chunks
+
+
+def lenuzen_model(size):
+    """Lenuzen with its two mixers in turn, of the width, heads and layers of the Qwen3-style decoder of ``sokevik_models`` and a
+    feed-forward of as many weights (two matrices instead of three)."""
+    z = SOKEVIK_SIZES[size]
+    rot = {"base": 500000.0, "dims": 128, "scaling": {"factor": 8.0, "fast": 32.0, "slow": 1.0, "original": 4096}}
+    m = {"heads": z["heads"], "kv_heads": z["kv"], "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": LENUZEN_WINDOW}, "rot": rot}
+    mlp = {"kind": "dense", "ff": 3 * z["ff"] // 2}
+    return {"architecture": "Lenuzen", "width": z["width"], "vocab": 32000, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0}, "logit_scale": 1.0,
+            "layers": [{"type": ("attention", "attention_2")[i % 2], "mixer": m, "mlp": mlp} for i in range(z["layers"])]}
+
+
+def bench_lenuzen(args, with_models=True):
+    """The Lenuzen design beside the Qwen3-style decoder, the nearest other design (grouped heads, dense feed-forwards), at equal
+    width, heads, layers and weights: whole-engine throughput, and every kernel beside the like kernel."""
+    import torch
+    out = {"models": {}, "kernels": {}}
+    for size in SOKEVIK_SIZES if with_models else ():
+        for prompts, prompt_len, new in ((4, 2048, 128), (32, 512, 128), (1, 16384, 64)):
+            leg = {}
+            for name, config in (("lenuzen", lenuzen_model(size)), ("qwen3", sokevik_models(size)[1])):
+                leg[name] = engine_throughput(args, config, prompts, prompt_len, new)
+                torch.cuda.empty_cache()
+            out["models"][f"{size}_{prompts}x{prompt_len}+{new}"] = leg
+            print(f"{size} {prompts}x{prompt_len}+{new}: {leg}", file=sys.stderr, flush=True)
+    for rows, calls in ((8192, 4), (64, 20)):
+        with torch.inference_mode():
+            out["kernels"][f"{rows}_rows"] = bench_lenuzen_kernels(args, rows, calls)
+        torch.cuda.empty_cache()
+    return out
+
+
+def bench_lenuzen_kernels(args, rows, calls):
+    """Kernels at width 4096 (mixed heads also at the 16 / 8 heads of width 2048): 8192 prompt rows (8 prompts of 1024, or one), or
+    64 decoded rows (attention: 256 sequences, or 16, of 1024 tokens)."""
+    import torch
+    from minivllm_amd.engine.hybrid_cache import HybridCacheManager
+    from minivllm_amd.engine.ragged import ragged_step
+    from minivllm_amd.engine.sequence import Sequence
+    from minivllm_amd.engine.windows import SlidingWindow
+    from minivllm_amd.layers.attention import flash_attention_prefill, paged_attention_decode
+    from minivllm_amd.layers.basic import RotaryEmbedding, rotary_pair_table
+    from minivllm_amd.layers.fused import add_rms_norm, gelu_tanh, head_rope_store, linear_small_m, post_norm, qk_norm_rope_store, silu_and_mul
+    from minivllm_amd.layers.talk import talk_decode, talk_prefill
+    from minivllm_amd.layers.window import window_decode, window_prefill
+
+    dev = torch.device("cuda:0")
+    gen = torch.Generator(device=dev).manual_seed(args.seed)
+    rnd = lambda *shape, dtype=torch.bfloat16: torch.randn(*shape, generator=gen, device=dev).to(dtype)
+    prefill = rows > 64
+    width, hq, hkv, d, window, bs, ff = 4096, 32, 8, 128, LENUZEN_WINDOW, 16, 3 * SOKEVIK_SIZES["w4096"]["ff"] // 2
+    views = [window, SlidingWindow(window)]
+
+    def step_of(lengths, before):
+        m = HybridCacheManager(views, sum(-(-min(n + p, views[1].places) // bs) for n, p in zip(lengths, before)), bs, len(lengths))
+        seqs = []
+        for n, p0 in zip(lengths, before):
+            q = Sequence([0] * (p0 + n), block_size=bs)
+            m.allocate(q)
+            q.num_computed_tokens, q.num_scheduled_tokens = p0, n
+            seqs.append(q)
+        return ragged_step(seqs, views, bs, dev), len(m.pools[0].blocks)
+
+    lengths = [window] * (rows // window) if prefill else [1] * rows
+    step, blocks = step_of(lengths, [0] * len(lengths) if prefill else [window - 1] * rows)
+    chunk, ring = step.windows
+    res = {}
+    leg = kernel_legs(args, res, calls)
+    scale, sinks = d ** -0.5, torch.zeros(hq, device=dev)
+    talk = lambda h: torch.eye(h, device=dev) + rnd(h, h).float() / 16
+
+    # ---- attention ----
+    if prefill:
+        pairs, cu = sum(n * (n + 1) // 2 for n in lengths), ring.cu_q
+        q, kv, gate, out = rnd(rows, hq, d), rnd(rows, hkv, 2 * d), rnd(rows, hq), torch.empty(rows, hq, d, dtype=torch.bfloat16, device=dev)
+        k, v = rnd(rows, hkv, d), rnd(rows, hkv, d)
+        moved, flops = rows * (2 * hq + 2 * hkv) * d * 2, 4.0 * hq * d * pairs
+        like = lambda: flash_attention_prefill(q, k, v, cu, scale, hq, hkv, d)
+        run = lambda c: window_prefill(out, q, kv[..., :d], c, c, scale, window, v=kv[..., d:], gate=gate)
+        leg("window_prefill", lambda: run(cu), moved, like, "packed prefill", moved, flops, flops)
+        whole = torch.tensor([0, rows], dtype=torch.int32, device=dev)
+        seen = window * (window + 1) // 2 + (rows - window) * window
+        leg("window_prefill_one_prompt", lambda: run(whole), moved, like, "packed prefill", moved, 4.0 * hq * d * seen, flops)
+        for h, g in ((hq, hkv), (16, 8)):
+            qh, kh, vh, oh, t = q[:, :h].contiguous(), k[:, :g].contiguous(), v[:, :g].contiguous(), out[:, :h].contiguous(), talk(h)
+            moved, s = rows * (2 * h + 2 * g) * d * 2, sinks[:h].contiguous()
+            leg(f"talk_prefill_{h}_{g}", lambda: talk_prefill(oh, qh, kh, vh, t, cu, sinks=s), moved,
+                lambda: flash_attention_prefill(qh, kh, vh, cu, scale, h, g, d, sink=s), "packed prefill with a sink", moved,
+                (4.0 * h * d + 2.0 * h * h) * pairs, 4.0 * h * d * pairs)
+        del q, kv, gate, out, k, v, qh, kh, vh, oh
+    else:
+        for name, batch in (("", 256), ("_16_rows", 16)):
+            st, n = step_of([1] * batch, [window - 1] * batch)
+            w, c = st.windows[1], st.windows[0]
+            cache, gate, q = rnd(n, bs, hkv, 2 * d), rnd(batch, hq), rnd(batch, hq, d)
+            kc, vc = rnd(n, bs, hkv, d), rnd(n, bs, hkv, d)
+            out = torch.empty(batch, hq, d, dtype=torch.bfloat16, device=dev)
+            nbytes = batch * (window * 2 * hkv * d * 2 + 2 * hq * d * 2 + 4 * window // bs)
+            like = lambda **kw: paged_attention_decode(q, kc, vc, c.decode_tables, c.chunk_lens, scale, hq, hkv, d, bs, **kw)
+            leg("window_decode" + name, lambda: window_decode(out, q, cache, w.tables, st.row_entry, w.lens, scale, window, views[1].places, gate=gate),
+                nbytes + batch * hq * 2, like, "paged decode", nbytes)
+            for h, g in ((hq, hkv), (16, 8)):
+                qh, kh, vh, oh, t, s = q[:, :h].contiguous(), kc[:, :, :g].contiguous(), vc[:, :, :g].contiguous(), out[:, :h].contiguous(), talk(h), sinks[:h].contiguous()
+                nbytes = batch * (window * 2 * g * d * 2 + 2 * h * d * 2 + 4 * window // bs)
+                leg(f"talk_decode_{h}_{g}{name}", lambda: talk_decode(oh, qh, kh, vh, c.decode_tables, c.chunk_lens, t, s), nbytes,
+                    lambda: paged_attention_decode(qh, kh, vh, c.decode_tables, c.chunk_lens, scale, h, g, d, bs, sink=s), "paged decode with a sink", nbytes)
+            del cache, kc, vc, kh, vh
+    # ---- in front of attention: norms, rotation, cache ----
+    cols = (hq + 2 * hkv) * d
+    proj, table = rnd(rows, cols + hq), rotary_pair_table(500000.0, d, 2048).to(dev)
+    rotary, one = RotaryEmbedding(1_000_000, d, 2048).to(dev), torch.ones(d, device=dev)
+    kc = torch.zeros(blocks, bs, hkv, d, dtype=torch.bfloat16, device=dev)
+    vc, both = torch.zeros_like(kc), torch.zeros(blocks, bs, hkv, 2 * d, dtype=torch.bfloat16, device=dev)
+    keys = torch.empty(rows, hkv, 2 * d, dtype=torch.bfloat16, device=dev) if prefill else None
+    moved = rows * (2 * cols + (hq + (4 if prefill else 2) * hkv) * d * 2 + 16)
+    q, k, v = proj[:, :hq * d].unflatten(-1, (hq, d)), proj[:, hq * d:(hq + hkv) * d].unflatten(-1, (hkv, d)), proj[:, (hq + hkv) * d:cols].unflatten(-1, (hkv, d))
+    like = lambda: qk_norm_rope_store(q, k, v, step.positions, rotary.cos_sin_cache, one, 1e-6, chunk.slots, kc, vc, need_kv=prefill)
+    factor, gain_q, gain_k = torch.ones(hq, device=dev), torch.ones(hq * d, device=dev), torch.ones(hkv * d, device=dev)
+    heads = lambda **kw: head_rope_store(proj, step.positions, hq, hkv, d, d, d, eps=1e-6, rot_table=table, **kw)
+    leg("head_norm_rope_store (unit heads)", lambda: heads(unit_qk=True, unit_v=True, head_scale=factor, kv_cache=both, slots=ring.slots, kv_out=keys,
+                                                           kv_rows=ring.key_rows), moved + rows * 8 * bool(prefill), like, "qk_norm_rope_store", moved)
+    leg("head_norm_rope_store (rows)", lambda: heads(gain_q=gain_q, gain_k=gain_k, row_norm=True, slots=chunk.slots, k_cache=kc, v_cache=vc, need_kv=prefill),
+        moved, like, "qk_norm_rope_store", moved)
+    # ---- behind the sublayers, between the feed-forward's products ----
+    x, y, z, gains = rnd(rows, width, dtype=torch.float32), rnd(rows, width), rnd(rows, width), torch.ones(width, device=dev)
+    leg("post_norm", lambda: post_norm(x, y, gains, 1e-6), rows * width * 12 + 4 * width, lambda: add_rms_norm(y, gains, 1e-6, z), "add_rms_norm", rows * width * 8)
+    act, wide = rnd(rows, ff), rnd(rows, 4 * ff // 3)
+    leg("gelu_tanh", lambda: gelu_tanh(act, out=act), rows * ff * 4, lambda: silu_and_mul(wide), "silu_and_mul", rows * 2 * ff // 3 * 6)
+    if not prefill:
+        w = rnd(ff, width)
+        nbytes = 2 * (ff * width + rows * width + rows * ff)
+        leg("linear_small_m with gelu", lambda: linear_small_m(y, w, None, True), nbytes, lambda: linear_small_m(y, w), "linear_small_m", nbytes)
+    return res
+
+
 def summary_of(line):
     """The figures of every quantity the metric names, in a few hundred characters, for the end of the JSON line."""
     ex = line["extra"]
@@ -1597,6 +1735,10 @@ def main():
         extra["fevosun"] = bench_fevosun(args)
     elif "fevosun_kernels" in only:
         extra["fevosun"] = bench_fevosun(args, with_models=False)
+    if "lenuzen" in only:
+        extra["lenuzen"] = bench_lenuzen(args)
+    elif "lenuzen_kernels" in only:
+        extra["lenuzen"] = bench_lenuzen(args, with_models=False)
 
     if "loads_only" in head:
         extra["decode_loads_only"] = head["loads_only"]

@@ -26,13 +26,16 @@ struct TalkArgs {
   float2* part_ml;            // [rows, parts, heads]: maximum (base 2), sum
   int64_t out_row, out_head, total_q, num_blocks;
   int num_seqs, heads, kv_heads, dim, table_width, block_size, parts;
-  int tiles_x, heads_y, band_bits, band_shift;     // the tiled prefill's item order
+  // the tiled prefill, filled in by its launcher: item order; query heads per kv head, pieces of them and 65536 / pieces_per_kv + 1
+  int tiles_x, heads_y, band_bits, band_shift, per, pieces, pieces_per_kv;
+  unsigned piece_magic;
 };
 
-// Heads in fours that share a kv head: what one wave makes raw scores of, and a 16-byte entry of the scores in LDS.
+// Heads, `most` at a time, that share a kv head: what one wave makes raw scores of.
 struct TalkPieces {
   int per_kv, count;
-  __host__ __device__ TalkPieces(int heads, int kv_heads) : per_kv((heads / kv_heads + 3) / 4), count(kv_heads * ((heads / kv_heads + 3) / 4)) {}
+  __host__ __device__ TalkPieces(int heads, int kv_heads, int most)
+      : per_kv((heads / kv_heads + most - 1) / most), count(kv_heads * ((heads / kv_heads + most - 1) / most)) {}
 };
 
 int launch_talk_prefill(const TalkArgs& a, hipStream_t stream);      // talk_prefill.hip; kNotBuilt where it takes nothing
