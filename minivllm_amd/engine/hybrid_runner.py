@@ -1,6 +1,6 @@
 """Runner of models that run ragged steps and keep recurrent state (models/sokevik.py, models/niridra.py, models/fevosun.py,
-models/lenuzen.py): portions of prompts and decoded tokens in one batch, a cache manager of its own, and the captured decode step of ``ModelRunner`` over
-more static buffers.
+models/lenuzen.py): portions of prompts and decoded tokens in one batch, a cache manager of its own, and the captured decode step
+of ``ModelRunner`` over more static buffers.
 
 Engine keys as for ``ModelRunner``; ``max_cached_blocks`` counts the blocks of each attention window's pool,
 ``max_num_sequences`` the slots of recurrent state, ``model_dir`` names a checkpoint folder (absent: random weights)."""

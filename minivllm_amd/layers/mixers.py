@@ -4,9 +4,9 @@ memories.
 ``RaggedAttention`` runs a step's pieces through the framework's decode, paged-prefill and packed-prefill kernels,
 ``LatentAttention`` through the latent decode and the same prefill kernels, ``SharedKeyAttention``, ``RotaryLatentAttention`` and
 ``UnitHeadAttention`` through the windowed kernels, ``TalkingAttention`` through the ones that mix heads' scores;
-``MatrixMemory`` runs it through the mLSTM recurrence, ``DecayMemory`` through the one with constant decays.  ``RaggedAttention`` and the memories take the packed
-projection of the step's rows and return what the output projection reads.  Caches and states are assigned from outside, as
-for ``layers.attention.Attention``."""
+``MatrixMemory`` runs it through the mLSTM recurrence, ``DecayMemory`` through the one with constant decays.  ``RaggedAttention``
+and the memories take the packed projection of the step's rows and return what the output projection reads.  Caches and states
+are assigned from outside, as for ``layers.attention.Attention``."""
 from __future__ import annotations
 
 import math

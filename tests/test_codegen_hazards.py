@@ -59,7 +59,7 @@ def test_checker_flags_a_bare_read_and_accepts_a_guarded_one():
 
 
 @pytest.mark.skipif(shutil.which("hipcc") is None, reason="hipcc not installed")
-@pytest.mark.parametrize("source,least", [("prefill_varlen.hip", 500), ("window_prefill.hip", 120), ("window_prefill_latent.hip", 240)])
+@pytest.mark.parametrize("source,least", [("prefill_varlen.hip", 500), ("window_prefill.hip", 120), ("window_prefill_latent.hip", 240), ("window_prefill_heads.hip", 120)])
 def test_prefill_kernel_has_no_asm_read_inside_mfma_latency(tmp_path, source, least):
     from minivllm_amd._build import HIPCC_FLAGS
     out = tmp_path / "prefill.s"
